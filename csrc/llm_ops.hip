@@ -31,6 +31,7 @@
 #include <cstdlib>
 
 #include "common.h"
+#include "gemm_tile.h"
 
 // ====================================================================
 // GEMV: y[N] = W[N,K] @ stage(x)[K]  (+ res)  (optional softcap, f32 out)
@@ -2552,10 +2553,7 @@ extern "C" hipError_t launch_sample(const void* logits, int V, int lbf16,
 
 // ====================================================================
 // Prefill GEMM: Y[M,N] = X[M,K] @ W[N,K]^T (+res), bf16 in/out, fp32 acc.
-// MFMA v_mfma_f32_16x16x32_bf16; 128x128 tile, BK=32, 4 waves (2x2),
-// each wave a 64x64 sub-tile (4x4 fragments).  LDS staged, padded rows.
-// Correctness-first structure (guide §5 ladder step ~0-2); prefill only —
-// decode uses k_gemv_bf16.
+// MFMA v_mfma_f32_16x16x32_bf16; prefill only — decode uses k_gemv_bf16.
 // ====================================================================
 
 typedef short bf16x8 __attribute__((ext_vector_type(8)));
@@ -2565,33 +2563,17 @@ typedef float f32x4 __attribute__((ext_vector_type(4)));
 #define BN 128
 #define BK 64
 
-// TS=BM=BN tile template (128 or 64), BK=64, 4 waves (2x2), each wave
-// a (TS/2)^2 sub-tile of 16x16 fragments.  Double-buffered LDS filled
-// by global_load_lds (async global->LDS DMA, 16 B/lane), one barrier
-// per K-tile (guide §5 "Minimum 2-phase": STAGE next ahead of
-// ds_read+MFMA).  LDS rows are XOR-swizzled st_8x16 (slot ^= row&7) so
-// ds_read_b128 fragment reads stay conflict-free; glds writes
-// lane-linear, so the swizzle is applied to the per-lane GLOBAL source
-// address (guide §5.4 rule 21) and to the read offsets — never the LDS
-// dest.  The 64-tile variant exists because M=N=2048-class prefill
-// GEMMs give the 128-tile only ~256 blocks = 1 block/CU — no occupancy
-// to hide the DMA/barrier latency (measured 250 TF; see
-// profiles/prefill_gemm_r02.md).
+// TS=BM=BN tile (128 or 64) over the shared MFMA main loop (gemm_tile.h).
+// The 64-tile variant exists because M=N=2048-class prefill GEMMs give
+// the 128-tile only ~256 blocks = 1 block/CU — no occupancy to hide the
+// DMA/barrier latency (measured 250 TF; see profiles/prefill_gemm_r02.md).
 template <int TS>
 __global__ void __launch_bounds__(256)
 k_gemm_bf16_t(const u16* __restrict__ X, const u16* __restrict__ W,
               u16* __restrict__ Y, const u16* __restrict__ res,
               float* __restrict__ accbuf, int M, int N, int K) {
-  constexpr int F = TS / 32;        // 16x16 frags per wave dim
-  constexpr int SUB = TS / 2;       // wave sub-tile span
-  __shared__ u16 As[2][TS * 64];
-  __shared__ u16 Bs[2][TS * 64];
-
-  const int tid = threadIdx.x;
-  const int wave = tid >> 6, lane = tid & 63;
-  const int wrow = wave >> 1, wcol = wave & 1;  // 2x2 waves
+  __shared__ __attribute__((aligned(16))) char lds[gemm_lds_bytes<TS, TS>()];
   const int bm = blockIdx.x * TS, bn = blockIdx.y * TS;
-
   const int SK = gridDim.z;
   const int kslices = (K / BK + SK - 1) / SK;
   const int k_lo = blockIdx.z * kslices * BK;
@@ -2600,81 +2582,20 @@ k_gemm_bf16_t(const u16* __restrict__ X, const u16* __restrict__ W,
   const int nt = (k_hi - k_lo) / BK;
   if (nt <= 0) return;
 
-  f4v acc[F][F];
-#pragma unroll
-  for (int i = 0; i < F; i++)
-#pragma unroll
-    for (int j = 0; j < F; j++) acc[i][j] = {0.f, 0.f, 0.f, 0.f};
+  f4v acc[TS / 32][TS / 32];
+  gemm_mainloop<TS, TS, u16>(
+      acc, lds,
+      [&](int r) { return X + (size_t)min(bm + r, M - 1) * K; },
+      [&](int r) { return W + (size_t)min(bn + r, N - 1) * K; }, k_lo, nt);
 
-  // glds staging: per call a wave fills 8 rows x 128 B (lane: row
-  // lane/8, slot lane%8); source col-slot pre-swizzled by row&7.
-  const int g_r = lane >> 3;             // row within the 8-row group
-  const int g_s = lane & 7;              // LDS slot
-  auto stage = [&](int buf, int kt) {
-    const int k0 = k_lo + kt * BK;
 #pragma unroll
-    for (int i = 0; i < TS / 32; i++) {
-      int r = wave * (TS / 4) + i * 8 + g_r;   // tile row 0..TS-1
-      int cs = g_s ^ (r & 7);            // source col-slot (involution)
-      int gr = bm + r;
-      int grc = gr < M ? gr : (M > 0 ? M - 1 : 0);
-      __builtin_amdgcn_global_load_lds(
-          (const __attribute__((address_space(1))) uint32_t*)(
-              X + (size_t)grc * K + k0 + cs * 8),
-          (__attribute__((address_space(3))) uint32_t*)(
-              &As[buf][(wave * (TS / 4) + i * 8) * 64]),
-          16, 0, 0);
-      int gb = bn + r;
-      int gbc = gb < N ? gb : N - 1;
-      __builtin_amdgcn_global_load_lds(
-          (const __attribute__((address_space(1))) uint32_t*)(
-              W + (size_t)gbc * K + k0 + cs * 8),
-          (__attribute__((address_space(3))) uint32_t*)(
-              &Bs[buf][(wave * (TS / 4) + i * 8) * 64]),
-          16, 0, 0);
-    }
-  };
-
-  stage(0, 0);
-  __syncthreads();
-
-  const int fr = lane & 15, fk = lane >> 4;  // fragment row / k-slot
-  int cur = 0;
-  for (int t = 0; t < nt; t++) {
-    if (t + 1 < nt) stage(cur ^ 1, t + 1);   // issue next tile's DMA
+  for (int i = 0; i < TS / 32; i++) {
 #pragma unroll
-    for (int sl = 0; sl < 2; sl++) {         // two 32-deep k-slices
-      bf16x8 a[F], b[F];
-#pragma unroll
-      for (int i = 0; i < F; i++) {
-        int ra = wrow * SUB + i * 16 + fr;
-        int sa = (sl * 4 + fk) ^ (ra & 7);
-        a[i] = *(bf16x8*)(&As[cur][ra * 64 + sa * 8]);
-        int rb = wcol * SUB + i * 16 + fr;
-        int sb = (sl * 4 + fk) ^ (rb & 7);
-        b[i] = *(bf16x8*)(&Bs[cur][rb * 64 + sb * 8]);
-      }
-#pragma unroll
-      for (int i = 0; i < F; i++)
-#pragma unroll
-        for (int j = 0; j < F; j++)
-          acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-              a[i], b[j], acc[i][j], 0, 0, 0);
-    }
-    __syncthreads();  // drains the in-flight DMA (vmcnt0) + read fence
-    cur ^= 1;
-  }
-
-  // epilogue: C layout col = lane&15, row = (lane>>4)*4 + reg
-  const int cc = lane & 15, cr = (lane >> 4) * 4;
-#pragma unroll
-  for (int i = 0; i < F; i++) {
-#pragma unroll
-    for (int j = 0; j < F; j++) {
+    for (int j = 0; j < TS / 32; j++) {
+      const int col = bn + gemm_col<TS>(j);
 #pragma unroll
       for (int r = 0; r < 4; r++) {
-        int row = bm + wrow * SUB + i * 16 + cr + r;
-        int col = bn + wcol * SUB + j * 16 + cc;
+        const int row = bm + gemm_row0<TS>(i) + r;
         if (row < M && col < N) {
           float v = acc[i][j][r];
           if (SK > 1) {

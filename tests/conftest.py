@@ -10,7 +10,9 @@ sys.path.insert(0, os.path.dirname(os.path.dirname(os.path.abspath(__file__))))
 # serialize them into a deadlock.  Must be set before HIP runtime init
 # (conftest imports before any CUDA call).  Real TP runs one process
 # per GPU and needs no such setting.
-os.environ.setdefault("GPU_MAX_HW_QUEUES", "10")
+# An environment that presets a smaller number is raised too.
+if int(os.environ.get("GPU_MAX_HW_QUEUES") or 0) < 10:
+    os.environ["GPU_MAX_HW_QUEUES"] = "10"
 
 
 def pytest_configure(config):
