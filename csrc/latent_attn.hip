@@ -1,0 +1,508 @@
+// latent_attn.hip — attention over a paged cache of latents.
+//
+// A cached token is one row [c (rank, zero-padded to RP) | rotated key part
+// (padded to RT)]; page p of a sequence holds positions 64p .. 64p+63.
+// Scores and outputs stay in latent space: the per-head up-projection of
+// the keys is folded into the query (q' = W_uk^T q), so every head reads
+// the same rows, and the value up-projection is applied to the attended
+// latent.  A query tile is 16 (token, head) pairs of one sequence.
+#include "gemm_tile.h"
+#include "hybrid.h"
+#include "moe.h"
+
+#define PAGE 64
+
+struct LatentArgs {
+  const float* P;        // fp32 projections [rows, ldp]
+  const void* Wuk;       // [H*d, RP]
+  const void* Wuv;       // [H*vd, RP]
+  const float* cnorm;    // [rank]
+  const float *cosT, *sinT;   // [positions, rdims/2]
+  const int *slot, *pos; // per row
+  const int* table;      // [slots, ldt] page numbers
+  void* cache;           // [pages, 64, RP+RT]
+  void* qn;              // [rows, H, dp]      (GEMM path)
+  void* qa;              // [rows, H, RP+RT]
+  float *part, *ml;      // split partials [NS, rows*H, RP], [NS, rows*H, 2]
+  void* olat;            // [rows, H, RP]
+  void* o;               // [rows, ldo]
+  const int *seg_row0, *seg_len, *seg_slot, *seg_pos0;
+  const int *tile_seg, *tile_rr0;    // null: one-token segments
+  int* ridx;             // router outputs (rows * (rtop + rextra))
+  float* rwt;
+  int ldp, oq, odkv, og, orouter;
+  int H, d, dp, rot, rdims, RT, rank, RP, vd, ldo, ldt;
+  int rows, rbase, NS;   // rows [rbase, rbase+rows) take part in the split
+  int E, rtop, rextra;
+  float eps, scale;
+};
+
+// element i (< rot) of the rotated part of v at position p
+DEVINL float rotated(const float* v, int i, int dims, const float* c,
+                     const float* s) {
+  const int half = dims >> 1;
+  if (i >= dims) return v[i];
+  if (i < half) return v[i] * c[i] - v[i + half] * s[i];
+  return v[i] * c[i - half] + v[i - half] * s[i - half];
+}
+
+// normed latent and rotated key part of one row -> its cache row
+template <typename T>
+DEVINL void latent_write(const LatentArgs& a, int r, float* red) {
+  const float* p = a.P + (size_t)r * a.ldp + a.odkv;
+  const int pos = a.pos[r], CS = a.RP + a.RT;
+  const int page = a.table[(size_t)a.slot[r] * a.ldt + pos / PAGE];
+  T* dst = (T*)a.cache + ((size_t)page * PAGE + pos % PAGE) * CS;
+  const float* c = a.cosT + (size_t)pos * (a.rdims >> 1);
+  const float* s = a.sinT + (size_t)pos * (a.rdims >> 1);
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < a.rank; i += blockDim.x) ss += p[i] * p[i];
+  const float rn = 1.f / sqrtf(block_sum(ss, red) / (float)a.rank + a.eps);
+  for (int i = threadIdx.x; i < CS; i += blockDim.x) {
+    float v = 0.f;
+    if (i < a.rank) v = p[i] * rn * a.cnorm[i];
+    else if (i >= a.RP && i < a.RP + a.rot)
+      v = rotated(p + a.rank, i - a.RP, a.rdims, c, s);
+    dst[i] = El<T>::st(v);
+  }
+}
+
+DEVINL void route_from_proj(const float* P, int ldp, int orouter, int E,
+                            int top, int extra, int* ridx, float* rwt, int r) {
+  const float* z = P + (size_t)r * ldp + orouter;
+  const int k1 = top + extra;
+  if (E <= 64) route_row<1>(z, E, top, extra, ridx + r * k1, rwt + r * k1);
+  else route_row<16>(z, E, top, extra, ridx + r * k1, rwt + r * k1);
+}
+
+// ---- many rows: split q, rotate, write the cache, route ----------------
+template <typename T>
+__global__ void __launch_bounds__(256) k_latent_prep(LatentArgs a) {
+  __shared__ float red[4];
+  const int r = blockIdx.x;
+  const float* q = a.P + (size_t)r * a.ldp + a.oq;
+  const int pos = a.pos[r], dq = a.d + a.rot, CS = a.RP + a.RT;
+  const float* c = a.cosT + (size_t)pos * (a.rdims >> 1);
+  const float* s = a.sinT + (size_t)pos * (a.rdims >> 1);
+  T* qn = (T*)a.qn + (size_t)r * a.H * a.dp;
+  for (int i = threadIdx.x; i < a.H * a.dp; i += 256) {
+    int h = i / a.dp, j = i - h * a.dp;
+    qn[i] = El<T>::st(j < a.d ? q[h * dq + j] : 0.f);
+  }
+  T* qa = (T*)a.qa + (size_t)r * a.H * CS;
+  for (int i = threadIdx.x; i < a.H * a.RT; i += 256) {
+    int h = i / a.RT, j = i - h * a.RT;
+    qa[(size_t)h * CS + a.RP + j] = El<T>::st(
+        j < a.rot ? rotated(q + h * dq + a.d, j, a.rdims, c, s) : 0.f);
+  }
+  latent_write<T>(a, r, red);
+  if (a.E > 0 && threadIdx.x < 64)
+    route_from_proj(a.P, a.ldp, a.orouter, a.E, a.rtop, a.rextra, a.ridx,
+                    a.rwt, r);
+}
+
+// ---- few rows: absorb W_uk per (head, row); one more block per row does
+// ---- the cache row and the routing ------------------------------------
+template <typename T>
+__global__ void __launch_bounds__(256) k_latent_dec_prep(LatentArgs a) {
+  __shared__ float red[256 * 8 + 256];
+  const int h = blockIdx.x, r = blockIdx.y;
+  if (h == a.H) {
+    latent_write<T>(a, r, red);
+    if (a.E > 0 && threadIdx.x < 64)
+      route_from_proj(a.P, a.ldp, a.orouter, a.E, a.rtop, a.rextra, a.ridx,
+                      a.rwt, r);
+    return;
+  }
+  constexpr int V = El<T>::V;
+  const int dq = a.d + a.rot, CS = a.RP + a.RT, pos = a.pos[r];
+  const float* q = a.P + (size_t)r * a.ldp + a.oq + (size_t)h * dq;
+  T* qa = (T*)a.qa + ((size_t)r * a.H + h) * CS;
+  // lanes own V latent columns each; the d axis is split over the groups
+  const int nv = a.RP / V, tid = threadIdx.x;
+  const int groups = 256 / nv;           // RP <= 512 (bf16) / 512 (fp32)
+  const int grp = tid / nv, cv = tid - grp * nv;
+  float acc[V];
+#pragma unroll
+  for (int j = 0; j < V; j++) acc[j] = 0.f;
+  if (grp < groups) {
+    const T* w = (const T*)a.Wuk + (size_t)h * a.d * a.RP + cv * V;
+#pragma unroll 4
+    for (int i = grp; i < a.d; i += groups) {
+      union { f4v f; T t[V]; } u;
+      u.f = ld16(w + (size_t)i * a.RP);
+      const float qi = El<T>::ld(El<T>::st(q[i]));
+#pragma unroll
+      for (int j = 0; j < V; j++) acc[j] = fmaf(qi, El<T>::ld(u.t[j]), acc[j]);
+    }
+#pragma unroll
+    for (int j = 0; j < V; j++) red[(grp * nv + cv) * V + j] = acc[j];
+  }
+  __syncthreads();
+  for (int i = tid; i < a.RP; i += 256) {
+    float v = 0.f;
+    for (int g = 0; g < groups; g++) v += red[g * a.RP + i];
+    qa[i] = El<T>::st(v);
+  }
+  const float* c = a.cosT + (size_t)pos * (a.rdims >> 1);
+  const float* s = a.sinT + (size_t)pos * (a.rdims >> 1);
+  for (int j = tid; j < a.RT; j += 256)
+    qa[a.RP + j] = El<T>::st(
+        j < a.rot ? rotated(q + a.d, j, a.rdims, c, s) : 0.f);
+}
+
+// ---- attention --------------------------------------------------------
+// S^T = K Q^T keeps a query's statistics in the lanes of its column; the
+// PV product accumulates O^T = V^T P^T from the same rows' first RP
+// columns.  bf16 keeps a transposed copy of the latent columns in LDS, in
+// the key order in which P^T leaves the score MFMA.
+#define KT 32
+
+template <typename T, int RP> struct AttnShape {
+  static constexpr int NC = RP * sizeof(T) / 64;        // latent chunks
+  static constexpr int NRM = 128 * sizeof(T) / 64;      // rotated, at most
+  static constexpr int VS = KT + 8;                     // V^T row stride
+};
+
+template <typename T>
+static size_t attn_lds(int RP, int RT) {
+  size_t b = (size_t)KT * ((RP + RT) * sizeof(T) + 16);
+  if (sizeof(T) == 2) b += (size_t)RP * (KT + 8) * 2;
+  return b;
+}
+
+template <typename T, int RP, int NW>
+__global__ void __launch_bounds__(64 * NW) k_latent_attn(LatentArgs a) {
+  using Sh = AttnShape<T, RP>;
+  extern __shared__ __attribute__((aligned(16))) char smem[];
+  const int CS = RP + a.RT;
+  const int KB = CS * (int)sizeof(T) + 16;              // K row bytes in LDS
+  char* kl = smem;
+  u16* vt = (u16*)(smem + (size_t)KT * KB);
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  const int qc = lane & 15, g = lane >> 4;
+  int seg, rr0;
+  if (a.tile_seg) {
+    seg = a.tile_seg[blockIdx.x];
+    rr0 = a.tile_rr0[blockIdx.x];
+  } else {
+    const int nth = (a.H + 16 * NW - 1) / (16 * NW);
+    seg = blockIdx.x / nth;
+    rr0 = (blockIdx.x - seg * nth) * 16 * NW;
+  }
+  const int row0 = a.seg_row0[seg], pos0 = a.seg_pos0[seg];
+  const int nrr = a.seg_len[seg] * a.H;
+  const int* pages = a.table + (size_t)a.seg_slot[seg] * a.ldt;
+  const int my = rr0 + wave * 16 + qc;
+  const int myc = my < nrr ? my : nrr - 1;
+  const int qpos = pos0 + myc / a.H;
+  const int last = min(rr0 + 16 * NW, nrr) - 1;
+  const int kend = pos0 + last / a.H + 1;               // keys [0, kend)
+  // key tiles of this split
+  const int ntile = (kend + KT - 1) / KT;
+  const int per = (ntile + a.NS - 1) / a.NS;
+  const int t_lo = blockIdx.y * per, t_hi = min(ntile, t_lo + per);
+
+  f4v qf[Sh::NC + Sh::NRM];
+  const int NR = a.RT * (int)sizeof(T) / 64;
+  {
+    const char* qp = (const char*)a.qa +
+                     ((size_t)row0 * a.H + myc) * CS * sizeof(T) + g * 16;
+#pragma unroll
+    for (int c = 0; c < Sh::NC; c++) qf[c] = ld16(qp + c * 64);
+#pragma unroll
+    for (int c = 0; c < Sh::NRM; c++)
+      if (c < NR) qf[Sh::NC + c] = ld16(qp + (Sh::NC + c) * 64);
+  }
+  f4v acc[RP / 16];
+#pragma unroll
+  for (int d = 0; d < RP / 16; d++) acc[d] = {0.f, 0.f, 0.f, 0.f};
+  float mrun = -INFINITY, lrun = 0.f;
+  const float sc = a.scale * 1.4426950408889634f;       // base-2 exponents
+
+  for (int t = t_lo; t < t_hi; t++) {
+    const int k0 = t * KT;
+    // rows past kend are stale or unwritten: read a valid row instead (the
+    // mask removes its score, and the value must stay finite)
+    const int nk = min(KT, kend - k0);
+    const char* src = (const char*)a.cache +
+        ((size_t)pages[k0 / PAGE] * PAGE + k0 % PAGE) * CS * sizeof(T);
+    if (NW > 1 || t > t_lo) __syncthreads();
+    {
+      // lanes take 16 row pairs x 16-byte columns
+      const int kp = tid & 15;
+      const int r0 = min(2 * kp, nk - 1), r1 = min(2 * kp + 1, nk - 1);
+      const int nvec = CS * (int)sizeof(T) / 16;
+      const int vpos = (kp < 8 ? (kp >> 1) * 8 : ((kp - 8) >> 1) * 8 + 4) +
+                       (kp & 1) * 2;
+      for (int cv = tid >> 4; cv < nvec; cv += NW * 4) {
+        f4v x0 = ld16(src + (size_t)r0 * CS * sizeof(T) + cv * 16);
+        f4v x1 = ld16(src + (size_t)r1 * CS * sizeof(T) + cv * 16);
+        *(f4v*)(kl + (2 * kp) * KB + cv * 16) = x0;
+        *(f4v*)(kl + (2 * kp + 1) * KB + cv * 16) = x1;
+        if (sizeof(T) == 2 && cv * 8 < RP) {
+          union { f4v f; uint32_t u[4]; } a0, a1;
+          a0.f = x0; a1.f = x1;
+#pragma unroll
+          for (int j = 0; j < 4; j++) {
+            *(uint32_t*)(vt + (cv * 8 + 2 * j) * Sh::VS + vpos) =
+                (a0.u[j] & 0xffffu) | (a1.u[j] << 16);
+            *(uint32_t*)(vt + (cv * 8 + 2 * j + 1) * Sh::VS + vpos) =
+                (a0.u[j] >> 16) | (a1.u[j] & 0xffff0000u);
+          }
+        }
+      }
+    }
+    __syncthreads();
+
+    f4v st[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+    const char* kr = kl + qc * KB + g * 16;
+#pragma unroll
+    for (int c = 0; c < Sh::NC; c++)
+#pragma unroll
+      for (int i = 0; i < 2; i++)
+        st[i] = GemmMma<T>::mma(ld16(kr + i * 16 * KB + c * 64), qf[c], st[i]);
+#pragma unroll
+    for (int c = 0; c < Sh::NRM; c++)
+      if (c < NR)
+#pragma unroll
+        for (int i = 0; i < 2; i++)
+          st[i] = GemmMma<T>::mma(ld16(kr + i * 16 * KB + (Sh::NC + c) * 64),
+                                  qf[Sh::NC + c], st[i]);
+    float sv[8], pmax = -INFINITY;
+#pragma unroll
+    for (int i = 0; i < 8; i++) {
+      const int key = k0 + (i >> 2) * 16 + g * 4 + (i & 3);
+      sv[i] = key <= qpos ? st[i >> 2][i & 3] * sc : -INFINITY;
+      pmax = fmaxf(pmax, sv[i]);
+    }
+    pmax = fmaxf(pmax, __shfl_xor(pmax, 16));
+    pmax = fmaxf(pmax, __shfl_xor(pmax, 32));
+    const float mnew = fmaxf(mrun, pmax);
+    const float base = mnew == -INFINITY ? 0.f : mnew;
+    const float alpha = exp2f(mrun - base);             // 0 while mrun = -inf
+    float psum = 0.f;
+#pragma unroll
+    for (int i = 0; i < 8; i++) {
+      sv[i] = exp2f(sv[i] - base);
+      psum += sv[i];
+    }
+    psum += __shfl_xor(psum, 16);
+    psum += __shfl_xor(psum, 32);
+    lrun = lrun * alpha + psum;
+    mrun = mnew;
+    if (__any(alpha != 1.f)) {
+#pragma unroll
+      for (int d = 0; d < RP / 16; d++)
+#pragma unroll
+        for (int j = 0; j < 4; j++) acc[d][j] *= alpha;
+    }
+    if constexpr (sizeof(T) == 2) {
+      union { f4v f; u16 h[8]; } p;
+#pragma unroll
+      for (int i = 0; i < 8; i++) p.h[i] = f2b(sv[i]);
+#pragma unroll
+      for (int d = 0; d < RP / 16; d++)
+        acc[d] = GemmMma<u16>::mma(
+            ld16(vt + (d * 16 + qc) * Sh::VS + g * 8), p.f, acc[d]);
+    } else {
+#pragma unroll
+      for (int d = 0; d < RP / 16; d++)
+#pragma unroll
+        for (int i = 0; i < 8; i++)
+          acc[d] = __builtin_amdgcn_mfma_f32_16x16x4f32(
+              *(const float*)(kl + ((i >> 2) * 16 + g * 4 + (i & 3)) * KB +
+                              (d * 16 + qc) * 4),
+              sv[i], acc[d], 0, 0, 0);
+    }
+  }
+
+  if (my >= nrr) return;
+  const size_t orow = (size_t)row0 * a.H + my;
+  if (a.NS == 1) {
+    const float inv = 1.f / lrun;
+    T* op = (T*)a.olat + orow * RP + g * 4;
+#pragma unroll
+    for (int d = 0; d < RP / 16; d++) {
+      union { T t[4]; uint64_t u; f4v f; } v;
+#pragma unroll
+      for (int j = 0; j < 4; j++) v.t[j] = El<T>::st(acc[d][j] * inv);
+      if constexpr (sizeof(T) == 2) *(uint64_t*)(op + d * 16) = v.u;
+      else *(f4v*)(op + d * 16) = v.f;
+    }
+  } else {
+    const size_t pr =
+        ((size_t)blockIdx.y * a.rows + row0 - a.rbase) * a.H + my;
+    if (g == 0) {
+      a.ml[pr * 2] = mrun;
+      a.ml[pr * 2 + 1] = lrun;
+    }
+    if (t_lo < t_hi) {
+      float* op = a.part + pr * RP + g * 4;
+#pragma unroll
+      for (int d = 0; d < RP / 16; d++) *(f4v*)(op + d * 16) = acc[d];
+    }
+  }
+}
+
+// merged latent of one (row, head) -> LDS (as T); sw holds NS weights
+template <typename T>
+DEVINL void latent_merge(const LatentArgs& a, size_t orow, T* dst, float* sw) {
+  const size_t n = (size_t)a.rows * a.H;
+  if (threadIdx.x < 64) {
+    float mt = -INFINITY;
+    for (int s = threadIdx.x; s < a.NS; s += 64)
+      mt = fmaxf(mt, a.ml[(s * n + orow) * 2]);
+    mt = wave_reduce_max(mt);
+    float lt = 0.f;
+    for (int s = threadIdx.x; s < a.NS; s += 64) {
+      float w = exp2f(a.ml[(s * n + orow) * 2] - mt);   // -inf: empty split
+      sw[s] = w;
+      lt += w * a.ml[(s * n + orow) * 2 + 1];
+    }
+    lt = wave_reduce_sum(lt);
+    for (int s = threadIdx.x; s < a.NS; s += 64) sw[s] /= lt;
+  }
+  __syncthreads();
+  for (int i = threadIdx.x * 4; i < a.RP; i += blockDim.x * 4) {
+    f4v v = {0.f, 0.f, 0.f, 0.f};
+    for (int s = 0; s < a.NS; s++) {
+      float w = sw[s];
+      if (w == 0.f) continue;              // empty splits wrote no partial
+      f4v p = *(const f4v*)(a.part + (s * n + orow) * a.RP + i);
+#pragma unroll
+      for (int j = 0; j < 4; j++) v[j] = fmaf(w, p[j], v[j]);
+    }
+#pragma unroll
+    for (int j = 0; j < 4; j++) dst[i + j] = El<T>::st(v[j]);
+  }
+}
+
+#define MAX_SPLITS 256
+
+template <typename T>
+__global__ void __launch_bounds__(128) k_latent_merge(LatentArgs a) {
+  __shared__ float sw[MAX_SPLITS];
+  latent_merge<T>(a, blockIdx.x,
+                  (T*)a.olat + ((size_t)a.rbase * a.H + blockIdx.x) * a.RP, sw);
+}
+
+// ---- few rows: merge + value up-projection + gate per (row, head); the
+// ---- experts' gate/up halves run beside it in the same launch ----------
+template <typename T>
+__global__ void __launch_bounds__(256) k_latent_dec_fin(LatentArgs a,
+                                                        MoeArgs m, int fblocks) {
+  __shared__ __attribute__((aligned(16))) T ol[512];
+  __shared__ float sw[MAX_SPLITS];
+  const int nmix = a.rows * a.H;
+  if ((int)blockIdx.x >= nmix) {
+    const int b = blockIdx.x - nmix;
+    expert_gu_block<T>(m, b / fblocks, b % fblocks);
+    return;
+  }
+  constexpr int V = El<T>::V;
+  const int r = blockIdx.x / a.H, h = blockIdx.x - r * a.H;
+  latent_merge<T>(a, blockIdx.x, ol, sw);
+  __syncthreads();
+  const float gate = sigmoid_f(a.P[(size_t)r * a.ldp + a.og + h]);
+  const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int nv = a.RP / V;                  // 16-byte vectors of a row
+  T* o = (T*)a.o + (size_t)r * a.ldo + h * a.vd;
+  for (int j0 = wave * 4; j0 < a.vd; j0 += 16) {
+    float acc[4] = {0.f, 0.f, 0.f, 0.f};
+    for (int k = lane; k < nv; k += 64) {
+      f4v x = ld16(ol + k * V);
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        int j = min(j0 + i, a.vd - 1);
+        acc[i] = dot16<T>(
+            ld16((const T*)a.Wuv + ((size_t)h * a.vd + j) * a.RP + k * V), x,
+            acc[i]);
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+      float v = wave_reduce_sum(acc[i]);
+      if (lane == 0 && j0 + i < a.vd) o[j0 + i] = El<T>::st(v * gate);
+    }
+  }
+}
+
+// ---- launchers ---------------------------------------------------------
+static bool bad_shape(const LatentArgs& a) {
+  return a.rows < 1 || a.H < 1 || a.RT % 32 || a.RT < a.rot || a.RT > 128 ||
+         a.RP < a.rank || a.rdims > a.rot || a.rdims % 2 || a.NS < 1 ||
+         a.NS > MAX_SPLITS || a.E > 1024 || (a.E > 0 && a.rtop > a.E) || a.dp % 64 ||
+         a.dp < a.d;
+}
+
+extern "C" hipError_t launch_latent_prep(int f32, const LatentArgs* a,
+                                         hipStream_t s) {
+  if (bad_shape(*a)) return hipErrorInvalidValue;
+  if (f32) hipLaunchKernelGGL(k_latent_prep<float>, dim3(a->rows), dim3(256), 0, s, *a);
+  else hipLaunchKernelGGL(k_latent_prep<u16>, dim3(a->rows), dim3(256), 0, s, *a);
+  return hipGetLastError();
+}
+
+extern "C" hipError_t launch_latent_dec_prep(int f32, const LatentArgs* a,
+                                             hipStream_t s) {
+  if (bad_shape(*a) || a->RP > 512) return hipErrorInvalidValue;
+  dim3 grid(a->H + 1, a->rows);
+  if (f32) hipLaunchKernelGGL(k_latent_dec_prep<float>, grid, dim3(256), 0, s, *a);
+  else hipLaunchKernelGGL(k_latent_dec_prep<u16>, grid, dim3(256), 0, s, *a);
+  return hipGetLastError();
+}
+
+template <typename T, int RP, int NW>
+static hipError_t attn_go(const LatentArgs& a, int tiles, hipStream_t s) {
+  size_t lds = attn_lds<T>(RP, a.RT);
+  RAISE_LDS((k_latent_attn<T, RP, NW>));
+  hipLaunchKernelGGL((k_latent_attn<T, RP, NW>), dim3(tiles, a.NS),
+                     dim3(64 * NW), lds, s, a);
+  return hipGetLastError();
+}
+
+template <typename T, int NW>
+static hipError_t attn_rp(const LatentArgs& a, int tiles, hipStream_t s) {
+  switch (a.RP) {
+    case 64: return attn_go<T, 64, NW>(a, tiles, s);
+    case 128: return attn_go<T, 128, NW>(a, tiles, s);
+    case 256: return attn_go<T, 256, NW>(a, tiles, s);
+    case 384: return attn_go<T, 384, NW>(a, tiles, s);
+    case 512: return attn_go<T, 512, NW>(a, tiles, s);
+  }
+  return hipErrorInvalidValue;
+}
+
+// tiles: number of query tiles of 16*NW (token, head) pairs
+extern "C" hipError_t launch_latent_attn(int f32, const LatentArgs* a, int nw,
+                                         int tiles, hipStream_t s) {
+  if (bad_shape(*a) || tiles < 1 || (nw != 1 && nw != 4))
+    return hipErrorInvalidValue;
+  if (f32)
+    return nw == 1 ? attn_rp<float, 1>(*a, tiles, s)
+                   : attn_rp<float, 4>(*a, tiles, s);
+  return nw == 1 ? attn_rp<u16, 1>(*a, tiles, s)
+                 : attn_rp<u16, 4>(*a, tiles, s);
+}
+
+extern "C" hipError_t launch_latent_merge(int f32, const LatentArgs* a,
+                                          hipStream_t s) {
+  if (bad_shape(*a)) return hipErrorInvalidValue;
+  dim3 grid(a->rows * a->H);
+  if (f32) hipLaunchKernelGGL(k_latent_merge<float>, grid, dim3(128), 0, s, *a);
+  else hipLaunchKernelGGL(k_latent_merge<u16>, grid, dim3(128), 0, s, *a);
+  return hipGetLastError();
+}
+
+extern "C" hipError_t launch_latent_dec_fin(int f32, const LatentArgs* a,
+                                            const MoeArgs* m, int pairs,
+                                            hipStream_t s) {
+  if (bad_shape(*a) || a->RP > 512 || a->NS < 2) return hipErrorInvalidValue;
+  int ffm = m->ff > m->ffs ? m->ff : m->ffs;
+  int fb = pairs ? (ffm + MOE_FPB - 1) / MOE_FPB : 1;
+  dim3 grid(a->rows * a->H + pairs * fb);
+  if (f32) hipLaunchKernelGGL(k_latent_dec_fin<float>, grid, dim3(256), 0, s, *a, *m, fb);
+  else hipLaunchKernelGGL(k_latent_dec_fin<u16>, grid, dim3(256), 0, s, *a, *m, fb);
+  return hipGetLastError();
+}

@@ -25,7 +25,8 @@ def main(argv=None):
     ap.add_argument("--backend", default="auto",
                     choices=["auto", "gpu", "numpy"])
     ap.add_argument("--dtype", default="bf16",
-                    choices=["bf16", "fp8", "fp4"])
+                    choices=["bf16", "fp8", "fp4", "fp32"],
+                    help="fp32: layer-list designs only")
     ap.add_argument("--kv-dtype", default="bf16", choices=["bf16", "fp8"])
     ap.add_argument("--strategy", default="min_p",
                     choices=["min_p", "greedy", "top_k", "top_p",

@@ -21,6 +21,8 @@ import os
 from dataclasses import dataclass, field
 from typing import Optional
 
+from .layered import LAYERED_PRESETS, LayeredConfig
+
 
 @dataclass
 class ModelConfig:
@@ -105,7 +107,9 @@ class ModelConfig:
                           "mixtral")
 
     @classmethod
-    def from_hf_dict(cls, d: dict) -> "ModelConfig":
+    def from_hf_dict(cls, d: dict):
+        if LayeredConfig.matches(d):
+            return LayeredConfig.from_dict(d)
         model_type = d.get("model_type", "llama")
         if model_type not in cls.SUPPORTED_FAMILIES:
             raise ValueError(
@@ -152,7 +156,7 @@ class ModelConfig:
         return cfg
 
     @classmethod
-    def from_json(cls, path: str) -> "ModelConfig":
+    def from_json(cls, path: str):
         with open(path) as f:
             return cls.from_hf_dict(json.load(f))
 
@@ -406,8 +410,18 @@ PRESETS = {
 }
 
 
-def preset_config(name: str) -> ModelConfig:
+def preset_names() -> list:
+    return sorted([*PRESETS, *LAYERED_PRESETS])
+
+
+def has_preset(name: str) -> bool:
+    return name.lower() in PRESETS or name.lower() in LAYERED_PRESETS
+
+
+def preset_config(name: str):
     key = name.lower()
+    if key in LAYERED_PRESETS:
+        return LayeredConfig.from_dict(LAYERED_PRESETS[key])
     if key not in PRESETS:
-        raise KeyError(f"unknown preset {name!r}; have {sorted(PRESETS)}")
+        raise KeyError(f"unknown preset {name!r}; have {preset_names()}")
     return ModelConfig(**PRESETS[key])

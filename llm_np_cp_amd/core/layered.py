@@ -1,0 +1,366 @@
+"""Configuration of layer-list designs.
+
+Where ``ModelConfig`` describes a stack of identical blocks, a layer-list
+``config.json`` names every layer: its mixer, the mixer's sizes, its
+feed-forward, and optionally a range of layers that runs several times.
+Each mechanism is a small spec class that reads its own keys and knows its
+tensors; a further design registers further specs in ``MIXERS`` and its
+name in ``DESIGNS``.
+
+Turudra: parallel blocks (one norm feeds mixer and experts), latent
+attention and matrix-memory LSTM mixers, clamped routed experts with a
+shared one, a looped range that mixes the embedding output back in, and a
+soft-capped head.
+"""
+
+from __future__ import annotations
+
+from dataclasses import dataclass, field
+from typing import Dict, List, Optional, Tuple
+
+Shapes = Dict[str, Tuple[int, ...]]
+
+
+def _get(d: dict, key: str, where: str):
+    if not isinstance(d, dict) or key not in d:
+        raise ValueError(f"config.json: {where} lacks {key!r}")
+    return d[key]
+
+
+def _positive(where: str, **kw):
+    for k, v in kw.items():
+        if isinstance(v, bool) or not isinstance(v, int) or v < 1:
+            raise ValueError(f"config.json: {where}.{k} must be a positive "
+                             f"integer, got {v!r}")
+
+
+@dataclass
+class LatentAttentionSpec:
+    heads: int
+    dim: int
+    rot_dim: int
+    vdim: int
+    kv_rank: int
+    scale: float
+    rot_base: float
+    rot_dims: int
+    kind = "latent_attention"
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str):
+        rot = _get(m, "rot", where)
+        s = cls(heads=_get(m, "heads", where), dim=_get(m, "dim", where),
+                rot_dim=_get(m, "rot_dim", where),
+                vdim=_get(m, "vdim", where),
+                kv_rank=_get(m, "kv_rank", where),
+                scale=float(_get(m, "scale", where)),
+                rot_base=float(_get(rot, "base", where + ".rot")),
+                rot_dims=_get(rot, "dims", where + ".rot"))
+        _positive(where, heads=s.heads, dim=s.dim, rot_dim=s.rot_dim,
+                  vdim=s.vdim, kv_rank=s.kv_rank, rot_dims=s.rot_dims)
+        if s.rot_dims % 2 or s.rot_dims > s.rot_dim:
+            raise ValueError(f"config.json: {where}.rot.dims {s.rot_dims} "
+                             f"must be even and at most {s.rot_dim}")
+        return s
+
+    def to_dict(self) -> dict:
+        return {"heads": self.heads, "dim": self.dim,
+                "rot_dim": self.rot_dim, "vdim": self.vdim,
+                "kv_rank": self.kv_rank, "scale": self.scale,
+                "rot": {"base": self.rot_base, "dims": self.rot_dims}}
+
+    def shapes(self, p: str, width: int) -> Shapes:
+        H = self.heads
+        return {p + "q": (H * (self.dim + self.rot_dim), width),
+                p + "dkv": (self.kv_rank + self.rot_dim, width),
+                p + "dkv.norm": (self.kv_rank,),
+                p + "uk": (H * self.dim, self.kv_rank),
+                p + "uv": (H * self.vdim, self.kv_rank),
+                p + "g": (H, width),
+                p + "o": (width, H * self.vdim)}
+
+
+@dataclass
+class MLSTMSpec:
+    heads: int
+    dim: int
+    vdim: int
+    gate_cap: float
+    kind = "mlstm"
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str):
+        s = cls(heads=_get(m, "heads", where), dim=_get(m, "dim", where),
+                vdim=_get(m, "vdim", where),
+                gate_cap=float(_get(m, "gate_cap", where)))
+        _positive(where, heads=s.heads, dim=s.dim, vdim=s.vdim)
+        return s
+
+    def to_dict(self) -> dict:
+        return {"heads": self.heads, "dim": self.dim, "vdim": self.vdim,
+                "gate_cap": self.gate_cap}
+
+    def shapes(self, p: str, width: int) -> Shapes:
+        H, qk, v = self.heads, self.heads * self.dim, self.heads * self.vdim
+        return {p + "q": (qk, width), p + "k": (qk, width),
+                p + "v": (v, width), p + "g": (v, width),
+                p + "o": (width, v), p + "norm": (v,),
+                p + "i": (H, width), p + "i.b": (H,),
+                p + "f": (H, width), p + "f.b": (H,)}
+
+
+@dataclass
+class ExpertSpec:
+    ff: int
+    limit: float
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str):
+        s = cls(ff=_get(m, "ff", where), limit=float(_get(m, "limit", where)))
+        _positive(where, ff=s.ff)
+        return s
+
+    def shapes(self, p: str, width: int) -> Shapes:
+        return {p + "gate": (self.ff, width), p + "up": (self.ff, width),
+                p + "down": (width, self.ff)}
+
+
+@dataclass
+class MoESpec:
+    experts: int
+    top: int
+    expert: ExpertSpec
+    shared: Optional[ExpertSpec] = None
+    kind = "moe"
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str):
+        r = _get(m, "router", where)
+        sh = m.get("shared")
+        s = cls(experts=_get(r, "experts", where + ".router"),
+                top=_get(r, "top", where + ".router"),
+                expert=ExpertSpec.from_dict(_get(m, "expert", where),
+                                            where + ".expert"),
+                shared=(ExpertSpec.from_dict(sh, where + ".shared")
+                        if sh else None))
+        _positive(where + ".router", experts=s.experts, top=s.top)
+        if s.top > s.experts or s.experts > 1024:
+            raise ValueError(f"config.json: {where}.router: top {s.top} of "
+                             f"{s.experts} experts (at most 1024) is not "
+                             f"possible")
+        return s
+
+    def to_dict(self) -> dict:
+        ex = lambda e: {"ff": e.ff, "limit": e.limit}
+        return {"kind": self.kind,
+                "router": {"experts": self.experts, "top": self.top},
+                "expert": ex(self.expert),
+                "shared": ex(self.shared) if self.shared else None}
+
+    def shapes(self, p: str, width: int) -> Shapes:
+        out = {p + "router": (self.experts, width)}
+        for e in range(self.experts):
+            out.update(self.expert.shapes(f"{p}e{e}.", width))
+        if self.shared:
+            out.update(self.shared.shapes(p + "shared.", width))
+        return out
+
+
+MIXERS = {c.kind: c for c in (LatentAttentionSpec, MLSTMSpec)}
+MLPS = {c.kind: c for c in (MoESpec,)}
+DESIGNS = {"Turudra": "turudra"}       # config "architecture" -> model_type
+
+
+@dataclass
+class LayerSpec:
+    mixer: object
+    mlp: Optional[MoESpec]
+
+
+@dataclass
+class LoopSpec:
+    start: int
+    stop: int
+    times: int
+
+
+@dataclass
+class LayeredConfig:
+    model_type: str
+    vocab_size: int
+    hidden_size: int
+    layers: List[LayerSpec]
+    loop: Optional[LoopSpec] = None
+    norm_eps: float = 1e-5
+    embed_scale: float = 1.0
+    residual_mult: float = 1.0
+    logit_softcap: Optional[float] = None
+    max_position_embeddings: int = 131072
+    bos_token_id: Optional[int] = None
+    eos_token_id: Optional[int] = None
+    runs: List[Tuple[int, bool]] = field(default_factory=list)
+
+    def __post_init__(self):
+        n, lp = len(self.layers), self.loop
+        if lp is None:
+            self.runs = [(i, False) for i in range(n)]
+            return
+        if not (0 <= lp.start < lp.stop <= n and lp.times >= 1):
+            raise ValueError(f"config.json: loop {lp} does not fit "
+                             f"{n} layers")
+        self.runs = [(i, False) for i in range(lp.start)]
+        for _ in range(lp.times):
+            self.runs += [(i, i == lp.start)
+                          for i in range(lp.start, lp.stop)]
+        self.runs += [(i, False) for i in range(lp.stop, n)]
+
+    # names the rest of the framework reads
+    @property
+    def num_hidden_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def rms_norm_eps(self) -> float:
+        return self.norm_eps
+
+    @property
+    def is_moe(self) -> bool:
+        return any(l.mlp is not None for l in self.layers)
+
+    @property
+    def recurrent(self) -> bool:
+        return any(l.mixer.kind == "mlstm" for l in self.layers)
+
+    @classmethod
+    def matches(cls, d: dict) -> bool:
+        return "architecture" in d
+
+    @classmethod
+    def from_dict(cls, d: dict) -> "LayeredConfig":
+        arch = _get(d, "architecture", "top level")
+        if arch not in DESIGNS:
+            raise ValueError(f"unsupported architecture {arch!r}; layer-list "
+                             f"designs: {sorted(DESIGNS)}")
+        layers = []
+        for i, l in enumerate(_get(d, "layers", "top level")):
+            w = f"layers[{i}]"
+            kind = _get(l, "type", w)
+            if kind not in MIXERS:
+                raise ValueError(f"config.json: {w}: unknown mixer {kind!r}")
+            mlp = l.get("mlp")
+            if mlp is not None and mlp.get("kind") not in MLPS:
+                raise ValueError(f"config.json: {w}: unknown feed-forward "
+                                 f"{mlp.get('kind')!r}")
+            layers.append(LayerSpec(
+                MIXERS[kind].from_dict(_get(l, "mixer", w), w + ".mixer"),
+                MLPS[mlp["kind"]].from_dict(mlp, w + ".mlp") if mlp
+                else None))
+        lp = d.get("loop")
+        width, vocab = _get(d, "width", "top level"), _get(d, "vocab",
+                                                           "top level")
+        _positive("top level", width=width, vocab=vocab)
+        cap = d.get("logit_softcap")
+        return cls(
+            model_type=DESIGNS[arch], vocab_size=vocab, hidden_size=width,
+            layers=layers,
+            loop=LoopSpec(_get(lp, "start", "loop"), _get(lp, "stop", "loop"),
+                          _get(lp, "times", "loop")) if lp else None,
+            norm_eps=float(_get(_get(d, "norm", "top level"), "eps", "norm")),
+            embed_scale=float(_get(_get(d, "embedding", "top level"),
+                                   "scale", "embedding")),
+            residual_mult=float(_get(d, "residual_mult", "top level")),
+            logit_softcap=float(cap) if cap else None,
+            max_position_embeddings=d.get("max_position_embeddings", 131072),
+            bos_token_id=d.get("bos_token_id"),
+            eos_token_id=d.get("eos_token_id"))
+
+    def to_dict(self) -> dict:
+        arch = {v: k for k, v in DESIGNS.items()}[self.model_type]
+        d = {"architecture": arch, "vocab": self.vocab_size,
+             "width": self.hidden_size, "norm": {"eps": self.norm_eps},
+             "embedding": {"scale": self.embed_scale},
+             "residual_mult": self.residual_mult,
+             "logit_softcap": self.logit_softcap,
+             "layers": [{"type": l.mixer.kind, "mixer": l.mixer.to_dict(),
+                         "mlp": l.mlp.to_dict() if l.mlp else None}
+                        for l in self.layers],
+             "loop": None}
+        if self.loop:
+            d["loop"] = {"start": self.loop.start, "stop": self.loop.stop,
+                         "times": self.loop.times}
+        for k in ("bos_token_id", "eos_token_id"):
+            if getattr(self, k) is not None:
+                d[k] = getattr(self, k)
+        return d
+
+    to_hf_dict = to_dict
+
+    def weight_shapes(self) -> Shapes:
+        W = self.hidden_size
+        out: Shapes = {"embed": (self.vocab_size, W), "final.norm": (W,),
+                       "head": (self.vocab_size, W)}
+        if self.loop:
+            out["loop.in"] = (W, 2 * W)
+        for i, l in enumerate(self.layers):
+            out[f"l{i}.norm1"] = (W,)
+            out.update(l.mixer.shapes(f"l{i}.mix.", W))
+            if l.mlp:
+                out.update(l.mlp.shapes(f"l{i}.mlp.", W))
+        return out
+
+
+# ----------------------------------------------------------------------
+# presets (random-init runs)
+# ----------------------------------------------------------------------
+
+def _layer(mixer: str, experts: int, top: int, ff: int, shared: int,
+           limit: float = 7.0, **m) -> dict:
+    mlp = {"kind": "moe", "router": {"experts": experts, "top": top},
+           "expert": {"ff": ff, "limit": limit},
+           "shared": {"ff": shared, "limit": limit} if shared else None}
+    return {"type": mixer, "mixer": m, "mlp": mlp if experts else None}
+
+
+def _latent(heads, dim, rot, vdim, rank, base=10000.0) -> dict:
+    return dict(heads=heads, dim=dim, rot_dim=rot, vdim=vdim, kv_rank=rank,
+                scale=(dim + rot) ** -0.5, rot={"base": base, "dims": rot})
+
+
+def _design(vocab, width, layers, loop=None, **kw) -> dict:
+    d = {"architecture": "Turudra", "vocab": vocab, "width": width,
+         "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
+         "residual_mult": 0.5, "logit_softcap": 30.0, "layers": layers,
+         "loop": loop}
+    d.update(kw)
+    return d
+
+
+def _moe_stack(n, mix, width, heads, moe) -> list:
+    """n layers: latent attention, or alternating with mLSTM (mix "both")."""
+    lat = _latent(heads, 128, 64, 128, 512)
+    mem = dict(heads=heads // 2, dim=128, vdim=2 * 128, gate_cap=15.0)
+    return [_layer("latent_attention", **moe, **lat)
+            if mix == "latent" or i % 2 == 0
+            else _layer("mlstm", **moe, **mem) for i in range(n)]
+
+
+LAYERED_PRESETS = {
+    "tiny-turudra": _design(
+        384, 96,
+        [_layer("latent_attention", 4, 2, 64, 48, 1.5,
+                **_latent(3, 24, 16, 40, 56)),
+         _layer("mlstm", 4, 2, 64, 48, 1.5, heads=2, dim=40, vdim=72,
+                gate_cap=12.0),
+         _layer("latent_attention", 4, 2, 64, 48, 1.5,
+                **_latent(3, 24, 16, 40, 56))],
+        loop={"start": 0, "stop": 2, "times": 2}),
+    # layers of real models' sizes
+    "turudra-2k": _design(
+        32000, 2048,
+        _moe_stack(8, "both", 2048, 16,
+                   dict(experts=8, top=2, ff=2048, shared=2048))),
+    "turudra-4k": _design(
+        32000, 4096,
+        _moe_stack(4, "both", 4096, 32,
+                   dict(experts=8, top=2, ff=4096, shared=4096))),
+}

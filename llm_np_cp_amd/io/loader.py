@@ -25,6 +25,7 @@ from typing import Dict, Iterator, Tuple
 import numpy as np
 
 from ..core.config import ModelConfig, preset_config
+from ..core.layered import LayeredConfig
 
 
 # ----------------------------------------------------------------------
@@ -135,7 +136,9 @@ class LazyCheckpointWeights:
 # ----------------------------------------------------------------------
 
 def hf_weight_shapes(cfg: ModelConfig) -> Dict[str, Tuple[int, ...]]:
-    """All HF state-dict tensor names and shapes for this architecture."""
+    """All checkpoint tensor names and shapes for this architecture."""
+    if isinstance(cfg, LayeredConfig):
+        return cfg.weight_shapes()
     h, hd = cfg.hidden_size, cfg.head_dim
     nh, kvh = cfg.num_attention_heads, cfg.num_key_value_heads
     im = cfg.intermediate_size

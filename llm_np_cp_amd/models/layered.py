@@ -1,0 +1,589 @@
+"""GPU engine of the layer-list designs: paged mixed-batch steps.
+
+One batch holds any mix of prompt portions and single decoded tokens, each
+row with its own sequence and position.  ``step()`` runs such a batch from
+the pages and state slots that earlier steps left; prompts, the row
+primitives of the batching server and the captured decode step all run
+the same layer stack over the same cache.
+
+The residual stream, projections, norms, scores, routing and recurrent
+state are fp32; dtype "bf16" keeps weights, the normed layer input and the
+cached latents in bf16 (fp32 accumulation), "fp32" everything in true
+fp32.
+"""
+
+from __future__ import annotations
+
+from dataclasses import dataclass, field
+from typing import Dict, List, Optional, Sequence as Seq
+
+import numpy as np
+import torch
+
+from ..core.layered import LayeredConfig
+from ..ops import hip_ops as ho
+from ..ops import hybrid_ops as hy
+from ..parallel import tp as tpu
+from ..runtime.cache_manager import CacheFull, CacheManager, Sequence
+from ..utils.tracing import trace_range
+from .decode_loop import DecodeLoop, DeviceCacheHandle
+from .mixers import MIXERS, Packer, RoutedExperts, pad_to
+
+FEW = 8             # rows up to which the single-token path is fused GEMVs
+PART_FLOATS = 1 << 25     # split-attention scratch for prompt portions
+
+
+@dataclass
+class StepEntry:
+    """The next tokens of one sequence; ``want`` are the places among them
+    whose logits are returned."""
+    seq: Sequence
+    tokens: np.ndarray
+    want: Seq[int] = ()
+
+
+@dataclass
+class Rows:
+    """One batch on the device.  Rows [0, nd) are single tokens; the rest
+    belong to nseg runs of at least two tokens."""
+    T: int
+    nd: int
+    ids: torch.Tensor
+    slot: torch.Tensor
+    pos: torch.Tensor
+    seg_row0: torch.Tensor
+    seg_len: torch.Tensor
+    seg_slot: torch.Tensor
+    seg_pos0: torch.Tensor
+    nseg: int = 0
+    nchunk: int = 0
+    seg_chunk0: object = 0
+    chunk_row0: object = 0
+    chunk_len: object = 0
+    tiles: Dict[int, tuple] = field(default_factory=dict)
+
+
+class _Layer:
+    def __init__(self, eng, spec, pk: Packer, i: int):
+        p = f"l{i}."
+        self.mixer = MIXERS[spec.mixer.kind](eng, spec.mixer, pk, p + "mix.")
+        names = [p + "mix." + n for n in self.mixer.IN]
+        self.orouter = sum(pk.w[n].shape[0] for n in names)
+        self.experts = None
+        if spec.mlp:
+            names.append(p + "mlp.router")
+            self.experts = RoutedExperts(eng, spec.mlp, pk, p + "mlp.")
+        self.win = pk.rows(names, eng.W)
+        self.ldp = self.win.shape[0]
+        self.g = pk.f32(p + "norm1")
+
+
+class LayeredModel(DecodeLoop):
+    def __init__(self, config: LayeredConfig, weights, dtype: str = "bf16",
+                 max_seq: Optional[int] = 4096, prefill_chunk: int = 2048,
+                 device: Optional[str] = None, seed: int = 0,
+                 kv_dtype: str = "bf16", max_batch: int = 1,
+                 pool_tokens: Optional[int] = None):
+        """``pool_tokens`` sizes the page pool (default: max_seq tokens for
+        each of max_batch sequences); ``max_batch`` is the number of
+        sequence slots."""
+        if dtype not in ("bf16", "fp32"):
+            raise ValueError(f"{config.model_type} runs in bf16 or fp32, "
+                             f"not {dtype!r}")
+        if kv_dtype != "bf16":
+            raise ValueError(f"{config.model_type} caches latents in the "
+                             f"compute dtype; kv_dtype {kv_dtype!r} is not "
+                             f"available")
+        if not torch.cuda.is_available():
+            raise RuntimeError("LayeredModel requires a GPU (MI355X)")
+        from ..io.loader import validate_weights
+        validate_weights(config, weights)
+        assert 1 <= max_batch <= 256
+        self.rank, self.world = tpu.init_distributed()
+        if self.world > 1:
+            raise ValueError(f"{config.model_type} runs on one GPU "
+                             f"(no tensor parallelism)")
+        self.config = self.cfg = config
+        self.seed, self.dtype, self.kv_dtype = seed, dtype, kv_dtype
+        self.f32 = 1 if dtype == "fp32" else 0
+        self.T = torch.float32 if self.f32 else torch.bfloat16
+        self.device = torch.device(device or "cuda:0")
+        torch.cuda.set_device(self.device)
+        self.W = config.hidden_size
+        self.Wp = pad_to(self.W, 64)
+        self.max_batch = max_batch
+        self.max_seq = max_seq or min(config.max_position_embeddings, 131072)
+        self.no_rewind = config.recurrent
+        pages = -(-(pool_tokens or max_batch * pad_to(self.max_seq, hy.PAGE))
+                  // hy.PAGE)
+        self.cache = CacheManager(pages, max_batch, hy.PAGE, self.max_seq)
+        self._ropes: Dict[tuple, tuple] = {}
+        self._upload(weights)
+        self._alloc(min(prefill_chunk, pad_to(self.max_seq * max_batch, 64)))
+        self._graph = None
+        self._graph_mode = None
+        self.reset()
+
+    # ------------------------------------------------------------------
+    # weights, cache, scratch
+    # ------------------------------------------------------------------
+    def rope_tables(self, base: float, dims: int):
+        """cos/sin of position * base**(-2i/dims), fp32 from fp64."""
+        key = (base, dims)
+        if key not in self._ropes:
+            n = self.cache.table.shape[1] * hy.PAGE
+            f = base ** (-2.0 * np.arange(dims // 2) / dims)
+            a = np.outer(np.arange(n, dtype=np.float64), f)
+            self._ropes[key] = tuple(
+                torch.from_numpy(t.astype(np.float32)).to(self.device)
+                for t in (np.cos(a), np.sin(a)))
+        return self._ropes[key]
+
+    def _upload(self, weights):
+        cfg = self.cfg
+        pk = Packer(weights, self.device, self.T)
+        self.embed = pk.raw("embed").to(self.T).contiguous()
+        self.head = pk.rows(["head"], self.W)
+        self.g_final = pk.f32("final.norm")
+        self.win_loop = pk.rows(["loop.in"], 2 * self.W) if cfg.loop else None
+        self.layers = [_Layer(self, s, pk, i)
+                       for i, s in enumerate(cfg.layers)]
+        # every run of a looped layer has its own cache or state
+        self.caches = [self.layers[i].mixer.new_cache(self)
+                       for i, _ in cfg.runs]
+
+    def decode_splits(self, rows: int) -> int:
+        """Key-range splits of single-token attention: fixed by the cache
+        size and the number of rows, so a captured step keeps its grid."""
+        tiles = -(-self.cache.table.shape[1] * hy.PAGE // 32)
+        return int(max(2, min(64, tiles // 2, 1024 // rows)))
+
+    def run_splits(self, tiles: int, longest: int) -> int:
+        """Splits for `tiles` query tiles against up to `longest` keys."""
+        if tiles >= 256:
+            return 1
+        return int(max(1, min(32, 512 // tiles, longest // 256)))
+
+    def _alloc(self, PC: int):
+        cfg, dev, B = self.cfg, self.device, self.max_batch
+        PC = self.PC = max(PC, B, FEW)
+        f32 = dict(dtype=torch.float32, device=dev)
+        i32 = dict(dtype=torch.int32, device=dev)
+        tt = dict(dtype=self.T, device=dev)
+        self.x = torch.zeros(PC, self.W, **f32)
+        self.xb = torch.zeros(PC, self.W, **f32)
+        self.x0 = torch.zeros(PC, self.W, **f32) if cfg.loop else None
+        self.h = torch.zeros(PC, self.Wp, **tt)
+        self.cat = (torch.zeros(PC, self.win_loop.shape[1], **tt)
+                    if cfg.loop else None)
+        self.P = torch.zeros(PC * max(l.ldp for l in self.layers), **f32)
+        rows_splits = max((r * self.decode_splits(r)
+                           for r in range(1, B + 1)), default=0)
+        need: Dict[str, int] = {}
+        for l in self.layers:
+            m = l.mixer
+            per = (max(rows_splits, PART_FLOATS //
+                       (m.spec.heads * m.RP)) if m.kind == "latent_attention"
+                   else B + 1)
+            for k, n in m.sizes(PC, per).items():
+                need[k] = max(need.get(k, 0), n)
+        for k in ("qn", "qa", "olat", "o", "part", "ml", "raw", "gF", "gi",
+                  "gm", "cm0", "U", "un"):
+            kw = tt if k in ("qn", "qa", "olat", "o") else f32
+            setattr(self, k, torch.zeros(max(need.get(k, 0), 1), **kw))
+        ex = [l.experts for l in self.layers if l.experts]
+        K1 = max((e.K1 for e in ex), default=1)
+        self.ridx = torch.zeros(PC * K1, **i32)
+        self.rwt = torch.zeros(PC * K1, **f32)
+        self.act = torch.zeros(max((PC * e.K1 * e.ffm for e in ex),
+                                   default=1), **tt)
+        self.ypair = torch.zeros(PC * K1 * self.W if ex else 1, **tt)
+        self.perm = torch.zeros(PC * K1, **i32)
+        nt = PC * K1 // 32 + max((e.spec.experts + 1 for e in ex), default=1)
+        self.tile_e, self.tile_row0, self.tile_n = (
+            torch.zeros(nt, **i32) for _ in range(3))
+        # block table and per-row decode state
+        self.table = torch.zeros(self.cache.table.shape, **i32)
+        self._table_version = -1
+        S, V = self.max_seq, cfg.vocab_size
+        i64 = dict(dtype=torch.int64, device=dev)
+        self.bt_slot = torch.zeros(B, **i32)
+        self.bt_lens = torch.zeros(B, **i32)
+        self.bt_next = torch.zeros(B, **i32)
+        self.bt_nout = torch.zeros(B, **i32)
+        self.bt_cnt = torch.zeros(B, **i32)
+        self.bt_gmax = torch.zeros(B, **i64)
+        self.bt_pick = torch.zeros(B, **i64)
+        self.bt_ring = torch.zeros(B, S + 16, **i32)
+        self.bt_logits32 = torch.zeros(B, V, **f32)
+        self.rng_ctr = torch.zeros(1, **i64)
+        self._iota = torch.arange(B, **i32)
+        self._ones = torch.ones(B, **i32)
+        # a single sequence is row 0 of the batch
+        self.b_logits = self.bt_logits32[0]
+        self.len_buf, self.next_token = self.bt_lens[:1], self.bt_next[:1]
+        self.nout, self.out_ring = self.bt_nout[:1], self.bt_ring[0]
+        self.s_gmax, self.s_pick = self.bt_gmax[:1], self.bt_pick[:1]
+        self.s_cnt = self.bt_cnt[:1]
+        heads = {l.mixer.spec.heads for l in self.layers
+                 if l.mixer.kind == "latent_attention"}
+        self._tile_heads = sorted(heads)
+        self._meta = torch.zeros(
+            3 * PC + 8 * (B + 2) + 2 * (PC // hy.CHUNK + B + 2) + PC +
+            sum(2 * (PC * h // 64 + B + 2) for h in heads), **i32)
+
+    # ------------------------------------------------------------------
+    # layer stack
+    # ------------------------------------------------------------------
+    def _sync_table(self):
+        if self._table_version != self.cache.version:
+            self.table.copy_(torch.from_numpy(self.cache.table))
+            self._table_version = self.cache.version
+
+    def _layer_stack(self, b: Rows, layer_hook=None):
+        """Embedding and every layer run over the batch; leaves the
+        residual stream of its rows in self.x."""
+        cfg, W, T = self.cfg, self.W, b.T
+        eps, mult = cfg.norm_eps, cfg.residual_mult
+        few = b.nseg == 0 and T <= FEW
+        hy.embed_rows(self.embed, b.ids, self.x, self.x0, T, cfg.embed_scale)
+        if layer_hook is not None:
+            layer_hook(-1, self.x[:T])
+        for j, (i, starts) in enumerate(cfg.runs):
+            l, cache = self.layers[i], self.caches[j]
+            m, ex = l.mixer, l.experts
+            if starts:         # x <- W_in [x; x0]
+                if few:
+                    hy.lin_rows(self.win_loop, self.x, self.xb, T, W, W, eps,
+                                x0=self.x0)
+                else:
+                    K = self.cat.shape[1]
+                    hy.norm_rows(self.x, None, self.cat, T, W, K, eps,
+                                 x0=self.x0)
+                    hy.gemm_rows(self.cat, self.win_loop, self.xb, T, K, W,
+                                 hy.EPI_F32)
+                self.x, self.xb = self.xb, self.x
+            if few:
+                # norm + every input projection (router too), the mixer,
+                # then output projection + experts' down + residual
+                hy.lin_rows(l.win, self.x, self.P, T, W, l.ldp, eps, g=l.g,
+                            hout=self.h)
+                m.few(self, b, cache, l)
+                hy.block_out(self.f32, m.wo, self.o, m.ldo,
+                             ex.bind(self) if ex else hy.MoeArgs(),
+                             ex.K1 if ex else 0, self.x, T, W, mult)
+            else:
+                hy.norm_rows(self.x, l.g, self.h, T, W, self.Wp, eps)
+                hy.gemm_rows(self.h, l.win, self.P, T, self.Wp, l.ldp,
+                             hy.EPI_F32)
+                m.many(self, b, cache, l)
+                hy.gemm_rows(self.o, m.wo, self.x, T, m.ldo, W,
+                             hy.EPI_RESADD, mult=mult)
+                if ex:
+                    ex.many(self, T)
+            if layer_hook is not None:
+                layer_hook(j, self.x[:T])
+
+    def _head(self, out: torch.Tensor, n: int, rows=None):
+        """Final norm, head and soft cap of n rows -> out [n, vocab]."""
+        cfg, V = self.cfg, self.cfg.vocab_size
+        cap = cfg.logit_softcap or 0.0
+        if n <= FEW:
+            hy.lin_rows(self.head, self.x, out, n, self.W, V, cfg.norm_eps,
+                        g=self.g_final, rows=rows, cap=cap)
+        else:
+            hy.norm_rows(self.x, self.g_final, self.h, n, self.W, self.Wp,
+                         cfg.norm_eps, rows=rows)
+            hy.gemm_rows(self.h, self.head, out, n, self.Wp, V,
+                         hy.EPI_SOFTCAP, mult=cap)
+
+    # ------------------------------------------------------------------
+    # mixed-batch step
+    # ------------------------------------------------------------------
+    def open_sequence(self) -> Sequence:
+        return self.cache.open()
+
+    def close_sequence(self, seq: Sequence) -> None:
+        self.cache.close(seq)
+
+    def step(self, entries: List[StepEntry], layer_hook=None) -> torch.Tensor:
+        """Run the entries' tokens as one batch and return the wanted
+        logits, [wanted, vocab] fp32 on the device, in entry order.  Pages
+        are reserved for the whole step first; CacheFull leaves everything
+        as it was.  A step beyond the scratch size runs as several
+        batches."""
+        entries = [StepEntry(e.seq, np.asarray(e.tokens, np.int32).ravel(),
+                             [int(k) for k in e.want]) for e in entries]
+        if len({id(e.seq) for e in entries}) != len(entries):
+            raise ValueError("a sequence appears twice in one step")
+        missing = 0
+        for e in entries:
+            n = len(e.tokens)
+            if n == 0:
+                raise ValueError("empty ids")
+            if e.tokens.min() < 0 or e.tokens.max() >= self.cfg.vocab_size:
+                raise ValueError("token id outside the vocabulary")
+            if any(not 0 <= k < n for k in e.want):
+                raise ValueError("wanted place outside the tokens")
+            if e.seq.length + n > self.max_seq:
+                raise ValueError(f"sequence {e.seq.length}+{n} exceeds "
+                                 f"max_seq {self.max_seq}")
+            missing += self.cache.missing(e.seq, e.seq.length + n)
+        if missing > self.cache.free_pages:
+            raise CacheFull(f"{missing} more pages needed, "
+                            f"{self.cache.free_pages} free")
+        for e in entries:
+            self.cache.reserve(e.seq, e.seq.length + len(e.tokens))
+        out = torch.empty(sum(len(e.want) for e in entries),
+                          self.cfg.vocab_size, dtype=torch.float32,
+                          device=self.device)
+        done = 0
+        parts, room = [], self.PC
+        for e in entries:
+            at = 0
+            while at < len(e.tokens):
+                n = min(room, len(e.tokens) - at)
+                parts.append((e.seq, e.tokens[at:at + n],
+                              [k - at for k in e.want if at <= k < at + n]))
+                at += n
+                room -= n
+                if room == 0:
+                    done += self._run_parts(parts, out[done:], layer_hook)
+                    parts, room = [], self.PC
+        if parts:
+            self._run_parts(parts, out[done:], layer_hook)
+        return out
+
+    def _run_parts(self, parts, out, layer_hook) -> int:
+        order = sorted(range(len(parts)), key=lambda k: len(parts[k][1]) > 1)
+        T = sum(len(p[1]) for p in parts)
+        nd = sum(len(p[1]) == 1 for p in parts)
+        row0, r = {}, 0
+        for k in order:
+            row0[k] = r
+            r += len(parts[k][1])
+        cols: Dict[str, list] = {n: [] for n in (
+            "ids", "slot", "pos", "seg_row0", "seg_len", "seg_slot",
+            "seg_pos0", "seg_chunk0", "chunk_row0", "chunk_len")}
+        for k in order:
+            seq, tok, _ = parts[k]
+            n = len(tok)
+            cols["ids"].append(tok)
+            cols["slot"].append(np.full(n, seq.slot, np.int32))
+            cols["pos"].append(np.arange(seq.length, seq.length + n,
+                                         dtype=np.int32))
+            cols["seg_row0"].append(row0[k])
+            cols["seg_len"].append(n)
+            cols["seg_slot"].append(seq.slot)
+            cols["seg_pos0"].append(seq.length)
+            if n > 1:
+                cols["seg_chunk0"].append(len(cols["chunk_row0"]))
+                for t in range(0, n, hy.CHUNK):
+                    cols["chunk_row0"].append(row0[k] + t)
+                    cols["chunk_len"].append(min(hy.CHUNK, n - t))
+        nchunk = len(cols["chunk_row0"])
+        # query tiles of the runs, latest (most keys) first
+        longest = max([parts[k][0].length + len(parts[k][1])
+                       for k in order[nd:]], default=0)
+        tiles = {}
+        for H in self._tile_heads:
+            t = [(seg, rr) for seg, k in enumerate(order) if seg >= nd
+                 for rr in range(0, len(parts[k][1]) * H, 64)]
+            t.sort(key=lambda s: -(parts[order[s[0]]][0].length + s[1] // H))
+            cols[f"ts{H}"] = [s for s, _ in t]
+            cols[f"tr{H}"] = [rr for _, rr in t]
+            tiles[H] = len(t)
+        want = [row0[k] + w for k in range(len(parts)) for w in parts[k][2]]
+        cols["want"] = want
+        flat, off = [], {}
+        at = 0
+        for name, v in cols.items():
+            a = (np.concatenate(v) if v and isinstance(v[0], np.ndarray)
+                 else np.asarray(v, dtype=np.int32))
+            off[name] = (at, len(a))
+            flat.append(a.astype(np.int32, copy=False))
+            at += len(a)
+        host = np.concatenate(flat)
+        assert len(host) <= self._meta.numel()
+        self._meta[:at].copy_(torch.from_numpy(host))
+        dev = {n: self._meta[a:a + c] for n, (a, c) in off.items()}
+        self._sync_table()
+        b = Rows(T=T, nd=nd, ids=dev["ids"], slot=dev["slot"],
+                 pos=dev["pos"], seg_row0=dev["seg_row0"],
+                 seg_len=dev["seg_len"], seg_slot=dev["seg_slot"],
+                 seg_pos0=dev["seg_pos0"], nseg=len(parts) - nd,
+                 nchunk=nchunk, seg_chunk0=dev["seg_chunk0"],
+                 chunk_row0=dev["chunk_row0"], chunk_len=dev["chunk_len"],
+                 tiles={H: (dev[f"ts{H}"], dev[f"tr{H}"], n, longest)
+                        for H, n in tiles.items()})
+        self._layer_stack(b, layer_hook)
+        if want:
+            self._head(out, len(want), dev["want"])
+        for seq, tok, _ in parts:
+            seq.length += len(tok)
+        return len(want)
+
+    # ------------------------------------------------------------------
+    # generation interface (rows of the lockstep group)
+    # ------------------------------------------------------------------
+    def reset(self):
+        self.cache.close_all()
+        self.rows: List[Optional[Sequence]] = [None] * self.max_batch
+        for t in (self.bt_lens, self.bt_nout, self.rng_ctr, self.bt_gmax,
+                  self.bt_pick, self.bt_cnt):
+            t.zero_()
+        self._host_len = 0
+        self._host_lens = [0] * self.max_batch
+        self._batch_n = 0
+
+    def _open_row(self, b: int) -> Sequence:
+        if self.rows[b] is not None:
+            self.cache.close(self.rows[b])
+        self.rows[b] = seq = self.cache.open()
+        self.bt_slot[b:b + 1].fill_(seq.slot)
+        return seq
+
+    def _reserve(self, lens):
+        for b, n in enumerate(lens):
+            self.cache.reserve(self.rows[b], n)
+        self._sync_table()
+
+    def _append_row0(self, ids, pos0: int, want, layer_hook=None):
+        ids = np.asarray(ids, dtype=np.int32).ravel()
+        if len(ids) == 0:
+            raise ValueError("empty ids")
+        if pos0 + len(ids) > self.max_seq:
+            raise ValueError(f"sequence {pos0}+{len(ids)} exceeds max_seq "
+                             f"{self.max_seq}")
+        seq = self.rows[0] or self._open_row(0)
+        seq.length = pos0        # the device loop advances on its own
+        out = self.step([StepEntry(seq, ids, want)], layer_hook)
+        self.bt_lens[:1].fill_(pos0 + len(ids))
+        self._host_len = pos0 + len(ids)
+        return out
+
+    def forward(self, ids: np.ndarray, cache: DeviceCacheHandle,
+                pos0: int) -> np.ndarray:
+        """Last-position logits (1, V) fp32."""
+        if pos0 != cache.seq_len:
+            raise ValueError("GPU engine requires sequential positions")
+        n = np.asarray(ids).size
+        out = self._append_row0(ids, pos0, [n - 1] if n else [])
+        self.b_logits.copy_(out[0])
+        cache.seq_len = pos0 + n
+        return out.cpu().numpy()
+
+    def forward_positions(self, ids: np.ndarray, pos0: int) -> np.ndarray:
+        """All-position logits (M, V), continuing from pos0."""
+        n = np.asarray(ids).size
+        return self._append_row0(ids, pos0, range(n)).cpu().numpy()
+
+    def forward_full(self, ids: np.ndarray,
+                     return_hidden_states: bool = False):
+        """All-position logits of a fresh sequence; optionally with the
+        residual stream after the embedding and after every layer run."""
+        self.reset()
+        n = np.asarray(ids).size
+        if not return_hidden_states:
+            return self.forward_positions(ids, 0)
+        hidden = [[] for _ in range(len(self.cfg.runs) + 1)]
+
+        def hook(i, x):
+            hidden[i + 1].append(x.cpu().numpy())
+        out = self._append_row0(ids, 0, range(n), hook)
+        return out.cpu().numpy(), [np.concatenate(h) for h in hidden]
+
+    def rewind(self, n: int):
+        """Drop the tokens from position n on.  Attention caches can; a
+        recurrent state cannot be rolled back, so with recurrent layers
+        only the current length (or 0) is possible."""
+        if not 0 <= n <= self.max_seq:
+            raise ValueError(f"rewind {n} outside [0, {self.max_seq}]")
+        if n == 0:
+            return self.reset()
+        cur = int(self.bt_lens[0].item())
+        if n > cur or (n < cur and self.no_rewind):
+            raise ValueError(f"cannot rewind from {cur} to {n}: "
+                             f"{self.cfg.model_type} carries recurrent state")
+        self.rows[0].length = n
+        self.bt_lens[:1].fill_(n)
+        self._host_len = n
+
+    def _decode_step(self, greedy: bool, min_p: float,
+                     temperature: float = 1.0):
+        self._decode_batch_step(1, greedy, min_p, temperature)
+
+    def _decode_batch_step(self, B: int, greedy: bool, min_p: float,
+                           temperature: float = 1.0):
+        """One token for rows [0, B); all state is on the device."""
+        b = Rows(T=B, nd=B, ids=self.bt_next, slot=self.bt_slot,
+                 pos=self.bt_lens, seg_row0=self._iota, seg_len=self._ones,
+                 seg_slot=self.bt_slot, seg_pos0=self.bt_lens)
+        x, xb = self.x, self.xb
+        self._layer_stack(b)
+        self._head(self.bt_logits32, B)
+        self.x, self.xb = x, xb      # a captured step ends where it began
+        ho.sample(self.bt_logits32[:B] if B > 1 else self.b_logits, min_p,
+                  greedy, self.seed, self.rng_ctr, self.bt_gmax,
+                  self.bt_pick, self.bt_next, self.bt_ring, self.bt_nout,
+                  self.bt_lens, bump_len=True, temperature=temperature,
+                  cnt=self.bt_cnt, batch=B)
+
+    def prefill_batch(self, prompts) -> None:
+        """Prefill B prompts (ragged lengths) as one mixed step."""
+        seqs = [np.asarray(p, dtype=np.int32).ravel() for p in prompts]
+        B = len(seqs)
+        assert 1 <= B <= self.max_batch
+        lens = [len(s) for s in seqs]
+        if min(lens) == 0:
+            raise ValueError("empty prompt in batch")
+        if max(lens) + 1 >= self.max_seq:
+            raise ValueError(f"prompt {max(lens)} fills the "
+                             f"{self.max_seq} pool")
+        self.reset()
+        rows = [self._open_row(b) for b in range(B)]
+        with trace_range(f"prefill_batch[{B}]"):
+            out = self.step([StepEntry(q, s, [len(s) - 1])
+                             for q, s in zip(rows, seqs)])
+        self.bt_logits32[:B].copy_(out)
+        self.bt_lens[:B].copy_(torch.tensor(lens, dtype=torch.int32))
+        self._host_lens = lens + [0] * (self.max_batch - B)
+        self._batch_n = B
+
+    def prefill_row(self, b: int, ids, greedy: bool = True,
+                    min_p: float = 0.1, temperature: float = 1.0):
+        """Prefill one sequence into row b and sample its first token (a
+        request joining the group between decode chunks)."""
+        ids = np.asarray(ids, dtype=np.int32).ravel()
+        P = len(ids)
+        if P == 0:
+            raise ValueError("empty prompt")
+        assert 0 <= b < self.max_batch
+        if P + 1 >= self.max_seq:
+            raise ValueError(f"prompt {P} fills the {self.max_seq} pool")
+        logits = self.step([StepEntry(self._open_row(b), ids, [P - 1])])
+        self.bt_lens[b:b + 1].fill_(P)
+        self.bt_nout[b:b + 1].zero_()
+        ho.sample(logits[0], min_p, greedy, self.seed, self.rng_ctr,
+                  self.bt_gmax[b:b + 1], self.bt_pick[b:b + 1],
+                  self.bt_next[b:b + 1], self.bt_ring[b:b + 1],
+                  self.bt_nout[b:b + 1], self.bt_lens[b:b + 1],
+                  bump_len=False, temperature=temperature,
+                  cnt=self.bt_cnt[b:b + 1], batch=1)
+        self._host_lens[b] = P
+        self._batch_n = max(self._batch_n, b + 1)
+
+    def compact_row(self, dst: int, src: int):
+        """Row dst is finished: its pages and slot are freed and row src
+        takes its place (no cache data moves)."""
+        if self.rows[dst] is not None:
+            self.cache.close(self.rows[dst])
+            self.rows[dst] = None
+        if dst == src:
+            return
+        self.rows[dst], self.rows[src] = self.rows[src], None
+        for t in (self.bt_slot, self.bt_lens, self.bt_next, self.bt_nout,
+                  self.bt_gmax, self.bt_pick, self.bt_cnt):
+            t[dst:dst + 1].copy_(t[src:src + 1])
+        self.bt_ring[dst].copy_(self.bt_ring[src])
+        self._host_lens[dst] = self._host_lens[src]

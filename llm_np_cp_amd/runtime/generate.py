@@ -299,7 +299,8 @@ def load_model(model_dir_or_preset: str, backend: str = "auto",
     mirrors the reference's ``snapshot_download`` flow
     (``llama3.2_model.py:1090``) and fails with a clear error when the
     machine has no network access.
-    ``backend``: "numpy" (CPU oracle), "gpu" (HIP engine), or "auto".
+    ``backend``: "numpy" (CPU oracle; Llama-style families only), "gpu"
+    (HIP engine), or "auto".
     ``max_batch``: >1 allocates per-sequence KV pools on the GPU engine
     (lockstep batched decode / continuous-batching server); ignored by
     the NumPy oracle.
@@ -310,14 +311,15 @@ def load_model(model_dir_or_preset: str, backend: str = "auto",
     """
     import os
 
-    from ..core.config import preset_config, PRESETS
+    from ..core.config import has_preset, preset_config, preset_names
     from ..io.loader import load_config, load_weights_numpy, random_weights
+    from ..models.registry import engine_class, oracle_class
 
     weights_dir = None
     if os.path.isdir(model_dir_or_preset):
         config = load_config(model_dir_or_preset)
         weights_dir = tok_dir = model_dir_or_preset
-    elif model_dir_or_preset.lower() in PRESETS:
+    elif has_preset(model_dir_or_preset):
         config = preset_config(model_dir_or_preset)
         weights = random_weights(config, seed=seed)
         tok_dir = None
@@ -328,7 +330,7 @@ def load_model(model_dir_or_preset: str, backend: str = "auto",
     else:
         raise FileNotFoundError(
             f"{model_dir_or_preset!r} is neither a directory, a preset "
-            f"({sorted(PRESETS)}), nor an HF repo id")
+            f"({preset_names()}), nor an HF repo id")
 
     if backend == "auto":
         try:
@@ -371,15 +373,18 @@ def load_model(model_dir_or_preset: str, backend: str = "auto",
         tokenizer = ByteTokenizer()
 
     if backend == "numpy":
-        from ..models.numpy_ref import NumpyModel, NumpyKVCache
+        from ..models.numpy_ref import NumpyKVCache
 
-        model = NumpyModel(config, weights)
+        cls = oracle_class(config)
+        if cls is None:
+            raise ValueError(f"{config.model_type} has no CPU backend; it "
+                             f"needs an MI355X (backend='gpu')")
+        model = cls(config, weights)
         model.make_cache = lambda n: NumpyKVCache(config, n)
     elif backend == "gpu":
-        from ..models.engine import GPUModel
-
-        model = GPUModel(config, weights, dtype=dtype, max_seq=max_seq,
-                         kv_dtype=kv_dtype, max_batch=max_batch)
+        model = engine_class(config)(config, weights, dtype=dtype,
+                                     max_seq=max_seq, kv_dtype=kv_dtype,
+                                     max_batch=max_batch)
     else:
         raise ValueError(f"unknown backend {backend!r}")
     return tokenizer, model, config

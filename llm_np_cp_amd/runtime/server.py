@@ -249,7 +249,7 @@ def build_app(model_name: str = "llama-3.2-1b", backend: str = "auto",
     else:
         # GPU engines built with batch pools serve the lockstep group
         can_batch = (max_batch > 1
-                     and type(model).__name__ == "GPUModel")
+                     and hasattr(model, "decode_rows"))
 
     eos = getattr(cfg, "eos_token_id", None)
     eos_set = (set() if eos is None else {int(eos)}
@@ -580,7 +580,7 @@ def main():
     ap.add_argument("--model", default="llama-3.2-1b")
     ap.add_argument("--backend", default="auto")
     ap.add_argument("--dtype", default="bf16",
-                    choices=["bf16", "fp8", "fp4"])
+                    choices=["bf16", "fp8", "fp4", "fp32"])
     ap.add_argument("--kv-dtype", default="bf16", choices=["bf16", "fp8"])
     ap.add_argument("--max-seq", type=int, default=4096)
     ap.add_argument("--max-batch", type=int, default=8)

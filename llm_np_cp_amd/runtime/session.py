@@ -88,7 +88,8 @@ class ChatSession:
         t1 = time.perf_counter()
         greedy_or_minp = self.params.strategy in ("greedy", "min_p")
         if (hasattr(self.model, "decode") and greedy_or_minp
-                and not self.params.logit_bias):
+                and not self.params.logit_bias
+                and not getattr(self.model, "no_rewind", False)):
             # GPU engine: continue with the device-side hipGraph loop
             # (the prefill logits above are already in b_logits)
             produced = 0

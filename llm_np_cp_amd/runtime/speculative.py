@@ -123,6 +123,11 @@ def generate_speculative(prompt: str, tokenizer, draft, target,
     """
     if k < 1:
         raise ValueError("k must be >= 1")
+    for m in (draft, target):
+        if getattr(m, "no_rewind", False):
+            raise ValueError(
+                f"speculative decoding rolls rejected drafts back; "
+                f"{m.config.model_type} carries recurrent state and cannot")
     if params is None:
         params = SamplingParams(strategy="greedy")
     rng = np.random.default_rng(params.seed)
