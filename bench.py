@@ -22,6 +22,81 @@ import time
 sys.path.insert(0, os.path.dirname(os.path.abspath(__file__)))
 
 
+def compare(cases, steps, warmup, prompt=2048, batches=(1, 4, 16)):
+    """One JSON line per model, size and batch: random weights, bf16,
+    synthetic prompts.  The transformer gets one more expert and one more
+    choice, so its experts match the design's routed + shared ones in
+    stored and in active parameters."""
+    import numpy as np
+    import torch
+
+    from csrc.build import ensure_built
+    ensure_built()
+    import llm_np_cp_amd as L
+    from llm_np_cp_amd.io.loader import LazyRandomWeights
+    from llm_np_cp_amd.models.registry import engine_class
+
+    def transformer(c):
+        lat = c.layers[0]
+        return L.ModelConfig(
+            model_type="mixtral", vocab_size=c.vocab_size,
+            hidden_size=c.hidden_size, intermediate_size=lat.mlp.expert.ff,
+            num_hidden_layers=len(c.runs),
+            num_attention_heads=lat.mixer.heads,
+            num_key_value_heads=max(1, lat.mixer.heads // 4), head_dim=128,
+            max_position_embeddings=32768, tie_word_embeddings=False,
+            num_local_experts=lat.mlp.experts + 1,
+            num_experts_per_tok=lat.mlp.top + 1)
+
+    def seconds(fn, n):
+        torch.cuda.synchronize()
+        t = time.perf_counter()
+        for _ in range(n):
+            fn()
+        torch.cuda.synchronize()
+        return (time.perf_counter() - t) / n
+
+    for case in cases:
+        size, _, side = case.partition(":")
+        design = L.preset_config(f"turudra-{size}")
+        for name, cfg in (("turudra", design),
+                          ("mixtral", transformer(design))):
+            if side and side != name:
+                continue
+            rng = np.random.default_rng(0)
+            ids = rng.integers(0, cfg.vocab_size, size=(max(batches),
+                                                        prompt))
+            line = {"model": f"{name}-{size}", "dtype": "bf16",
+                    "data": "synthetic",
+                    "layers": len(getattr(cfg, "runs", ())) or
+                    cfg.num_hidden_layers}
+
+            def show(what, dt, tokens):
+                print(json.dumps({**line, "what": what, "ms": dt * 1e3,
+                                  "tokens/s": tokens / dt}), flush=True)
+
+            # a single-sequence engine for batch 1 (its own fused path in
+            # the transformer), then one with rows for the batches
+            for rows in (1, max(batches)):
+                model = engine_class(cfg)(
+                    cfg, LazyRandomWeights(cfg, seed=0), max_seq=4096,
+                    max_batch=rows, seed=0)
+                if rows == 1:
+                    model.prefill(ids[0])
+                    show(f"prefill {prompt}",
+                         seconds(lambda: model.prefill(ids[0]), 5), prompt)
+                    model.decode(max(warmup, 3), greedy=True)
+                    show(f"decode batch 1 at {prompt}+",
+                         seconds(lambda: model._graph.replay(), steps), 1)
+                for B in [b for b in batches if b > 1 and rows > 1]:
+                    model.prefill_batch(ids[:B])
+                    model.decode_batch(max(warmup, 3), greedy=True)
+                    show(f"decode batch {B} at {prompt}+",
+                         seconds(lambda: model._graph.replay(), steps), B)
+                del model
+                torch.cuda.empty_cache()
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -46,7 +121,15 @@ def main():
                     help="lockstep batched decode (throughput mode; "
                          "value = aggregate tokens/s over the batch)")
     ap.add_argument("--no-graph", action="store_true")
+    ap.add_argument("--compare", nargs="*", default=None, metavar="CASE",
+                    help="instead of the default workload: prefill and "
+                         "decode throughput of the layer-list design beside "
+                         "the MoE transformer of equal size; cases "
+                         "2k, 4k (default both), each optionally with "
+                         ":turudra or :mixtral for one side only")
     args = ap.parse_args()
+    if args.compare is not None:
+        return compare(args.compare or ["2k", "4k"], args.steps, args.warmup)
 
     import numpy as np
     import torch

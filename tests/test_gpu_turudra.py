@@ -1,0 +1,696 @@
+"""Turudra on the GPU against the plain oracle (float64): every mechanism
+alone, any cut of the tokens, mixed batches, reused pages and slots, keys
+that stand out, long decoding and the framework's generation paths.
+
+Caches and states start filled with NaN, so reading a position or a state
+that the sequence has not written fails the comparison.
+"""
+
+import json
+import os
+import subprocess
+import sys
+
+import numpy as np
+import pytest
+import torch
+
+from turudra_cases import (config, default, greedy, latent, mlstm, moe, rel,
+                           save, tokens, weights, worst)
+from turudra_oracle import Oracle, expert, route
+
+pytestmark = pytest.mark.gpu
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+
+EXACT = 2e-4        # fp32 engine against float64, worst row
+ROUNDED = 6e-2      # bf16 engine, all rows together
+
+
+def engine(cfg, w, dtype="fp32", max_seq=320, max_batch=4, **kw):
+    from llm_np_cp_amd.core.layered import LayeredConfig
+    from llm_np_cp_amd.models.layered import LayeredModel
+
+    m = LayeredModel(LayeredConfig.from_dict(cfg), w, dtype=dtype,
+                     max_seq=max_seq, max_batch=max_batch, **kw)
+    for c in m.caches:
+        for t in (c if isinstance(c, tuple) else (c,)):
+            t.fill_(float("nan"))
+    return m
+
+
+def entry(seq, toks, want=None):
+    from llm_np_cp_amd.models.layered import StepEntry
+    return StepEntry(seq, toks, range(len(toks)) if want is None else want)
+
+
+def run(m, t, cuts=None):
+    """Logits of every token of t fed in portions of the given sizes."""
+    s, out, at = m.open_sequence(), [], 0
+    for n in cuts or [len(t)]:
+        out.append(m.step([entry(s, t[at:at + n])]).cpu().numpy())
+        at += n
+    assert at == len(t)
+    m.close_sequence(s)
+    return np.concatenate(out)
+
+
+def cut(total, sizes):
+    out, i = [], 0
+    while sum(out) < total:
+        out.append(min(sizes[i % len(sizes)], total - sum(out)))
+        i += 1
+    return out
+
+
+# ---------------------------------------------------------------- kernels
+
+def _dev(a, dtype=torch.float32):
+    return torch.from_numpy(np.asarray(a, np.float32)).to("cuda", dtype)
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("rows, width", [(1, 88), (2, 200), (3, 64), (5, 513),
+                                         (7, 320), (8, 136), (13, 96),
+                                         (16, 1030)])
+def test_few_row_linear(dtype, rows, width):
+    """Fused norm / concatenation + projection + soft cap of a few rows."""
+    from llm_np_cp_amd.ops import hybrid_ops as hy
+
+    rng = np.random.default_rng(rows)
+    N, Kp = 77, -(-width // 64) * 64
+    x = rng.standard_normal((rows + 2, width)) * 3
+    x0 = rng.standard_normal((rows + 2, width))
+    g = rng.standard_normal(width) + 1
+    pick = rng.permutation(rows + 2)[:rows].astype(np.int32)
+    tol = 1e-5 if dtype == torch.float32 else 1e-2
+    W = rng.standard_normal((N, width)) / np.sqrt(width)
+    Wp = torch.zeros(N, Kp, dtype=dtype, device="cuda")
+    Wp[:, :width] = _dev(W, dtype)
+    Wr = Wp[:, :width].double().cpu().numpy()
+    y = torch.full((rows, N + 3), 7.0, device="cuda")
+    h = torch.full((rows, Kp), float("nan"), dtype=dtype, device="cuda")
+    hy.lin_rows(Wp, _dev(x), y, rows, width, N + 3, 1e-5, g=_dev(g),
+                rows=torch.from_numpy(pick).cuda(), hout=h, cap=2.5)
+    n = x[pick] / np.sqrt((x[pick] ** 2).mean(-1, keepdims=True) + 1e-5) * g
+    assert rel(y[:, :N].cpu(), 2.5 * np.tanh(n @ Wr.T / 2.5)) < tol
+    assert (y[:, N:] == 7.0).all()
+    assert rel(h[:, :width].double().cpu(), n) < tol
+    assert (h[:, width:] == 0).all()
+    K2 = -(-2 * width // 64) * 64
+    W2 = torch.zeros(N, K2, dtype=dtype, device="cuda")
+    W2[:, :2 * width] = _dev(rng.standard_normal((N, 2 * width)), dtype)
+    y2 = torch.empty(rows, N, device="cuda")
+    hy.lin_rows(W2, _dev(x), y2, rows, width, N, 1e-5, x0=_dev(x0))
+    both = np.concatenate([x, x0], -1)[:rows]
+    assert rel(y2.cpu(), both @ W2[:, :2 * width].double().cpu().numpy().T) \
+        < tol
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("M, N, K", [(2, 40, 64), (16, 33, 192), (17, 70, 64),
+                                     (33, 130, 128), (64, 65, 320),
+                                     (65, 64, 64), (200, 257, 448),
+                                     (2500, 2049, 64)])
+def test_gemm_epilogues(dtype, M, N, K):
+    from llm_np_cp_amd.ops import hybrid_ops as hy
+
+    g = torch.Generator(device="cuda").manual_seed(M)
+    R = lambda *s: torch.randn(*s, device="cuda", generator=g)
+    X, W = R(M, K + 64).to(dtype), (R(N, K) / K ** 0.5).to(dtype)
+    ref = (X[:, :K].double() @ W.double().T).cpu().numpy()
+    tol = 1e-5
+    tt = 1e-5 if dtype == torch.float32 else 5e-3
+    Y = torch.full((M, N + 5), 3.0, device="cuda")
+    hy.gemm_rows(X, W, Y, M, K + 64, N + 5, hy.EPI_F32)
+    assert rel(Y[:, :N].cpu(), ref) < tol and (Y[:, N:] == 3.0).all()
+    x = R(M, N)
+    want = x.double().cpu().numpy() + 0.3 * ref
+    hy.gemm_rows(X, W, x, M, K + 64, N, hy.EPI_RESADD, mult=0.3)
+    assert rel(x.cpu(), want) < tol
+    hy.gemm_rows(X, W, x, M, K + 64, N, hy.EPI_SOFTCAP, mult=1.5)
+    assert rel(x.cpu(), 1.5 * np.tanh(ref / 1.5)) < tol
+    hy.gemm_rows(X, W, x, M, K + 64, N, hy.EPI_SOFTCAP, mult=0.0)
+    assert rel(x.cpu(), ref) < tol
+    T = torch.empty(M, N, dtype=dtype, device="cuda")
+    hy.gemm_rows(X, W, T, M, K + 64, N, hy.EPI_T)
+    assert rel(T.double().cpu(), ref) < tt
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("M", [3, 40, 90])
+def test_gemm_per_head_with_gate(dtype, M):
+    from llm_np_cp_amd.ops import hybrid_ops as hy
+
+    Z, N, K = 3, 20, 64
+    g = torch.Generator(device="cuda").manual_seed(1)
+    R = lambda *s: torch.randn(*s, device="cuda", generator=g)
+    X, W, G = R(M, Z, K).to(dtype), R(Z, N, K).to(dtype), R(M, Z + 2)
+    out = torch.zeros(M, 64, dtype=dtype, device="cuda")
+    hy.gemm_rows(X, W, out, M, Z * K, 64, hy.EPI_TGATE, N=N, K=K, Z=Z, xz=K,
+                 wz=N * K, yz=N, gate=G[:, 1:], ldg=Z + 2)
+    ref = torch.stack([X[:, z].double() @ W[z].double().T *
+                       torch.sigmoid(G[:, 1 + z].double())[:, None]
+                       for z in range(Z)], 1).reshape(M, Z * N)
+    assert rel(out[:, :Z * N].double().cpu(), ref.cpu()) < (
+        1e-5 if dtype == torch.float32 else 5e-3)
+    assert (out[:, Z * N:] == 0).all()
+
+
+@pytest.mark.parametrize("E, top, shared, ff, sff", [
+    (5, 2, True, 40, 72), (4, 4, True, 72, 24), (6, 1, False, 16, 0),
+    (1, 1, True, 64, 64), (70, 5, True, 8, 200), (130, 7, False, 24, 0)])
+@pytest.mark.parametrize("T", [1, 4, 6, 23, 180])
+def test_experts_alone(E, top, shared, ff, sff, T):
+    """A block whose mixer writes nothing: routing, clamps and weights."""
+    cfg = config([(latent(2), moe(E, top, ff, 0.7, sff if shared else None,
+                                  0.4))], width=72)
+    w = weights(cfg)
+    w["l0.mix.o"] *= 0
+    t = tokens(cfg, T)
+    want, _ = Oracle(cfg, w).run(t)
+    m = engine(cfg, w)
+    assert worst(run(m, t), want) < EXACT
+    if T <= 23:
+        assert worst(run(m, t, [1] * T), want) < EXACT
+
+
+def test_clamps_and_choice_matter():
+    """The limits bind and the choice is uneven in the expert tests."""
+    cfg = config([(latent(2), moe(5, 2, 40, 0.7, 72, 0.4))], width=72)
+    w = weights(cfg)
+    h = np.random.default_rng(0).standard_normal((60, 72))
+    g, u = h @ w["l0.mlp.e0.gate"].T, h @ w["l0.mlp.e0.up"].T
+    assert (g > 0.7).mean() > 0.1 and (abs(u) > 0.7).mean() > 0.2
+    idx, wt = route(h @ w["l0.mlp.router"].T, 2)
+    assert len(np.unique(idx)) == 5 and wt[:, 0].min() >= 0.5
+    assert rel(expert(w, "l0.mlp.e0.", 1e9, h),
+               expert(w, "l0.mlp.e0.", 0.7, h)) > 0.1
+
+
+LATENTS = [latent(), latent(1, 8, 4, 8, 16), latent(2, 33, 34, 65, 64, 20),
+           latent(7, 64, 32, 16, 65, base=77.0), latent(17, 16, 16, 24, 128),
+           latent(70, 8, 8, 4, 130), latent(2, 130, 64, 130, 257),
+           latent(4, 40, 128, 72, 385, scale=0.02),
+           latent(3, 16, 36, 12, 512, 2)]
+
+
+@pytest.mark.parametrize("k", range(len(LATENTS)))
+@pytest.mark.parametrize("dtype", ["fp32", "bf16"])
+def test_latent_attention_alone(k, dtype):
+    cfg = config([(LATENTS[k], None)])
+    w, t = weights(cfg), None
+    t = tokens(cfg, 150)
+    want, _ = Oracle(cfg, w).run(t)
+    m = engine(cfg, w, dtype)
+    for cuts in (None, [1] * 70 + [2, 78], [64, 1, 65, 20]):
+        got = run(m, t, cuts)
+        if dtype == "fp32":
+            assert worst(got, want) < EXACT, cuts
+        else:
+            assert rel(got, want) < ROUNDED, cuts
+
+
+MEMORIES = [mlstm(), mlstm(1, 4, 4), mlstm(3, 64, 64, 2.0), mlstm(2, 100, 30),
+            mlstm(5, 16, 130), mlstm(1, 200, 200, 30.0)]
+
+
+@pytest.mark.parametrize("k", range(len(MEMORIES)))
+@pytest.mark.parametrize("dtype", ["fp32", "bf16"])
+def test_mlstm_alone(k, dtype):
+    cfg = config([(MEMORIES[k], None)])
+    w, t = weights(cfg, k), tokens(cfg, 200)
+    want, _ = Oracle(cfg, w).run(t)
+    m = engine(cfg, w, dtype)
+    for cuts in (None, [1] * 70 + [2, 128], [63, 1, 65, 64, 7]):
+        got = run(m, t, cuts)
+        if dtype == "fp32":
+            assert worst(got, want) < EXACT, cuts
+        else:
+            assert rel(got, want) < ROUNDED, cuts
+
+
+@pytest.mark.parametrize("ib, fb", [(-40.0, 40.0), (40.0, 40.0),
+                                    (-40.0, -40.0), (40.0, -40.0)])
+def test_mlstm_gates_at_their_caps(ib, fb):
+    """Both gates saturated either way: pure integration, overwriting, and
+    inputs small enough that the e^-m floor of the divisor decides."""
+    cfg = config([(mlstm(2, 24, 40, 12.0), None)])
+    w, t = weights(cfg), tokens(cfg, 190)
+    w["l0.mix.i.b"][:] = ib
+    w["l0.mix.f.b"][:] = fb
+    want, _ = Oracle(cfg, w).run(t)
+    m = engine(cfg, w)
+    assert worst(run(m, t), want) < EXACT
+    assert worst(run(m, t, cut(190, [5, 1, 70, 2])), want) < EXACT
+
+
+@pytest.mark.parametrize("loop", [(0, 1, 1), (0, 2, 3), (1, 2, 2), (1, 3, 4)])
+def test_loop_alone(loop):
+    """Mixers that write nothing: only W_in [x; x0] per pass is left."""
+    cfg = config([(latent(2), None), (mlstm(), None), (latent(2), None)],
+                 loop=loop)
+    w, t = weights(cfg), tokens(cfg, 9)
+    for i in range(3):
+        w[f"l{i}.mix.o"] *= 0
+    want, _ = Oracle(cfg, w).run(t)
+    m = engine(cfg, w)
+    assert worst(run(m, t), want) < EXACT
+    assert worst(run(m, t, [1] * 9), want) < EXACT
+
+
+def test_loop_passes_keep_their_own_cache():
+    cfg = config([(latent(), None), (mlstm(), None)], loop=(0, 2, 3))
+    w, t = weights(cfg), tokens(cfg, 80)
+    want, _ = Oracle(cfg, w).run(t)
+    m = engine(cfg, w)
+    assert len(m.caches) == 6
+    assert worst(run(m, t), want) < EXACT
+    assert worst(run(m, t, [1] * 80), want) < EXACT
+
+
+@pytest.mark.parametrize("kw", [dict(cap=None), dict(emb=1.0, mult=1.0),
+                                dict(width=64, vocab=64), dict(width=130),
+                                dict(eps=0.3), dict(vocab=1001)])
+def test_stack_constants(kw):
+    cfg = config([(latent(2), moe()), (mlstm(), None)], **kw)
+    w, t = weights(cfg), tokens(cfg, 21)
+    want, _ = Oracle(cfg, w).run(t)
+    m = engine(cfg, w)
+    assert worst(run(m, t), want) < EXACT
+    assert worst(run(m, t, [1] * 21), want) < EXACT
+
+
+# ------------------------------------------------------------- whole model
+
+@pytest.fixture(scope="module")
+def model():
+    cfg = default()
+    w = weights(cfg)
+    t = tokens(cfg, 300)
+    return cfg, w, t, Oracle(cfg, w).run(t)[0]
+
+
+def test_residual_after_every_layer_run(model):
+    cfg, w, t, _ = model
+    trace = []
+    logits, _ = Oracle(cfg, w).run(t[:30], trace=trace)
+    m = engine(cfg, w)
+    got, hidden = m.forward_full(t[:30], return_hidden_states=True)
+    assert len(hidden) == len(trace) + 1
+    for a, b in zip(hidden[1:], trace):
+        assert worst(a, b) < EXACT
+    assert worst(got, logits) < EXACT
+
+
+@pytest.mark.parametrize("sizes", [[300], [1], [2], [3, 1], [5, 2, 1],
+                                   [63, 65], [64], [100, 1, 1, 27],
+                                   [17, 2, 2, 130]])
+def test_any_cut_gives_the_same_logits(model, sizes):
+    cfg, w, t, want = model
+    m = engine(cfg, w)
+    assert worst(run(m, t, cut(300, sizes)), want) < EXACT
+
+
+def test_scratch_smaller_than_the_step(model):
+    """A step beyond the scratch rows runs as several batches."""
+    cfg, w, t, want = model
+    m = engine(cfg, w, prefill_chunk=64)
+    assert m.PC == 64
+    assert worst(run(m, t), want) < EXACT
+    a, b = m.open_sequence(), m.open_sequence()
+    got = m.step([entry(a, t[:50]), entry(b, t[:70])]).cpu().numpy()
+    assert worst(got, np.concatenate([want[:50], want[:70]])) < EXACT
+
+
+def test_bf16_whole_model():
+    """Rounding only: with every expert chosen no close call can flip."""
+    cfg = config([(latent(), moe(3, 3)), (mlstm(), moe(3, 3)),
+                  (latent(5, 12, 8, 16, 70, 6), None)], loop=(0, 2, 2))
+    w, t = weights(cfg), tokens(cfg, 200)
+    want, _ = Oracle(cfg, w).run(t)
+    m = engine(cfg, w, "bf16")
+    for sizes in ([200], [1], [2, 70, 1]):
+        assert rel(run(m, t, cut(200, sizes)), want) < ROUNDED
+
+
+def test_mixed_batches_with_reuse(model):
+    """Random schedules over four live requests in a pool that is smaller
+    than their sum: every logit equals the request's own run."""
+    cfg, w, _, _ = model
+    o = Oracle(cfg, w)
+    reqs = [tokens(cfg, n, 10 + i) for i, n in enumerate(
+        [150, 3, 64, 97, 1, 130, 65, 40, 128, 2, 77])]
+    want = [o.run(t)[0] for t in reqs]
+    m = engine(cfg, w, max_seq=192, pool_tokens=64 * 8)
+    rng = np.random.default_rng(5)
+    todo, live, at, used = list(range(len(reqs))), {}, {}, set()
+    while todo or live:
+        while todo and len(live) < 4:
+            r = todo[0]
+            held = sum(-(-len(reqs[k]) // 64) for k in live)
+            if held + -(-len(reqs[r]) // 64) > 8:
+                break
+            live[todo.pop(0)] = m.open_sequence()
+            at[r] = 0
+        step, refs = [], []
+        for r in rng.permutation(list(live)):
+            if len(live) > 1 and rng.random() < 0.2:
+                continue                       # left out of this step
+            left = len(reqs[r]) - at[r]
+            n = min(left, int(rng.choice([1, 1, 2, 3, 17, 63, 64, 65])))
+            step.append(entry(live[r], reqs[r][at[r]:at[r] + n]))
+            refs.append(want[r][at[r]:at[r] + n])
+            at[r] += n
+        if not step:
+            continue
+        got = m.step(step).cpu().numpy()
+        assert worst(got, np.concatenate(refs)) < EXACT
+        for r in list(live):
+            used |= {(r, p) for p in live[r].pages}
+            if at[r] == len(reqs[r]):
+                m.close_sequence(live.pop(r))
+    pages = [p for _, p in used]
+    assert len(pages) > len(set(pages))        # pages did change hands
+    assert m.cache.free_pages == 8 and m.cache.free_slots == 4
+
+
+@pytest.mark.parametrize("rows", [2, 3, 5, 8, 9, 16, 19, 40])
+def test_many_single_tokens_in_one_step(model, rows):
+    """Decode batches of every size class, at unequal lengths."""
+    cfg, w, t, want = model
+    m = engine(cfg, w, max_batch=rows)
+    seqs = [m.open_sequence() for _ in range(rows)]
+    lens = [1 + (7 * i) % 90 for i in range(rows)]
+    m.step([entry(s, t[:n], []) for s, n in zip(seqs, lens)])
+    for k in range(3):
+        got = m.step([entry(s, t[n + k:n + k + 1])
+                      for s, n in zip(seqs, lens)]).cpu().numpy()
+        assert worst(got, np.stack([want[n + k] for n in lens])) < EXACT
+
+
+def test_wanted_places_and_order(model):
+    cfg, w, t, want = model
+    m = engine(cfg, w)
+    a, b, c = (m.open_sequence() for _ in range(3))
+    got = m.step([entry(a, t[:20], [19, 0, 7]), entry(b, t[:1], [0]),
+                  entry(c, t[:33], [])]).cpu().numpy()
+    assert worst(got, want[[19, 0, 7, 0]]) < EXACT
+    assert m.step([entry(c, t[33:40], [])]).shape == (0, cfg["vocab"])
+
+
+def test_step_errors_leave_the_cache_usable(model):
+    from llm_np_cp_amd.runtime.cache_manager import CacheFull
+
+    cfg, w, t, want = model
+    m = engine(cfg, w, max_seq=256, pool_tokens=128, max_batch=2)
+    a, b = m.open_sequence(), m.open_sequence()
+    m.step([entry(a, t[:60], [])])
+    with pytest.raises(CacheFull):
+        m.step([entry(a, t[60:70]), entry(b, t[:65])])
+    assert (a.length, b.length, m.cache.free_pages) == (60, 0, 1)
+    for bad in ([entry(a, t[:0])], [entry(a, t[:2], [2])],
+                [entry(a, [cfg["vocab"]])], [entry(a, [-1])],
+                [entry(a, t[:2]), entry(a, t[:2])],
+                [entry(a, np.zeros(200, np.int32))]):
+        with pytest.raises(ValueError):
+            m.step(bad)
+    got = m.step([entry(a, t[60:64])]).cpu().numpy()
+    assert worst(got, want[60:64]) < EXACT
+
+
+# ------------------------------------------------------ keys that stand out
+
+def _needle(at, total):
+    """A model and prompt in which the last token attends to one position
+    almost alone: only token 1, placed there, writes the latent direction
+    that only token 2, placed last, asks for."""
+    cfg = config([(latent(2, 24, 8, 32, 40, base=1e6, scale=0.4), None)],
+                 width=64, emb=1.0, cap=None, mult=1.0)
+    w = weights(cfg, 9)
+    w["embed"][:, :8] = 0
+    w["embed"][2, :4] = w["embed"][1, 4:8] = 3.0
+    w["l0.mix.q"][:, 4:8] = w["l0.mix.dkv"][:, :4] = 0
+    w["l0.mix.dkv"][:4, 4:8] = 2.0
+    w["l0.mix.o"] *= 4.0
+    q = np.random.default_rng(2).standard_normal(24)
+    for h in range(2):
+        w["l0.mix.q"][h * 32:h * 32 + 24, :4] = q[:, None] * 0.6
+        w["l0.mix.uk"][h * 24:(h + 1) * 24, :4] = q[:, None] * 0.6
+    t = 3 + tokens(cfg, total) % (cfg["vocab"] - 3)
+    t[at], t[-1] = 1, 2
+    return cfg, w, t.astype(np.int32)
+
+
+@pytest.mark.parametrize("total", [64, 65, 130, 257])
+@pytest.mark.parametrize("at", [0, 1, 15, 16, 31, 32, 62, 63, 64, 127, 128])
+def test_key_that_stands_out(at, total):
+    if at >= total - 1:
+        pytest.skip("beyond the prompt")
+    cfg, w, t = _needle(at, total)
+    o = Oracle(cfg, w)
+    want, _ = o.run(t)
+    gone = t.copy()
+    gone[at] = 3
+    assert worst(o.run(gone)[0][-1:], want[-1:]) > 0.1     # it does show
+    m = engine(cfg, w)
+    for cuts in ([total], [total - 1, 1], [total - 2, 2],
+                 cut(total - 1, [50, 3]) + [1]):
+        assert worst(run(m, t, cuts)[-1:], want[-1:]) < EXACT
+    b = engine(cfg, w, "bf16")
+    for cuts in ([total], [total - 1, 1]):
+        assert rel(run(b, t, cuts)[-1:], want[-1:]) < ROUNDED
+
+
+def test_far_key_while_decoding():
+    """The asking token comes at every place after a long decode."""
+    cfg, w, t = _needle(5, 200)
+    o = Oracle(cfg, w)
+    m = engine(cfg, w)
+    s = m.open_sequence()
+    m.step([entry(s, t[:10], [])])
+    _, st = o.run(t[:10])
+    for k in range(10, 150):
+        ask = 2 if k % 9 == 0 else int(t[k])
+        z, st = o.run([ask], st)
+        got = m.step([entry(s, [ask])]).cpu().numpy()
+        assert worst(got, z) < EXACT, k
+
+
+def test_memory_reaches_back():
+    """With the forget gate open, the first token still shapes the memory
+    200 tokens on; swapping it must show, and the engine must follow."""
+    cfg = config([(mlstm(2, 24, 40, 20.0), None)])
+    w, t = weights(cfg), tokens(cfg, 200)
+    w["l0.mix.f.b"][:] = 8.0
+    w["l0.mix.i"] *= 0
+    w["l0.mix.i.b"][:] = 0
+    other = t.copy()
+    other[0] = (t[0] + 5) % cfg["vocab"]
+    o = Oracle(cfg, w)
+    want, _ = o.run(t)
+    assert worst(o.run(other)[0][-1:], want[-1:]) > 10 * EXACT
+    m = engine(cfg, w)
+    for cuts in ([200], [199, 1], cut(200, [64, 1, 2])):
+        assert worst(run(m, t, cuts), want) < EXACT
+
+
+# ---------------------------------------------------- generation and serving
+
+def test_long_greedy_decode_graph_and_eager(model):
+    cfg, w, t, _ = model
+    want, margin = greedy(cfg, w, t[:5], 180)
+    assert margin > 1e-4
+    m = engine(cfg, w)
+    for graph in (True, False, True):
+        m.prefill(t[:5])
+        ids = m.decode(180, greedy=True, use_graph=graph)
+        assert ids.tolist() == want
+    assert m._graph_mode is not None and not getattr(m, "_graph_failed", 0)
+    # chunks of the loop, and a token fed by hand afterwards
+    m.prefill(t[:5])
+    ids = np.concatenate([m.decode(n, greedy=True, first_from_logits=k == 0)
+                          for k, n in enumerate([3, 16, 1, 60])])
+    assert ids.tolist() == want[:80]
+
+
+@pytest.mark.parametrize("B", [2, 4, 11])
+def test_batched_generation(model, B):
+    cfg, w, t, _ = model
+    prompts = [t[i:i + 1 + 13 * i % 70] for i in range(B)]
+    m = engine(cfg, w, max_batch=B)
+    out = m.generate_tokens_batch(prompts, 40)
+    for p, ids in zip(prompts, out):
+        want, margin = greedy(cfg, w, p, 40)
+        assert margin < 1e-4 or ids.tolist() == want
+
+
+def test_rows_join_and_leave(model):
+    """The server's row primitives: join, decode, retire, compact."""
+    cfg, w, t, _ = model
+    m = engine(cfg, w, max_batch=3)
+    prompts = {0: t[:9], 1: t[20:85], 2: t[40:43], 3: t[:70]}
+    want = {k: greedy(cfg, w, p, 20)[0] for k, p in prompts.items()}
+    rows, got = [], {}
+    for k in (0, 1, 2):
+        m.prefill_row(k, prompts[k])
+        rows.append(k)
+        got[k] = [int(m.bt_next[k].item())]
+    free = m.cache.free_pages
+    for k, ids in zip(rows, m.decode_rows(3, 4)):
+        got[k] += ids.tolist()
+    m.compact_row(0, 2)                        # request 0 leaves
+    rows = [2, 1]
+    assert m.cache.free_pages > free - 1 and m.rows[2] is None
+    for k, ids in zip(rows, m.decode_rows(2, 5)):
+        got[k] += ids.tolist()
+    m.prefill_row(2, prompts[3])
+    rows.append(3)
+    got[3] = [int(m.bt_next[2].item())]
+    for k, ids in zip(rows, m.decode_rows(3, 6)):
+        got[k] += ids.tolist()
+    m.compact_row(2, 2)
+    assert m.rows[2] is None
+    for k in got:
+        assert got[k] == want[k][:len(got[k])], k
+
+
+def test_generate_session_and_rewind(model, tmp_path):
+    import llm_np_cp_amd as L
+
+    cfg, w, _, _ = model
+    cfg = config([(l["type"], l["mixer"]) and ((l["type"], l["mixer"]),
+                                              l["mlp"])
+                  for l in cfg["layers"]], vocab=300, loop=(1, 3, 2))
+    w = weights(cfg)
+    save(cfg, w, tmp_path / "m")
+    tok, m, c = L.load_model(str(tmp_path / "m"), dtype="fp32", max_seq=256)
+    p = L.SamplingParams(strategy="greedy")
+    prompt = "Once upon a time"
+    ids = list(prompt.encode())
+    want, _ = greedy(cfg, w, ids, 30)
+    fast = L.generate(prompt, tok, m, max_tokens=30, params=p, stream=False)
+    slow = L.generate(prompt, tok, m, max_tokens=30, params=p, stream=False,
+                      logprobs=2)
+    assert fast.token_ids == want and slow.token_ids == want
+    z, _ = Oracle(cfg, w).run(ids)
+    lp = z[-1] - z[-1].max()
+    lp -= np.log(np.exp(lp).sum())
+    assert abs(slow.logprobs[0]["logprob"] - lp[want[0]]) < 1e-3
+    assert len(L.generate(prompt, tok, m, max_tokens=12, params=L.
+               SamplingParams(strategy="min_p", seed=1), stream=False,
+               ).token_ids) == 12
+    s = L.ChatSession(tok, m)
+    a = s.send("Hi", max_tokens=6).token_ids
+    b = s.send("more", max_tokens=6).token_ids
+    hist = list(b"Hi")
+    assert a == greedy(cfg, w, hist, 6)[0]
+    assert b == greedy(cfg, w, hist + a + list(b"more"), 6)[0]
+    m.prefill(np.asarray(ids))
+    m.rewind(len(ids))
+    with pytest.raises(ValueError, match="recurrent"):
+        m.rewind(3)
+
+
+def test_rewind_without_recurrence():
+    cfg = config([(latent(), moe()), (latent(2), None)])
+    w, t = weights(cfg), tokens(cfg, 40)
+    m = engine(cfg, w)
+    m.prefill(t)
+    m.rewind(25)
+    want, _ = Oracle(cfg, w).run(np.concatenate([t[:25], t[:9]]))
+    assert worst(m.forward_positions(t[:9], 25), want[25:]) < EXACT
+
+
+def test_server_batches_requests(tmp_path):
+    """The HTTP scheduler: concurrent greedy requests in one lockstep
+    group give what each gives alone."""
+    pytest.importorskip("fastapi")
+    from concurrent.futures import ThreadPoolExecutor
+
+    from fastapi.testclient import TestClient
+
+    from llm_np_cp_amd.runtime.server import build_app
+
+    cfg = config([(latent(), moe()), (mlstm(), moe())], vocab=280)
+    w = weights(cfg)
+    save(cfg, w, tmp_path / "m")
+    app = build_app(str(tmp_path / "m"), backend="gpu", dtype="fp32",
+                    max_seq=256, max_batch=3, batch_window_ms=60)
+    prompts = ["a", "hello there", "x" * 70, "four", "The end."]
+    want = [bytes(i % 256 for i in greedy(cfg, w, list(p.encode()), 12)[0])
+            .decode("utf-8", errors="replace") for p in prompts]
+    with TestClient(app) as c:
+        def ask(p):
+            return c.post("/v1/completions", json={
+                "prompt": p, "max_tokens": 12, "strategy": "greedy",
+                "stop_on_eos": False}).json()["choices"][0]["text"]
+        with ThreadPoolExecutor(5) as ex:
+            got = list(ex.map(ask, prompts))
+        assert got == want
+        assert c.get("/stats").json()["max_group"] > 1
+
+
+def test_command_line(tmp_path):
+    cfg = config([(latent(), moe()), (mlstm(), None)], vocab=300)
+    w = weights(cfg)
+    save(cfg, w, tmp_path / "m")
+    p = subprocess.run(
+        [sys.executable, "-m", "llm_np_cp_amd", "abc", "--model",
+         str(tmp_path / "m"), "--backend", "gpu", "--dtype", "fp32",
+         "--strategy", "greedy", "--max-tokens", "8"], cwd=ROOT,
+        capture_output=True, timeout=100)
+    assert p.returncode == 0, p.stderr.decode()[-2000:]
+    want, _ = greedy(cfg, w, list(b"abc"), 8)
+    text = bytes(i % 256 for i in want).decode("utf-8", errors="replace")
+    assert text in p.stdout.decode("utf-8", errors="replace")
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_trace_run(tmp_path, dtype):
+    """The command: portions beside single tokens, slots given back and
+    taken again, more requests over time than slots."""
+    cfg = config([(latent(), moe(3, 3)), (mlstm(), moe(2, 2))],
+                 loop=(0, 1, 2))
+    w = weights(cfg)
+    save(cfg, w, tmp_path / "m")
+    (tmp_path / "out").mkdir()
+    o = Oracle(cfg, w)
+    reqs = {f"q{i}": tokens(cfg, n, i) for i, n in enumerate(
+        [70, 5, 64, 2, 66, 30])}
+    plan = [{"q0": 66, "q1": 2, "q2": 1}, {"q0": 1, "q1": 2, "q2": 60},
+            {"q0": 1, "q3": 2, "q1": 1}, {"q2": 3, "q4": 65}, {"q0": 2},
+            {"q4": 1, "q5": 29}, {"q5": 1}]
+    at, lines, refs = dict.fromkeys(reqs, 0), [], []
+    full = {k: o.run(t)[0] for k, t in reqs.items()}
+    for n, step in enumerate(plan):
+        entries, end, rows = [], [], []
+        for k, c in step.items():
+            lo, hi = at[k], at[k] + c
+            want = [] if n == 3 else [c - 1] if c < 4 else [0, c - 1]
+            entries.append({"id": k, "tokens": reqs[k][lo:hi].tolist(),
+                            "want": want})
+            rows += [full[k][lo + x] for x in want]
+            at[k] = hi
+            if hi == len(reqs[k]):
+                end.append(k)
+        lines.append(json.dumps({"step": n, "entries": entries, "end": end}))
+        refs.append(rows)
+    assert all(at[k] == len(reqs[k]) for k in reqs)
+    p = subprocess.run(
+        [os.path.join(ROOT, "bin", "trace_run"), "--model",
+         str(tmp_path / "m"), "--dtype", dtype, "--out",
+         str(tmp_path / "out"), "--max-tokens", "320"],
+        input=("\n".join(lines) + "\n").encode(), capture_output=True,
+        timeout=100)
+    assert p.returncode == 0, p.stderr.decode()[-2000:]
+    done = [l for l in p.stdout.decode().splitlines() if l.startswith("done")]
+    assert done == [f"done {n}" for n in range(len(plan))]
+    for n, rows in enumerate(refs):
+        f = tmp_path / "out" / f"{n}.f32"
+        assert f.exists() == bool(rows)
+        if rows:
+            got = np.fromfile(f, "<f4").reshape(-1, cfg["vocab"])
+            if dtype == "float32":
+                assert worst(got, np.stack(rows)) < EXACT
+            else:
+                assert rel(got, np.stack(rows)) < ROUNDED
