@@ -101,49 +101,51 @@ __global__ void __launch_bounds__(256) k_latent_prep(LatentArgs a) {
                     a.rwt, r);
 }
 
-// ---- few rows: absorb W_uk per (head, row); one more block per row does
-// ---- the cache row and the routing ------------------------------------
+// ---- few rows: absorb W_uk per (head, latent columns, row); two more
+// ---- blocks per row do the cache row and the routing --------------------
+#define AB_COLS 128
 template <typename T>
 __global__ void __launch_bounds__(256) k_latent_dec_prep(LatentArgs a) {
-  __shared__ float red[256 * 8 + 256];
-  const int h = blockIdx.x, r = blockIdx.y;
-  if (h == a.H) {
-    latent_write<T>(a, r, red);
-    if (a.E > 0 && threadIdx.x < 64)
+  constexpr int V = El<T>::V;
+  __shared__ float red[256 * V];
+  const int r = blockIdx.y;
+  const int cb = a.RP < AB_COLS ? a.RP : AB_COLS, ncb = a.RP / cb;
+  const int h = blockIdx.x / ncb, c0 = (blockIdx.x - h * ncb) * cb;
+  if (h >= a.H) {
+    if ((int)blockIdx.x == a.H * ncb) latent_write<T>(a, r, red);
+    else if (threadIdx.x < 64)
       route_from_proj(a.P, a.ldp, a.orouter, a.E, a.rtop, a.rextra, a.ridx,
                       a.rwt, r);
     return;
   }
-  constexpr int V = El<T>::V;
-  const int dq = a.d + a.rot, CS = a.RP + a.RT, pos = a.pos[r];
+  const int dq = a.d + a.rot, CS = a.RP + a.RT, tid = threadIdx.x;
   const float* q = a.P + (size_t)r * a.ldp + a.oq + (size_t)h * dq;
   T* qa = (T*)a.qa + ((size_t)r * a.H + h) * CS;
   // lanes own V latent columns each; the d axis is split over the groups
-  const int nv = a.RP / V, tid = threadIdx.x;
-  const int groups = 256 / nv;           // RP <= 512 (bf16) / 512 (fp32)
+  const int nv = cb / V, groups = 256 / nv;
   const int grp = tid / nv, cv = tid - grp * nv;
   float acc[V];
 #pragma unroll
   for (int j = 0; j < V; j++) acc[j] = 0.f;
-  if (grp < groups) {
-    const T* w = (const T*)a.Wuk + (size_t)h * a.d * a.RP + cv * V;
-#pragma unroll 4
-    for (int i = grp; i < a.d; i += groups) {
-      union { f4v f; T t[V]; } u;
-      u.f = ld16(w + (size_t)i * a.RP);
-      const float qi = El<T>::ld(El<T>::st(q[i]));
+  const T* w = (const T*)a.Wuk + (size_t)h * a.d * a.RP + c0 + cv * V;
+#pragma unroll 8
+  for (int i = grp; i < a.d; i += groups) {
+    union { f4v f; T t[V]; } u;
+    u.f = ld16(w + (size_t)i * a.RP);
+    const float qi = El<T>::ld(El<T>::st(q[i]));
 #pragma unroll
-      for (int j = 0; j < V; j++) acc[j] = fmaf(qi, El<T>::ld(u.t[j]), acc[j]);
-    }
-#pragma unroll
-    for (int j = 0; j < V; j++) red[(grp * nv + cv) * V + j] = acc[j];
+    for (int j = 0; j < V; j++) acc[j] = fmaf(qi, El<T>::ld(u.t[j]), acc[j]);
   }
+#pragma unroll
+  for (int j = 0; j < V; j++) red[grp * cb + cv * V + j] = acc[j];
   __syncthreads();
-  for (int i = tid; i < a.RP; i += 256) {
+  for (int i = tid; i < cb; i += 256) {
     float v = 0.f;
-    for (int g = 0; g < groups; g++) v += red[g * a.RP + i];
-    qa[i] = El<T>::st(v);
+    for (int g = 0; g < groups; g++) v += red[g * cb + i];
+    qa[c0 + i] = El<T>::st(v);
   }
+  if (c0) return;
+  const int pos = a.pos[r];
   const float* c = a.cosT + (size_t)pos * (a.rdims >> 1);
   const float* s = a.sinT + (size_t)pos * (a.rdims >> 1);
   for (int j = tid; j < a.RT; j += 256)
@@ -171,9 +173,17 @@ static size_t attn_lds(int RP, int RT) {
   return b;
 }
 
-template <typename T, int RP, int NW>
+// SHARE: the NW waves hold the same 16 queries and split the latent columns
+// of the output (single tokens); otherwise each wave has 16 queries of its
+// own.  Where registers allow (AHEAD), the next key tile is loaded while one
+// is worked on.
+template <typename T, int RP, int NW, bool SHARE>
 __global__ void __launch_bounds__(64 * NW) k_latent_attn(LatentArgs a) {
+  constexpr bool AHEAD = SHARE && sizeof(T) == 2;
   using Sh = AttnShape<T, RP>;
+  constexpr int QW = SHARE ? 1 : NW;                    // query groups
+  constexpr int ND = SHARE ? RP / 16 / NW : RP / 16;    // output fragments
+  constexpr int PF = ((RP + 128) * (int)sizeof(T) / 16 + 4 * NW - 1) / (4 * NW);
   extern __shared__ __attribute__((aligned(16))) char smem[];
   const int CS = RP + a.RT;
   const int KB = CS * (int)sizeof(T) + 16;              // K row bytes in LDS
@@ -181,27 +191,54 @@ __global__ void __launch_bounds__(64 * NW) k_latent_attn(LatentArgs a) {
   u16* vt = (u16*)(smem + (size_t)KT * KB);
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
   const int qc = lane & 15, g = lane >> 4;
+  const int d0 = SHARE ? wave * ND : 0;
   int seg, rr0;
   if (a.tile_seg) {
     seg = a.tile_seg[blockIdx.x];
     rr0 = a.tile_rr0[blockIdx.x];
   } else {
-    const int nth = (a.H + 16 * NW - 1) / (16 * NW);
+    const int nth = (a.H + 16 * QW - 1) / (16 * QW);
     seg = blockIdx.x / nth;
-    rr0 = (blockIdx.x - seg * nth) * 16 * NW;
+    rr0 = (blockIdx.x - seg * nth) * 16 * QW;
   }
   const int row0 = a.seg_row0[seg], pos0 = a.seg_pos0[seg];
   const int nrr = a.seg_len[seg] * a.H;
   const int* pages = a.table + (size_t)a.seg_slot[seg] * a.ldt;
-  const int my = rr0 + wave * 16 + qc;
+  const int my = rr0 + (SHARE ? 0 : wave * 16) + qc;
   const int myc = my < nrr ? my : nrr - 1;
   const int qpos = pos0 + myc / a.H;
-  const int last = min(rr0 + 16 * NW, nrr) - 1;
+  const int last = min(rr0 + 16 * QW, nrr) - 1;
   const int kend = pos0 + last / a.H + 1;               // keys [0, kend)
   // key tiles of this split
   const int ntile = (kend + KT - 1) / KT;
   const int per = (ntile + a.NS - 1) / a.NS;
   const int t_lo = blockIdx.y * per, t_hi = min(ntile, t_lo + per);
+
+  // loading: lanes take 16 row pairs x 16-byte columns
+  const int kp = tid & 15, cv0 = tid >> 4;
+  const int nvec = CS * (int)sizeof(T) / 16;
+  const int vpos = (kp < 8 ? (kp >> 1) * 8 : ((kp - 8) >> 1) * 8 + 4) +
+                   (kp & 1) * 2;
+  f4v p0[PF], p1[PF];
+  auto fetch = [&](int t) {
+    const int k0 = t * KT;
+    // rows past kend are stale or unwritten: read a valid row instead (the
+    // mask removes its score, and the value must stay finite)
+    const int nk = min(KT, kend - k0);
+    const char* src = (const char*)a.cache +
+        ((size_t)pages[k0 / PAGE] * PAGE + k0 % PAGE) * CS * sizeof(T);
+    const char* s0 = src + (size_t)min(2 * kp, nk - 1) * CS * sizeof(T);
+    const char* s1 = src + (size_t)min(2 * kp + 1, nk - 1) * CS * sizeof(T);
+#pragma unroll
+    for (int i = 0; i < PF; i++) {
+      const int cv = cv0 + i * NW * 4;
+      if (cv < nvec) {
+        p0[i] = ld16(s0 + cv * 16);
+        p1[i] = ld16(s1 + cv * 16);
+      }
+    }
+  };
+  if (AHEAD && t_lo < t_hi) fetch(t_lo);
 
   f4v qf[Sh::NC + Sh::NRM];
   const int NR = a.RT * (int)sizeof(T) / 64;
@@ -214,35 +251,25 @@ __global__ void __launch_bounds__(64 * NW) k_latent_attn(LatentArgs a) {
     for (int c = 0; c < Sh::NRM; c++)
       if (c < NR) qf[Sh::NC + c] = ld16(qp + (Sh::NC + c) * 64);
   }
-  f4v acc[RP / 16];
+  f4v acc[ND];
 #pragma unroll
-  for (int d = 0; d < RP / 16; d++) acc[d] = {0.f, 0.f, 0.f, 0.f};
+  for (int d = 0; d < ND; d++) acc[d] = {0.f, 0.f, 0.f, 0.f};
   float mrun = -INFINITY, lrun = 0.f;
   const float sc = a.scale * 1.4426950408889634f;       // base-2 exponents
 
   for (int t = t_lo; t < t_hi; t++) {
     const int k0 = t * KT;
-    // rows past kend are stale or unwritten: read a valid row instead (the
-    // mask removes its score, and the value must stay finite)
-    const int nk = min(KT, kend - k0);
-    const char* src = (const char*)a.cache +
-        ((size_t)pages[k0 / PAGE] * PAGE + k0 % PAGE) * CS * sizeof(T);
-    if (NW > 1 || t > t_lo) __syncthreads();
-    {
-      // lanes take 16 row pairs x 16-byte columns
-      const int kp = tid & 15;
-      const int r0 = min(2 * kp, nk - 1), r1 = min(2 * kp + 1, nk - 1);
-      const int nvec = CS * (int)sizeof(T) / 16;
-      const int vpos = (kp < 8 ? (kp >> 1) * 8 : ((kp - 8) >> 1) * 8 + 4) +
-                       (kp & 1) * 2;
-      for (int cv = tid >> 4; cv < nvec; cv += NW * 4) {
-        f4v x0 = ld16(src + (size_t)r0 * CS * sizeof(T) + cv * 16);
-        f4v x1 = ld16(src + (size_t)r1 * CS * sizeof(T) + cv * 16);
-        *(f4v*)(kl + (2 * kp) * KB + cv * 16) = x0;
-        *(f4v*)(kl + (2 * kp + 1) * KB + cv * 16) = x1;
+    if (!AHEAD) fetch(t);
+    if (t > t_lo) __syncthreads();
+#pragma unroll
+    for (int i = 0; i < PF; i++) {
+      const int cv = cv0 + i * NW * 4;
+      if (cv < nvec) {
+        *(f4v*)(kl + (2 * kp) * KB + cv * 16) = p0[i];
+        *(f4v*)(kl + (2 * kp + 1) * KB + cv * 16) = p1[i];
         if (sizeof(T) == 2 && cv * 8 < RP) {
           union { f4v f; uint32_t u[4]; } a0, a1;
-          a0.f = x0; a1.f = x1;
+          a0.f = p0[i]; a1.f = p1[i];
 #pragma unroll
           for (int j = 0; j < 4; j++) {
             *(uint32_t*)(vt + (cv * 8 + 2 * j) * Sh::VS + vpos) =
@@ -254,6 +281,7 @@ __global__ void __launch_bounds__(64 * NW) k_latent_attn(LatentArgs a) {
       }
     }
     __syncthreads();
+    if (AHEAD && t + 1 < t_hi) fetch(t + 1);
 
     f4v st[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
     const char* kr = kl + qc * KB + g * 16;
@@ -293,7 +321,7 @@ __global__ void __launch_bounds__(64 * NW) k_latent_attn(LatentArgs a) {
     mrun = mnew;
     if (__any(alpha != 1.f)) {
 #pragma unroll
-      for (int d = 0; d < RP / 16; d++)
+      for (int d = 0; d < ND; d++)
 #pragma unroll
         for (int j = 0; j < 4; j++) acc[d][j] *= alpha;
     }
@@ -302,17 +330,17 @@ __global__ void __launch_bounds__(64 * NW) k_latent_attn(LatentArgs a) {
 #pragma unroll
       for (int i = 0; i < 8; i++) p.h[i] = f2b(sv[i]);
 #pragma unroll
-      for (int d = 0; d < RP / 16; d++)
+      for (int d = 0; d < ND; d++)
         acc[d] = GemmMma<u16>::mma(
-            ld16(vt + (d * 16 + qc) * Sh::VS + g * 8), p.f, acc[d]);
+            ld16(vt + ((d0 + d) * 16 + qc) * Sh::VS + g * 8), p.f, acc[d]);
     } else {
 #pragma unroll
-      for (int d = 0; d < RP / 16; d++)
+      for (int d = 0; d < ND; d++)
 #pragma unroll
         for (int i = 0; i < 8; i++)
           acc[d] = __builtin_amdgcn_mfma_f32_16x16x4f32(
               *(const float*)(kl + ((i >> 2) * 16 + g * 4 + (i & 3)) * KB +
-                              (d * 16 + qc) * 4),
+                              ((d0 + d) * 16 + qc) * 4),
               sv[i], acc[d], 0, 0, 0);
     }
   }
@@ -321,9 +349,9 @@ __global__ void __launch_bounds__(64 * NW) k_latent_attn(LatentArgs a) {
   const size_t orow = (size_t)row0 * a.H + my;
   if (a.NS == 1) {
     const float inv = 1.f / lrun;
-    T* op = (T*)a.olat + orow * RP + g * 4;
+    T* op = (T*)a.olat + orow * RP + d0 * 16 + g * 4;
 #pragma unroll
-    for (int d = 0; d < RP / 16; d++) {
+    for (int d = 0; d < ND; d++) {
       union { T t[4]; uint64_t u; f4v f; } v;
 #pragma unroll
       for (int j = 0; j < 4; j++) v.t[j] = El<T>::st(acc[d][j] * inv);
@@ -333,95 +361,122 @@ __global__ void __launch_bounds__(64 * NW) k_latent_attn(LatentArgs a) {
   } else {
     const size_t pr =
         ((size_t)blockIdx.y * a.rows + row0 - a.rbase) * a.H + my;
-    if (g == 0) {
+    if (g == 0 && (!SHARE || wave == 0)) {
       a.ml[pr * 2] = mrun;
       a.ml[pr * 2 + 1] = lrun;
     }
     if (t_lo < t_hi) {
-      float* op = a.part + pr * RP + g * 4;
+      float* op = a.part + pr * RP + d0 * 16 + g * 4;
 #pragma unroll
-      for (int d = 0; d < RP / 16; d++) *(f4v*)(op + d * 16) = acc[d];
+      for (int d = 0; d < ND; d++) *(f4v*)(op + d * 16) = acc[d];
     }
   }
 }
 
-// merged latent of one (row, head) -> LDS (as T); sw holds NS weights
+// merged latent of one (row, head) -> dst (as T).  256 threads; sh holds
+// MAX_SPLITS + 1024 floats.  Splits with keys come first; only they wrote
+// partials.
+#define MAX_SPLITS 256
+#define MERGE_LDS (MAX_SPLITS + 1024)
 template <typename T>
-DEVINL void latent_merge(const LatentArgs& a, size_t orow, T* dst, float* sw) {
+DEVINL void latent_merge(const LatentArgs& a, size_t orow, T* dst, float* sh) {
   const size_t n = (size_t)a.rows * a.H;
+  float *sw = sh, *part = sh + MAX_SPLITS;
+  __shared__ int live;
   if (threadIdx.x < 64) {
     float mt = -INFINITY;
     for (int s = threadIdx.x; s < a.NS; s += 64)
       mt = fmaxf(mt, a.ml[(s * n + orow) * 2]);
     mt = wave_reduce_max(mt);
     float lt = 0.f;
+    int top = 0;
     for (int s = threadIdx.x; s < a.NS; s += 64) {
-      float w = exp2f(a.ml[(s * n + orow) * 2] - mt);   // -inf: empty split
+      float w = exp2f(a.ml[(s * n + orow) * 2] - mt);   // -inf: nothing seen
       sw[s] = w;
+      if (w > 0.f) top = s + 1;
       lt += w * a.ml[(s * n + orow) * 2 + 1];
     }
     lt = wave_reduce_sum(lt);
+#pragma unroll
+    for (int m = 1; m < 64; m <<= 1) top = max(top, __shfl_xor(top, m));
     for (int s = threadIdx.x; s < a.NS; s += 64) sw[s] /= lt;
+    if (threadIdx.x == 0) live = top;
   }
   __syncthreads();
-  for (int i = threadIdx.x * 4; i < a.RP; i += blockDim.x * 4) {
+  const int nv = a.RP / 4, groups = 256 / nv;           // RP <= 1024
+  const int grp = threadIdx.x / nv, cv = threadIdx.x - grp * nv;
+  if (grp < groups) {
     f4v v = {0.f, 0.f, 0.f, 0.f};
-    for (int s = 0; s < a.NS; s++) {
-      float w = sw[s];
-      if (w == 0.f) continue;              // empty splits wrote no partial
-      f4v p = *(const f4v*)(a.part + (s * n + orow) * a.RP + i);
+#pragma unroll 8
+    for (int s = grp; s < live; s += groups) {
+      const float w = sw[s];
+      f4v p = *(const f4v*)(a.part + (s * n + orow) * a.RP + cv * 4);
 #pragma unroll
       for (int j = 0; j < 4; j++) v[j] = fmaf(w, p[j], v[j]);
     }
-#pragma unroll
-    for (int j = 0; j < 4; j++) dst[i + j] = El<T>::st(v[j]);
+    *(f4v*)(part + (grp * nv + cv) * 4) = v;
+  }
+  __syncthreads();
+  for (int i = threadIdx.x; i < a.RP; i += 256) {
+    float v = 0.f;
+    for (int k = 0; k < groups; k++) v += part[k * a.RP + i];
+    dst[i] = El<T>::st(v);
   }
 }
 
-#define MAX_SPLITS 256
-
 template <typename T>
-__global__ void __launch_bounds__(128) k_latent_merge(LatentArgs a) {
-  __shared__ float sw[MAX_SPLITS];
+__global__ void __launch_bounds__(256) k_latent_merge(LatentArgs a) {
+  __shared__ __attribute__((aligned(16))) float sh[MERGE_LDS];
   latent_merge<T>(a, blockIdx.x,
-                  (T*)a.olat + ((size_t)a.rbase * a.H + blockIdx.x) * a.RP, sw);
+                  (T*)a.olat + ((size_t)a.rbase * a.H + blockIdx.x) * a.RP,
+                  sh);
 }
 
-// ---- few rows: merge + value up-projection + gate per (row, head); the
-// ---- experts' gate/up halves run beside it in the same launch ----------
+// ---- few rows: merge + value up-projection + gate, in `nub` blocks per
+// ---- (row, head); the experts' gate/up halves run beside it ------------
+#define UVW 8      // outputs of a wave at a time
 template <typename T>
-__global__ void __launch_bounds__(256) k_latent_dec_fin(LatentArgs a,
+__global__ void __launch_bounds__(256) k_latent_dec_fin(LatentArgs a, int nub,
                                                         MoeArgs m, int fblocks) {
   __shared__ __attribute__((aligned(16))) T ol[512];
-  __shared__ float sw[MAX_SPLITS];
-  const int nmix = a.rows * a.H;
+  __shared__ __attribute__((aligned(16))) float sh[MERGE_LDS];
+  const int nmix = a.rows * a.H * nub;
   if ((int)blockIdx.x >= nmix) {
     const int b = blockIdx.x - nmix;
     expert_gu_block<T>(m, b / fblocks, b % fblocks);
     return;
   }
   constexpr int V = El<T>::V;
-  const int r = blockIdx.x / a.H, h = blockIdx.x - r * a.H;
-  latent_merge<T>(a, blockIdx.x, ol, sw);
-  __syncthreads();
-  const float gate = sigmoid_f(a.P[(size_t)r * a.ldp + a.og + h]);
+  const int rh = blockIdx.x / nub, ub = blockIdx.x - rh * nub;
+  const int r = rh / a.H, h = rh - r * a.H;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   const int nv = a.RP / V;                  // 16-byte vectors of a row
+  const T* wb = (const T*)a.Wuv + (size_t)h * a.vd * a.RP;
   T* o = (T*)a.o + (size_t)r * a.ldo + h * a.vd;
-  for (int j0 = wave * 4; j0 < a.vd; j0 += 16) {
-    float acc[4] = {0.f, 0.f, 0.f, 0.f};
+  int j0 = (ub * 4 + wave) * UVW;
+  f4v w[UVW];                               // on its way during the merge
+  auto slab = [&](int k) {
+#pragma unroll
+    for (int i = 0; i < UVW; i++)
+      w[i] = k < nv ? ld16(wb + (size_t)min(j0 + i, a.vd - 1) * a.RP + k * V)
+                    : f4v{0.f, 0.f, 0.f, 0.f};
+  };
+  slab(lane);
+  latent_merge<T>(a, rh, ol, sh);
+  __syncthreads();
+  const float gate = sigmoid_f(a.P[(size_t)r * a.ldp + a.og + h]);
+  for (int first = 1; j0 < a.vd; j0 += nub * 4 * UVW, first = 0) {
+    float acc[UVW];
+#pragma unroll
+    for (int i = 0; i < UVW; i++) acc[i] = 0.f;
     for (int k = lane; k < nv; k += 64) {
+      if (!first || k != lane) slab(k);
       f4v x = ld16(ol + k * V);
 #pragma unroll
-      for (int i = 0; i < 4; i++) {
-        int j = min(j0 + i, a.vd - 1);
-        acc[i] = dot16<T>(
-            ld16((const T*)a.Wuv + ((size_t)h * a.vd + j) * a.RP + k * V), x,
-            acc[i]);
-      }
+      for (int i = 0; i < UVW; i++) acc[i] = dot16<T>(w[i], x, acc[i]);
     }
 #pragma unroll
-    for (int i = 0; i < 4; i++) {
+    for (int i = 0; i < UVW; i++) {
       float v = wave_reduce_sum(acc[i]);
       if (lane == 0 && j0 + i < a.vd) o[j0 + i] = El<T>::st(v * gate);
     }
@@ -447,51 +502,60 @@ extern "C" hipError_t launch_latent_prep(int f32, const LatentArgs* a,
 extern "C" hipError_t launch_latent_dec_prep(int f32, const LatentArgs* a,
                                              hipStream_t s) {
   if (bad_shape(*a) || a->RP > 512) return hipErrorInvalidValue;
-  dim3 grid(a->H + 1, a->rows);
+  const int cb = a->RP < AB_COLS ? a->RP : AB_COLS;
+  if (a->RP % cb) return hipErrorInvalidValue;
+  // the last head's blocks: cache row, then routing (RP / cb may be 1)
+  dim3 grid(a->H * (a->RP / cb) + (a->E > 0 ? 2 : 1), a->rows);
   if (f32) hipLaunchKernelGGL(k_latent_dec_prep<float>, grid, dim3(256), 0, s, *a);
   else hipLaunchKernelGGL(k_latent_dec_prep<u16>, grid, dim3(256), 0, s, *a);
   return hipGetLastError();
 }
 
-template <typename T, int RP, int NW>
-static hipError_t attn_go(const LatentArgs& a, int tiles, hipStream_t s) {
+template <typename T, int RP>
+static hipError_t attn_go(const LatentArgs& a, int share, int tiles,
+                          hipStream_t s) {
   size_t lds = attn_lds<T>(RP, a.RT);
-  RAISE_LDS((k_latent_attn<T, RP, NW>));
-  hipLaunchKernelGGL((k_latent_attn<T, RP, NW>), dim3(tiles, a.NS),
-                     dim3(64 * NW), lds, s, a);
+  dim3 grid(tiles, a.NS);
+  if (share) {
+    RAISE_LDS((k_latent_attn<T, RP, 4, true>));
+    hipLaunchKernelGGL((k_latent_attn<T, RP, 4, true>), grid, dim3(256), lds,
+                       s, a);
+  } else {
+    RAISE_LDS((k_latent_attn<T, RP, 4, false>));
+    hipLaunchKernelGGL((k_latent_attn<T, RP, 4, false>), grid, dim3(256), lds,
+                       s, a);
+  }
   return hipGetLastError();
 }
 
-template <typename T, int NW>
-static hipError_t attn_rp(const LatentArgs& a, int tiles, hipStream_t s) {
+template <typename T>
+static hipError_t attn_rp(const LatentArgs& a, int share, int tiles,
+                          hipStream_t s) {
   switch (a.RP) {
-    case 64: return attn_go<T, 64, NW>(a, tiles, s);
-    case 128: return attn_go<T, 128, NW>(a, tiles, s);
-    case 256: return attn_go<T, 256, NW>(a, tiles, s);
-    case 384: return attn_go<T, 384, NW>(a, tiles, s);
-    case 512: return attn_go<T, 512, NW>(a, tiles, s);
+    case 64: return attn_go<T, 64>(a, share, tiles, s);
+    case 128: return attn_go<T, 128>(a, share, tiles, s);
+    case 256: return attn_go<T, 256>(a, share, tiles, s);
+    case 384: return attn_go<T, 384>(a, share, tiles, s);
+    case 512: return attn_go<T, 512>(a, share, tiles, s);
   }
   return hipErrorInvalidValue;
 }
 
-// tiles: number of query tiles of 16*NW (token, head) pairs
-extern "C" hipError_t launch_latent_attn(int f32, const LatentArgs* a, int nw,
-                                         int tiles, hipStream_t s) {
-  if (bad_shape(*a) || tiles < 1 || (nw != 1 && nw != 4))
-    return hipErrorInvalidValue;
-  if (f32)
-    return nw == 1 ? attn_rp<float, 1>(*a, tiles, s)
-                   : attn_rp<float, 4>(*a, tiles, s);
-  return nw == 1 ? attn_rp<u16, 1>(*a, tiles, s)
-                 : attn_rp<u16, 4>(*a, tiles, s);
+// tiles: query tiles of 16 (share) or 64 (token, head) pairs
+extern "C" hipError_t launch_latent_attn(int f32, const LatentArgs* a,
+                                         int share, int tiles,
+                                         hipStream_t s) {
+  if (bad_shape(*a) || tiles < 1) return hipErrorInvalidValue;
+  return f32 ? attn_rp<float>(*a, share, tiles, s)
+             : attn_rp<u16>(*a, share, tiles, s);
 }
 
 extern "C" hipError_t launch_latent_merge(int f32, const LatentArgs* a,
                                           hipStream_t s) {
   if (bad_shape(*a)) return hipErrorInvalidValue;
   dim3 grid(a->rows * a->H);
-  if (f32) hipLaunchKernelGGL(k_latent_merge<float>, grid, dim3(128), 0, s, *a);
-  else hipLaunchKernelGGL(k_latent_merge<u16>, grid, dim3(128), 0, s, *a);
+  if (f32) hipLaunchKernelGGL(k_latent_merge<float>, grid, dim3(256), 0, s, *a);
+  else hipLaunchKernelGGL(k_latent_merge<u16>, grid, dim3(256), 0, s, *a);
   return hipGetLastError();
 }
 
@@ -501,8 +565,11 @@ extern "C" hipError_t launch_latent_dec_fin(int f32, const LatentArgs* a,
   if (bad_shape(*a) || a->RP > 512 || a->NS < 2) return hipErrorInvalidValue;
   int ffm = m->ff > m->ffs ? m->ff : m->ffs;
   int fb = pairs ? (ffm + MOE_FPB - 1) / MOE_FPB : 1;
-  dim3 grid(a->rows * a->H + pairs * fb);
-  if (f32) hipLaunchKernelGGL(k_latent_dec_fin<float>, grid, dim3(256), 0, s, *a, *m, fb);
-  else hipLaunchKernelGGL(k_latent_dec_fin<u16>, grid, dim3(256), 0, s, *a, *m, fb);
+  int nub = 1;               // spread the heads while there are few of them
+  while (nub < 4 && a->rows * a->H * nub < 128 && nub * 4 * UVW < a->vd)
+    nub *= 2;
+  dim3 grid(a->rows * a->H * nub + pairs * fb);
+  if (f32) hipLaunchKernelGGL(k_latent_dec_fin<float>, grid, dim3(256), 0, s, *a, nub, *m, fb);
+  else hipLaunchKernelGGL(k_latent_dec_fin<u16>, grid, dim3(256), 0, s, *a, nub, *m, fb);
   return hipGetLastError();
 }

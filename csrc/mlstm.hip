@@ -31,7 +31,7 @@ struct MlstmArgs {
   const int *slot, *pos;      // per row
   const int *seg_row0, *seg_len, *seg_slot, *seg_pos0, *seg_chunk0;
   const int *chunk_row0, *chunk_len;
-  float *gF, *gi, *gm;        // [rows, H]
+  float *gF, *gi, *gm;        // [rows, H]: F, i, max of i - F so far
   float* cm0;                 // [chunks, H] maximum before the chunk
   float *U, *un;              // [chunks, H, d, vd], [chunks, H, d]
   int* ridx;
@@ -51,9 +51,14 @@ DEVINL float gate_f(const MlstmArgs& a, int r, int h) {
 }
 
 // ---- one token per row ------------------------------------------------
-__global__ void __launch_bounds__(256) k_mlstm_step(MlstmArgs a) {
-  extern __shared__ float sm[];           // q[d], k[d], v[64], red[4*64]
-  __shared__ float red[4];
+// 16 waves per (head, column tile): a wave's lanes own the 64 columns, the
+// rows of S are dealt to the waves.  The first rows are on their way while
+// the gates are worked out.
+#define SW 16
+#define SPRE 8
+__global__ void __launch_bounds__(64 * SW) k_mlstm_step(MlstmArgs a) {
+  extern __shared__ float sm[];           // q[d], k[d], part[SW*64]
+  __shared__ float red[SW];
   const int r = blockIdx.y;
   if ((int)blockIdx.x == a.H * a.nvt) {
     if (threadIdx.x < 64) {
@@ -68,10 +73,20 @@ __global__ void __launch_bounds__(256) k_mlstm_step(MlstmArgs a) {
   }
   const int h = blockIdx.x / a.nvt, vtile = blockIdx.x - h * a.nvt;
   const int tid = threadIdx.x, c = tid & 63, w = tid >> 6;
-  float *qs = sm, *ks = sm + a.d, *vs = sm + 2 * a.d, *part = vs + VT;
+  float *qs = sm, *ks = sm + a.d, *part = sm + 2 * a.d;
   const float* p = a.P + (size_t)r * a.ldp;
   const size_t sl = a.slot[r];
   const bool fresh = a.pos[r] == 0;
+  const int col = vtile * VT + c;
+  const bool live = col < a.vd;
+  float* S = a.S + ((sl * a.H + h) * a.d) * (size_t)a.vd + col;
+  float pre[SPRE];
+#pragma unroll
+  for (int u = 0; u < SPRE; u++) {
+    const int i = w + u * SW;
+    pre[u] = (live && !fresh && i < a.d) ? S[(size_t)i * a.vd] : 0.f;
+  }
+  const float v = live ? p[a.ov + h * a.vd + col] : 0.f;
   float* np = a.n + ((sl * a.H + h) * a.nvt + vtile) * a.d;
   float* mp = a.m + (sl * a.H + h) * a.nvt + vtile;
   const float m0 = fresh ? 0.f : *mp;
@@ -80,24 +95,28 @@ __global__ void __launch_bounds__(256) k_mlstm_step(MlstmArgs a) {
   const float keep = fresh ? 0.f : expf(gf + m0 - m1), add = expf(gi - m1);
   const float qscale = 1.f / sqrtf((float)a.d);
   float nq = 0.f;
-  for (int i = tid; i < a.d; i += 256) {
-    float q = p[a.oq + h * a.d + i] * qscale, k = p[a.ok + h * a.d + i];
+  for (int i = tid; i < a.d; i += 64 * SW) {
+    float q = p[a.oq + h * a.d + i] * qscale, k = p[a.ok + h * a.d + i] * add;
     qs[i] = q;
-    ks[i] = k * add;
-    float nv = fresh ? k * add : keep * np[i] + k * add;
+    ks[i] = k;
+    float nv = fresh ? k : keep * np[i] + k;
     np[i] = nv;
     nq += nv * q;
   }
-  const int col = vtile * VT + c;
-  const bool live = col < a.vd;
-  if (tid < VT) vs[tid] = live ? p[a.ov + h * a.vd + col] : 0.f;
-  nq = block_sum(nq, red);                 // its barriers publish qs/ks/vs
-  float* S = a.S + ((sl * a.H + h) * a.d) * (size_t)a.vd + col;
+  nq = block_sum(nq, red);                 // its barriers publish qs and ks
   float acc = 0.f;
   if (live) {
-    const float v = vs[c];
-#pragma unroll 8
-    for (int i = w; i < a.d; i += 4) {
+#pragma unroll
+    for (int u = 0; u < SPRE; u++) {
+      const int i = w + u * SW;
+      if (i < a.d) {
+        const float s = keep * pre[u] + ks[i] * v;
+        S[(size_t)i * a.vd] = s;
+        acc = fmaf(s, qs[i], acc);
+      }
+    }
+#pragma unroll 4
+    for (int i = w + SPRE * SW; i < a.d; i += SW) {
       float s = ks[i] * v;
       if (!fresh) s += keep * S[(size_t)i * a.vd];
       S[(size_t)i * a.vd] = s;
@@ -107,7 +126,9 @@ __global__ void __launch_bounds__(256) k_mlstm_step(MlstmArgs a) {
   part[w * VT + c] = acc;
   __syncthreads();
   if (tid < VT && live) {
-    float num = (part[c] + part[VT + c]) + (part[2 * VT + c] + part[3 * VT + c]);
+    float num = 0.f;
+#pragma unroll
+    for (int u = 0; u < SW; u++) num += part[u * VT + c];
     a.o[(size_t)r * a.H * a.vd + h * a.vd + col] =
         num / (fmaxf(fabsf(nq), expf(-m1)) + 1e-6f);
   }
@@ -115,36 +136,50 @@ __global__ void __launch_bounds__(256) k_mlstm_step(MlstmArgs a) {
 }
 
 // ---- runs of tokens -----------------------------------------------------
-// gates and running maxima: one wave per (head, segment)
+// gates inside a chunk, one wave per (head, chunk): F and the running
+// maximum M of i - F; m_t follows once the maximum before the chunk is known
 __global__ void __launch_bounds__(64) k_mlstm_gates(MlstmArgs a) {
+  const int h = blockIdx.x, c = blockIdx.y, lane = threadIdx.x;
+  const int r = a.chunk_row0[c] + lane;
+  const bool live = lane < a.chunk_len[c];
+  const float gi = live ? gate_i(a, r, h) : 0.f;
+  float F = live ? gate_f(a, r, h) : 0.f;
+#pragma unroll
+  for (int s = 1; s < 64; s <<= 1) {
+    float o = __shfl_up(F, s);
+    if (lane >= s) F += o;
+  }
+  float M = live ? gi - F : -INFINITY;
+#pragma unroll
+  for (int s = 1; s < 64; s <<= 1) {
+    float o = __shfl_up(M, s);
+    if (lane >= s) M = fmaxf(M, o);
+  }
+  if (live) {
+    a.gF[(size_t)r * a.H + h] = F;
+    a.gi[(size_t)r * a.H + h] = gi;
+    a.gm[(size_t)r * a.H + h] = M;
+  }
+}
+
+// m before every chunk, and the new state maximum: one wave per (head,
+// segment), 64 chunks at a time.  gM = max(m0, .) + F at a chunk's end.
+__global__ void __launch_bounds__(64) k_mlstm_chain(MlstmArgs a) {
   const int h = blockIdx.x, sg = blockIdx.y, lane = threadIdx.x;
-  const int row0 = a.seg_row0[sg], len = a.seg_len[sg], c0 = a.seg_chunk0[sg];
+  const int c0 = a.seg_chunk0[sg], nc = (a.seg_len[sg] + CH - 1) / CH;
   float* mp = a.m + ((size_t)a.seg_slot[sg] * a.H + h) * a.nvt;
   float m0 = a.seg_pos0[sg] == 0 ? 0.f : mp[0];
-  for (int t0 = 0, c = c0; t0 < len; t0 += CH, c++) {
-    const int nt = min(CH, len - t0), r = row0 + t0 + lane;
-    const bool live = lane < nt;
-    const float gi = live ? gate_i(a, r, h) : 0.f;
-    float F = live ? gate_f(a, r, h) : 0.f;
-#pragma unroll
-    for (int s = 1; s < 64; s <<= 1) {
-      float o = __shfl_up(F, s);
-      if (lane >= s) F += o;
+  for (int b = 0; b < nc; b += 64) {
+    const int n = min(64, nc - b), c = c0 + b + min(lane, n - 1);
+    const size_t last =
+        (size_t)(a.chunk_row0[c] + a.chunk_len[c] - 1) * a.H + h;
+    const float F = a.gF[last], M = a.gm[last];
+    float mine = m0;
+    for (int k = 0; k < n; k++) {
+      if (lane == k) mine = m0;
+      m0 = __shfl(F, k) + fmaxf(m0, __shfl(M, k));
     }
-    float M = live ? gi - F : -INFINITY;
-#pragma unroll
-    for (int s = 1; s < 64; s <<= 1) {
-      float o = __shfl_up(M, s);
-      if (lane >= s) M = fmaxf(M, o);
-    }
-    const float mt = F + fmaxf(m0, M);
-    if (live) {
-      a.gF[(size_t)r * a.H + h] = F;
-      a.gi[(size_t)r * a.H + h] = gi;
-      a.gm[(size_t)r * a.H + h] = mt;
-    }
-    if (lane == 0) a.cm0[(size_t)c * a.H + h] = m0;
-    m0 = __shfl(mt, nt - 1);
+    if (lane < n) a.cm0[(size_t)c * a.H + h] = mine;
   }
   for (int i = lane; i < a.nvt; i += 64) mp[i] = m0;
 }
@@ -153,25 +188,37 @@ __global__ void __launch_bounds__(64) k_mlstm_gates(MlstmArgs a) {
 #define LS 68     // LDS row stride of a 64-wide fp32 tile
 __global__ void __launch_bounds__(256) k_mlstm_local(MlstmArgs a) {
   __shared__ __attribute__((aligned(16))) float kl[CH * LS], vl[CH * LS];
+  __shared__ float wl[CH];
   const int c = blockIdx.y, h = blockIdx.z;
   const int ndt = (a.d + 63) / 64;
   const int vtile = blockIdx.x / ndt, dt = blockIdx.x - vtile * ndt;
   const int row0 = a.chunk_row0[c], len = a.chunk_len[c];
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
   const size_t last = (size_t)(row0 + len - 1) * a.H + h;
-  const float Fe = a.gF[last], me = a.gm[last];
-  for (int i = tid; i < CH * 64; i += 256) {
-    const int s = i >> 6, j = i & 63;
-    float kv = 0.f, vv = 0.f;
-    if (s < len) {
-      const float* p = a.P + (size_t)(row0 + s) * a.ldp;
-      const size_t gx = (size_t)(row0 + s) * a.H + h;
-      const float w = expf(Fe - a.gF[gx] + a.gi[gx] - me);
-      if (dt * 64 + j < a.d) kv = w * p[a.ok + h * a.d + dt * 64 + j];
-      if (vtile * VT + j < a.vd) vv = p[a.ov + h * a.vd + vtile * VT + j];
-    }
-    kl[s * LS + j] = kv;
-    vl[s * LS + j] = vv;
+  const float Fe = a.gF[last];
+  const float me = Fe + fmaxf(a.cm0[(size_t)c * a.H + h], a.gm[last]);
+  if (tid < CH) {
+    const size_t gx = (size_t)(row0 + min(tid, len - 1)) * a.H + h;
+    wl[tid] = tid < len ? expf(Fe - a.gF[gx] + a.gi[gx] - me) : 0.f;
+  }
+  const int j = tid & 63;
+  const bool dl = dt * 64 + j < a.d, vl_ = vtile * VT + j < a.vd;
+  const float* pk = a.P + a.ok + h * a.d + dt * 64 + j;
+  const float* pv = a.P + a.ov + h * a.vd + vtile * VT + j;
+  float kv[16], vv[16];
+#pragma unroll
+  for (int u = 0; u < 16; u++) {
+    const int s = wave + u * 4;
+    const size_t ro = (size_t)(row0 + min(s, len - 1)) * a.ldp;
+    kv[u] = dl ? pk[ro] : 0.f;
+    vv[u] = vl_ ? pv[ro] : 0.f;
+  }
+  __syncthreads();
+#pragma unroll
+  for (int u = 0; u < 16; u++) {
+    const int s = wave + u * 4;
+    kl[s * LS + j] = kv[u] * wl[s];          // 0 past the chunk
+    vl[s * LS + j] = vv[u];
   }
   __syncthreads();
   const int lr = lane & 15, g = lane >> 4;
@@ -216,8 +263,8 @@ __global__ void __launch_bounds__(256) k_mlstm_scan(MlstmArgs a) {
   for (int c = c0; c < c0 + nc; c++) {
     const size_t last =
         (size_t)(a.chunk_row0[c] + a.chunk_len[c] - 1) * a.H + h;
-    const float keep = expf(a.gF[last] + a.cm0[(size_t)c * a.H + h] -
-                            a.gm[last]);
+    const float mc = a.cm0[(size_t)c * a.H + h];
+    const float keep = expf(mc - fmaxf(mc, a.gm[last]));
     float* u = isn ? a.un + ((size_t)c * a.H + h) * a.d + (i - dv)
                    : a.U + ((size_t)c * a.H + h) * (size_t)dv + i;
     const float add = *u;
@@ -248,25 +295,34 @@ __global__ void __launch_bounds__(256) k_mlstm_out(MlstmArgs a) {
     const size_t gx = (size_t)(row0 + min(tid, len - 1)) * a.H + h;
     Fl[tid] = a.gF[gx];
     il[tid] = a.gi[gx];
-    ml[tid] = a.gm[gx];
+    ml[tid] = a.gF[gx] + fmaxf(m0, a.gm[gx]);
   }
   f4v sc[4], acc[4];
 #pragma unroll
   for (int j = 0; j < 4; j++)
     sc[j] = acc[j] = f4v{0.f, 0.f, 0.f, 0.f};
-  float nq = 0.f;        // thread t < 64: q_t . n before the chunk
+  float nq = 0.f;        // q_t . n before the chunk, a quarter per thread
   for (int d0 = 0; d0 < a.d; d0 += 64) {
+    const int j = tid & 63, v = vtile * VT + j;
+    const bool dl = d0 + j < a.d, vlive = v < a.vd;
+    const float* pq = a.P + a.oq + h * a.d + d0 + j;
+    const float* pk = a.P + a.ok + h * a.d + d0 + j;
+    float qv[16], kv[16], uv[16];
+#pragma unroll
+    for (int u = 0; u < 16; u++) {
+      const int s = wave + u * 4;            // a token, and a row of U
+      const size_t ro = (size_t)(row0 + min(s, len - 1)) * a.ldp;
+      qv[u] = dl ? pq[ro] : 0.f;
+      kv[u] = dl ? pk[ro] : 0.f;
+      uv[u] = (d0 + s < a.d && vlive) ? U[(size_t)(d0 + s) * a.vd + v] : 0.f;
+    }
     __syncthreads();
-    for (int i = tid; i < CH * 64; i += 256) {
-      const int s = i >> 6, j = i & 63;
-      const bool dl = d0 + j < a.d;
-      const float* p = a.P + (size_t)(row0 + s) * a.ldp + h * a.d + d0 + j;
-      const bool on = s < len && dl;
-      ql[s * LS + j] = on ? p[a.oq] * qscale : 0.f;
-      kl[s * LS + j] = on ? p[a.ok] : 0.f;
-      const int v = vtile * VT + j;        // here s runs over d
-      sl[s * LS + j] = (d0 + s < a.d && v < a.vd)
-                           ? U[(size_t)(d0 + s) * a.vd + v] : 0.f;
+#pragma unroll
+    for (int u = 0; u < 16; u++) {
+      const int s = wave + u * 4;
+      ql[s * LS + j] = s < len ? qv[u] * qscale : 0.f;
+      kl[s * LS + j] = s < len ? kv[u] : 0.f;
+      sl[s * LS + j] = uv[u];
     }
     if (tid < 64) nl[tid] = d0 + tid < a.d ? un[d0 + tid] : 0.f;
     __syncthreads();
@@ -280,18 +336,30 @@ __global__ void __launch_bounds__(256) k_mlstm_out(MlstmArgs a) {
             av, sl[(k + g) * LS + j * 16 + lr], acc[j], 0, 0, 0);
       }
     }
-    if (tid < CH)
-      for (int j = 0; j < 64; j++) nq += ql[tid * LS + j] * nl[j];
+#pragma unroll
+    for (int j = 0; j < 16; j++)
+      nq += ql[(tid >> 2) * LS + j * 4 + (tid & 3)] * nl[j * 4 + (tid & 3)];
   }
+  nq += __shfl_xor(nq, 1);
+  nq += __shfl_xor(nq, 2);
   __syncthreads();
   // values of the tile, and q.n per token
-  for (int i = tid; i < CH * 64; i += 256) {
-    const int s = i >> 6, j = i & 63;
-    sl[s * LS + j] = (s < len && vtile * VT + j < a.vd)
-        ? a.P[(size_t)(row0 + s) * a.ldp + a.ov + h * a.vd + vtile * VT + j]
-        : 0.f;
+  {
+    const int j = tid & 63;
+    const bool vlive = vtile * VT + j < a.vd;
+    const float* pv = a.P + a.ov + h * a.vd + vtile * VT + j;
+    float vv[16];
+#pragma unroll
+    for (int u = 0; u < 16; u++)
+      vv[u] = vlive
+          ? pv[(size_t)(row0 + min(wave + u * 4, len - 1)) * a.ldp] : 0.f;
+#pragma unroll
+    for (int u = 0; u < 16; u++) {
+      const int s = wave + u * 4;
+      sl[s * LS + j] = s < len ? vv[u] : 0.f;
+    }
   }
-  if (tid < CH) nl[tid] = nq;
+  if ((tid & 3) == 0) nl[tid >> 2] = nq;
   __syncthreads();
   float den[4];
 #pragma unroll
@@ -393,11 +461,11 @@ static bool bad_shape(const MlstmArgs& a) {
 
 extern "C" hipError_t launch_mlstm_step(const MlstmArgs* a, hipStream_t s) {
   if (bad_shape(*a)) return hipErrorInvalidValue;
-  size_t lds = (size_t)(2 * a->d + VT + 4 * VT) * sizeof(float);
+  size_t lds = (size_t)(2 * a->d + SW * VT) * sizeof(float);
   RAISE_LDS(k_mlstm_step);
   hipLaunchKernelGGL(k_mlstm_step,
                      dim3(a->H * a->nvt + (a->E > 0 ? 1 : 0), a->rows),
-                     dim3(256), lds, s, *a);
+                     dim3(64 * SW), lds, s, *a);
   return hipGetLastError();
 }
 
@@ -406,7 +474,8 @@ extern "C" hipError_t launch_mlstm_chunks(const MlstmArgs* a, hipStream_t s) {
   if (bad_shape(*a) || a->nseg < 1 || a->nchunk < 1)
     return hipErrorInvalidValue;
   const int ndt = (a->d + 63) / 64;
-  hipLaunchKernelGGL(k_mlstm_gates, dim3(a->H, a->nseg), dim3(64), 0, s, *a);
+  hipLaunchKernelGGL(k_mlstm_gates, dim3(a->H, a->nchunk), dim3(64), 0, s, *a);
+  hipLaunchKernelGGL(k_mlstm_chain, dim3(a->H, a->nseg), dim3(64), 0, s, *a);
   hipLaunchKernelGGL(k_mlstm_local, dim3(ndt * a->nvt, a->nchunk, a->H),
                      dim3(256), 0, s, *a);
   hipLaunchKernelGGL(k_mlstm_scan,

@@ -266,9 +266,8 @@ class LayeredConfig:
             loop=LoopSpec(_get(lp, "start", "loop"), _get(lp, "stop", "loop"),
                           _get(lp, "times", "loop")) if lp else None,
             norm_eps=float(_get(_get(d, "norm", "top level"), "eps", "norm")),
-            embed_scale=float(_get(_get(d, "embedding", "top level"),
-                                   "scale", "embedding")),
-            residual_mult=float(_get(d, "residual_mult", "top level")),
+            embed_scale=float(d.get("embedding", {}).get("scale", 1.0)),
+            residual_mult=float(d.get("residual_mult", 1.0)),
             logit_softcap=float(cap) if cap else None,
             max_position_embeddings=d.get("max_position_embeddings", 131072),
             bos_token_id=d.get("bos_token_id"),

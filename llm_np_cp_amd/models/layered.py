@@ -29,7 +29,8 @@ from ..utils.tracing import trace_range
 from .decode_loop import DecodeLoop, DeviceCacheHandle
 from .mixers import MIXERS, Packer, RoutedExperts, pad_to
 
-FEW = 8             # rows up to which the single-token path is fused GEMVs
+FEW = 16            # single tokens that take the fused few-row kernels
+FUSE = 4            # of them, those whose experts run as fused GEMVs
 PART_FLOATS = 1 << 25     # split-attention scratch for prompt portions
 
 
@@ -156,7 +157,7 @@ class LayeredModel(DecodeLoop):
         """Key-range splits of single-token attention: fixed by the cache
         size and the number of rows, so a captured step keeps its grid."""
         tiles = -(-self.cache.table.shape[1] * hy.PAGE // 32)
-        return int(max(2, min(64, tiles // 2, 1024 // rows)))
+        return int(max(2, min(64, tiles // 4, 1024 // rows)))
 
     def run_splits(self, tiles: int, longest: int) -> int:
         """Splits for `tiles` query tiles against up to `longest` keys."""
@@ -244,7 +245,7 @@ class LayeredModel(DecodeLoop):
         """Embedding and every layer run over the batch; leaves the
         residual stream of its rows in self.x."""
         cfg, W, T = self.cfg, self.W, b.T
-        eps, mult = cfg.norm_eps, cfg.residual_mult
+        mult = cfg.residual_mult
         few = b.nseg == 0 and T <= FEW
         hy.embed_rows(self.embed, b.ids, self.x, self.x0, T, cfg.embed_scale)
         if layer_hook is not None:
@@ -253,30 +254,20 @@ class LayeredModel(DecodeLoop):
             l, cache = self.layers[i], self.caches[j]
             m, ex = l.mixer, l.experts
             if starts:         # x <- W_in [x; x0]
-                if few:
-                    hy.lin_rows(self.win_loop, self.x, self.xb, T, W, W, eps,
-                                x0=self.x0)
-                else:
-                    K = self.cat.shape[1]
-                    hy.norm_rows(self.x, None, self.cat, T, W, K, eps,
-                                 x0=self.x0)
-                    hy.gemm_rows(self.cat, self.win_loop, self.xb, T, K, W,
-                                 hy.EPI_F32)
+                self._project(self.win_loop, self.cat, self.xb, T, x0=self.x0)
                 self.x, self.xb = self.xb, self.x
+            # norm + every input projection (the router's too)
+            self._project(l.win, self.h, self.P, T, g=l.g)
+            fuse = few and T <= FUSE
             if few:
-                # norm + every input projection (router too), the mixer,
-                # then output projection + experts' down + residual
-                hy.lin_rows(l.win, self.x, self.P, T, W, l.ldp, eps, g=l.g,
-                            hout=self.h)
-                m.few(self, b, cache, l)
+                m.few(self, b, cache, l, fuse)
+            else:
+                m.many(self, b, cache, l)
+            if fuse:           # output projection + experts' down + residual
                 hy.block_out(self.f32, m.wo, self.o, m.ldo,
                              ex.bind(self) if ex else hy.MoeArgs(),
                              ex.K1 if ex else 0, self.x, T, W, mult)
             else:
-                hy.norm_rows(self.x, l.g, self.h, T, W, self.Wp, eps)
-                hy.gemm_rows(self.h, l.win, self.P, T, self.Wp, l.ldp,
-                             hy.EPI_F32)
-                m.many(self, b, cache, l)
                 hy.gemm_rows(self.o, m.wo, self.x, T, m.ldo, W,
                              hy.EPI_RESADD, mult=mult)
                 if ex:
@@ -284,18 +275,25 @@ class LayeredModel(DecodeLoop):
             if layer_hook is not None:
                 layer_hook(j, self.x[:T])
 
+    def _project(self, w, staged, out, T: int, g=None, x0=None, rows=None,
+                 cap=None):
+        """out[T, N] fp32 = w . norm(x) (g) or w . [x | x0]; the staged
+        input stays in `staged`.  One row runs as a single fused GEMV."""
+        N, K = w.shape
+        W, eps = self.W, self.cfg.norm_eps
+        if T == 1 and K * w.element_size() <= 1 << 17:
+            hy.lin_row(w, self.x, out, W, eps, g=g, x0=x0, rows=rows,
+                       hout=staged, cap=cap or 0.0)
+            return
+        hy.norm_rows(self.x, g, staged, T, W, K, eps, rows=rows, x0=x0)
+        hy.gemm_rows(staged, w, out, T, K, N,
+                     hy.EPI_F32 if cap is None else hy.EPI_SOFTCAP,
+                     mult=cap or 0.0)
+
     def _head(self, out: torch.Tensor, n: int, rows=None):
         """Final norm, head and soft cap of n rows -> out [n, vocab]."""
-        cfg, V = self.cfg, self.cfg.vocab_size
-        cap = cfg.logit_softcap or 0.0
-        if n <= FEW:
-            hy.lin_rows(self.head, self.x, out, n, self.W, V, cfg.norm_eps,
-                        g=self.g_final, rows=rows, cap=cap)
-        else:
-            hy.norm_rows(self.x, self.g_final, self.h, n, self.W, self.Wp,
-                         cfg.norm_eps, rows=rows)
-            hy.gemm_rows(self.h, self.head, out, n, self.Wp, V,
-                         hy.EPI_SOFTCAP, mult=cap)
+        self._project(self.head, self.h, out, n, g=self.g_final, rows=rows,
+                      cap=self.cfg.logit_softcap or 0.0)
 
     # ------------------------------------------------------------------
     # mixed-batch step

@@ -3,8 +3,8 @@ cache or state of each layer run, and the kernel sequence for a batch.
 
 Every mechanism has two sequences over the same cache and state:
 
-    few()   up to a handful of rows, one token each (decode): fused
-            GEMV-shaped launches
+    few()   up to 16 rows, one token each (decode): fused small launches;
+            with `fuse` the experts' gate/up halves ride along
     many()  any mix of single tokens and runs of tokens: MFMA GEMMs, run
             kernels over the runs, single-token kernels over the rest
 
@@ -162,15 +162,13 @@ class LatentAttention:
     def _single(self, eng, a, n):
         """Split attention of the first n rows, partials left in part/ml."""
         a.put(rows=n, rbase=0, NS=eng.decode_splits(n))
-        H = self.spec.heads
-        nw = 1 if H <= 16 else 4
-        hy.latent_attn(eng.f32, a, nw, n * (-(-H // (16 * nw))))
+        hy.latent_attn(eng.f32, a, 1, n * (-(-self.spec.heads // 16)))
 
-    def few(self, eng, b, cache, layer):
+    def few(self, eng, b, cache, layer, fuse):
         a = self._bind(eng, b, cache, layer)
         hy.latent_dec_prep(eng.f32, a)
         self._single(eng, a, b.T)
-        x = layer.experts
+        x = layer.experts if fuse else None
         hy.latent_dec_fin(eng.f32, a, x.bind(eng) if x else hy.MoeArgs(),
                           b.T * x.K1 if x else 0)
 
@@ -192,7 +190,7 @@ class LatentAttention:
                      eng.ml.numel() // (rows * H * 2))
             a.put(tile_seg=seg, tile_rr0=rr0, rows=rows, rbase=b.nd,
                   NS=max(1, ns))
-            hy.latent_attn(eng.f32, a, 4, n)
+            hy.latent_attn(eng.f32, a, 0, n)
             if ns > 1:
                 hy.latent_merge(eng.f32, a)
         hy.gemm_rows(eng.olat, self.wuv, eng.o, b.T, H * RP, self.ldo,
@@ -251,8 +249,9 @@ class MLSTM:
             nchunk=b.nchunk, E=x.spec.experts if x else 0,
             rtop=x.top if x else 0, rextra=x.extra if x else 0)
 
-    def few(self, eng, b, cache, layer):
-        a, x = self._bind(eng, b, cache, layer), layer.experts
+    def few(self, eng, b, cache, layer, fuse):
+        a = self._bind(eng, b, cache, layer)
+        x = layer.experts if fuse else None
         hy.mlstm_step(a)
         hy.mlstm_dec_fin(eng.f32, a, x.bind(eng) if x else hy.MoeArgs(),
                          b.T * x.K1 if x else 0)

@@ -72,7 +72,7 @@ MoeSort = _struct(
 _SIGS = {
     "launch_embed_rows": [_i, _p, _p, _p, _p, _i, _i, _f, _p],
     "launch_norm_rows": [_i, _p, _p, _p, _p, _p, _i, _i, _i, _f, _p],
-    "launch_lin_rows": [_i] + [_p] * 7 + [_i] * 5 + [_f, _f, _p],
+    "launch_lin_row": [_i] + [_p] * 7 + [_i] * 3 + [_f, _f, _p],
     "launch_gemm_rows": [_i] + [_p] * 4 + [_i] * 8 + [_f, _i, _l, _l, _l, _p],
     "launch_latent_prep": [_i, _p, _p],
     "launch_latent_dec_prep": [_i, _p, _p],
@@ -136,15 +136,15 @@ def norm_rows(x, g, out, M: int, W: int, Kp: int, eps: float, rows=None,
         _ptr(rows), _ptr(out), M, W, Kp, eps)
 
 
-def lin_rows(Wt, x, y, M: int, W: int, ldy: int, eps: float, g=None, x0=None,
-             rows=None, hout=None, cap: float = 0.0):
-    """y[r, n] = Wt[n] . stage(x_r) for a few rows; stage = norm (g) or the
-    concatenation [x | x0].  hout receives the staged rows."""
+def lin_row(Wt, x, y, W: int, eps: float, g=None, x0=None, rows=None,
+            hout=None, cap: float = 0.0):
+    """y[n] = Wt[n] . stage(x) for one row; stage = norm (g) or the
+    concatenation [x | x0].  hout receives the staged row."""
     N, Kp = Wt.shape
     assert Kp % 64 == 0 and Kp >= (W if g is not None else 2 * W)
-    assert y.numel() >= (M - 1) * ldy + N and y.dtype == torch.float32
-    _go("launch_lin_rows", _f32(Wt), _ptr(Wt), _ptr(x), _ptr(x0), _ptr(g),
-        _ptr(rows), _ptr(hout), _ptr(y), M, N, W, Kp, ldy, eps, cap)
+    assert y.numel() >= N and y.dtype == torch.float32
+    _go("launch_lin_row", _f32(Wt), _ptr(Wt), _ptr(x), _ptr(x0), _ptr(g),
+        _ptr(rows), _ptr(hout), _ptr(y), N, W, Kp, eps, cap)
 
 
 def gemm_rows(X, Wt, Y, M: int, ldx: int, ldy: int, epi: int,
@@ -169,8 +169,9 @@ def latent_dec_prep(f32, a):
     _go("launch_latent_dec_prep", f32, ctypes.byref(a))
 
 
-def latent_attn(f32, a, nw: int, tiles: int):
-    _go("launch_latent_attn", f32, ctypes.byref(a), nw, tiles)
+def latent_attn(f32, a, share: int, tiles: int):
+    """tiles of 16 (share: single tokens) or 64 (token, head) pairs."""
+    _go("launch_latent_attn", f32, ctypes.byref(a), share, tiles)
 
 
 def latent_merge(f32, a):

@@ -69,41 +69,48 @@ def _dev(a, dtype=torch.float32):
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("rows, width", [(1, 88), (2, 200), (3, 64), (5, 513),
-                                         (7, 320), (8, 136), (13, 96),
-                                         (16, 1030)])
-def test_few_row_linear(dtype, rows, width):
-    """Fused norm / concatenation + projection + soft cap of a few rows."""
+@pytest.mark.parametrize("width", [8, 64, 88, 513, 1030, 2048, 2113, 5000])
+def test_norm_and_single_row_projection(dtype, width):
+    """Norm / concatenation of rows, alone and fused with a projection and
+    soft cap of one row."""
     from llm_np_cp_amd.ops import hybrid_ops as hy
 
-    rng = np.random.default_rng(rows)
-    N, Kp = 77, -(-width // 64) * 64
-    x = rng.standard_normal((rows + 2, width)) * 3
-    x0 = rng.standard_normal((rows + 2, width))
+    rng = np.random.default_rng(width)
+    N, Kp, n = 77, -(-width // 64) * 64, 6
+    x = rng.standard_normal((n, width)) * 3
+    x0 = rng.standard_normal((n, width))
     g = rng.standard_normal(width) + 1
-    pick = rng.permutation(rows + 2)[:rows].astype(np.int32)
+    X, X0, G = _dev(x), _dev(x0), _dev(g)
     tol = 1e-5 if dtype == torch.float32 else 1e-2
-    W = rng.standard_normal((N, width)) / np.sqrt(width)
-    Wp = torch.zeros(N, Kp, dtype=dtype, device="cuda")
-    Wp[:, :width] = _dev(W, dtype)
-    Wr = Wp[:, :width].double().cpu().numpy()
-    y = torch.full((rows, N + 3), 7.0, device="cuda")
-    h = torch.full((rows, Kp), float("nan"), dtype=dtype, device="cuda")
-    hy.lin_rows(Wp, _dev(x), y, rows, width, N + 3, 1e-5, g=_dev(g),
-                rows=torch.from_numpy(pick).cuda(), hout=h, cap=2.5)
-    n = x[pick] / np.sqrt((x[pick] ** 2).mean(-1, keepdims=True) + 1e-5) * g
-    assert rel(y[:, :N].cpu(), 2.5 * np.tanh(n @ Wr.T / 2.5)) < tol
-    assert (y[:, N:] == 7.0).all()
-    assert rel(h[:, :width].double().cpu(), n) < tol
+    normed = x / np.sqrt((x ** 2).mean(-1, keepdims=True) + 1e-5) * g
+    pick = np.array([4, 0, 3], np.int32)
+    rows = torch.from_numpy(pick).cuda()
+    h = torch.full((3, Kp), float("nan"), dtype=dtype, device="cuda")
+    hy.norm_rows(X, G, h, 3, width, Kp, 1e-5, rows=rows)
+    assert rel(h[:, :width].double().cpu(), normed[pick]) < tol
     assert (h[:, width:] == 0).all()
     K2 = -(-2 * width // 64) * 64
+    c = torch.full((n, K2), float("nan"), dtype=dtype, device="cuda")
+    hy.norm_rows(X, None, c, n, width, K2, 1e-5, x0=X0)
+    both = np.concatenate([x, x0], -1)
+    assert rel(c[:, :2 * width].double().cpu(), both) < tol
+    assert (c[:, 2 * width:] == 0).all()
+
+    Wp = torch.zeros(N, Kp, dtype=dtype, device="cuda")
+    Wp[:, :width] = _dev(rng.standard_normal((N, width)) / width ** .5, dtype)
+    Wr = Wp[:, :width].double().cpu().numpy()
+    y = torch.full((N + 3,), 7.0, device="cuda")
+    h.fill_(float("nan"))
+    hy.lin_row(Wp, X, y, width, 1e-5, g=G, rows=rows, hout=h, cap=2.5)
+    assert rel(y[:N].cpu(), 2.5 * np.tanh(normed[4] @ Wr.T / 2.5)) < tol
+    assert (y[N:] == 7.0).all()
+    assert rel(h[0, :width].double().cpu(), normed[4]) < tol
+    assert (h[0, width:] == 0).all() and h[1].isnan().all()
     W2 = torch.zeros(N, K2, dtype=dtype, device="cuda")
     W2[:, :2 * width] = _dev(rng.standard_normal((N, 2 * width)), dtype)
-    y2 = torch.empty(rows, N, device="cuda")
-    hy.lin_rows(W2, _dev(x), y2, rows, width, N, 1e-5, x0=_dev(x0))
-    both = np.concatenate([x, x0], -1)[:rows]
-    assert rel(y2.cpu(), both @ W2[:, :2 * width].double().cpu().numpy().T) \
-        < tol
+    hy.lin_row(W2, X, y, width, 1e-5, x0=X0)
+    assert rel(y[:N].cpu(), both[0] @
+               W2[:, :2 * width].double().cpu().numpy().T) < tol
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
