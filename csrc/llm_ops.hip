@@ -194,7 +194,7 @@ DEVINL const u16* gemv_stage(char* smem, const u16* x, const u16* x2,
 }
 
 // f32 variant of the staging pass, used by the fp8 GEMV: x lands in LDS
-// as fp32 PAIRS so the inner loop can feed v_pk_fma_f32 directly from
+// as fp32 PAIRS so the inner loop can feed its FMAs directly from
 // the v_cvt_pk_f32_fp8 outputs (the round-1 fp8 stream was
 // conversion-VALU-bound at 4.3 TB/s — this halves the VALU work per
 // weight byte).  Semantics match gemv_stage: the NORM2-persisted h' is
@@ -459,7 +459,7 @@ extern "C" hipError_t launch_gemv_bf16(const void* W, const void* x,
 typedef uint32_t u4v __attribute__((ext_vector_type(4)));  // = u4v_ alias
 
 // Inner loop is PACKED: x is staged as fp32 in LDS (gemv_stage_f32),
-// each v_cvt_pk_f32_fp8 output pair feeds one v_pk_fma_f32 against an
+// each v_cvt_pk_f32_fp8 output pair feeds two FMAs against an
 // LDS fp32 pair — ~16 VALU per 16 weight bytes vs ~40 for the round-1
 // scalar form (the fp8 stream was conversion-bound at 4.3 TB/s while
 // bf16 hit 6.4; see profiles/decode_kernels_r01.md).
@@ -672,7 +672,7 @@ extern "C" hipError_t launch_gemv_fp8(const void* W, const void* scales,
 // turns B-way decode into ~single-sequence step time (the 128-row MFMA
 // GEMM path wastes >90% of each tile at B<=8).  All staging modes of
 // the single-x GEMV, applied per row; XF32 stages fp32 pairs for
-// v_pk_fma_f32 (LDS B*K*4), falling back to bf16 staging (B*K*2) for
+// fp32 FMAs (LDS B*K*4), falling back to bf16 staging (B*K*2) for
 // deep-K shapes.  BT = compile-time row capacity (2/4/8); the actual
 // B <= BT, with clamped source rows.
 // ====================================================================
@@ -906,7 +906,7 @@ extern "C" hipError_t launch_gemv_fp8_mx(
 // ====================================================================
 // Skinny fp8 MFMA GEMM pair (batched decode, B = 3..16): matrix cores
 // own the MACs — the multi-x GEMV above is VALU-ISSUE-bound beyond B=2
-// (64 irreducible v_pk_fma per 16 weight bytes at B=8).
+// (128 irreducible FMAs per 16 weight bytes at B=8).
 //   1. k_stage_quant_mx: per sequence row, apply the staging op
 //      (RAW/NORM/GLU/NORM2/NORM_EMBED) and quantize to e4m3 + scale
 //      (one block per row; row stats need full-K visibility).
@@ -1139,7 +1139,7 @@ extern "C" hipError_t launch_gemm_fp8_skinny(
 // ====================================================================
 // MXFP4 GEMV: y[N] = W4[N,K] @ stage(x)[K] (+res); 2 fp4/byte with one
 // e8m0 scale per 32 elements.  Same packed structure as the fp8 GEMV
-// (fp32 x staging or XDIR direct reads feeding v_pk_fma_f32) — the
+// (fp32 x staging or XDIR direct reads feeding fp32 FMAs) — the
 // block scale rides inside v_cvt_scalef32_pk_f32_fp4, so per-ELEMENT
 // VALU matches fp8 at HALF the weight bytes.
 // ====================================================================

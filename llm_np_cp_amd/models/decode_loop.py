@@ -224,8 +224,8 @@ class DecodeLoop:
     def capture_decode_graph(self, greedy: bool = True, min_p: float = 0.1,
                              temperature: float = 1.0):
         """Capture one decode step into a hipGraph (fixed shapes: KV pool
-        is preallocated and the position is a device scalar — SURVEY §7
-        'graph must be shape-stable').
+        is preallocated and the position is a device scalar, so the graph
+        is shape-stable).
 
         NOTE: the warm-up executes ONE REAL decode step (advances the
         sequence by one token).  Returns ``(steps_taken, ok)``:
@@ -254,7 +254,7 @@ class DecodeLoop:
         except Exception as e:
             # the warm-up step above DID run (token committed to
             # out_ring, len_buf advanced) — report it so decode() does
-            # not double-count (ADVICE r1 medium)
+            # not double-count
             self._graph_failed = True
             self._graph_error = e
             torch.cuda.synchronize()

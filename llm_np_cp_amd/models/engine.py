@@ -1047,8 +1047,8 @@ class GPUModel(DecodeLoop):
         cfg = self.config
         # measured (profiles/decode_kernels_r02.md): the SKINNY fp8 MFMA
         # GEMM wins at every B (even B=2: 1.34 vs the multi-x GEMV's
-        # 1.44 ms — the GEMV is VALU-ISSUE-bound, 64 irreducible
-        # v_pk_fma per 16 weight bytes at B=8).  The multi-x path stays
+        # 1.44 ms — the GEMV is VALU-ISSUE-bound, 128 irreducible
+        # FMAs per 16 weight bytes at B=8).  The multi-x path stays
         # available via LLM_BATCH_MX_MAX for comparison.
         import os as _os  # noqa: delayed so env changes apply per call
         mx_max = int(_os.environ.get("LLM_BATCH_MX_MAX", "0"))
