@@ -94,7 +94,7 @@ DEVINL float fast_sigmoid(float z) {
 }
 DEVINL float fast_silu(float z) { return z * fast_sigmoid(z); }
 
-// clamped GLU of the routed experts:
+// GLUs of the routed experts (glu_act): silu(gate)*up, or clamped,
 //   g = min(gate, lim), u = clamp(up, -lim, lim), g*sigmoid(1.702 g)*(u+1)
 DEVINL float clamped_glu(float gate, float up, float lim) {
   float g = fminf(gate, lim);
@@ -102,11 +102,16 @@ DEVINL float clamped_glu(float gate, float up, float lim) {
   return g * sigmoid_f(1.702f * g) * (u + 1.f);
 }
 
+DEVINL float glu_act(int kind, float gate, float up, float lim) {
+  return kind ? gate * sigmoid_f(gate) * up : clamped_glu(gate, up, lim);
+}
+
 // logits of one row (already fp32, in global or LDS) -> the `top` largest
-// and the softmax over them.  One wave; E <= 64*EPL.
+// and the softmax over them, or with `scores` their sigmoids as they are.
+// One wave; E <= 64*EPL.
 template <int EPL>
 DEVINL void route_row(const float* z, int E, int top, int extra, int* idx,
-                      float* wt) {
+                      float* wt, int scores = 0) {
   const int lane = threadIdx.x & 63;
   float v[EPL];
 #pragma unroll
@@ -135,7 +140,7 @@ DEVINL void route_row(const float* z, int E, int top, int extra, int* idx,
     }
     if (be >= E) be = 0;   // NaN logits: stay in range
     if (j == 0) zmax = bv;
-    float w = expf(bv - zmax);
+    float w = scores ? sigmoid_f(bv) : expf(bv - zmax);
     sum += w;
     if (lane == 0) { idx[j] = be; wt[j] = w; }
 #pragma unroll
@@ -143,7 +148,8 @@ DEVINL void route_row(const float* z, int E, int top, int extra, int* idx,
       if (lane + i * 64 == be) v[i] = -INFINITY;
   }
   if (lane == 0) {
-    for (int j = 0; j < top; j++) wt[j] = wt[j] / sum;
+    if (!scores)
+      for (int j = 0; j < top; j++) wt[j] = wt[j] / sum;
     if (extra) { idx[top] = E; wt[top] = 1.f; }   // the shared expert
   }
 }

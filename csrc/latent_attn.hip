@@ -5,7 +5,9 @@
 // Scores and outputs stay in latent space: the per-head up-projection of
 // the keys is folded into the query (q' = W_uk^T q), so every head reads
 // the same rows, and the value up-projection is applied to the attended
-// latent.  A query tile is 16 (token, head) pairs of one sequence.
+// latent.  A query tile is 16 (token, head) pairs of one sequence.  Optional:
+// queries that go through a normed latent of their own, a sliding window, a
+// sink per head in the softmax, gates per element.
 #include "attn_split.h"
 #include "gemm_tile.h"
 #include "hybrid.h"
@@ -15,6 +17,11 @@
 
 struct LatentArgs {
   const float* P;        // fp32 projections [rows, ldp]
+  const float* Q;        // few rows: queries [rows, ldq]; head h's unrotated
+                         // part at h*qh, its rotated one at oqr + h*qrh
+  void* cq;              // normed query latents [rows, QRp]
+  const float* qnorm;    // [qrank]
+  const float* sink;     // nullable: [H]
   const void* Wuk;       // [H*d, RP]
   const void* Wuv;       // [H*vd, RP]
   const float* cnorm;    // [rank]
@@ -35,14 +42,23 @@ struct LatentArgs {
   int H, d, dp, rot, rdims, RT, rank, RP, vd, ldo, ldt;
   int rows, rbase, NS;   // rows [rbase, rbase+rows) take part in the split
   int E, rtop, rextra;
+  int ldq, qh, oqr, qrh, qrank, QRp;
+  int pairs;             // 1: rotation pairs are (2i, 2i+1), else (i, i+half)
+  int win;               // keys a token sees, itself included (0: all)
+  int gz, gc;            // gate of (head h, element j): P[og + h*gz + j*gc]
+  int written;           // the cache rows are there already
   float eps, scale;
 };
 
 // element i (< rot) of the rotated part of v at position p
 DEVINL float rotated(const float* v, int i, int dims, const float* c,
-                     const float* s) {
+                     const float* s, int pairs) {
   const int half = dims >> 1;
   if (i >= dims) return v[i];
+  if (pairs) {
+    const float o = v[i ^ 1];
+    return v[i] * c[i >> 1] + (i & 1 ? o : -o) * s[i >> 1];
+  }
   if (i < half) return v[i] * c[i] - v[i + half] * s[i];
   return v[i] * c[i - half] + v[i - half] * s[i - half];
 }
@@ -63,7 +79,7 @@ DEVINL void latent_write(const LatentArgs& a, int r, float* red) {
     float v = 0.f;
     if (i < a.rank) v = p[i] * rn * a.cnorm[i];
     else if (i >= a.RP && i < a.RP + a.rot)
-      v = rotated(p + a.rank, i - a.RP, a.rdims, c, s);
+      v = rotated(p + a.rank, i - a.RP, a.rdims, c, s, a.pairs);
     dst[i] = El<T>::st(v);
   }
 }
@@ -94,12 +110,31 @@ __global__ void __launch_bounds__(256) k_latent_prep(LatentArgs a) {
   for (int i = threadIdx.x; i < a.H * a.RT; i += 256) {
     int h = i / a.RT, j = i - h * a.RT;
     qa[(size_t)h * CS + a.RP + j] = El<T>::st(
-        j < a.rot ? rotated(q + h * dq + a.d, j, a.rdims, c, s) : 0.f);
+        j < a.rot ? rotated(q + h * dq + a.d, j, a.rdims, c, s, a.pairs) : 0.f);
   }
   latent_write<T>(a, r, red);
   if (a.E > 0 && threadIdx.x < 64)
     route_from_proj(a.P, a.ldp, a.orouter, a.E, a.rtop, a.rextra, a.ridx,
                     a.rwt, r);
+}
+
+// ---- normed query latent and cache row (rows of P whose queries are still
+// ---- to be projected) ------------------------------------------------------
+template <typename T>
+__global__ void __launch_bounds__(256) k_latent_mid(LatentArgs a) {
+  __shared__ float red[4];
+  const int r = blockIdx.x;
+  if (blockIdx.y) {
+    latent_write<T>(a, r, red);
+    return;
+  }
+  const float* q = a.P + (size_t)r * a.ldp + a.oq;
+  float ss = 0.f;
+  for (int i = threadIdx.x; i < a.qrank; i += 256) ss += q[i] * q[i];
+  const float rn = 1.f / sqrtf(block_sum(ss, red) / (float)a.qrank + a.eps);
+  for (int i = threadIdx.x; i < a.QRp; i += 256)
+    ((T*)a.cq)[(size_t)r * a.QRp + i] =
+        El<T>::st(i < a.qrank ? q[i] * rn * a.qnorm[i] : 0.f);
 }
 
 // ---- few rows: absorb W_uk per (head, latent columns, row); two more
@@ -113,14 +148,16 @@ __global__ void __launch_bounds__(256) k_latent_dec_prep(LatentArgs a) {
   const int cb = a.RP < AB_COLS ? a.RP : AB_COLS, ncb = a.RP / cb;
   const int h = blockIdx.x / ncb, c0 = (blockIdx.x - h * ncb) * cb;
   if (h >= a.H) {
-    if ((int)blockIdx.x == a.H * ncb) latent_write<T>(a, r, red);
-    else if (threadIdx.x < 64)
+    if ((int)blockIdx.x == a.H * ncb) {
+      if (!a.written) latent_write<T>(a, r, red);
+    } else if (threadIdx.x < 64)
       route_from_proj(a.P, a.ldp, a.orouter, a.E, a.rtop, a.rextra, a.ridx,
                       a.rwt, r);
     return;
   }
-  const int dq = a.d + a.rot, CS = a.RP + a.RT, tid = threadIdx.x;
-  const float* q = a.P + (size_t)r * a.ldp + a.oq + (size_t)h * dq;
+  const int CS = a.RP + a.RT, tid = threadIdx.x;
+  const float* q = a.Q + (size_t)r * a.ldq + (size_t)h * a.qh;
+  const float* qr = a.Q + (size_t)r * a.ldq + a.oqr + (size_t)h * a.qrh;
   T* qa = (T*)a.qa + ((size_t)r * a.H + h) * CS;
   // lanes own V latent columns each; the d axis is split over the groups
   const int nv = cb / V, groups = 256 / nv;
@@ -151,7 +188,7 @@ __global__ void __launch_bounds__(256) k_latent_dec_prep(LatentArgs a) {
   const float* s = a.sinT + (size_t)pos * (a.rdims >> 1);
   for (int j = tid; j < a.RT; j += 256)
     qa[a.RP + j] = El<T>::st(
-        j < a.rot ? rotated(q + a.d, j, a.rdims, c, s) : 0.f);
+        j < a.rot ? rotated(qr, j, a.rdims, c, s, a.pairs) : 0.f);
 }
 
 // ---- attention --------------------------------------------------------
@@ -210,10 +247,12 @@ __global__ void __launch_bounds__(64 * NW) k_latent_attn(LatentArgs a) {
   const int qpos = pos0 + myc / a.H;
   const int last = min(rr0 + 16 * QW, nrr) - 1;
   const int kend = pos0 + last / a.H + 1;               // keys [0, kend)
-  // key tiles of this split
-  const int ntile = (kend + KT - 1) / KT;
-  const int per = (ntile + a.NS - 1) / a.NS;
-  const int t_lo = blockIdx.y * per, t_hi = min(ntile, t_lo + per);
+  // key tiles of this split, from the first one that the first query sees
+  const int tbeg = a.win ? max(0, pos0 + rr0 / a.H - a.win + 1) / KT : 0;
+  const int tend = (kend + KT - 1) / KT;
+  const int per = (tend - tbeg + a.NS - 1) / a.NS;
+  const int t_lo = tbeg + blockIdx.y * per, t_hi = min(tend, t_lo + per);
+  const int before = a.win ? qpos - a.win : -1;         // keys this one hides
 
   // loading: lanes take 16 row pairs x 16-byte columns
   const int kp = tid & 15, cv0 = tid >> 4;
@@ -256,6 +295,10 @@ __global__ void __launch_bounds__(64 * NW) k_latent_attn(LatentArgs a) {
 #pragma unroll
   for (int d = 0; d < ND; d++) acc[d] = {0.f, 0.f, 0.f, 0.f};
   float mrun = -INFINITY, lrun = 0.f;
+  if (a.sink && blockIdx.y == 0) {      // a score without a value
+    mrun = a.sink[myc % a.H] * 1.4426950408889634f;
+    lrun = 1.f;
+  }
   const float sc = a.scale * 1.4426950408889634f;       // base-2 exponents
 
   for (int t = t_lo; t < t_hi; t++) {
@@ -302,7 +345,7 @@ __global__ void __launch_bounds__(64 * NW) k_latent_attn(LatentArgs a) {
 #pragma unroll
     for (int i = 0; i < 8; i++) {
       const int key = k0 + (i >> 2) * 16 + g * 4 + (i & 3);
-      sv[i] = key <= qpos ? st[i >> 2][i & 3] * sc : -INFINITY;
+      sv[i] = key <= qpos && key > before ? st[i >> 2][i & 3] * sc : -INFINITY;
       pmax = fmaxf(pmax, sv[i]);
     }
     pmax = fmaxf(pmax, __shfl_xor(pmax, 16));
@@ -421,9 +464,11 @@ __global__ void __launch_bounds__(256) k_latent_dec_fin(LatentArgs a, int nub,
   slab(lane);
   latent_merge<T>(a, rh, ol, sh);
   __syncthreads();
-  const float gate = sigmoid_f(a.P[(size_t)r * a.ldp + a.og + h]);
+  const float* gate = a.P + (size_t)r * a.ldp + a.og + h * a.gz;
   for (int first = 1; j0 < a.vd; j0 += nub * 4 * UVW, first = 0) {
-    float acc[UVW];
+    float acc[UVW], out = 0.f;
+    const bool mine = lane < UVW && j0 + lane < a.vd;
+    const float gt = mine ? sigmoid_f(gate[(j0 + lane) * a.gc]) : 0.f;
 #pragma unroll
     for (int i = 0; i < UVW; i++) acc[i] = 0.f;
     for (int k = lane; k < nv; k += 64) {
@@ -435,8 +480,9 @@ __global__ void __launch_bounds__(256) k_latent_dec_fin(LatentArgs a, int nub,
 #pragma unroll
     for (int i = 0; i < UVW; i++) {
       float v = wave_reduce_sum(acc[i]);
-      if (lane == 0 && j0 + i < a.vd) o[j0 + i] = El<T>::st(v * gate);
+      if (lane == i) out = v;
     }
+    if (mine) o[j0 + lane] = El<T>::st(out * gt);
   }
 }
 
@@ -445,7 +491,7 @@ static bool bad_shape(const LatentArgs& a) {
   return a.rows < 1 || a.H < 1 || a.RT % 32 || a.RT < a.rot || a.RT > 128 ||
          a.RP < a.rank || a.rdims > a.rot || a.rdims % 2 || a.NS < 1 ||
          a.NS > MAX_SPLITS || a.E > 1024 || (a.E > 0 && a.rtop > a.E) || a.dp % 64 ||
-         a.dp < a.d;
+         a.dp < a.d || a.win < 0;
 }
 
 extern "C" hipError_t launch_latent_prep(int f32, const LatentArgs* a,
@@ -456,9 +502,19 @@ extern "C" hipError_t launch_latent_prep(int f32, const LatentArgs* a,
   return hipGetLastError();
 }
 
+extern "C" hipError_t launch_latent_mid(int f32, const LatentArgs* a,
+                                        hipStream_t s) {
+  if (bad_shape(*a) || a->qrank < 1 || a->QRp < a->qrank || !a->cq ||
+      !a->qnorm)
+    return hipErrorInvalidValue;
+  if (f32) hipLaunchKernelGGL(k_latent_mid<float>, dim3(a->rows, 2), dim3(256), 0, s, *a);
+  else hipLaunchKernelGGL(k_latent_mid<u16>, dim3(a->rows, 2), dim3(256), 0, s, *a);
+  return hipGetLastError();
+}
+
 extern "C" hipError_t launch_latent_dec_prep(int f32, const LatentArgs* a,
                                              hipStream_t s) {
-  if (bad_shape(*a) || a->RP > 512) return hipErrorInvalidValue;
+  if (bad_shape(*a) || a->RP > 512 || !a->Q) return hipErrorInvalidValue;
   const int cb = a->RP < AB_COLS ? a->RP : AB_COLS;
   if (a->RP % cb) return hipErrorInvalidValue;
   // the last head's blocks: cache row, then routing (RP / cb may be 1)

@@ -23,6 +23,9 @@ k_embed_rows(const T* __restrict__ table, const int* __restrict__ ids,
 // ---- staging a row of the residual for a projection --------------------
 // v = x [+ y / rms(y) * gb] [+ xadd]            (y: the last sublayer's output)
 // out = v / rms(v) * g [* sigmoid(gate)]
+// or, with CONV, v + a causal convolution over time on each channel,
+//   out = v + sum_j cw[taps-1-j] v(pos - j),    zero before position 0.
+// The last inputs v of a sequence are kept in a ring, ring[slot][pos % taps].
 // A row of up to NT*U elements stays in the registers of NT threads.
 struct RowStage {
   const float* x;
@@ -31,11 +34,14 @@ struct RowStage {
   const float* g;           // null: only v is wanted
   const float* gate;        // nullable, [rows, ldg]
   float* xout;              // nullable: receives v
-  int W, Kp, ldg;
+  const float* cw;          // CONV: [taps, W]
+  float* ring;              // CONV: [slots, taps, W]
+  const int *slot, *pos;    // CONV: per row
+  int W, Kp, ldg, taps;
   float eps;
 };
 
-template <int NT, int U, class Put>
+template <int NT, int U, bool CONV = false, class Put>
 DEVINL void stage_row(const RowStage& s, size_t row, bool keep, float* red,
                       Put put) {
   const int tid = threadIdx.x, W = s.W;
@@ -47,6 +53,28 @@ DEVINL void stage_row(const RowStage& s, size_t row, bool keep, float* red,
     xv[u] = i < W ? s.x[o + i] : 0.f;
     gv[u] = s.g && i < W ? s.g[i] : 0.f;
     if (s.y) yv[u] = i < W ? s.y[o + i] : 0.f;
+  }
+  [[maybe_unused]] int pos = 0;
+  [[maybe_unused]] float* ring = nullptr;
+  [[maybe_unused]] float cv[U], cl[U];   // earlier inputs' part, newest tap
+  if constexpr (CONV) {
+    pos = s.pos[row];
+    ring = s.ring + (size_t)s.slot[row] * s.taps * W;
+#pragma unroll
+    for (int u = 0; u < U; u++) {
+      const int i = tid + u * NT;
+      cv[u] = 0.f;
+      cl[u] = i < W ? s.cw[(size_t)(s.taps - 1) * W + i] : 0.f;
+    }
+    for (int j = 1; j < s.taps && j <= pos; j++) {
+      const float* h = ring + (size_t)((pos - j) % s.taps) * W;
+      const float* c = s.cw + (size_t)(s.taps - 1 - j) * W;
+#pragma unroll
+      for (int u = 0; u < U; u++) {
+        const int i = tid + u * NT;
+        if (i < W) cv[u] = fmaf(c[i], h[i], cv[u]);
+      }
+    }
   }
   float rb = 0.f;
   if (s.y) {
@@ -89,8 +117,30 @@ DEVINL void stage_row(const RowStage& s, size_t row, bool keep, float* red,
   auto finish = [&](int i, float v, float g) {
     if (s.g && i < s.Kp)
       put(i, i < W ? v * rn * g * (gt ? sigmoid_f(gt[i]) : 1.f) : 0.f);
-    if (keep && i < W) s.xout[o + i] = v;    // may be x: its reads are done
+    // xout may be x: its reads are done
+    if (keep && s.xout && i < W) s.xout[o + i] = v;
   };
+  if constexpr (CONV) {
+    auto mix = [&](int i, float v, float c, float before) {
+      if (i < s.Kp) put(i, i < W ? v + fmaf(c, v, before) : 0.f);
+      if (keep && i < W) {
+        if (s.xout) s.xout[o + i] = v;
+        ring[(size_t)(pos % s.taps) * W + i] = v;   // nobody reads this entry
+      }
+    };
+#pragma unroll
+    for (int u = 0; u < U; u++) mix(tid + u * NT, xv[u], cl[u], cv[u]);
+    for (int i = tid + U * NT; i < max(W, s.Kp); i += NT) {
+      float before = 0.f;
+      if (i < W)
+        for (int j = 1; j < s.taps && j <= pos; j++)
+          before = fmaf(s.cw[(size_t)(s.taps - 1 - j) * W + i],
+                        ring[(size_t)((pos - j) % s.taps) * W + i], before);
+      mix(i, i < W ? late(i) : 0.f,
+          i < W ? s.cw[(size_t)(s.taps - 1) * W + i] : 0.f, before);
+    }
+    return;
+  }
 #pragma unroll
   for (int u = 0; u < U; u++) finish(tid + u * NT, xv[u], gv[u]);
   for (int i = tid + U * NT; i < max(W, s.Kp); i += NT)
@@ -104,8 +154,273 @@ __global__ void __launch_bounds__(256)
 k_norm_rows(RowStage s, const int* __restrict__ rows, T* __restrict__ out) {
   __shared__ float red[4];
   T* o = out + (size_t)blockIdx.x * s.Kp;
-  stage_row<256, U>(s, rows ? rows[blockIdx.x] : blockIdx.x, s.xout != nullptr, red,
+  stage_row<256, U>(s, rows ? rows[blockIdx.x] : blockIdx.x, true, red,
                [&](int i, float v) { o[i] = El<T>::st(v); });
+}
+
+// ---- rows with their input convolution -----------------------------------
+// out[r] = v_r + conv(v)_r with v = x [+ y / rms(y) * gb], for single tokens
+// and runs of tokens.  A block takes one single token, or CR rows of a chunk
+// of a run; it computes the rows ahead of its own again.  The block at the
+// head of a run reads the ring and, channel by channel in the same thread,
+// leaves the run's last inputs in it.
+#define CR 8
+#define CHUNK 64
+
+struct ConvRows {
+  RowStage s;               // x, y, gb, xout (beside x), cw, ring, slot, pos
+  void* out;                // [rows, Kp] T
+  const int *seg_row0, *seg_len, *seg_slot, *seg_pos0;   // runs
+  const int *chunk_row0, *chunk_len, *chunk_seg;
+  int nd, nseg, nchunk;     // rows [0, nd) are single tokens
+};
+
+struct ConvBlock {
+  int row0, n, seg0, len, slot, pos0;   // rows of the block, its sequence's run
+};
+
+DEVINL ConvBlock conv_block(const ConvRows& a) {
+  const int b = blockIdx.x;
+  if (b < a.nd) return {b, 1, b, 1, a.s.slot[b], a.s.pos[b]};
+  const int c = (b - a.nd) / (CHUNK / CR), at = (b - a.nd) % (CHUNK / CR) * CR;
+  const int g = a.chunk_seg[c];
+  return {a.chunk_row0[c] + at, min(CR, a.chunk_len[c] - at), a.seg_row0[g],
+          a.seg_len[g], a.seg_slot[g], a.seg_pos0[g]};
+}
+
+// 1 / rms of one row of y, by one wave
+DEVINL float wave_rms(const RowStage& s, int row) {
+  const float* y = s.y + (size_t)row * s.W;
+  const int lane = threadIdx.x & 63;
+  float ss = 0.f;
+  if (s.W % 4 == 0) {
+#pragma unroll 4
+    for (int i = lane * 4; i < s.W; i += 256) {
+      f4v v = *(const f4v*)(y + i);
+      ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+    }
+  } else {
+    for (int i = lane; i < s.W; i += 64) ss += y[i] * y[i];
+  }
+  return 1.f / sqrtf(wave_reduce_sum(ss) / (float)s.W + s.eps);
+}
+
+template <int V> struct Vec { float f[V]; };
+template <int V> DEVINL Vec<V> ldv(const float* p) {
+  Vec<V> r;
+  if constexpr (V == 4) {
+    f4v v = *(const f4v*)p;
+#pragma unroll
+    for (int c = 0; c < 4; c++) r.f[c] = v[c];
+  } else r.f[0] = *p;
+  return r;
+}
+template <int V> DEVINL void stv(float* p, const Vec<V>& v) {
+  if constexpr (V == 4) *(f4v*)p = f4v{v.f[0], v.f[1], v.f[2], v.f[3]};
+  else *p = v.f[0];
+}
+template <int V, typename T> DEVINL void stv_as(T* p, const Vec<V>& v) {
+  union { T t[V]; uint64_t u; f4v f; } o;
+#pragma unroll
+  for (int c = 0; c < V; c++) o.t[c] = El<T>::st(v.f[c]);
+  if constexpr (V * sizeof(T) == 8) *(uint64_t*)p = o.u;
+  else if constexpr (V * sizeof(T) == 16) *(f4v*)p = o.f;
+  else *p = o.t[0];
+}
+
+// TAPS - 1 <= CR; V = 4 needs W % 4 == 0
+template <typename T, int TAPS, int V>
+__global__ void __launch_bounds__(256) k_conv_rows(ConvRows a) {
+  constexpr int B = TAPS - 1;
+  __shared__ float rn[CR + 2 * B];      // the block's rows, the run's last
+  const RowStage& s = a.s;
+  const ConvBlock k = conv_block(a);
+  if (k.n <= 0) return;
+  const int W = s.W, tid = threadIdx.x;
+  const bool head = k.row0 == k.seg0;
+  const int tail0 = k.seg0 + k.len - B;
+  if (s.y) {
+    for (int e = tid >> 6; e < CR + 2 * B; e += 4) {
+      const int row = e < CR + B ? k.row0 - B + e : tail0 + e - (CR + B);
+      if (row < k.seg0 || (e < CR + B ? row >= k.row0 + k.n : !head)) continue;
+      const float r = wave_rms(s, row);
+      if ((tid & 63) == 0) rn[e] = r;
+    }
+    __syncthreads();
+  }
+  float* ring = s.ring + (size_t)k.slot * TAPS * W;
+  for (int i = tid * V; i < s.Kp; i += 256 * V) {
+    if (i >= W) {
+      const Vec<V> z = {};
+      for (int e = 0; e < k.n; e++)
+        stv_as<V>((T*)a.out + (size_t)(k.row0 + e) * s.Kp + i, z);
+      continue;
+    }
+    const Vec<V> gb = s.y ? ldv<V>(s.gb + i) : Vec<V>{};
+    auto value = [&](int row, int e) {
+      Vec<V> v = ldv<V>(s.x + (size_t)row * W + i);
+      if (s.y) {
+        const Vec<V> y = ldv<V>(s.y + (size_t)row * W + i);
+#pragma unroll
+        for (int c = 0; c < V; c++) v.f[c] += y.f[c] * rn[e] * gb.f[c];
+      }
+      return v;
+    };
+    Vec<V> w[TAPS], v[CR + B];
+#pragma unroll
+    for (int j = 0; j < TAPS; j++) w[j] = ldv<V>(s.cw + (size_t)j * W + i);
+#pragma unroll
+    for (int e = 0; e < B; e++) {
+      const int back = k.row0 - B + e - k.seg0;     // < 0: before this run
+      if (back >= 0) v[e] = value(k.row0 - B + e, e);
+      else if (k.pos0 + back >= 0)
+        v[e] = ldv<V>(ring + (size_t)((k.pos0 + back) % TAPS) * W + i);
+      else v[e] = {};
+    }
+#pragma unroll
+    for (int e = 0; e < CR; e++)
+      if (e < k.n) v[B + e] = value(k.row0 + e, B + e);
+#pragma unroll
+    for (int e = 0; e < CR; e++)
+      if (e < k.n) {
+        Vec<V> o;
+#pragma unroll
+        for (int c = 0; c < V; c++) {
+          float sum = 0.f;
+#pragma unroll
+          for (int j = 0; j < TAPS; j++) sum = fmaf(w[j].f[c], v[e + j].f[c], sum);
+          o.f[c] = v[B + e].f[c] + sum;
+        }
+        stv_as<V>((T*)a.out + (size_t)(k.row0 + e) * s.Kp + i, o);
+        if (s.xout) stv<V>(s.xout + (size_t)(k.row0 + e) * W + i, v[B + e]);
+      }
+    if (head)
+#pragma unroll
+      for (int e = 0; e < B; e++) {
+        const int row = tail0 + e;
+        if (row >= k.seg0)
+          stv<V>(ring + (size_t)((k.pos0 + row - k.seg0) % TAPS) * W + i,
+                 value(row, CR + B + e));
+      }
+  }
+}
+
+// any number of taps; the ring is written by a launch of its own
+template <typename T>
+__global__ void __launch_bounds__(256) k_conv_rows_any(ConvRows a) {
+  extern __shared__ float rnx[];        // CR + taps - 1
+  const RowStage& s = a.s;
+  const ConvBlock k = conv_block(a);
+  if (k.n <= 0) return;
+  const int W = s.W, B = s.taps - 1, tid = threadIdx.x;
+  if (s.y)
+    for (int e = tid >> 6; e < k.n + B; e += 4) {
+      const int row = k.row0 - B + e;
+      if (row < k.seg0) continue;
+      const float r = wave_rms(s, row);
+      if ((tid & 63) == 0) rnx[e] = r;
+    }
+  __syncthreads();
+  const float* ring = s.ring + (size_t)k.slot * s.taps * W;
+  for (int i = tid; i < s.Kp; i += 256)
+    for (int e = 0; e < k.n; e++) {
+      T* o = (T*)a.out + (size_t)(k.row0 + e) * s.Kp + i;
+      if (i >= W) {
+        *o = El<T>::st(0.f);
+        continue;
+      }
+      float sum = 0.f, v = 0.f;
+      for (int j = 0; j < s.taps; j++) {
+        const int row = k.row0 + e - B + j, back = row - k.seg0;
+        v = 0.f;
+        if (back >= 0) {
+          v = s.x[(size_t)row * W + i];
+          if (s.y) v += s.y[(size_t)row * W + i] * rnx[e + j] * s.gb[i];
+        } else if (k.pos0 + back >= 0) {
+          v = ring[(size_t)((k.pos0 + back) % s.taps) * W + i];
+        }
+        sum = fmaf(s.cw[(size_t)j * W + i], v, sum);
+      }
+      *o = El<T>::st(v + sum);
+      if (s.xout) s.xout[(size_t)(k.row0 + e) * W + i] = v;
+    }
+}
+
+// last inputs of every sequence of the batch -> its ring; v holds the rows
+__global__ void __launch_bounds__(256)
+k_conv_ring(ConvRows a, const float* __restrict__ v) {
+  const int b = blockIdx.x, W = a.s.W, taps = a.s.taps, g = b - a.nd;
+  const bool one = b < a.nd;
+  const int row0 = one ? b : a.seg_row0[g], len = one ? 1 : a.seg_len[g];
+  const int slot = one ? a.s.slot[b] : a.seg_slot[g];
+  const int pos0 = one ? a.s.pos[b] : a.seg_pos0[g];
+  float* ring = a.s.ring + (size_t)slot * taps * W;
+  for (int t = max(0, len - taps + 1); t < len; t++)
+    for (int i = threadIdx.x; i < W; i += 256)
+      ring[(size_t)((pos0 + t) % taps) * W + i] = v[(size_t)(row0 + t) * W + i];
+}
+
+// ---- polynomial activation of whole rows ---------------------------------
+// out = c0 N(z) + c1 N(z^2) + c2 N(z^3) + c3, N dividing by the root mean
+// square over the row's W values; zero from W to Kp.
+struct PolyNorm {
+  float r1, r2, r3, e;
+  DEVINL float operator()(float z) const {
+    const float z2 = z * z;
+    return r1 * z + (r2 * z2 + (r3 * (z2 * z) + e));
+  }
+};
+
+// NT threads hold z[u] = element tid + u*NT, late(i) reads the others
+template <int NT, int U, class Late>
+DEVINL PolyNorm poly_moments(const float (&z)[U], Late late, int W,
+                             const float* coef, float eps, float* red) {
+  float m[3] = {0.f, 0.f, 0.f};
+  auto add = [&](float v) {
+    const float v2 = v * v, v4 = v2 * v2;
+    m[0] += v2; m[1] += v4; m[2] += v4 * v2;
+  };
+#pragma unroll
+  for (int u = 0; u < U; u++) add(z[u]);
+  for (int i = threadIdx.x + U * NT; i < W; i += NT) add(late(i));
+#pragma unroll
+  for (int k = 0; k < 3; k++) m[k] = wave_reduce_sum(m[k]);
+  if ((threadIdx.x & 63) == 0)
+#pragma unroll
+    for (int k = 0; k < 3; k++) red[(threadIdx.x >> 6) * 3 + k] = m[k];
+  __syncthreads();
+  float r[3];
+#pragma unroll
+  for (int k = 0; k < 3; k++) {
+    float t = 0.f;
+    for (int w = 0; w < NT / 64; w++) t += red[w * 3 + k];
+    r[k] = coef[k] / sqrtf(t / (float)W + eps);
+  }
+  return {r[0], r[1], r[2], coef[3]};
+}
+
+template <typename T, int U>
+__global__ void __launch_bounds__(256)
+k_poly_rows(const float* __restrict__ z, int ldz, const float* __restrict__ coef,
+            T* __restrict__ out, int W, int Kp, float eps) {
+  __shared__ float red[12];
+  const float* zr = z + (size_t)blockIdx.x * ldz;
+  T* o = out + (size_t)blockIdx.x * Kp;
+  float v[U];
+#pragma unroll
+  for (int u = 0; u < U; u++) {
+    const int i = threadIdx.x + u * 256;
+    v[u] = i < W ? zr[i] : 0.f;
+  }
+  auto late = [&](int i) { return zr[i]; };
+  const PolyNorm f = poly_moments<256, U>(v, late, W, coef, eps, red);
+#pragma unroll
+  for (int u = 0; u < U; u++) {
+    const int i = threadIdx.x + u * 256;
+    if (i < Kp) o[i] = El<T>::st(i < W ? f(v[u]) : 0.f);
+  }
+  for (int i = threadIdx.x + U * 256; i < Kp; i += 256)
+    o[i] = El<T>::st(i < W ? f(late(i)) : 0.f);
 }
 
 // cast of [x | x0] with zero padding
@@ -121,13 +436,13 @@ k_cat_rows(const float* __restrict__ x, const float* __restrict__ x0,
 }
 
 // ---- one row: y[n] = W[n] . staged row, one wave per NR outputs ----------
-// The row is staged into LDS as T: normed (stage_row) or concatenated [x |
-// x0]; block 0 can persist it to hout, and the residual to xout.  A row
+// The row is staged into LDS as T: normed or convolved (stage_row),
+// concatenated [x | x0], or through the polynomial activation; block 0 can persist it to hout, and the residual to xout.  A row
 // that is T already (hin) is read where it lies.  A wave always has its
 // next slab of weights on the way, the first one during the staging.
 enum { EPI_F32 = 0, EPI_RESADD = 1, EPI_SOFTCAP = 2, EPI_T = 3, EPI_TGATE = 4,
-       EPI_RELU2 = 5 };
-enum { ROW_NORM = 0, ROW_CAT = 1, ROW_PLAIN = 2 };
+       EPI_RELU2 = 5, EPI_ROTARY = 6 };
+enum { ROW_NORM = 0, ROW_CAT = 1, ROW_PLAIN = 2, ROW_CONV = 3, ROW_POLY = 4 };
 
 struct LinRowArgs {
   const void* Wt;           // [N, Kp]
@@ -136,6 +451,7 @@ struct LinRowArgs {
   const void* hin;          // ROW_PLAIN
   void* hout;               // nullable
   const float* bias;        // nullable
+  const float* act;         // ROW_POLY: four coefficients; the row is s.x
   void* y;                  // fp32, or T for EPI_RELU2
   int N, stage, epi;
   float cap;
@@ -150,7 +466,7 @@ DEVINL float relu2_f(float v) {
 template <typename T, int MODE, int U, int NR>
 __global__ void __launch_bounds__(LIN_NT) k_lin_row(LinRowArgs a) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  __shared__ float red[LIN_NT / 64];
+  __shared__ float red[LIN_NT / 64 * (MODE == ROW_POLY ? 3 : 1)];
   constexpr int V = El<T>::V, S = 64 * V, NK = 8 / NR;
   T* xs = (T*)smem;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
@@ -172,13 +488,31 @@ __global__ void __launch_bounds__(LIN_NT) k_lin_row(LinRowArgs a) {
   slab(w, n, 0);
   const size_t row = a.rows ? a.rows[0] : 0;
   const bool first = blockIdx.x == 0;
-  if constexpr (MODE == ROW_NORM) {
-    stage_row<LIN_NT, U>(a.s, row, first && a.s.xout, red,
-                         [&](int i, float f) {
+  if constexpr (MODE == ROW_NORM || MODE == ROW_CONV) {
+    stage_row<LIN_NT, U, MODE == ROW_CONV>(a.s, row, first, red,
+                                           [&](int i, float f) {
       T v = El<T>::st(f);
       xs[i] = v;
       if (a.hout && first) ((T*)a.hout)[i] = v;
     });
+  } else if constexpr (MODE == ROW_POLY) {
+    const int W = a.s.W;
+    const float* z = a.s.x + row * W;
+    float v[U];
+#pragma unroll
+    for (int u = 0; u < U; u++) {
+      const int i = tid + u * LIN_NT;
+      v[u] = i < W ? z[i] : 0.f;
+    }
+    auto late = [&](int i) { return z[i]; };
+    const PolyNorm f = poly_moments<LIN_NT, U>(v, late, W, a.act, a.s.eps, red);
+#pragma unroll
+    for (int u = 0; u < U; u++) {
+      const int i = tid + u * LIN_NT;
+      if (i < Kp) xs[i] = El<T>::st(i < W ? f(v[u]) : 0.f);
+    }
+    for (int i = tid + U * LIN_NT; i < Kp; i += LIN_NT)
+      xs[i] = El<T>::st(i < W ? f(late(i)) : 0.f);
   } else if constexpr (MODE == ROW_CAT) {
     const int W = a.s.W;
     const float *x = a.s.x + row * W, *x0 = a.s.xadd + row * W;
@@ -228,19 +562,47 @@ __global__ void __launch_bounds__(LIN_NT) k_lin_row(LinRowArgs a) {
 }
 
 // ---- many rows: MFMA GEMM ---------------------------------------------
+// EPI_ROTARY: columns from `split` on are heads of RT values, of which the
+// first `dims` rotate in pairs (2i, 2i+1); they go to y[row*ld + head*hs].
+struct Rotary {
+  const int* pos;
+  const float *cosT, *sinT;   // [positions, dims/2]
+  void* y;
+  int split, RT, dims, ld, hs;
+};
+
 struct GemmArgs {
   const void *X, *W;
   void* Y;
-  const float* gate;        // EPI_TGATE: sigmoid(gate[row*ldg + z])
+  const float* gate;        // EPI_TGATE: sigmoid(gate[row*ldg + z*gz + col*gc])
   const float* bias;        // nullable: added per column
-  int M, N, K, ldx, ldw, ldy, ldg, epi;
+  int M, N, K, ldx, ldw, ldy, ldg, epi, gz, gc;
   float mult;               // EPI_RESADD multiplier / EPI_SOFTCAP cap
   long xz, wz, yz;          // per-z (head) element offsets
+  struct Rotary r;          // EPI_ROTARY
 };
 
 template <typename T, int EPI>
 DEVINL void gemm_store(const GemmArgs& a, int z, int row, int col, float v) {
   const size_t o = (size_t)z * a.yz + (size_t)row * a.ldy + col;
+  if constexpr (EPI == EPI_ROTARY) {
+    // every lane of the wave comes here, neighbours with neighbouring columns
+    const Rotary& r = a.r;
+    const float other = __shfl_xor(v, 1);
+    if (row >= a.M || col >= a.N) return;
+    if (col < r.split) {
+      ((T*)a.Y)[o] = El<T>::st(v);
+      return;
+    }
+    const int c = col - r.split, h = c / r.RT, j = c - h * r.RT;
+    if (j < r.dims) {
+      const size_t t = (size_t)r.pos[row] * (r.dims >> 1) + (j >> 1);
+      v = v * r.cosT[t] + (j & 1 ? other : -other) * r.sinT[t];
+    }
+    ((T*)r.y)[(size_t)row * r.ld + (size_t)h * r.hs + j] = El<T>::st(v);
+    return;
+  }
+  if (row >= a.M || col >= a.N) return;
   if constexpr (EPI == EPI_F32) ((float*)a.Y)[o] = v;
   else if constexpr (EPI == EPI_RESADD) ((float*)a.Y)[o] += a.mult * v;
   else if constexpr (EPI == EPI_SOFTCAP)
@@ -249,7 +611,7 @@ DEVINL void gemm_store(const GemmArgs& a, int z, int row, int col, float v) {
   else if constexpr (EPI == EPI_RELU2) ((T*)a.Y)[o] = El<T>::st(relu2_f(v));
   else
     ((T*)a.Y)[o] = El<T>::st(
-        v * sigmoid_f(a.gate[(size_t)row * a.ldg + z]));
+        v * sigmoid_f(a.gate[(size_t)row * a.ldg + z * a.gz + col * a.gc]));
 }
 
 // run body(integral constant of the epilogue)
@@ -261,6 +623,7 @@ template <class Body> DEVINL void with_epilogue(int epi, Body body) {
     case EPI_T: body(std::integral_constant<int, EPI_T>()); break;
     case EPI_TGATE: body(std::integral_constant<int, EPI_TGATE>()); break;
     case EPI_RELU2: body(std::integral_constant<int, EPI_RELU2>()); break;
+    case EPI_ROTARY: body(std::integral_constant<int, EPI_ROTARY>()); break;
   }
 }
 
@@ -289,9 +652,8 @@ __global__ void __launch_bounds__(256) k_gemm(GemmArgs a) {
 #pragma unroll
         for (int r = 0; r < 4; r++) {
           const int row = bm + gemm_row0<BM>(i) + r;
-          if (row < a.M && col < a.N)
-            gemm_store<T, decltype(epi)::value>(a, z, row, col,
-                                                acc[i][j][r] + bias[j]);
+          gemm_store<T, decltype(epi)::value>(a, z, row, col,
+                                              acc[i][j][r] + bias[j]);
         }
       }
   });
@@ -345,12 +707,10 @@ __global__ void __launch_bounds__(64 * NW) k_gemm_skinny(GemmArgs a) {
 #pragma unroll
     for (int u = 0; u < NW; u++) v += red[u * MF * 256 + e];
     const int row = e >> 4, col = n0 + (e & 15);
-    if (row < a.M && col < a.N) {
-      if (a.bias) v += a.bias[col];
-      with_epilogue(a.epi, [&](auto epi) {
-        gemm_store<T, decltype(epi)::value>(a, z, row, col, v);
-      });
-    }
+    if (a.bias) v += a.bias[min(col, a.N - 1)];
+    with_epilogue(a.epi, [&](auto epi) {
+      gemm_store<T, decltype(epi)::value>(a, z, row, col, v);
+    });
   }
 }
 
@@ -399,6 +759,74 @@ extern "C" hipError_t launch_norm_rows(int f32, const RowStage* s,
   return hipGetLastError();
 }
 
+static bool bad_conv(const RowStage& s) {
+  return bad_stage(s) || !s.cw || !s.ring || !s.slot || !s.pos || s.taps < 1 ||
+         s.Kp < s.W || s.xadd || s.g || s.gate || (s.y && !s.xout);
+}
+
+template <typename T, int V>
+static bool conv_go(const ConvRows& a, int blocks, hipStream_t st) {
+#define CONV_TAPS(n)                                                         \
+  case n:                                                                    \
+    hipLaunchKernelGGL((k_conv_rows<T, n, V>), dim3(blocks), dim3(256), 0,   \
+                       st, a);                                               \
+    return true
+  switch (a.s.taps) {
+    CONV_TAPS(1);
+    CONV_TAPS(2);
+    CONV_TAPS(3);
+    CONV_TAPS(4);
+  }
+#undef CONV_TAPS
+  return false;
+}
+
+template <typename T>
+static hipError_t conv_rows(const ConvRows& a, hipStream_t st) {
+  const int blocks = a.nd + a.nchunk * (CHUNK / CR);
+  const bool done = a.s.W % 4 ? conv_go<T, 1>(a, blocks, st)
+                              : conv_go<T, 4>(a, blocks, st);
+  if (!done) {
+    const size_t lds = (CR + a.s.taps - 1) * sizeof(float);
+    hipLaunchKernelGGL(k_conv_rows_any<T>, dim3(blocks), dim3(256), lds, st, a);
+    hipLaunchKernelGGL(k_conv_ring, dim3(a.nd + a.nseg), dim3(256), 0, st, a,
+                       a.s.xout ? a.s.xout : a.s.x);
+  }
+  return hipGetLastError();
+}
+
+extern "C" hipError_t launch_conv_rows(int f32, const ConvRows* a,
+                                       hipStream_t st) {
+  if (bad_conv(a->s) || a->s.xout == a->s.x || !a->out || a->nd < 0 ||
+      a->nchunk < 0 || a->nd + a->nchunk < 1 || !a->nseg != !a->nchunk ||
+      a->s.taps > 8192)
+    return hipErrorInvalidValue;
+  return f32 ? conv_rows<float>(*a, st) : conv_rows<u16>(*a, st);
+}
+
+template <typename T>
+static void poly_rows(const void* z, int ldz, const void* coef, void* out,
+                      int M, int W, int Kp, float eps, hipStream_t s) {
+  if (W <= 4096)
+    hipLaunchKernelGGL((k_poly_rows<T, 16>), dim3(M), dim3(256), 0, s,
+                       (const float*)z, ldz, (const float*)coef, (T*)out, W,
+                       Kp, eps);
+  else
+    hipLaunchKernelGGL((k_poly_rows<T, 40>), dim3(M), dim3(256), 0, s,
+                       (const float*)z, ldz, (const float*)coef, (T*)out, W,
+                       Kp, eps);
+}
+
+extern "C" hipError_t launch_poly_rows(int f32, const void* z, int ldz,
+                                       const void* coef, void* out, int M,
+                                       int W, int Kp, float eps,
+                                       hipStream_t s) {
+  if (M < 1 || W < 1 || Kp < W || ldz < W) return hipErrorInvalidValue;
+  if (f32) poly_rows<float>(z, ldz, coef, out, M, W, Kp, eps, s);
+  else poly_rows<u16>(z, ldz, coef, out, M, W, Kp, eps, s);
+  return hipGetLastError();
+}
+
 extern "C" hipError_t launch_cat_rows(int f32, const void* x, const void* x0,
                                       void* out, int M, int W, int Kp,
                                       hipStream_t s) {
@@ -441,8 +869,20 @@ static hipError_t lin_row(const LinRowArgs& a, hipStream_t s) {
   if (a.stage == ROW_CAT)
     return a.s.xadd && a.s.Kp >= 2 * a.s.W ? lin_row_go<T, ROW_CAT, 1>(a, s)
                                            : hipErrorInvalidValue;
+  if (a.stage == ROW_POLY) {
+    if (!a.s.x || !a.act || a.s.W < 1 || a.s.Kp < a.s.W)
+      return hipErrorInvalidValue;
+    return a.s.W <= 4096 ? lin_row_go<T, ROW_POLY, 8>(a, s)
+                         : lin_row_go<T, ROW_POLY, 20>(a, s);
+  }
+  if (a.stage == ROW_CONV) {
+    if (bad_conv(a.s) || a.s.xout == a.s.x || a.rows)
+      return hipErrorInvalidValue;
+    return a.s.W <= 2048 ? lin_row_go<T, ROW_CONV, 4>(a, s)
+                         : lin_row_go<T, ROW_CONV, 8>(a, s);
+  }
   // other blocks read x while block 0 writes xout
-  if (bad_stage(a.s) || !a.s.g || a.s.xout == a.s.x) return hipErrorInvalidValue;
+  if (a.stage != ROW_NORM || bad_stage(a.s) || !a.s.g || a.s.xout == a.s.x) return hipErrorInvalidValue;
   return a.s.W <= 2048 ? lin_row_go<T, ROW_NORM, 4>(a, s)
                        : lin_row_go<T, ROW_NORM, 8>(a, s);
 }
@@ -486,12 +926,20 @@ extern "C" hipError_t launch_gemm_rows(int f32, const void* X, const void* W,
                                        int N, int K, int ldx, int ldw,
                                        int ldy, int ldg, int epi, float mult,
                                        int Z, long xz, long wz, long yz,
+                                       int gz, int gc, const Rotary* rotary,
                                        hipStream_t s) {
   if (M < 1 || N < 1 || K < 64 || K % 64 || ldx < K || ldw < K || Z < 1 ||
-      epi < 0 || epi > EPI_RELU2)
+      epi < 0 || epi > EPI_ROTARY || (epi == EPI_TGATE && !gate))
     return hipErrorInvalidValue;
   GemmArgs a = {X, W, Y, (const float*)gate, (const float*)bias, M, N, K, ldx,
-                ldw, ldy, ldg, epi, mult, xz, wz, yz};
+                ldw, ldy, ldg, epi, gz, gc, mult, xz, wz, yz, {}};
+  if (epi == EPI_ROTARY) {
+    if (!rotary || rotary->split % 2 || rotary->RT < 2 || rotary->RT % 2 ||
+        rotary->dims % 2 || rotary->dims > rotary->RT || Z != 1 ||
+        (N - rotary->split) % rotary->RT)
+      return hipErrorInvalidValue;
+    a.r = *rotary;
+  }
   if (f32) gemm_go<float>(a, Z, s);
   else gemm_go<u16>(a, Z, s);
   return hipGetLastError();

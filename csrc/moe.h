@@ -4,7 +4,9 @@
 // A (token, choice) pair p = token*K1 + j uses expert idx[p] with weight
 // wt[p]; K1 = top (+1 when a shared expert exists: it is expert number E,
 // runs for every token with weight 1 and may have its own width and
-// limit).  Gate and up rows are interleaved in groups of 16 (16 gate rows,
+// limit).  Weights apply to the outputs, or (win) to the inputs of the
+// routed experts, which for the bias-free halves is a factor on their
+// products.  Gate and up rows are interleaved in groups of 16 (16 gate rows,
 // then the 16 up rows of the same hidden units), so one MFMA wave holds
 // both halves of the GLU.
 #pragma once
@@ -18,8 +20,13 @@ struct MoeArgs {
   const float* wt;          // [rows*K1]
   void* act;                // [rows*K1, ldact] T
   int ldh, ldact, W, E, K1, ff, ffs;   // ff, ffs padded to 64
+  int glu, win;             // 1: silu; 1: weights on the inputs
   float lim, lims;
 };
+
+// factor of pair p's gate/up products, and of its output
+DEVINL float pair_in(const MoeArgs& a, int p) { return a.win ? a.wt[p] : 1.f; }
+DEVINL float pair_out(const MoeArgs& a, int p) { return a.win ? 1.f : a.wt[p]; }
 
 DEVINL int gu_row(int f) { return (f >> 4) * 32 + (f & 15); }
 
@@ -34,12 +41,12 @@ DEVINL const T* moe_down_base(const MoeArgs& a, int e) {
 
 #define MOE_FPB 8   // hidden units of a block: 4 waves x 2
 
-// one block: pair p, hidden units [fb*8, fb*8+8)
+// one block: pair p of expert e, hidden units [fb*8, fb*8+8); the products
+// with the input come times wp
 template <typename T>
-DEVINL void expert_gu_block(const MoeArgs& a, int p, int fb) {
+DEVINL void expert_gu_block(const MoeArgs& a, int p, int e, float wp, int fb) {
   constexpr int V = El<T>::V;
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-  const int e = a.idx[p];
   const int ff = e == a.E ? a.ffs : a.ff;
   const int f0 = fb * MOE_FPB + wave * 2;
   if (f0 >= ff) return;
@@ -60,8 +67,14 @@ DEVINL void expert_gu_block(const MoeArgs& a, int p, int fb) {
     for (int i = 0; i < 4; i++) acc[i] = dot16<T>(ld16nt(w[i] + k), x, acc[i]);
   }
 #pragma unroll
-  for (int i = 0; i < 4; i++) acc[i] = wave_reduce_sum(acc[i]);
+  for (int i = 0; i < 4; i++) acc[i] = wave_reduce_sum(acc[i]) * wp;
   if (lane < 2)
-    ((T*)a.act)[(size_t)p * a.ldact + f0 + lane] = El<T>::st(
-        clamped_glu(lane ? acc[2] : acc[0], lane ? acc[3] : acc[1], lim));
+    ((T*)a.act)[(size_t)p * a.ldact + f0 + lane] = El<T>::st(glu_act(
+        a.glu, lane ? acc[2] : acc[0], lane ? acc[3] : acc[1], lim));
+}
+
+// the same for a pair that is routed already
+template <typename T>
+DEVINL void expert_gu_block(const MoeArgs& a, int p, int fb) {
+  expert_gu_block<T>(a, p, a.idx[p], pair_in(a, p), fb);
 }

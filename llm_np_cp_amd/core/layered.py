@@ -4,8 +4,7 @@ Where ``ModelConfig`` describes a stack of identical blocks, a layer-list
 ``config.json`` names every layer: its mixer, the mixer's sizes, its
 feed-forward, and optionally a range of layers that runs several times.
 Each mechanism is a small spec class that reads its own keys and knows its
-tensors; a further design registers further specs in ``MIXERS`` and its
-name in ``DESIGNS``.
+tensors; a further design lists its specs under its name in ``DESIGNS``.
 
 Turudra: parallel blocks (one norm feeds mixer and experts), latent
 attention and matrix-memory LSTM mixers, clamped routed experts with a
@@ -16,6 +15,12 @@ Garupel: sandwich blocks (a norm before and after each sublayer), grouped
 attention without rotation, gated linear recurrence and decaying linear
 attention mixers, dense feed-forwards, a looped range to which the
 embedding output is added ahead of every pass but the first.
+
+Fidizen: post-norm blocks (a norm on each sublayer's output only) whose
+sublayers read the residual through a short causal convolution, latent
+attention with a query latent, a sliding window and a sink, polynomial
+dense feed-forwards or sigmoid-routed experts, layers that use another
+layer's tensors.
 """
 
 from __future__ import annotations
@@ -43,6 +48,11 @@ def _positive(where: str, **kw):
 class LatentAttentionSpec:
     libs = ("latent",)
     recurrent = False
+    inputs = ("q", "dkv", "g")   # matrices that read the mixer's input
+    interleaved = False          # rotation pairs (i, i + dims/2)
+    gate = "head"                # the output gate is one number per head
+    q_rank = window = None       # no query latent, every earlier key
+    sink = False
     heads: int
     dim: int
     rot_dim: int
@@ -88,6 +98,41 @@ class LatentAttentionSpec:
 
 
 @dataclass
+class WindowedLatentSpec(LatentAttentionSpec):
+    """Latent attention whose queries go through a latent of their own
+    (q_rank), over the last `window` tokens, with a sink per head in the
+    softmax, interleaved rotation and an output gate per element."""
+    inputs = ("dq", "dkv", "g")
+    interleaved = True
+    gate = "element"
+    sink = True
+    q_rank: int = 0
+    window: int = 0
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str):
+        s = super().from_dict(m, where)
+        s.q_rank = _get(m, "q_rank", where)
+        s.window = _get(_get(m, "mask", where), "size", where + ".mask")
+        _positive(where, q_rank=s.q_rank)
+        _positive(where + ".mask", size=s.window)
+        return s
+
+    def to_dict(self) -> dict:
+        return {**super().to_dict(), "q_rank": self.q_rank,
+                "mask": {"size": self.window}}
+
+    def shapes(self, p: str, width: int) -> Shapes:
+        out = super().shapes(p, width)
+        H, Q = self.heads, self.q_rank
+        out.pop(p + "q")
+        out.update({p + "dq": (Q, width), p + "dq.norm": (Q,),
+                    p + "uq": (H * (self.dim + self.rot_dim), Q),
+                    p + "sink": (H,), p + "g": (H * self.vdim, width)})
+        return out
+
+
+@dataclass
 class MLSTMSpec:
     libs = ("mlstm",)
     recurrent = True
@@ -120,14 +165,18 @@ class MLSTMSpec:
 
 @dataclass
 class ExpertSpec:
+    """W_down (act(W_gate h, W_up h)), act = silu(gate) up."""
     ff: int
-    limit: float
+    limit = 0.0
 
     @classmethod
     def from_dict(cls, m: dict, where: str):
-        s = cls(ff=_get(m, "ff", where), limit=float(_get(m, "limit", where)))
+        s = cls(ff=_get(m, "ff", where))
         _positive(where, ff=s.ff)
         return s
+
+    def to_dict(self) -> dict:
+        return {"ff": self.ff}
 
     def shapes(self, p: str, width: int) -> Shapes:
         return {p + "gate": (self.ff, width), p + "up": (self.ff, width),
@@ -135,13 +184,34 @@ class ExpertSpec:
 
 
 @dataclass
+class ClampedExpertSpec(ExpertSpec):
+    """The GLU clamps both halves at `limit`."""
+    limit: float = 0.0
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str):
+        s = super().from_dict(m, where)
+        s.limit = float(_get(m, "limit", where))
+        return s
+
+    def to_dict(self) -> dict:
+        return {"ff": self.ff, "limit": self.limit}
+
+
+@dataclass
 class MoESpec:
+    """Routed experts and an optional shared one.  The chosen experts'
+    weights are the softmax over their logits, applied to the outputs."""
     experts: int
     top: int
     expert: ExpertSpec
     shared: Optional[ExpertSpec] = None
     kind = "moe"
     libs = ("moe",)
+    expert_class = ClampedExpertSpec
+    glu = "clamped"
+    score = "softmax"
+    weigh = "output"
 
     @classmethod
     def from_dict(cls, m: dict, where: str):
@@ -149,9 +219,9 @@ class MoESpec:
         sh = m.get("shared")
         s = cls(experts=_get(r, "experts", where + ".router"),
                 top=_get(r, "top", where + ".router"),
-                expert=ExpertSpec.from_dict(_get(m, "expert", where),
-                                            where + ".expert"),
-                shared=(ExpertSpec.from_dict(sh, where + ".shared")
+                expert=cls.expert_class.from_dict(
+                    _get(m, "expert", where), where + ".expert"),
+                shared=(cls.expert_class.from_dict(sh, where + ".shared")
                         if sh else None))
         _positive(where + ".router", experts=s.experts, top=s.top)
         if s.top > s.experts or s.experts > 1024:
@@ -161,11 +231,10 @@ class MoESpec:
         return s
 
     def to_dict(self) -> dict:
-        ex = lambda e: {"ff": e.ff, "limit": e.limit}
         return {"kind": self.kind,
                 "router": {"experts": self.experts, "top": self.top},
-                "expert": ex(self.expert),
-                "shared": ex(self.shared) if self.shared else None}
+                "expert": self.expert.to_dict(),
+                "shared": self.shared.to_dict() if self.shared else None}
 
     def shapes(self, p: str, width: int) -> Shapes:
         out = {p + "router": (self.experts, width)}
@@ -174,6 +243,16 @@ class MoESpec:
         if self.shared:
             out.update(self.shared.shapes(p + "shared.", width))
         return out
+
+
+@dataclass
+class SigmoidMoESpec(MoESpec):
+    """Every expert has a score sigmoid(logit); the scores of the chosen
+    ones, as they are, weigh the experts' inputs."""
+    expert_class = ExpertSpec
+    glu = "silu"
+    score = "sigmoid"
+    weigh = "input"
 
 
 @dataclass
@@ -300,6 +379,7 @@ class DenseSpec:
     ff: int
     kind = "dense"
     libs = ()
+    act = "relu2"
 
     @classmethod
     def from_dict(cls, m: dict, where: str):
@@ -314,28 +394,47 @@ class DenseSpec:
         return {p + "up": (self.ff, width), p + "down": (width, self.ff)}
 
 
+@dataclass
+class PolyDenseSpec(DenseSpec):
+    """act(z) = a N(z) + b N(z^2) + c N(z^3) + e with learned a, b, c, e;
+    N divides a token's vector by its root mean square."""
+    act = "polynorm"
+
+    def shapes(self, p: str, width: int) -> Shapes:
+        return {**super().shapes(p, width), p + "act": (4,)}
+
+
 @dataclass(frozen=True)
 class Design:
     """What a design fixes about its layers.  ``parallel``: one norm feeds
     mixer and feed-forward; ``sandwich``: each has a norm before and after
-    it.  ``project``: W_in [x; x0] ahead of every pass of the loop; ``add``:
-    x + x0 ahead of every pass but the first."""
+    it; ``post``: each has a norm after it and a short convolution over
+    time ahead of it.  ``project``: W_in [x; x0] ahead of every pass of the
+    loop; ``add``: x + x0 ahead of every pass but the first.  ``share``: a
+    layer may use another one's tensors."""
     model_type: str
     block: str
-    loop: str
-    mixers: Tuple[str, ...]
-    mlps: Tuple[str, ...]
+    loop: Optional[str]
+    mixers: Tuple[type, ...]
+    mlps: Tuple[type, ...]
+    share: bool = False
+
+    def mixer(self, kind):
+        return next((c for c in self.mixers if c.kind == kind), None)
+
+    def mlp(self, kind):
+        return next((c for c in self.mlps if c.kind == kind), None)
 
 
-MIXERS = {c.kind: c for c in (LatentAttentionSpec, MLSTMSpec, AttentionSpec,
-                              RGLRUSpec, LightningSpec)}
-MLPS = {c.kind: c for c in (MoESpec, DenseSpec)}
 # config "architecture" -> design
 DESIGNS = {
     "Turudra": Design("turudra", "parallel", "project",
-                      ("latent_attention", "mlstm"), ("moe",)),
+                      (LatentAttentionSpec, MLSTMSpec), (MoESpec,)),
     "Garupel": Design("garupel", "sandwich", "add",
-                      ("attention", "rglru", "lightning"), ("dense",)),
+                      (AttentionSpec, RGLRUSpec, LightningSpec),
+                      (DenseSpec,)),
+    "Fidizen": Design("fidizen", "post", None, (WindowedLatentSpec,),
+                      (PolyDenseSpec, SigmoidMoESpec), share=True),
 }
 
 
@@ -343,6 +442,7 @@ DESIGNS = {
 class LayerSpec:
     mixer: object
     mlp: Optional[object]
+    weights_of: Optional[int] = None   # the layer whose tensors it uses
 
 
 @dataclass
@@ -363,16 +463,17 @@ class LayeredConfig:
     embed_scale: float = 1.0
     residual_mult: float = 1.0
     logit_softcap: Optional[float] = None
+    conv_taps: int = 1            # of the sublayers' input convolutions
     max_position_embeddings: int = 131072
     bos_token_id: Optional[int] = None
     eos_token_id: Optional[int] = None
-    # (layer, the embedding output comes in ahead of it)
+    # (layer whose tensors run, the embedding output comes in ahead of it)
     runs: List[Tuple[int, bool]] = field(default_factory=list)
 
     def __post_init__(self):
         n, lp = len(self.layers), self.loop
         if lp is None:
-            self.runs = [(i, False) for i in range(n)]
+            self.runs = [(self._owner(i), False) for i in range(n)]
             return
         if not (0 <= lp.start < lp.stop <= n and lp.times >= 1):
             raise ValueError(f"config.json: loop {lp} does not fit "
@@ -383,6 +484,23 @@ class LayeredConfig:
             self.runs += [(i, i == lp.start and k >= first)
                           for i in range(lp.start, lp.stop)]
         self.runs += [(i, False) for i in range(lp.stop, n)]
+
+    def _owner(self, i: int) -> int:
+        """The layer whose tensors layer i uses."""
+        seen = [i]
+        while self.layers[i].weights_of is not None:
+            j = self.layers[i].weights_of
+            if (isinstance(j, bool) or not isinstance(j, int) or
+                    not 0 <= j < len(self.layers) or j in seen):
+                raise ValueError(f"config.json: layers[{i}].weights_of {j!r} "
+                                 f"is not possible")
+            a, b = self.layers[seen[0]], self.layers[j]
+            if (a.mixer, a.mlp) != (b.mixer, b.mlp):
+                raise ValueError(f"config.json: layers[{seen[0]}] differs "
+                                 f"from layers[{j}], whose tensors it uses")
+            seen.append(j)
+            i = j
+        return i
 
     @property
     def architecture(self) -> str:
@@ -419,7 +537,8 @@ class LayeredConfig:
 
     @property
     def recurrent(self) -> bool:
-        return any(l.mixer.recurrent for l in self.layers)
+        return self.conv_taps > 1 or any(l.mixer.recurrent
+                                         for l in self.layers)
 
     @classmethod
     def matches(cls, d: dict) -> bool:
@@ -435,17 +554,28 @@ class LayeredConfig:
         for i, l in enumerate(_get(d, "layers", "top level")):
             w = f"layers[{i}]"
             kind = _get(l, "type", w)
-            if kind not in design.mixers:
+            if design.mixer(kind) is None:
                 raise ValueError(f"config.json: {w}: unknown mixer {kind!r}")
             mlp = l.get("mlp")
-            if mlp is not None and mlp.get("kind") not in design.mlps:
+            if mlp is not None and design.mlp(mlp.get("kind")) is None:
                 raise ValueError(f"config.json: {w}: unknown feed-forward "
                                  f"{mlp.get('kind')!r}")
+            share = l.get("weights_of")
+            if share is not None and not design.share:
+                raise ValueError(f"config.json: {w}: {arch} does not share "
+                                 f"tensors between layers")
             layers.append(LayerSpec(
-                MIXERS[kind].from_dict(_get(l, "mixer", w), w + ".mixer"),
-                MLPS[mlp["kind"]].from_dict(mlp, w + ".mlp") if mlp
-                else None))
+                design.mixer(kind).from_dict(_get(l, "mixer", w),
+                                             w + ".mixer"),
+                design.mlp(mlp["kind"]).from_dict(mlp, w + ".mlp") if mlp
+                else None, share))
         lp = d.get("loop")
+        if lp and not design.loop:
+            raise ValueError(f"config.json: {arch} has no loop")
+        taps = 1
+        if design.block == "post":
+            taps = _get(_get(d, "canon", "top level"), "taps", "canon")
+            _positive("canon", taps=taps)
         width, vocab = _get(d, "width", "top level"), _get(d, "vocab",
                                                            "top level")
         _positive("top level", width=width, vocab=vocab)
@@ -459,6 +589,7 @@ class LayeredConfig:
             embed_scale=float(d.get("embedding", {}).get("scale", 1.0)),
             residual_mult=float(d.get("residual_mult", 1.0)),
             logit_softcap=float(cap) if cap else None,
+            conv_taps=taps,
             max_position_embeddings=d.get("max_position_embeddings", 131072),
             bos_token_id=d.get("bos_token_id"),
             eos_token_id=d.get("eos_token_id"))
@@ -468,8 +599,15 @@ class LayeredConfig:
              "width": self.hidden_size, "norm": {"eps": self.norm_eps},
              "layers": [{"type": l.mixer.kind, "mixer": l.mixer.to_dict(),
                          "mlp": l.mlp.to_dict() if l.mlp else None}
-                        for l in self.layers],
-             "loop": None}
+                        for l in self.layers]}
+        for entry, l in zip(d["layers"], self.layers):
+            if l.weights_of is not None:
+                entry["weights_of"] = l.weights_of
+        if self.design.loop:
+            d["loop"] = None
+        if self.design.block == "post":
+            d.update({"embedding": {"scale": self.embed_scale},
+                      "canon": {"taps": self.conv_taps}})
         if self.design.block == "parallel":
             d.update({"embedding": {"scale": self.embed_scale},
                       "residual_mult": self.residual_mult,
@@ -491,8 +629,16 @@ class LayeredConfig:
         if self.loop and self.design.loop == "project":
             out["loop.in"] = (W, 2 * W)
         sandwich = self.design.block == "sandwich"
+        post = self.design.block == "post"
         for i, l in enumerate(self.layers):
+            if l.weights_of is not None:
+                continue
             out[f"l{i}.norm1"] = (W,)
+            if post:
+                out[f"l{i}.canon1"] = (W, self.conv_taps)
+                if l.mlp:
+                    out[f"l{i}.norm2"] = (W,)
+                    out[f"l{i}.canon2"] = (W, self.conv_taps)
             if sandwich:
                 out[f"l{i}.norm1b"] = (W,)
             out.update(l.mixer.shapes(f"l{i}.mix.", W))
@@ -569,7 +715,47 @@ def _recurrent_stack(n, width, heads) -> list:
     return [kinds[i % 4] for i in range(n)]
 
 
+def _fidizen(vocab, width, layers, taps=4, scale=1.0) -> dict:
+    return {"architecture": "Fidizen", "vocab": vocab, "width": width,
+            "norm": {"eps": 1e-6}, "embedding": {"scale": scale},
+            "canon": {"taps": taps}, "layers": layers}
+
+
+def _windowed(mlp, heads, dim, rot, vdim, rank, q_rank, window,
+              of=None) -> dict:
+    mix = {**_latent(heads, dim, rot, vdim, rank), "q_rank": q_rank,
+           "mask": {"size": window}}
+    d = {"type": "latent_attention", "mixer": mix, "mlp": mlp}
+    return d if of is None else {**d, "weights_of": of}
+
+
+def _poly(ff) -> dict:
+    return {"kind": "dense", "ff": ff}
+
+
+def _sigmoid_moe(experts, top, ff, shared) -> dict:
+    return {"kind": "moe", "router": {"experts": experts, "top": top},
+            "expert": {"ff": ff}, "shared": {"ff": shared} if shared else None}
+
+
+def _windowed_stack(n, heads, ff) -> list:
+    """Dense and routed layers in turn; two matrices of a dense one are as
+    large as the three of the experts that a token uses."""
+    mlps = [_poly(9 * ff // 2), _sigmoid_moe(8, 2, ff, ff)]
+    return [_windowed(mlps[i % 2], heads, 128, 64, 128, 512, 1024, 1024)
+            for i in range(n)]
+
+
 LAYERED_PRESETS = {
+    "tiny-fidizen": _fidizen(
+        352, 72,
+        [_windowed(_poly(104), 5, 20, 12, 28, 44, 36, 70),
+         _windowed(_sigmoid_moe(6, 2, 40, 24), 3, 28, 16, 20, 60, 52, 33),
+         _windowed(_poly(104), 5, 20, 12, 28, 44, 36, 70, of=0)],
+        taps=4, scale=2.0),
+    "fidizen-2k": _fidizen(32000, 2048, _windowed_stack(8, 16, 2048)),
+    "fidizen-4k": _fidizen(32000, 4096, _windowed_stack(4, 32, 4096)),
+
     "tiny-garupel": _garupel(
         320, 80,
         [_grouped(6, 3, 20, 28),

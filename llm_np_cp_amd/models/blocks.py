@@ -9,13 +9,19 @@ norm and addition are still pending (eng.pend).
 from __future__ import annotations
 
 from ..ops import hybrid_ops as hy
-from .mixers import MIXERS, DenseFF, Packer, RoutedExperts
-
-FEW = 16            # single tokens that take the fused few-row kernels
-FUSE = 5            # of them, those whose experts run as fused GEMVs
+from .mixers import (FEED_FORWARDS, FEW, FUSE, MIXERS, DenseFF, InputConv,
+                     Packer, RoutedExperts)
 
 
-class ParallelBlock:
+class Block:
+    experts = None
+
+    def new_cache(self, eng):
+        """The cache or state of one run of the layer."""
+        return self.mixer.new_cache(eng)
+
+
+class ParallelBlock(Block):
     """x += m (mixer(h) + experts(h)), h the norm of x; the router's rows
     ride along in the input projection."""
 
@@ -29,7 +35,7 @@ class ParallelBlock:
             names.append(p + "mlp.router")
             self.experts = RoutedExperts(eng, spec.mlp, pk, p + "mlp.")
         self.win = pk.rows(names, eng.W)
-        self.ldp = self.win.shape[0]
+        self.ldp = self.p_floats = self.win.shape[0]
         self.act_floats = (self.experts.K1 * self.experts.ffm
                            if self.experts else 0)
         self.g = pk.f32(p + "norm1")
@@ -53,13 +59,12 @@ class ParallelBlock:
             hy.gemm_rows(eng.o, m.wo, eng.x, T, m.ldo, eng.W, hy.EPI_RESADD,
                          mult=mult)
             if ex:
-                ex.many(eng, T)
+                ex.many(eng, T, eng.x, mult)
 
 
-class SandwichBlock:
+class SandwichBlock(Block):
     """x += norm1b(mixer(norm1(x))), x += norm2b(ff(norm2(x))).  Each post
     norm and addition happens in the staging of the projection after it."""
-    experts = None
 
     def __init__(self, eng, spec, pk: Packer, i: int):
         p = f"l{i}."
@@ -67,7 +72,7 @@ class SandwichBlock:
                                                  p + "mix.")
         self.win = pk.rows([p + "mix." + n for n in m.IN], eng.W)
         self.bias = m.biases(eng, pk, p + "mix.")
-        self.ldp = self.win.shape[0]
+        self.ldp = self.p_floats = self.win.shape[0]
         self.g1, self.g1b = pk.f32(p + "norm1"), pk.f32(p + "norm1b")
         self.ff = None
         self.act_floats = 0
@@ -89,4 +94,42 @@ class SandwichBlock:
             eng.pend = self.g2b
 
 
-BLOCKS = {"parallel": ParallelBlock, "sandwich": SandwichBlock}
+class PostNormBlock(Block):
+    """x += norm1(mixer(c1(x))), x += norm2(ff(c2(x))), c a short causal
+    convolution over time added to its input.  Norm and addition happen in
+    the staging of the projection after them, together with its
+    convolution."""
+
+    def __init__(self, eng, spec, pk: Packer, i: int):
+        p = f"l{i}."
+        self.mixer = m = MIXERS[spec.mixer.kind](eng, spec.mixer, pk,
+                                                 p + "mix.")
+        self.win = pk.rows([p + "mix." + n for n in m.IN], eng.W)
+        self.ldp = self.p_floats = self.win.shape[0]
+        self.orouter = self.act_floats = 0
+        self.c1, self.g1 = InputConv(pk, p + "canon1"), pk.f32(p + "norm1")
+        self.ff = None
+        if spec.mlp:
+            self.ff = FEED_FORWARDS[spec.mlp.kind](eng, spec.mlp, pk,
+                                                   p + "mlp.")
+            self.c2, self.g2 = InputConv(pk, p + "canon2"), pk.f32(p + "norm2")
+            self.act_floats = self.ff.act_floats
+            self.p_floats = max(self.ldp, self.ff.p_floats)
+
+    def new_cache(self, eng):
+        convs = [self.c1, self.c2] if self.ff else [self.c1]
+        return (self.mixer.new_cache(eng), *(c.new_ring(eng) for c in convs))
+
+    def run(self, eng, b, cache):
+        eng.conv_project(self.win, self.c1.w, cache[1], b, eng.P)
+        self.mixer.run(eng, b, cache[0], self)
+        self.mixer.out(eng, b, self)
+        eng.pend = self.g1
+        if self.ff:
+            eng.conv_project(self.ff.up, self.c2.w, cache[2], b, eng.P)
+            self.ff.after_up(eng, b)
+            eng.pend = self.g2
+
+
+BLOCKS = {"parallel": ParallelBlock, "sandwich": SandwichBlock,
+          "post": PostNormBlock}

@@ -26,9 +26,9 @@ from ..ops import hybrid_ops as hy
 from ..parallel import tp as tpu
 from ..runtime.cache_manager import CacheFull, CacheManager, Sequence
 from ..utils.tracing import trace_range
-from .blocks import BLOCKS, FEW
+from .blocks import BLOCKS
 from .decode_loop import DecodeLoop, DeviceCacheHandle
-from .mixers import Packer, pad_to
+from .mixers import FEW, Packer, pad_to
 
 
 @dataclass
@@ -140,11 +140,11 @@ class LayeredModel(DecodeLoop):
                          if cfg.loop and cfg.design.loop == "project"
                          else None)
         block = BLOCKS[cfg.design.block]
-        self.layers = [block(self, s, pk, i)
-                       for i, s in enumerate(cfg.layers)]
-        # every run of a looped layer has its own cache or state
-        self.caches = [self.layers[i].mixer.new_cache(self)
-                       for i, _ in cfg.runs]
+        # layers that use another one's tensors have none of their own
+        self.layers = {i: block(self, cfg.layers[i], pk, i)
+                       for i in sorted({i for i, _ in cfg.runs})}
+        # every run of a looped or shared layer has its own cache or state
+        self.caches = [self.layers[i].new_cache(self) for i, _ in cfg.runs]
 
     def decode_splits(self, rows: int) -> int:
         """Key-range splits of single-token attention: fixed by the cache
@@ -176,23 +176,25 @@ class LayeredModel(DecodeLoop):
         self.cat = (torch.zeros(PC, self.win_loop.shape[1], **tt)
                     if self.win_loop is not None else None)
         self.y = (torch.zeros(PC, self.W, **f32)
-                  if cfg.design.block == "sandwich" else None)
+                  if cfg.design.block != "parallel" else None)
         self.pend, self.add0 = None, False
-        self.P = torch.zeros(PC * max(l.ldp for l in self.layers), **f32)
+        layers = self.layers.values()
+        self.P = torch.zeros(PC * max(l.p_floats for l in layers), **f32)
         need: Dict[str, int] = {}
-        for l in self.layers:
+        for l in layers:
             for k, n in l.mixer.sizes(self, PC).items():
                 need[k] = max(need.get(k, 0), n)
         for k in ("q", "qn", "qa", "olat", "o", "part", "ml", "raw", "gF",
-                  "gi", "gm", "cm0", "U", "un", "decay", "local"):
-            kw = tt if k in ("q", "qn", "qa", "olat", "o") else f32
+                  "gi", "gm", "cm0", "U", "un", "decay", "local", "cq", "qf"):
+            kw = tt if k in ("q", "qn", "qa", "olat", "o", "cq") else f32
             setattr(self, k, torch.zeros(max(need.get(k, 0), 1), **kw))
-        ex = [l.experts for l in self.layers if l.experts]
+        ex = [l.experts or l.ff.experts for l in layers
+              if l.experts or getattr(l, "ff", None) and l.ff.experts]
         K1 = max((e.K1 for e in ex), default=1)
         self.ridx = torch.zeros(PC * K1, **i32)
         self.rwt = torch.zeros(PC * K1, **f32)
         self.act = torch.zeros(
-            max(1, PC * max(l.act_floats for l in self.layers)), **tt)
+            max(1, PC * max(l.act_floats for l in layers)), **tt)
         self.ypair = torch.zeros(PC * K1 * self.W if ex else 1, **tt)
         self.perm = torch.zeros(PC * K1, **i32)
         nt = PC * K1 // 32 + max((e.spec.experts + 1 for e in ex), default=1)
@@ -221,7 +223,7 @@ class LayeredModel(DecodeLoop):
         self.nout, self.out_ring = self.bt_nout[:1], self.bt_ring[0]
         self.s_gmax, self.s_pick = self.bt_gmax[:1], self.bt_pick[:1]
         self.s_cnt = self.bt_cnt[:1]
-        heads = {l.mixer.tile_pairs for l in self.layers} - {None}
+        heads = {l.mixer.tile_pairs for l in layers} - {None}
         self._tile_pairs = sorted(heads)
         self._meta = torch.zeros(
             3 * PC + 8 * (B + 2) + 3 * (PC // hy.CHUNK + B + 2) + PC +
@@ -271,7 +273,7 @@ class LayeredModel(DecodeLoop):
             hy.norm_rows(self.x, None, None, T, self.W, self.W,
                          self.cfg.norm_eps, xout=self.x, **kw)
 
-    def _one_row(self, w, T: int) -> bool:
+    def one_row(self, w, T: int) -> bool:
         return T == 1 and w.shape[1] * w.element_size() <= 1 << 17
 
     def project(self, w, staged, out, T: int, g=None, rows=None, cap=None,
@@ -282,7 +284,7 @@ class LayeredModel(DecodeLoop):
         (N, K), W, eps = w.shape, self.W, self.cfg.norm_eps
         kw = self._pending()
         keep = bool(kw) and rows is None
-        if self._one_row(w, T):
+        if self.one_row(w, T):
             if keep:           # other blocks still read x: write beside it
                 kw["xout"] = self.xb
             res = {"res": kw.pop("y")} if "y" in kw else {}
@@ -306,7 +308,7 @@ class LayeredModel(DecodeLoop):
     def linear(self, w, src, out, T: int):
         """out[T, N] fp32 = w . src, rows of src as wide as w's."""
         N, K = w.shape
-        if self._one_row(w, T):
+        if self.one_row(w, T):
             hy.lin_row(w, None, out, 0, 0.0, hin=src)
         else:
             hy.gemm_rows(src, w, out, T, K, N, hy.EPI_F32)
@@ -315,10 +317,38 @@ class LayeredModel(DecodeLoop):
                       ldg: int):
         """out[T, N] fp32 = w . (norm(src) sigmoid(gate)), src [T, W]."""
         (N, K), eps = w.shape, self.cfg.norm_eps
-        if self._one_row(w, T):
+        if self.one_row(w, T):
             hy.lin_row(w, src, out, W, eps, g=g, gate=gate, ldg=ldg)
         else:
             hy.norm_rows(src, g, staged, T, W, K, eps, gate=gate, ldg=ldg)
+            hy.gemm_rows(staged, w, out, T, K, N, hy.EPI_F32)
+
+    def conv_project(self, w, kernel, ring, b: Rows, out):
+        """out[T, N] fp32 = w . (v + conv(v)), v the residual with what is
+        pending on it; the staged input stays in self.h."""
+        (N, K), W, eps, T = w.shape, self.W, self.cfg.norm_eps, b.T
+        kw = self._pending()
+        keep = bool(kw)
+        if keep:               # earlier rows are read again: write beside
+            kw["xout"] = self.xb
+        conv = (kernel, ring, b.slot, b.pos)
+        if self.one_row(w, T):
+            res = {"res": kw.pop("y")} if keep else {}
+            hy.lin_row(w, self.x, out, W, eps, hout=self.h, conv=conv, **res,
+                       **kw)
+        else:
+            hy.conv_rows(self.x, self.h, b, W, K, eps, conv, **kw)
+            hy.gemm_rows(self.h, w, out, T, K, N, hy.EPI_F32)
+        if keep:
+            self.x, self.xb = self.xb, self.x
+
+    def poly_linear(self, w, z, W: int, coef, staged, out, T: int):
+        """out[T, N] fp32 = w . polynorm(z), rows of W values in z."""
+        (N, K), eps = w.shape, self.cfg.norm_eps
+        if self.one_row(w, T):
+            hy.lin_row(w, z, out, W, eps, act=coef)
+        else:
+            hy.poly_rows(z, K, coef, staged, T, W, eps)
             hy.gemm_rows(staged, w, out, T, K, N, hy.EPI_F32)
 
     def _head(self, out: torch.Tensor, n: int, rows=None):

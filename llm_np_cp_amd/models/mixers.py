@@ -10,9 +10,9 @@ Every mechanism has two sequences over the same cache and state:
 
 A batch lists its single-token rows first.  Both leave the mixer's output
 (before the output projection) in eng.o and, in a parallel block, the
-expert choice in eng.ridx / eng.rwt.  Mixers of sandwich blocks have one
-sequence (the single-token kernels are the fused ones) and apply their
-output projection themselves, in out().
+expert choice in eng.ridx / eng.rwt.  Mixers of sandwich and post blocks
+have run(), which picks the sequence, and apply their output projection
+themselves, in out().
 """
 
 from __future__ import annotations
@@ -23,6 +23,8 @@ import torch
 from ..ops import hybrid_ops as hy
 
 PART_FLOATS = 1 << 25     # split-attention scratch for prompt portions
+FEW = 16            # single tokens that take the fused few-row kernels
+FUSE = 5            # of them, those whose experts run as fused GEMVs
 
 
 def pad_to(n: int, m: int) -> int:
@@ -54,9 +56,10 @@ class Packer:
 
 
 class RoutedExperts:
-    """Clamped-GLU experts and their shared one (see csrc/moe.h for the
-    weight layout); routing logits are columns of the block's input
-    projection, so the router costs no launch of its own."""
+    """Routed experts and their shared one (see csrc/moe.h for the weight
+    layout).  Routing logits are columns of a parallel block's input
+    projection, so the router costs no launch of its own there; elsewhere
+    they are a projection by themselves."""
 
     def __init__(self, eng, spec, pk: Packer, p: str):
         W, Wp = eng.W, eng.Wp
@@ -86,13 +89,34 @@ class RoutedExperts:
             fill(p + "shared.", E, sh.ff, ffs)
         self.args = hy.MoeArgs().put(
             gu=self.gu, down=self.down, ldh=Wp, ldact=self.ffm, W=W, E=E,
-            K1=self.K1, ff=ff, ffs=ffs, lim=spec.expert.limit,
+            K1=self.K1, ff=ff, ffs=ffs, glu=int(spec.glu == "silu"),
+            win=int(spec.weigh == "input"), lim=spec.expert.limit,
             lims=sh.limit if sh else 0.0)
 
     def bind(self, eng):
         return self.args.put(h=eng.h, idx=eng.ridx, wt=eng.rwt, act=eng.act)
 
-    def many(self, eng, T: int):
+    def route(self, eng, T: int):
+        """Routing of the logits in eng.P."""
+        E = self.spec.experts
+        return hy.RouteArgs().put(
+            z=eng.P, idx=eng.ridx, wt=eng.rwt, ldz=E, rows=T, E=E,
+            top=self.top, extra=self.extra,
+            scores=int(self.spec.score == "sigmoid"))
+
+    def apart(self, eng, T: int, few: bool):
+        """eng.y = the experts' sum for the rows of eng.h, from the logits
+        in eng.P."""
+        m, route = self.bind(eng), self.route(eng, T)
+        if few and T <= FUSE:
+            hy.moe_gu_few(eng.f32, m, route)
+            hy.block_out(eng.f32, None, None, 0, m, self.K1, eng.y, T, eng.W,
+                         1.0, set=True)
+        else:
+            hy.moe_route(m, route)
+            self.many(eng, T, eng.y, 1.0, True)
+
+    def many(self, eng, T: int, out, mult: float, set: bool = False):
         avg = T * self.top / self.spec.experts
         bm = 128 if avg >= 160 else 64 if avg >= 24 else 32
         pairs, groups = T * self.K1, self.spec.experts + self.extra
@@ -101,13 +125,11 @@ class RoutedExperts:
             tile_n=eng.tile_n, pairs=pairs, groups=groups, bm=bm,
             maxtiles=pairs // bm + groups)
         assert s.maxtiles <= eng.tile_e.numel()
-        hy.moe_rows(eng.f32, self.bind(eng), s, eng.ypair, eng.x, T,
-                    eng.cfg.residual_mult)
+        hy.moe_rows(eng.f32, self.bind(eng), s, eng.ypair, out, T, mult, set)
 
 
 class LatentAttention:
     kind = "latent_attention"
-    IN = ("q", "dkv", "g")           # rows of the input projection
 
     def __init__(self, eng, spec, pk: Packer, p: str):
         self.spec = s = spec
@@ -117,6 +139,7 @@ class LatentAttention:
                 f"latent attention: kv_rank {s.kv_rank} / rot_dim "
                 f"{s.rot_dim} exceed the built kernels "
                 f"({hy.RANKS[-1]} / 128)")
+        self.IN = s.inputs                 # rows of the input projection
         self.RP, self.RT = fit[0], pad_to(s.rot_dim, 32)
         self.tile_pairs = s.heads          # pairs a token adds to a tile
         self.CS, self.dp = self.RP + self.RT, pad_to(s.dim, 64)
@@ -134,17 +157,49 @@ class LatentAttention:
         self.wo = pk.rows([p + "o"], H * vd)
         self.cnorm = pk.f32(p + "dkv.norm")
         self.cosT, self.sinT = eng.rope_tables(s.rot_base, s.rot_dims)
-        nq = H * (d + s.rot_dim)
+        nq = s.q_rank or H * (d + s.rot_dim)
+        self.og = nq + s.kv_rank + s.rot_dim
+        each = s.gate == "element"
         self.args = hy.LatentArgs().put(
             Wuk=self.wuk, Wuv=self.wuv, cnorm=self.cnorm, cosT=self.cosT,
-            sinT=self.sinT, oq=0, odkv=nq, og=nq + s.kv_rank + s.rot_dim,
-            H=H, d=d, dp=self.dp, rot=s.rot_dim, rdims=s.rot_dims,
-            RT=self.RT, rank=s.kv_rank, RP=RP, vd=vd, ldo=self.ldo,
-            eps=eng.cfg.norm_eps, scale=s.scale)
+            sinT=self.sinT, oq=0, odkv=nq, og=self.og, H=H, d=d, dp=self.dp,
+            rot=s.rot_dim, rdims=s.rot_dims, RT=self.RT, rank=s.kv_rank,
+            RP=RP, vd=vd, ldo=self.ldo, qh=d + s.rot_dim, oqr=d,
+            qrh=d + s.rot_dim, pairs=int(s.interleaved), win=s.window or 0,
+            gz=vd if each else 1, gc=int(each), eps=eng.cfg.norm_eps,
+            scale=s.scale)
+        if s.sink:
+            self.sink = pk.f32(p + "sink")
+            self.args.put(sink=self.sink)
+        if s.q_rank:
+            self._query_latent(pk, p)
+
+    def _query_latent(self, pk: Packer, p: str):
+        """W_uq with the unrotated parts of all heads first, each padded to
+        dp rows, then the rotated ones, each padded to RT."""
+        s, H, dp, RT = self.spec, self.spec.heads, self.dp, self.RT
+        uq = pk.rows([p + "uq"], s.q_rank)
+        self.QRp = uq.shape[1]
+        uq = uq.view(H, s.dim + s.rot_dim, self.QRp)
+        self.wuq = torch.zeros(H * (dp + RT), self.QRp, dtype=pk.dtype,
+                               device=pk.device)
+        flat, rot = self.wuq[:H * dp], self.wuq[H * dp:]
+        flat.view(H, dp, -1)[:, :s.dim].copy_(uq[:, :s.dim])
+        rot.view(H, RT, -1)[:, :s.rot_dim].copy_(uq[:, s.dim:])
+        self.qnorm = pk.f32(p + "dq.norm")
+        self.args.put(qnorm=self.qnorm, qrank=s.q_rank, QRp=self.QRp,
+                      ldq=H * (dp + RT), qh=dp, oqr=H * dp, qrh=RT)
 
     def new_cache(self, eng):
         return torch.zeros(eng.cache.num_pages, hy.PAGE, self.CS,
                            dtype=eng.T, device=eng.device)
+
+    def token_splits(self, eng, rows: int) -> int:
+        """Key splits of single tokens, at most one per key tile of the
+        window."""
+        n = eng.decode_splits(rows)
+        return max(2, min(n, self.spec.window // 32 + 1)) \
+            if self.spec.window else n
 
     def sizes(self, eng, rows):
         """Scratch elements for `rows` rows, and fp32 partials."""
@@ -152,29 +207,50 @@ class LatentAttention:
         splits = max(PART_FLOATS // (H * self.RP),
                      *(r * eng.decode_splits(r)
                        for r in range(1, eng.max_batch + 1)), 1)
-        return dict(qn=rows * H * self.dp, qa=rows * H * self.CS,
+        need = dict(qn=rows * H * self.dp, qa=rows * H * self.CS,
                     olat=rows * H * self.RP, o=rows * self.ldo,
                     part=splits * H * self.RP, ml=splits * H * 2)
+        if self.spec.q_rank:
+            need.update(cq=rows * self.QRp,
+                        qf=min(rows, FEW) * self.wuq.shape[0])
+        return need
 
     def _bind(self, eng, b, cache, layer):
-        x = layer.experts
+        x, latent = layer.experts, self.spec.q_rank
+        if not latent:
+            self.args.put(ldq=layer.ldp)
         return self.args.put(
-            P=eng.P, slot=b.slot, pos=b.pos, table=eng.table, cache=cache,
-            qn=eng.qn, qa=eng.qa, part=eng.part, ml=eng.ml, olat=eng.olat,
-            o=eng.o, seg_row0=b.seg_row0, seg_len=b.seg_len,
-            seg_slot=b.seg_slot, seg_pos0=b.seg_pos0, tile_seg=0,
-            tile_rr0=0, ridx=eng.ridx, rwt=eng.rwt, ldp=layer.ldp,
-            orouter=layer.orouter, ldt=eng.table.shape[1], rows=b.T, rbase=0,
-            NS=1, E=x.spec.experts if x else 0, rtop=x.top if x else 0,
+            P=eng.P, Q=eng.qf if latent else eng.P, cq=eng.cq, slot=b.slot,
+            pos=b.pos, table=eng.table, cache=cache, qn=eng.qn, qa=eng.qa,
+            part=eng.part, ml=eng.ml, olat=eng.olat, o=eng.o,
+            seg_row0=b.seg_row0, seg_len=b.seg_len, seg_slot=b.seg_slot,
+            seg_pos0=b.seg_pos0, tile_seg=0, tile_rr0=0, ridx=eng.ridx,
+            rwt=eng.rwt, ldp=layer.ldp, orouter=layer.orouter,
+            ldt=eng.table.shape[1], rows=b.T, rbase=0, NS=1, written=0,
+            E=x.spec.experts if x else 0, rtop=x.top if x else 0,
             rextra=x.extra if x else 0)
 
     def _single(self, eng, a, n):
         """Split attention of the first n rows, partials left in part/ml."""
-        a.put(rows=n, rbase=0, NS=eng.decode_splits(n))
+        a.put(rows=n, rbase=0, NS=self.token_splits(eng, n))
         hy.latent_attn(eng.f32, a, 1, n * (-(-self.spec.heads // 16)))
+
+    def _queries(self, eng, a, T):
+        """Queries of a few rows, fp32, from their latents."""
+        s = self.spec
+        if eng.one_row(self.wuq, T):
+            hy.lin_row(self.wuq, eng.P, eng.qf, s.q_rank, eng.cfg.norm_eps,
+                       g=self.qnorm)
+        else:
+            hy.latent_mid(eng.f32, a)
+            a.put(written=1)
+            hy.gemm_rows(eng.cq, self.wuq, eng.qf, T, self.QRp,
+                         self.wuq.shape[0], hy.EPI_F32)
 
     def few(self, eng, b, cache, layer, fuse):
         a = self._bind(eng, b, cache, layer)
+        if self.spec.q_rank:
+            self._queries(eng, a, b.T)
         hy.latent_dec_prep(eng.f32, a)
         self._single(eng, a, b.T)
         x = layer.experts if fuse else None
@@ -184,7 +260,16 @@ class LatentAttention:
     def many(self, eng, b, cache, layer):
         s, H, CS, RP = self.spec, self.spec.heads, self.CS, self.RP
         a = self._bind(eng, b, cache, layer)
-        hy.latent_prep(eng.f32, a)
+        if s.q_rank:
+            hy.latent_mid(eng.f32, a)
+            rot = hy.Rotary().put(
+                pos=b.pos, cosT=self.cosT, sinT=self.sinT, y=eng.qa[RP:],
+                split=H * self.dp, RT=self.RT, dims=s.rot_dims, ld=H * CS,
+                hs=CS)
+            hy.gemm_rows(eng.cq, self.wuq, eng.qn, b.T, self.QRp,
+                         H * self.dp, hy.EPI_ROTARY, rotary=rot)
+        else:
+            hy.latent_prep(eng.f32, a)
         hy.gemm_rows(eng.qn, self.wukT, eng.qa, b.T, H * self.dp, H * CS,
                      hy.EPI_T, N=RP, K=self.dp, Z=H, xz=self.dp,
                      wz=RP * self.dp, yz=CS)
@@ -193,6 +278,8 @@ class LatentAttention:
             hy.latent_merge(eng.f32, a)
         if b.nd < b.T:
             seg, rr0, n, longest = b.tiles[H]
+            if s.window:
+                longest = min(longest, s.window + hy.TILE // H)
             rows = b.T - b.nd
             ns = min(eng.run_splits(n, longest),
                      eng.part.numel() // (rows * H * RP),
@@ -204,8 +291,17 @@ class LatentAttention:
                 hy.latent_merge(eng.f32, a)
         hy.gemm_rows(eng.olat, self.wuv, eng.o, b.T, H * RP, self.ldo,
                      hy.EPI_TGATE, N=s.vdim, K=RP, Z=H, xz=RP,
-                     wz=s.vdim * RP, yz=s.vdim,
-                     gate=eng.P[a.og:], ldg=layer.ldp)
+                     wz=s.vdim * RP, yz=s.vdim, gate=eng.P[self.og:],
+                     ldg=layer.ldp, gz=a.gz, gc=a.gc)
+
+    def run(self, eng, b, cache, layer):
+        if b.nseg == 0 and b.T <= FEW:
+            self.few(eng, b, cache, layer, False)
+        else:
+            self.many(eng, b, cache, layer)
+
+    def out(self, eng, b, layer):
+        eng.linear(self.wo, eng.o, eng.y, b.T)
 
 
 class MLSTM:
@@ -470,17 +566,53 @@ class Lightning(SandwichMixer):
                           gate=eng.P[self.og:], ldg=layer.ldp)
 
 
+class InputConv:
+    """A sublayer's input plus its causal convolution over time, channel by
+    channel; a ring per sequence keeps the inputs that later steps need."""
+
+    def __init__(self, pk: Packer, name: str):
+        self.w = pk.f32(name).t().contiguous()         # [taps, width]
+
+    def new_ring(self, eng):
+        return torch.zeros(eng.cache.num_slots, *self.w.shape,
+                           dtype=torch.float32, device=eng.device)
+
+
 class DenseFF:
-    """W_down relu(W_up h)^2; the hidden size is zero-padded to 64."""
+    """W_down act(W_up h); the hidden size is zero-padded to 64."""
+    experts = None
 
     def __init__(self, eng, spec, pk: Packer, p: str):
-        self.ffp = pad_to(spec.ff, 64)
+        self.ff, self.ffp = spec.ff, pad_to(spec.ff, 64)
         up = pk.rows([p + "up"], eng.W)
         self.up = torch.zeros(self.ffp, up.shape[1], dtype=pk.dtype,
                               device=pk.device)
         self.up[:spec.ff].copy_(up)
         self.down = pk.rows([p + "down"], spec.ff)
+        self.coef = pk.f32(p + "act") if spec.act == "polynorm" else None
+        self.act_floats = self.ffp
+        self.p_floats = self.ffp if self.coef is not None else 0
+
+    def after_up(self, eng, b):
+        """eng.y from the up products in eng.P, a polynomial activation of
+        the whole row between the two matrices."""
+        eng.poly_linear(self.down, eng.P, self.ff, self.coef, eng.act,
+                        eng.y, b.T)
 
 
+class RoutedFF:
+    """Routed experts of a block that does not route in its mixer."""
+
+    def __init__(self, eng, spec, pk: Packer, p: str):
+        self.experts = RoutedExperts(eng, spec, pk, p)
+        self.up = pk.rows([p + "router"], eng.W)
+        self.act_floats = self.experts.K1 * self.experts.ffm
+        self.p_floats = spec.experts
+
+    def after_up(self, eng, b):
+        self.experts.apart(eng, b.T, b.nseg == 0)
+
+
+FEED_FORWARDS = {"dense": DenseFF, "moe": RoutedFF}
 MIXERS = {c.kind: c for c in (LatentAttention, MLSTM, GroupedAttention,
                               RGLRU, Lightning)}

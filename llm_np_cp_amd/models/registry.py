@@ -28,7 +28,7 @@ def _numpy():
 # pass; None: the config names them)
 MODELS = {t: (_dense, _numpy, ("llmops",))
           for t in ("llama", "gemma2", "qwen2", "mistral", "mixtral")}
-MODELS.update({t: (_layered, None, None) for t in ("turudra", "garupel")})
+MODELS.update({t: (_layered, None, None) for t in ("turudra", "garupel", "fidizen")})
 
 
 def _entry(config):

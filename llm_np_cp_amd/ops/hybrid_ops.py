@@ -17,10 +17,11 @@ import torch
 _PKG = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 _FNS = {}
 
-EPI_F32, EPI_RESADD, EPI_SOFTCAP, EPI_T, EPI_TGATE, EPI_RELU2 = range(6)
-ROW_NORM, ROW_CAT, ROW_PLAIN = range(3)
+(EPI_F32, EPI_RESADD, EPI_SOFTCAP, EPI_T, EPI_TGATE, EPI_RELU2,
+ EPI_ROTARY) = range(7)
+ROW_NORM, ROW_CAT, ROW_PLAIN, ROW_CONV, ROW_POLY = range(5)
 PAGE = 64           # tokens of a cache page (latent_attn.hip, gqa_attn.hip)
-CHUNK = 64          # tokens of a recurrence chunk (mlstm, rglru, lightning)
+CHUNK = 64          # tokens of a chunk (linear, mlstm, rglru, lightning)
 MAX_SPLITS = 256
 TILE = 64           # (token, head) pairs of an attention block over runs
 RANKS = (64, 128, 256, 384, 512)      # padded latent sizes that are built
@@ -53,10 +54,11 @@ def _struct(name, *fields):
 
 LatentArgs = _struct(
     "LatentArgs",
-    (_p, "P Wuk Wuv cnorm cosT sinT slot pos table cache qn qa part ml olat "
+    (_p, "P Q cq qnorm sink Wuk Wuv cnorm cosT sinT slot pos table cache qn qa part ml olat "
          "o seg_row0 seg_len seg_slot seg_pos0 tile_seg tile_rr0 ridx rwt"),
     (_i, "ldp oq odkv og orouter H d dp rot rdims RT rank RP vd ldo ldt rows "
-         "rbase NS E rtop rextra"),
+         "rbase NS E rtop rextra ldq qh oqr qrh qrank QRp pairs win gz gc "
+         "written"),
     (_f, "eps scale"))
 MlstmArgs = _struct(
     "MlstmArgs",
@@ -83,14 +85,22 @@ LightningArgs = _struct(
          "chunk_row0 chunk_len"),
     (_i, "ldp oq ok ov H d vd nvt rows nseg nchunk"))
 RowStage = _struct(
-    "RowStage", (_p, "x y gb xadd g gate xout"), (_i, "W Kp ldg"),
-    (_f, "eps"))
+    "RowStage", (_p, "x y gb xadd g gate xout cw ring slot pos"),
+    (_i, "W Kp ldg taps"), (_f, "eps"))
+ConvRows = _struct(
+    "ConvRows", (RowStage, "s"),
+    (_p, "out seg_row0 seg_len seg_slot seg_pos0 chunk_row0 chunk_len "
+         "chunk_seg"), (_i, "nd nseg nchunk"))
 LinRowArgs = _struct(
-    "LinRowArgs", (_p, "Wt"), (RowStage, "s"), (_p, "rows hin hout bias y"),
-    (_i, "N stage epi"), (_f, "cap"))
+    "LinRowArgs", (_p, "Wt"), (RowStage, "s"),
+    (_p, "rows hin hout bias act y"), (_i, "N stage epi"), (_f, "cap"))
+Rotary = _struct(
+    "Rotary", (_p, "pos cosT sinT y"), (_i, "split RT dims ld hs"))
 MoeArgs = _struct(
     "MoeArgs", (_p, "h gu down idx wt act"),
-    (_i, "ldh ldact W E K1 ff ffs"), (_f, "lim lims"))
+    (_i, "ldh ldact W E K1 ff ffs glu win"), (_f, "lim lims"))
+RouteArgs = _struct(
+    "RouteArgs", (_p, "z idx wt"), (_i, "ldz rows E top extra scores"))
 MoeSort = _struct(
     "MoeSort", (_p, "perm tile_e tile_row0 tile_n"),
     (_i, "pairs groups bm maxtiles"))
@@ -102,9 +112,13 @@ _SIGS = {
         "launch_cat_rows": [_i, _p, _p, _p, _i, _i, _i, _p],
         "launch_lin_row": [_i, _p, _p],
         "launch_gemm_rows":
-            [_i] + [_p] * 5 + [_i] * 8 + [_f, _i, _l, _l, _l, _p]},
+            [_i] + [_p] * 5 + [_i] * 8 + [_f, _i, _l, _l, _l, _i, _i, _p,
+                                          _p],
+        "launch_conv_rows": [_i, _p, _p],
+        "launch_poly_rows": [_i, _p, _i, _p, _p, _i, _i, _i, _f, _p]},
     "latent": {
         "launch_latent_prep": [_i, _p, _p],
+        "launch_latent_mid": [_i, _p, _p],
         "launch_latent_dec_prep": [_i, _p, _p],
         "launch_latent_attn": [_i, _p, _i, _i, _p],
         "launch_latent_merge": [_i, _p, _p],
@@ -126,8 +140,10 @@ _SIGS = {
         "launch_lightning_step": [_p, _p],
         "launch_lightning_run": [_p, _p]},
     "moe": {
-        "launch_block_out": [_i, _p, _p, _i, _p, _i, _p, _i, _i, _f, _p],
-        "launch_moe_rows": [_i, _p, _p, _p, _p, _i, _f, _p]},
+        "launch_block_out": [_i, _p, _p, _i, _p, _i, _p, _i, _i, _f, _i, _p],
+        "launch_moe_gu_few": [_i, _p, _p, _p],
+        "launch_moe_route": [_p, _p, _p],
+        "launch_moe_rows": [_i, _p, _p, _p, _p, _i, _f, _i, _p]},
 }
 _LIB_OF = {fn: name for name, sigs in _SIGS.items() for fn in sigs}
 
@@ -173,13 +189,20 @@ def embed_rows(table, ids, x, x0, M: int, scale: float):
 
 
 def _stage(x, W: int, Kp: int, eps: float, g=None, y=None, gb=None,
-           xadd=None, gate=None, ldg: int = 0, xout=None):
+           xadd=None, gate=None, ldg: int = 0, xout=None, conv=None):
     """Staging of residual rows: v = x [+ y/rms(y) gb] [+ xadd], then
-    v/rms(v) g [sigmoid(gate)]; xout receives v."""
+    v/rms(v) g [sigmoid(gate)]; xout receives v.  conv = (kernel [taps, W],
+    ring [slots, taps, W], slots, positions): v + its convolution over time
+    instead of the norm."""
     assert (y is None) == (gb is None) and (g is None or Kp >= W)
-    return RowStage().put(x=_ptr(x), y=_ptr(y), gb=_ptr(gb), xadd=_ptr(xadd),
-                          g=_ptr(g), gate=_ptr(gate), xout=_ptr(xout), W=W,
-                          Kp=Kp, ldg=ldg, eps=eps)
+    s = RowStage().put(x=_ptr(x), y=_ptr(y), gb=_ptr(gb), xadd=_ptr(xadd),
+                       g=_ptr(g), gate=_ptr(gate), xout=_ptr(xout), W=W,
+                       Kp=Kp, ldg=ldg, eps=eps)
+    if conv is not None:
+        cw, ring, slot, pos = conv
+        assert cw.shape[1] == W and ring.shape[1:] == cw.shape
+        s.put(cw=cw, ring=ring, slot=slot, pos=pos, taps=cw.shape[0])
+    return s
 
 
 def norm_rows(x, g, out, M: int, W: int, Kp: int, eps: float, rows=None,
@@ -201,43 +224,76 @@ def norm_rows(x, g, out, M: int, W: int, Kp: int, eps: float, rows=None,
 
 def lin_row(Wt, x, y, W: int, eps: float, g=None, x0=None, rows=None,
             hout=None, cap: float = 0.0, bias=None, epi: int = EPI_F32,
-            hin=None, res=None, gb=None, **kw):
+            hin=None, res=None, gb=None, conv=None, act=None, **kw):
     """y[n] = Wt[n] . stage(x) [+ bias] for one row; stage is the norm of x
-    with g (see _stage; `res` is its y), the concatenation [x | x0], or the
-    finished row hin.  hout receives the staged row."""
+    with g or its convolution (see _stage; `res` is its y), the
+    concatenation [x | x0], the polynomial activation of x with
+    coefficients act, or the finished row hin.  hout receives the staged
+    row (norm and convolution)."""
     N, Kp = Wt.shape
     stage = (ROW_NORM if g is not None else ROW_CAT if x0 is not None
-             else ROW_PLAIN)
+             else ROW_CONV if conv is not None
+             else ROW_POLY if act is not None else ROW_PLAIN)
     assert Kp % 64 == 0 and y.numel() >= N
     assert stage != ROW_PLAIN or hin.numel() >= Kp and hin.dtype == Wt.dtype
     assert stage != ROW_CAT or Kp >= 2 * W
     assert y.dtype == (Wt.dtype if epi == EPI_RELU2 else torch.float32)
     a = LinRowArgs().put(
         Wt=Wt, rows=_ptr(rows), hin=_ptr(hin), hout=_ptr(hout),
-        bias=_ptr(bias), y=y, N=N, stage=stage, epi=epi, cap=cap)
+        bias=_ptr(bias), act=_ptr(act), y=y, N=N, stage=stage, epi=epi, cap=cap)
     if stage == ROW_CAT:
         kw["xadd"] = x0
-    a.s = _stage(x, W, Kp, eps, g, y=res, gb=gb, **kw)
+    a.s = _stage(x, W, Kp, eps, g, y=res, gb=gb, conv=conv, **kw)
     _go("launch_lin_row", _f32(Wt), ctypes.byref(a))
+
+
+def conv_rows(x, out, b, W: int, Kp: int, eps: float, conv, **kw):
+    """out[r] = v + conv(v) for the rows of batch b (see _stage; takes y,
+    gb, xout)."""
+    assert out.numel() >= b.T * Kp and Kp % 64 == 0
+    nd = b.nd
+    a = ConvRows().put(
+        out=out, seg_row0=b.seg_row0[nd:], seg_len=b.seg_len[nd:],
+        seg_slot=b.seg_slot[nd:], seg_pos0=b.seg_pos0[nd:],
+        chunk_row0=b.chunk_row0, chunk_len=b.chunk_len, chunk_seg=b.chunk_seg,
+        nd=nd, nseg=b.nseg, nchunk=b.nchunk)
+    a.s = _stage(x, W, Kp, eps, conv=conv, **kw)
+    _go("launch_conv_rows", _f32(out), ctypes.byref(a))
+
+
+def poly_rows(z, ldz: int, act, out, M: int, W: int, eps: float):
+    """out[M, W padded to 64] = a N(z) + b N(z^2) + c N(z^3) + e."""
+    Kp = -(-W // 64) * 64
+    assert z.numel() >= (M - 1) * ldz + W and out.numel() >= M * Kp
+    _go("launch_poly_rows", _f32(out), _ptr(z), ldz, _ptr(act), _ptr(out), M,
+        W, Kp, eps)
 
 
 def gemm_rows(X, Wt, Y, M: int, ldx: int, ldy: int, epi: int,
               mult: float = 0.0, N: int = 0, K: int = 0, Z: int = 1,
               xz: int = 0, wz: int = 0, yz: int = 0, gate=None, ldg: int = 0,
-              bias=None):
+              bias=None, gz: int = 1, gc: int = 0, rotary=None):
     """Y[M, N] = X[M, K] Wt[N, K]^T with one of the EPI_* epilogues, for
-    each of Z heads (element offsets xz/wz/yz)."""
+    each of Z heads (element offsets xz/wz/yz).  Gates are at row*ldg +
+    z*gz + column*gc.  EPI_ROTARY: the columns from rotary.split on go,
+    rotated, to rotary.y."""
     N = N or Wt.shape[0]
     K = K or Wt.shape[-1]
     assert X.numel() >= (M - 1) * ldx + (Z - 1) * xz + K
-    assert Y.numel() >= (M - 1) * ldy + (Z - 1) * yz + N
+    cols = rotary.split if epi == EPI_ROTARY else N
+    assert Y.numel() >= (M - 1) * ldy + (Z - 1) * yz + cols
     assert Wt.numel() >= (Z - 1) * wz + N * K
     _go("launch_gemm_rows", _f32(Wt), _ptr(X), _ptr(Wt), _ptr(Y), _ptr(gate),
-        _ptr(bias), M, N, K, ldx, K, ldy, ldg, epi, mult, Z, xz, wz, yz)
+        _ptr(bias), M, N, K, ldx, K, ldy, ldg, epi, mult, Z, xz, wz, yz, gz, gc,
+        ctypes.byref(rotary) if rotary is not None else 0)
 
 
 def latent_prep(f32, a):
     _go("launch_latent_prep", f32, ctypes.byref(a))
+
+
+def latent_mid(f32, a):
+    _go("launch_latent_mid", f32, ctypes.byref(a))
 
 
 def latent_dec_prep(f32, a):
@@ -307,11 +363,22 @@ def mlstm_dec_fin(f32, a, m, pairs: int):
 
 
 def block_out(f32, Wo, o, ldo: int, m, K1: int, x, rows: int, W: int,
-              mult: float):
+              mult: float, set: bool = False):
+    """x[r] += mult (Wo o_r + the experts' outputs), or with `set` x[r] =
+    that; without Wo where ldo is 0."""
     _go("launch_block_out", f32, _ptr(Wo), _ptr(o), ldo, ctypes.byref(m), K1,
-        _ptr(x), rows, W, mult)
+        _ptr(x), rows, W, mult, int(set))
 
 
-def moe_rows(f32, m, s, y, x, rows: int, mult: float):
+def moe_gu_few(f32, m, route):
+    """Routing and the experts' gate/up halves, one block row per pair."""
+    _go("launch_moe_gu_few", f32, ctypes.byref(m), ctypes.byref(route))
+
+
+def moe_route(m, route):
+    _go("launch_moe_route", ctypes.byref(m), ctypes.byref(route))
+
+
+def moe_rows(f32, m, s, y, x, rows: int, mult: float, set: bool = False):
     _go("launch_moe_rows", f32, ctypes.byref(m), ctypes.byref(s), _ptr(y),
-        _ptr(x), rows, mult)
+        _ptr(x), rows, mult, int(set))
