@@ -22,13 +22,17 @@ import time
 sys.path.insert(0, os.path.dirname(os.path.abspath(__file__)))
 
 
-COMPARE = ("turudra-2k", "turudra-4k", "garupel-2k", "garupel-4k")
+COMPARE = ("turudra-2k", "turudra-4k", "garupel-2k", "garupel-4k",
+           "fidizen-2k", "fidizen-4k")
 
 
 def compare(cases, steps, warmup, prompt=2048, batches=(1, 4, 16)):
     """One JSON line per model, size and batch: random weights, bf16,
-    synthetic prompts.  Beside each design stands the closest transformer
-    of equal width, heads and layer runs.  An MoE one gets one more expert
+    synthetic prompts.  Beside each design stands the closest other model
+    of equal width, heads and layer runs.  Windowed latent attention stands
+    beside unwindowed one, a dense feed-forward beside two experts, both
+    chosen, and a shared one that hold as much; other designs stand beside
+    a transformer.  An MoE one gets one more expert
     and one more choice, so its experts match the design's routed + shared
     ones in stored and in active parameters; a dense one gets two thirds of
     the hidden size, so its three matrices match the design's two."""
@@ -41,7 +45,29 @@ def compare(cases, steps, warmup, prompt=2048, batches=(1, 4, 16)):
     from llm_np_cp_amd.io.loader import LazyRandomWeights
     from llm_np_cp_amd.models.registry import engine_class
 
-    def transformer(c):
+    def latent_design(c):
+        def layer(l):
+            m, f = l.mixer, l.mlp
+            if f.kind == "dense":     # 2 matrices -> 3 experts of 3
+                n, top, ff = 2, 2, f.ff * 2 // 9
+            else:
+                n, top, ff = f.experts, f.top, f.expert.ff
+            e = {"ff": ff, "limit": 7.0}
+            keep = ("heads", "dim", "rot_dim", "vdim", "kv_rank", "scale",
+                    "rot")
+            d = m.to_dict()
+            return {"type": "latent_attention",
+                    "mixer": {k: d[k] for k in keep},
+                    "mlp": {"kind": "moe", "expert": e, "shared": e,
+                            "router": {"experts": n, "top": top}}}
+        return "turudra", L.ModelConfig.from_hf_dict({
+            "architecture": "Turudra", "vocab": c.vocab_size,
+            "width": c.hidden_size, "norm": {"eps": 1e-6},
+            "residual_mult": 0.5, "layers": [layer(l) for l in c.layers]})
+
+    def closest(c):
+        if c.model_type == "fidizen":
+            return latent_design(c)
         att, ff = c.layers[0].mixer, c.layers[0].mlp
         kw = dict(vocab_size=c.vocab_size, hidden_size=c.hidden_size,
                   num_hidden_layers=len(c.runs), head_dim=128,
@@ -71,7 +97,7 @@ def compare(cases, steps, warmup, prompt=2048, batches=(1, 4, 16)):
             preset = "turudra-" + preset
         family, _, size = preset.partition("-")
         design = L.preset_config(preset)
-        for name, cfg in ((family, design), transformer(design)):
+        for name, cfg in ((family, design), closest(design)):
             if side and side != name:
                 continue
             rng = np.random.default_rng(0)
@@ -135,11 +161,11 @@ def main():
     ap.add_argument("--compare", nargs="*", default=None, metavar="CASE",
                     help="instead of the default workload: prefill and "
                          "decode throughput of the layer-list designs "
-                         "beside the closest transformer of equal size; "
+                         "beside the closest other model of equal size; "
                          "cases turudra-2k (or 2k), turudra-4k, garupel-2k, "
-                         "garupel-4k (default all), each optionally with "
-                         ":turudra, :mixtral, :garupel or :qwen2 for one "
-                         "side only")
+                         "garupel-4k, fidizen-2k, fidizen-4k (default all), "
+                         "each optionally with :turudra, :mixtral, :garupel, "
+                         ":qwen2 or :fidizen for one side only")
     args = ap.parse_args()
     if args.compare is not None:
         return compare(args.compare or COMPARE, args.steps, args.warmup)
