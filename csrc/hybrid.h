@@ -111,13 +111,13 @@ DEVINL float glu_act(int kind, float gate, float up, float lim) {
 // One wave; E <= 64*EPL.
 template <int EPL>
 DEVINL void route_row(const float* z, int E, int top, int extra, int* idx,
-                      float* wt, int scores = 0) {
+                      float* wt, int scores = 0, int lde = 1) {
   const int lane = threadIdx.x & 63;
   float v[EPL];
 #pragma unroll
   for (int i = 0; i < EPL; i++) {
     int e = lane + i * 64;
-    v[i] = e < E ? z[e] : -INFINITY;
+    v[i] = e < E ? z[(size_t)e * lde] : -INFINITY;
   }
   float zmax = 0.f, sum = 0.f;
   for (int j = 0; j < top; j++) {

@@ -217,7 +217,7 @@ static size_t attn_lds(int RP, int RT) {
 // is worked on.
 template <typename T, int RP, int NW, bool SHARE>
 __global__ void __launch_bounds__(64 * NW) k_latent_attn(LatentArgs a) {
-  constexpr bool AHEAD = SHARE && sizeof(T) == 2;
+  constexpr bool AHEAD = sizeof(T) == 2;
   using Sh = AttnShape<T, RP>;
   constexpr int QW = SHARE ? 1 : NW;                    // query groups
   constexpr int ND = SHARE ? RP / 16 / NW : RP / 16;    // output fragments

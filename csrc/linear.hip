@@ -60,19 +60,38 @@ DEVINL void stage_row(const RowStage& s, size_t row, bool keep, float* red,
   if constexpr (CONV) {
     pos = s.pos[row];
     ring = s.ring + (size_t)s.slot[row] * s.taps * W;
+    const int now = pos % s.taps;
+    // input j places back; the first three without branches, so that their
+    // loads are on the way together
+    float h[3][U], c[3][U];
+#pragma unroll
+    for (int j = 1; j <= 3; j++) {
+      const bool ok = j < s.taps && j <= pos;
+      const float* hp = ring + (ok ? now - j + (now < j ? s.taps : 0) : 0) * W;
+      const float* cp = s.cw + (ok ? s.taps - 1 - j : 0) * W;
+#pragma unroll
+      for (int u = 0; u < U; u++) {
+        const int i = min(tid + u * NT, W - 1);
+        h[j - 1][u] = hp[i];
+        c[j - 1][u] = cp[i];
+        if (!ok) h[j - 1][u] = c[j - 1][u] = 0.f;     // may hold anything
+      }
+    }
 #pragma unroll
     for (int u = 0; u < U; u++) {
       const int i = tid + u * NT;
-      cv[u] = 0.f;
       cl[u] = i < W ? s.cw[(size_t)(s.taps - 1) * W + i] : 0.f;
+      cv[u] = 0.f;
+#pragma unroll
+      for (int j = 0; j < 3; j++) cv[u] = fmaf(c[j][u], h[j][u], cv[u]);
     }
-    for (int j = 1; j < s.taps && j <= pos; j++) {
-      const float* h = ring + (size_t)((pos - j) % s.taps) * W;
-      const float* c = s.cw + (size_t)(s.taps - 1 - j) * W;
+    for (int j = 4; j < s.taps && j <= pos; j++) {
+      const float* hp = ring + (size_t)((pos - j) % s.taps) * W;
+      const float* cp = s.cw + (size_t)(s.taps - 1 - j) * W;
 #pragma unroll
       for (int u = 0; u < U; u++) {
         const int i = tid + u * NT;
-        if (i < W) cv[u] = fmaf(c[i], h[i], cv[u]);
+        if (i < W) cv[u] = fmaf(cp[i], hp[i], cv[u]);
       }
     }
   }
@@ -160,11 +179,10 @@ k_norm_rows(RowStage s, const int* __restrict__ rows, T* __restrict__ out) {
 
 // ---- rows with their input convolution -----------------------------------
 // out[r] = v_r + conv(v)_r with v = x [+ y / rms(y) * gb], for single tokens
-// and runs of tokens.  A block takes one single token, or CR rows of a chunk
+// and runs of tokens.  A block takes one single token, or R rows of a chunk
 // of a run; it computes the rows ahead of its own again.  The block at the
 // head of a run reads the ring and, channel by channel in the same thread,
 // leaves the run's last inputs in it.
-#define CR 8
 #define CHUNK 64
 
 struct ConvRows {
@@ -179,138 +197,185 @@ struct ConvBlock {
   int row0, n, seg0, len, slot, pos0;   // rows of the block, its sequence's run
 };
 
-DEVINL ConvBlock conv_block(const ConvRows& a) {
-  const int b = blockIdx.x;
+template <int R> DEVINL ConvBlock conv_block(const ConvRows& a) {
+  int b = blockIdx.x;
   if (b < a.nd) return {b, 1, b, 1, a.s.slot[b], a.s.pos[b]};
-  const int c = (b - a.nd) / (CHUNK / CR), at = (b - a.nd) % (CHUNK / CR) * CR;
+  b -= a.nd;                // neighbours on one XCD: they share rows in its L2
+  b = b % 8 * (a.nchunk * (CHUNK / R) / 8) + b / 8;
+  const int c = b / (CHUNK / R), at = b % (CHUNK / R) * R;
   const int g = a.chunk_seg[c];
-  return {a.chunk_row0[c] + at, min(CR, a.chunk_len[c] - at), a.seg_row0[g],
+  return {a.chunk_row0[c] + at, min(R, a.chunk_len[c] - at), a.seg_row0[g],
           a.seg_len[g], a.seg_slot[g], a.seg_pos0[g]};
+}
+
+// sums over the wave of N values a lane, N a power of two: lane l < N gets
+// the sum of value sum_slot<N>(l)
+template <int N> DEVINL float wave_sums(float (&v)[N]) {
+  const int lane = threadIdx.x & 63;
+  int mask = 1;
+#pragma unroll
+  for (int half = N / 2; half >= 1; half /= 2, mask *= 2) {
+    const bool up = lane & mask;
+#pragma unroll
+    for (int i = 0; i < half; i++) {
+      const float keep = up ? v[i + half] : v[i];
+      const float give = up ? v[i] : v[i + half];
+      v[i] = keep + __shfl_xor(give, mask);
+    }
+  }
+  float t = v[0];
+#pragma unroll
+  for (int m = N; m < 64; m *= 2) t += __shfl_xor(t, m);
+  return t;
+}
+template <int N> DEVINL int sum_slot(int lane) {
+  return N == 1 ? 0 : (int)(__brev((unsigned)lane) >> (32 - __builtin_ctz(N)));
+}
+
+DEVINL f4v mix4(f4v x, f4v y, f4v gb, float rn) {
+  f4v v;
+#pragma unroll
+  for (int c = 0; c < 4; c++) v[c] = x[c] + y[c] * rn * gb[c];
+  return v;
+}
+
+template <typename T> DEVINL void st4(T* p, f4v v) {
+  if constexpr (sizeof(T) == 2) {
+    union { T t[4]; uint64_t u; } o;
+#pragma unroll
+    for (int c = 0; c < 4; c++) o.t[c] = El<T>::st(v[c]);
+    *(uint64_t*)p = o.u;
+  } else *(f4v*)p = v;
+}
+
+// a thread owns four channels: 4 NT >= W, W % 4 == 0, TAPS - 1 <= R; R = 1
+// where the batch has single tokens only
+template <typename T, int TAPS, int NT, int R>
+__global__ void __launch_bounds__(NT) k_conv_rows(ConvRows a) {
+  constexpr int B = TAPS - 1, NW = NT / 64;
+  constexpr int N = R == 1 ? 1 : R + B <= 8 ? 8 : 16;
+  constexpr int E0 = R == 1 ? B : 0;    // first row whose norm may be needed
+  static_assert(R + B <= 16 && (B <= R || R == 1));
+  __shared__ float red[NW][N];
+  const RowStage& s = a.s;
+  const ConvBlock k = R == 1 ? ConvBlock{(int)blockIdx.x, 1, (int)blockIdx.x, 1,
+                                         s.slot[blockIdx.x], s.pos[blockIdx.x]}
+                             : conv_block<R>(a);
+  if (k.n <= 0) return;
+  const int W = s.W, tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
+  const int c0 = tid * 4;
+  const bool mine = c0 < W;
+  const f4v zero = {0.f, 0.f, 0.f, 0.f};
+  float* ring = s.ring + (size_t)k.slot * TAPS * W + c0;
+  // 1 / rms of the rows whose squares' sums each thread has in ss
+  auto rms_all = [&](float (&ss)[N]) {
+    const float t = wave_sums<N>(ss);
+    if (lane < N) red[wave][sum_slot<N>(lane)] = t;
+    __syncthreads();
+    if (tid < N) {
+      float sum = 0.f;
+#pragma unroll
+      for (int w = 0; w < NW; w++) sum += red[w][tid];
+      red[0][tid] = 1.f / sqrtf(sum / (float)W + s.eps);
+    }
+    __syncthreads();
+  };
+  auto square = [](f4v v) {
+    return v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+  };
+
+  f4v v[R + B], y[R + B], w[TAPS], gb = zero;
+  float ss[N];
+#pragma unroll
+  for (int e = 0; e < N; e++) ss[e] = 0.f;
+#pragma unroll
+  for (int e = 0; e < R + B; e++) {
+    v[e] = y[e] = zero;
+    const int row = k.row0 - B + e, back = row - k.seg0;   // < 0: before it
+    if (!mine || e - B >= k.n) continue;
+    if (back >= 0) {
+      v[e] = *(const f4v*)(s.x + (size_t)row * W + c0);
+      if (s.y) y[e] = *(const f4v*)(s.y + (size_t)row * W + c0);
+    } else if (k.pos0 + back >= 0) {
+      v[e] = *(const f4v*)(ring + (size_t)((k.pos0 + back) % TAPS) * W);
+    }
+  }
+#pragma unroll
+  for (int j = 0; j < TAPS; j++)
+    w[j] = mine ? *(const f4v*)(s.cw + (size_t)j * W + c0) : zero;
+  if (s.y) {
+    if (mine) gb = *(const f4v*)(s.gb + c0);
+#pragma unroll
+    for (int e = E0; e < R + B; e++) ss[e - E0] = square(y[e]);
+    rms_all(ss);
+#pragma unroll
+    for (int e = E0; e < R + B; e++)
+      v[e] = mix4(v[e], y[e], gb, red[0][e - E0]);
+  }
+#pragma unroll
+  for (int e = 0; e < R; e++) {
+    if (e >= k.n) break;
+    f4v o = v[B + e];
+#pragma unroll
+    for (int c = 0; c < 4; c++) {
+      float sum = 0.f;
+#pragma unroll
+      for (int j = 0; j < TAPS; j++) sum = fmaf(w[j][c], v[e + j][c], sum);
+      o[c] += sum;
+    }
+    if (c0 < s.Kp)
+      st4((T*)a.out + (size_t)(k.row0 + e) * s.Kp + c0, mine ? o : zero);
+    if (mine && s.xout)
+      *(f4v*)(s.xout + (size_t)(k.row0 + e) * W + c0) = v[B + e];
+  }
+  if (k.row0 != k.seg0 || B == 0) return;
+  if (R == 1 || k.len == 1) {
+    if (mine) *(f4v*)(ring + (size_t)(k.pos0 % TAPS) * W) = v[B];
+    return;
+  }
+  if constexpr (R > 1) {
+  // the run's last inputs
+  f4v xt[TAPS], yt[TAPS];
+#pragma unroll
+  for (int e = 0; e < N; e++) ss[e] = 0.f;
+#pragma unroll
+  for (int e = 0; e < B; e++) {
+    const int row = k.seg0 + k.len - B + e;
+    const bool in = mine && row >= k.seg0;
+    xt[e] = in ? *(const f4v*)(s.x + (size_t)row * W + c0) : zero;
+    yt[e] = in && s.y ? *(const f4v*)(s.y + (size_t)row * W + c0) : zero;
+    ss[e] = square(yt[e]);
+  }
+  if (s.y) {
+    __syncthreads();                    // red[0] has been read
+    rms_all(ss);
+  }
+#pragma unroll
+  for (int e = 0; e < B; e++) {
+    const int at = k.len - B + e;
+    if (mine && at >= 0)
+      *(f4v*)(ring + (size_t)((k.pos0 + at) % TAPS) * W) =
+          s.y ? mix4(xt[e], yt[e], gb, red[0][e]) : xt[e];
+  }
+  }
 }
 
 // 1 / rms of one row of y, by one wave
 DEVINL float wave_rms(const RowStage& s, int row) {
   const float* y = s.y + (size_t)row * s.W;
-  const int lane = threadIdx.x & 63;
   float ss = 0.f;
-  if (s.W % 4 == 0) {
-#pragma unroll 4
-    for (int i = lane * 4; i < s.W; i += 256) {
-      f4v v = *(const f4v*)(y + i);
-      ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
-    }
-  } else {
-    for (int i = lane; i < s.W; i += 64) ss += y[i] * y[i];
-  }
+#pragma unroll 8
+  for (int i = threadIdx.x & 63; i < s.W; i += 64) ss += y[i] * y[i];
   return 1.f / sqrtf(wave_reduce_sum(ss) / (float)s.W + s.eps);
 }
 
-template <int V> struct Vec { float f[V]; };
-template <int V> DEVINL Vec<V> ldv(const float* p) {
-  Vec<V> r;
-  if constexpr (V == 4) {
-    f4v v = *(const f4v*)p;
-#pragma unroll
-    for (int c = 0; c < 4; c++) r.f[c] = v[c];
-  } else r.f[0] = *p;
-  return r;
-}
-template <int V> DEVINL void stv(float* p, const Vec<V>& v) {
-  if constexpr (V == 4) *(f4v*)p = f4v{v.f[0], v.f[1], v.f[2], v.f[3]};
-  else *p = v.f[0];
-}
-template <int V, typename T> DEVINL void stv_as(T* p, const Vec<V>& v) {
-  union { T t[V]; uint64_t u; f4v f; } o;
-#pragma unroll
-  for (int c = 0; c < V; c++) o.t[c] = El<T>::st(v.f[c]);
-  if constexpr (V * sizeof(T) == 8) *(uint64_t*)p = o.u;
-  else if constexpr (V * sizeof(T) == 16) *(f4v*)p = o.f;
-  else *p = o.t[0];
-}
-
-// TAPS - 1 <= CR; V = 4 needs W % 4 == 0
-template <typename T, int TAPS, int V>
-__global__ void __launch_bounds__(256) k_conv_rows(ConvRows a) {
-  constexpr int B = TAPS - 1;
-  __shared__ float rn[CR + 2 * B];      // the block's rows, the run's last
-  const RowStage& s = a.s;
-  const ConvBlock k = conv_block(a);
-  if (k.n <= 0) return;
-  const int W = s.W, tid = threadIdx.x;
-  const bool head = k.row0 == k.seg0;
-  const int tail0 = k.seg0 + k.len - B;
-  if (s.y) {
-    for (int e = tid >> 6; e < CR + 2 * B; e += 4) {
-      const int row = e < CR + B ? k.row0 - B + e : tail0 + e - (CR + B);
-      if (row < k.seg0 || (e < CR + B ? row >= k.row0 + k.n : !head)) continue;
-      const float r = wave_rms(s, row);
-      if ((tid & 63) == 0) rn[e] = r;
-    }
-    __syncthreads();
-  }
-  float* ring = s.ring + (size_t)k.slot * TAPS * W;
-  for (int i = tid * V; i < s.Kp; i += 256 * V) {
-    if (i >= W) {
-      const Vec<V> z = {};
-      for (int e = 0; e < k.n; e++)
-        stv_as<V>((T*)a.out + (size_t)(k.row0 + e) * s.Kp + i, z);
-      continue;
-    }
-    const Vec<V> gb = s.y ? ldv<V>(s.gb + i) : Vec<V>{};
-    auto value = [&](int row, int e) {
-      Vec<V> v = ldv<V>(s.x + (size_t)row * W + i);
-      if (s.y) {
-        const Vec<V> y = ldv<V>(s.y + (size_t)row * W + i);
-#pragma unroll
-        for (int c = 0; c < V; c++) v.f[c] += y.f[c] * rn[e] * gb.f[c];
-      }
-      return v;
-    };
-    Vec<V> w[TAPS], v[CR + B];
-#pragma unroll
-    for (int j = 0; j < TAPS; j++) w[j] = ldv<V>(s.cw + (size_t)j * W + i);
-#pragma unroll
-    for (int e = 0; e < B; e++) {
-      const int back = k.row0 - B + e - k.seg0;     // < 0: before this run
-      if (back >= 0) v[e] = value(k.row0 - B + e, e);
-      else if (k.pos0 + back >= 0)
-        v[e] = ldv<V>(ring + (size_t)((k.pos0 + back) % TAPS) * W + i);
-      else v[e] = {};
-    }
-#pragma unroll
-    for (int e = 0; e < CR; e++)
-      if (e < k.n) v[B + e] = value(k.row0 + e, B + e);
-#pragma unroll
-    for (int e = 0; e < CR; e++)
-      if (e < k.n) {
-        Vec<V> o;
-#pragma unroll
-        for (int c = 0; c < V; c++) {
-          float sum = 0.f;
-#pragma unroll
-          for (int j = 0; j < TAPS; j++) sum = fmaf(w[j].f[c], v[e + j].f[c], sum);
-          o.f[c] = v[B + e].f[c] + sum;
-        }
-        stv_as<V>((T*)a.out + (size_t)(k.row0 + e) * s.Kp + i, o);
-        if (s.xout) stv<V>(s.xout + (size_t)(k.row0 + e) * W + i, v[B + e]);
-      }
-    if (head)
-#pragma unroll
-      for (int e = 0; e < B; e++) {
-        const int row = tail0 + e;
-        if (row >= k.seg0)
-          stv<V>(ring + (size_t)((k.pos0 + row - k.seg0) % TAPS) * W + i,
-                 value(row, CR + B + e));
-      }
-  }
-}
-
-// any number of taps; the ring is written by a launch of its own
+// any number of taps and any width; the ring is written by a launch of its own
+#define ANY_R 8
 template <typename T>
 __global__ void __launch_bounds__(256) k_conv_rows_any(ConvRows a) {
-  extern __shared__ float rnx[];        // CR + taps - 1
+  extern __shared__ float rnx[];        // ANY_R + taps - 1
   const RowStage& s = a.s;
-  const ConvBlock k = conv_block(a);
+  const ConvBlock k = conv_block<ANY_R>(a);
   if (k.n <= 0) return;
   const int W = s.W, B = s.taps - 1, tid = threadIdx.x;
   if (s.y)
@@ -585,23 +650,6 @@ struct GemmArgs {
 template <typename T, int EPI>
 DEVINL void gemm_store(const GemmArgs& a, int z, int row, int col, float v) {
   const size_t o = (size_t)z * a.yz + (size_t)row * a.ldy + col;
-  if constexpr (EPI == EPI_ROTARY) {
-    // every lane of the wave comes here, neighbours with neighbouring columns
-    const Rotary& r = a.r;
-    const float other = __shfl_xor(v, 1);
-    if (row >= a.M || col >= a.N) return;
-    if (col < r.split) {
-      ((T*)a.Y)[o] = El<T>::st(v);
-      return;
-    }
-    const int c = col - r.split, h = c / r.RT, j = c - h * r.RT;
-    if (j < r.dims) {
-      const size_t t = (size_t)r.pos[row] * (r.dims >> 1) + (j >> 1);
-      v = v * r.cosT[t] + (j & 1 ? other : -other) * r.sinT[t];
-    }
-    ((T*)r.y)[(size_t)row * r.ld + (size_t)h * r.hs + j] = El<T>::st(v);
-    return;
-  }
   if (row >= a.M || col >= a.N) return;
   if constexpr (EPI == EPI_F32) ((float*)a.Y)[o] = v;
   else if constexpr (EPI == EPI_RESADD) ((float*)a.Y)[o] += a.mult * v;
@@ -612,6 +660,42 @@ DEVINL void gemm_store(const GemmArgs& a, int z, int row, int col, float v) {
   else
     ((T*)a.Y)[o] = El<T>::st(
         v * sigmoid_f(a.gate[(size_t)row * a.ldg + z * a.gz + col * a.gc]));
+}
+
+// the same for NR consecutive rows, v[r] of row0 + r
+template <typename T, int EPI, int NR>
+DEVINL void gemm_store_rows(const GemmArgs& a, int z, int row0, int col,
+                            const float* v) {
+  if constexpr (EPI != EPI_ROTARY) {
+#pragma unroll
+    for (int r = 0; r < NR; r++)
+      gemm_store<T, EPI>(a, z, row0 + r, col, v[r]);
+  } else {
+    // every lane of the wave comes here, neighbours with neighbouring columns
+    const Rotary& t = a.r;
+    const int c = max(col - t.split, 0), h = c / t.RT, j = c - h * t.RT;
+    const bool rot = col >= t.split, turn = rot && j < t.dims;
+    float cs[NR], sn[NR], other[NR];
+    if (__any(turn))
+#pragma unroll
+      for (int r = 0; r < NR; r++) {
+        const size_t k = (size_t)t.pos[min(row0 + r, a.M - 1)] * (t.dims >> 1) +
+                         (turn ? j >> 1 : 0);
+        cs[r] = t.cosT[k];
+        sn[r] = t.sinT[k];
+      }
+#pragma unroll
+    for (int r = 0; r < NR; r++) other[r] = __shfl_xor(v[r], 1);
+#pragma unroll
+    for (int r = 0; r < NR; r++) {
+      const int row = row0 + r;
+      const float o =
+          turn ? v[r] * cs[r] + (j & 1 ? other[r] : -other[r]) * sn[r] : v[r];
+      T* to = rot ? (T*)t.y + (size_t)row * t.ld + (size_t)h * t.hs + j
+                  : (T*)a.Y + (size_t)row * a.ldy + col;
+      if (row < a.M && col < a.N) *to = El<T>::st(o);
+    }
+  }
 }
 
 // run body(integral constant of the epilogue)
@@ -649,25 +733,25 @@ __global__ void __launch_bounds__(256) k_gemm(GemmArgs a) {
 #pragma unroll
       for (int j = 0; j < BN / 32; j++) {
         const int col = bn + gemm_col<BN>(j);
+        float v[4];
 #pragma unroll
-        for (int r = 0; r < 4; r++) {
-          const int row = bm + gemm_row0<BM>(i) + r;
-          gemm_store<T, decltype(epi)::value>(a, z, row, col,
-                                              acc[i][j][r] + bias[j]);
-        }
+        for (int r = 0; r < 4; r++) v[r] = acc[i][j][r] + bias[j];
+        gemm_store_rows<T, decltype(epi)::value, 4>(
+            a, z, bm + gemm_row0<BM>(i), col, v);
       }
   });
 }
 
-// up to 16*MF rows: a tile of 16 outputs per block, K over NW waves, both
-// operands straight from memory (the weights are read once)
-template <typename T, int MF, int NW>
+// up to 16*MF rows: a tile of NB (16, or 8 to have more blocks) outputs per
+// block, K over NW waves, both operands straight from memory (the weights are
+// read once)
+template <typename T, int MF, int NW, int NB = 16>
 __global__ void __launch_bounds__(64 * NW) k_gemm_skinny(GemmArgs a) {
   __shared__ float red[NW * MF * 256];
   constexpr int U = MF == 1 ? 8 : 4;
   const int tid = threadIdx.x, wave = wave_index(), lane = tid & 63;
   const int lr = lane & 15, gq = lane >> 4, z = blockIdx.z;
-  const int n0 = blockIdx.x * 16, nch = a.K * (int)sizeof(T) / 64;
+  const int n0 = blockIdx.x * NB, nch = a.K * (int)sizeof(T) / 64;
   const char* wr = (const char*)((const T*)a.W + (size_t)z * a.wz +
                                  (size_t)min(n0 + lr, a.N - 1) * a.ldw) +
                    gq * 16;
@@ -685,7 +769,7 @@ __global__ void __launch_bounds__(64 * NW) k_gemm_skinny(GemmArgs a) {
     for (int u = 0; u < U; u++) {
       const int cu = c + u * NW;
       const bool in = cu < nch;
-      w[u] = in ? ld16nt(wr + (size_t)cu * 64) : f4v{0.f, 0.f, 0.f, 0.f};
+      w[u] = in && lr < NB ? ld16nt(wr + (size_t)cu * 64) : f4v{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int i = 0; i < MF; i++)
         xv[u][i] = in ? ld16(xr[i] + cu * 64) : f4v{0.f, 0.f, 0.f, 0.f};
@@ -706,10 +790,10 @@ __global__ void __launch_bounds__(64 * NW) k_gemm_skinny(GemmArgs a) {
     float v = 0.f;
 #pragma unroll
     for (int u = 0; u < NW; u++) v += red[u * MF * 256 + e];
-    const int row = e >> 4, col = n0 + (e & 15);
+    const int row = e >> 4, col = (e & 15) < NB ? n0 + (e & 15) : a.N;
     if (a.bias) v += a.bias[min(col, a.N - 1)];
     with_epilogue(a.epi, [&](auto epi) {
-      gemm_store<T, decltype(epi)::value>(a, z, row, col, v);
+      gemm_store_rows<T, decltype(epi)::value, 1>(a, z, row, col, &v);
     });
   }
 }
@@ -764,13 +848,13 @@ static bool bad_conv(const RowStage& s) {
          s.Kp < s.W || s.xadd || s.g || s.gate || (s.y && !s.xout);
 }
 
-template <typename T, int V>
-static bool conv_go(const ConvRows& a, int blocks, hipStream_t st) {
+template <typename T, int NT, int R>
+static void conv_go(const ConvRows& a, hipStream_t st) {
+  const dim3 grid(a.nd + a.nchunk * (CHUNK / R));
 #define CONV_TAPS(n)                                                         \
   case n:                                                                    \
-    hipLaunchKernelGGL((k_conv_rows<T, n, V>), dim3(blocks), dim3(256), 0,   \
-                       st, a);                                               \
-    return true
+    hipLaunchKernelGGL((k_conv_rows<T, n, NT, R>), grid, dim3(NT), 0, st, a); \
+    break
   switch (a.s.taps) {
     CONV_TAPS(1);
     CONV_TAPS(2);
@@ -778,17 +862,23 @@ static bool conv_go(const ConvRows& a, int blocks, hipStream_t st) {
     CONV_TAPS(4);
   }
 #undef CONV_TAPS
-  return false;
 }
 
 template <typename T>
 static hipError_t conv_rows(const ConvRows& a, hipStream_t st) {
-  const int blocks = a.nd + a.nchunk * (CHUNK / CR);
-  const bool done = a.s.W % 4 ? conv_go<T, 1>(a, blocks, st)
-                              : conv_go<T, 4>(a, blocks, st);
-  if (!done) {
-    const size_t lds = (CR + a.s.taps - 1) * sizeof(float);
-    hipLaunchKernelGGL(k_conv_rows_any<T>, dim3(blocks), dim3(256), lds, st, a);
+  const int W = a.s.W;
+  if (a.s.taps <= 4 && W % 4 == 0 && W <= 4096) {
+    if (W <= 1024)
+      a.nchunk ? conv_go<T, 256, 4>(a, st) : conv_go<T, 256, 1>(a, st);
+    else if (W <= 2048)
+      a.nchunk ? conv_go<T, 512, 4>(a, st) : conv_go<T, 512, 1>(a, st);
+    else
+      a.nchunk ? conv_go<T, 1024, 4>(a, st) : conv_go<T, 1024, 1>(a, st);
+  } else {
+    const size_t lds = (ANY_R + a.s.taps - 1) * sizeof(float);
+    hipLaunchKernelGGL(k_conv_rows_any<T>,
+                       dim3(a.nd + a.nchunk * (CHUNK / ANY_R)), dim3(256), lds,
+                       st, a);
     hipLaunchKernelGGL(k_conv_ring, dim3(a.nd + a.nseg), dim3(256), 0, st, a,
                        a.s.xout ? a.s.xout : a.s.x);
   }
@@ -799,6 +889,7 @@ extern "C" hipError_t launch_conv_rows(int f32, const ConvRows* a,
                                        hipStream_t st) {
   if (bad_conv(a->s) || a->s.xout == a->s.x || !a->out || a->nd < 0 ||
       a->nchunk < 0 || a->nd + a->nchunk < 1 || !a->nseg != !a->nchunk ||
+      a->s.Kp % 64 || a->s.Kp >= a->s.W + 64 ||
       a->s.taps > 8192)
     return hipErrorInvalidValue;
   return f32 ? conv_rows<float>(*a, st) : conv_rows<u16>(*a, st);
@@ -846,7 +937,8 @@ static hipError_t lin_row_nr(const LinRowArgs& a, hipStream_t s) {
   constexpr int per = LIN_NT / 64 * NR;
   RAISE_LDS((k_lin_row<T, MODE, U, NR>));
   int blocks = (a.N + per - 1) / per;
-  if (blocks > 512) blocks = 512;
+  const int rounds = (blocks + 511) / 512;       // alike in every block
+  blocks = (blocks + rounds - 1) / rounds;
   hipLaunchKernelGGL((k_lin_row<T, MODE, U, NR>), dim3(blocks), dim3(LIN_NT),
                      MODE == ROW_PLAIN ? 0 : (size_t)a.s.Kp * sizeof(T), s, a);
   return hipGetLastError();
@@ -896,7 +988,10 @@ template <typename T>
 static void gemm_go(const GemmArgs& a, int Z, hipStream_t s) {
   long b128 = (long)((a.M + 127) / 128) * ((a.N + 127) / 128) * Z;
   dim3 sk((a.N + 15) / 16, 1, Z);
-  if (a.M <= 16 && sk.x * Z <= 256 && a.K >= 4096) {   // few blocks, deep K
+  if (a.M <= 16 && sk.x * Z <= 128 && a.K >= 4096) {   // few blocks, deep K
+    hipLaunchKernelGGL((k_gemm_skinny<T, 1, 16, 8>), dim3((a.N + 7) / 8, 1, Z),
+                       dim3(1024), 0, s, a);
+  } else if (a.M <= 16 && sk.x * Z <= 256 && a.K >= 4096) {
     hipLaunchKernelGGL((k_gemm_skinny<T, 1, 16>), sk, dim3(1024), 0, s, a);
   } else if (a.M <= 16) {
     hipLaunchKernelGGL((k_gemm_skinny<T, 1, 8>), sk, dim3(512), 0, s, a);

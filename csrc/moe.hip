@@ -6,17 +6,17 @@
 
 // logits of the rows; routed inside the gate/up kernel, or ahead of the sort
 struct RouteArgs {
-  const float* z;           // [rows, ldz]
+  const float* z;           // row r, expert e: z[r*ldz + e*lde]
   int* idx;                 // [rows*K1]
   float* wt;
-  int ldz, rows, E, top, extra, scores;
+  int ldz, lde, rows, E, top, extra, scores;
 };
 
 DEVINL void route(const RouteArgs& a, int r, int top, int extra, int* idx,
                   float* wt) {
   const float* z = a.z + (size_t)r * a.ldz;
-  if (a.E <= 64) route_row<1>(z, a.E, top, extra, idx, wt, a.scores);
-  else route_row<16>(z, a.E, top, extra, idx, wt, a.scores);
+  if (a.E <= 64) route_row<1>(z, a.E, top, extra, idx, wt, a.scores, a.lde);
+  else route_row<16>(z, a.E, top, extra, idx, wt, a.scores, a.lde);
 }
 
 __global__ void __launch_bounds__(256) k_moe_route(RouteArgs a) {
@@ -248,7 +248,7 @@ extern "C" hipError_t launch_block_out(int f32, const void* Wo, const void* o,
 
 static bool bad_route(const MoeArgs& m, const RouteArgs& a) {
   return bad_shape(m) || a.rows < 1 || a.E != m.E || a.E > 1024 ||
-         a.ldz < a.E || a.top < 1 || a.top > a.E || a.top + a.extra != m.K1 ||
+         a.ldz < 1 || a.lde < 1 || a.top < 1 || a.top > a.E || a.top + a.extra != m.K1 ||
          !a.z || a.idx != m.idx || a.wt != m.wt;
 }
 

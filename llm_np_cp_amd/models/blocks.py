@@ -126,8 +126,9 @@ class PostNormBlock(Block):
         self.mixer.out(eng, b, self)
         eng.pend = self.g1
         if self.ff:
-            eng.conv_project(self.ff.up, self.c2.w, cache[2], b, eng.P)
-            self.ff.after_up(eng, b)
+            across = eng.conv_project(self.ff.up, self.c2.w, cache[2], b,
+                                      eng.P, self.ff.experts is not None)
+            self.ff.after_up(eng, b, across)
             eng.pend = self.g2
 
 

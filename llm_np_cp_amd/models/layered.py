@@ -323,9 +323,10 @@ class LayeredModel(DecodeLoop):
             hy.norm_rows(src, g, staged, T, W, K, eps, gate=gate, ldg=ldg)
             hy.gemm_rows(staged, w, out, T, K, N, hy.EPI_F32)
 
-    def conv_project(self, w, kernel, ring, b: Rows, out):
+    def conv_project(self, w, kernel, ring, b: Rows, out, narrow=False):
         """out[T, N] fp32 = w . (v + conv(v)), v the residual with what is
-        pending on it; the staged input stays in self.h."""
+        pending on it; the staged input stays in self.h.  True where a
+        `narrow` w (up to 64 rows) ran as the other operand: out[N, T]."""
         (N, K), W, eps, T = w.shape, self.W, self.cfg.norm_eps, b.T
         kw = self._pending()
         keep = bool(kw)
@@ -338,9 +339,15 @@ class LayeredModel(DecodeLoop):
                        **kw)
         else:
             hy.conv_rows(self.x, self.h, b, W, K, eps, conv, **kw)
-            hy.gemm_rows(self.h, w, out, T, K, N, hy.EPI_F32)
         if keep:
             self.x, self.xb = self.xb, self.x
+        if self.one_row(w, T):
+            return False
+        if narrow and N <= 64 < T:
+            hy.gemm_rows(w, self.h, out, N, K, T, hy.EPI_F32, N=T)
+            return True
+        hy.gemm_rows(self.h, w, out, T, K, N, hy.EPI_F32)
+        return False
 
     def poly_linear(self, w, z, W: int, coef, staged, out, T: int):
         """out[T, N] fp32 = w . polynorm(z), rows of W values in z."""

@@ -96,18 +96,19 @@ class RoutedExperts:
     def bind(self, eng):
         return self.args.put(h=eng.h, idx=eng.ridx, wt=eng.rwt, act=eng.act)
 
-    def route(self, eng, T: int):
-        """Routing of the logits in eng.P."""
+    def route(self, eng, T: int, across: bool):
+        """Routing of the logits in eng.P, [T, E] or (across) [E, T]."""
         E = self.spec.experts
         return hy.RouteArgs().put(
-            z=eng.P, idx=eng.ridx, wt=eng.rwt, ldz=E, rows=T, E=E,
+            z=eng.P, idx=eng.ridx, wt=eng.rwt, ldz=1 if across else E,
+            lde=T if across else 1, rows=T, E=E,
             top=self.top, extra=self.extra,
             scores=int(self.spec.score == "sigmoid"))
 
-    def apart(self, eng, T: int, few: bool):
+    def apart(self, eng, T: int, few: bool, across: bool):
         """eng.y = the experts' sum for the rows of eng.h, from the logits
         in eng.P."""
-        m, route = self.bind(eng), self.route(eng, T)
+        m, route = self.bind(eng), self.route(eng, T, across)
         if few and T <= FUSE:
             hy.moe_gu_few(eng.f32, m, route)
             hy.block_out(eng.f32, None, None, 0, m, self.K1, eng.y, T, eng.W,
@@ -593,7 +594,7 @@ class DenseFF:
         self.act_floats = self.ffp
         self.p_floats = self.ffp if self.coef is not None else 0
 
-    def after_up(self, eng, b):
+    def after_up(self, eng, b, across):
         """eng.y from the up products in eng.P, a polynomial activation of
         the whole row between the two matrices."""
         eng.poly_linear(self.down, eng.P, self.ff, self.coef, eng.act,
@@ -609,8 +610,8 @@ class RoutedFF:
         self.act_floats = self.experts.K1 * self.experts.ffm
         self.p_floats = spec.experts
 
-    def after_up(self, eng, b):
-        self.experts.apart(eng, b.T, b.nseg == 0)
+    def after_up(self, eng, b, across):
+        self.experts.apart(eng, b.T, b.nseg == 0, across)
 
 
 FEED_FORWARDS = {"dense": DenseFF, "moe": RoutedFF}

@@ -100,7 +100,7 @@ MoeArgs = _struct(
     "MoeArgs", (_p, "h gu down idx wt act"),
     (_i, "ldh ldact W E K1 ff ffs glu win"), (_f, "lim lims"))
 RouteArgs = _struct(
-    "RouteArgs", (_p, "z idx wt"), (_i, "ldz rows E top extra scores"))
+    "RouteArgs", (_p, "z idx wt"), (_i, "ldz lde rows E top extra scores"))
 MoeSort = _struct(
     "MoeSort", (_p, "perm tile_e tile_row0 tile_n"),
     (_i, "pairs groups bm maxtiles"))

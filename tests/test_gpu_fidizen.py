@@ -57,7 +57,7 @@ def _batch(nd, runs, slots, pos):
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("taps", [1, 2, 3, 4, 5, 9, 13])
-@pytest.mark.parametrize("width", [40, 66, 1029, 2048])
+@pytest.mark.parametrize("width", [40, 66, 1029, 2048, 3000, 4096, 4100])
 def test_input_convolution_of_rows(dtype, taps, width):
     """Post norm + addition + convolution, single tokens beside runs, at
     the start of a sequence and later, and the inputs left for later."""
@@ -223,7 +223,7 @@ def test_launchers_refuse_bad_shapes():
         m = hy.MoeArgs().put(idx=i, wt=t, ldh=64, ldact=64, W=64, E=2, K1=3,
                              ff=64, ffs=64)
         hy.moe_gu_few(1, m, hy.RouteArgs().put(z=t, idx=i, wt=t, ldz=2,
-                                               rows=1, E=2, top=3))
+                                               lde=1, rows=1, E=2, top=3))
     with pytest.raises(RuntimeError):
         hy.gemm_rows(t, t, t, 2, 64, 64, hy.EPI_ROTARY, rotary=hy.Rotary().put(
             split=33, RT=31, dims=2))
