@@ -331,32 +331,29 @@ __global__ void __launch_bounds__(NT) k_conv_rows(ConvRows a) {
   if (k.row0 != k.seg0 || B == 0) return;
   if (R == 1 || k.len == 1) {
     if (mine) *(f4v*)(ring + (size_t)(k.pos0 % TAPS) * W) = v[B];
-    return;
-  }
-  if constexpr (R > 1) {
-  // the run's last inputs
-  f4v xt[TAPS], yt[TAPS];
+  } else if constexpr (R > 1) {         // the run's last inputs
+    f4v xt[TAPS], yt[TAPS];
 #pragma unroll
-  for (int e = 0; e < N; e++) ss[e] = 0.f;
+    for (int e = 0; e < N; e++) ss[e] = 0.f;
 #pragma unroll
-  for (int e = 0; e < B; e++) {
-    const int row = k.seg0 + k.len - B + e;
-    const bool in = mine && row >= k.seg0;
-    xt[e] = in ? *(const f4v*)(s.x + (size_t)row * W + c0) : zero;
-    yt[e] = in && s.y ? *(const f4v*)(s.y + (size_t)row * W + c0) : zero;
-    ss[e] = square(yt[e]);
-  }
-  if (s.y) {
-    __syncthreads();                    // red[0] has been read
-    rms_all(ss);
-  }
+    for (int e = 0; e < B; e++) {
+      const int row = k.seg0 + k.len - B + e;
+      const bool in = mine && row >= k.seg0;
+      xt[e] = in ? *(const f4v*)(s.x + (size_t)row * W + c0) : zero;
+      yt[e] = in && s.y ? *(const f4v*)(s.y + (size_t)row * W + c0) : zero;
+      ss[e] = square(yt[e]);
+    }
+    if (s.y) {
+      __syncthreads();                  // red[0] has been read
+      rms_all(ss);
+    }
 #pragma unroll
-  for (int e = 0; e < B; e++) {
-    const int at = k.len - B + e;
-    if (mine && at >= 0)
-      *(f4v*)(ring + (size_t)((k.pos0 + at) % TAPS) * W) =
-          s.y ? mix4(xt[e], yt[e], gb, red[0][e]) : xt[e];
-  }
+    for (int e = 0; e < B; e++) {
+      const int at = k.len - B + e;
+      if (mine && at >= 0)
+        *(f4v*)(ring + (size_t)((k.pos0 + at) % TAPS) * W) =
+            s.y ? mix4(xt[e], yt[e], gb, red[0][e]) : xt[e];
+    }
   }
 }
 
