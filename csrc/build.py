@@ -14,6 +14,8 @@ and the paged mixed-batch kernels of the layer-list designs:
     latent     attention over a cache of latents
     gqa        grouped-query attention
     mlstm      matrix-memory LSTM
+    mingru     gated recurrence of single tokens' gates
+    ssd        state-space recurrence behind a short convolution
     rglru      gated linear recurrence behind a short convolution
     lightning  linear attention with a decay per head
     moe        routed experts
@@ -33,11 +35,14 @@ LIBS = {
     "latent": ["latent_attn.hip"],
     "gqa": ["gqa_attn.hip"],
     "mlstm": ["mlstm.hip"],
+    "mingru": ["mingru.hip"],
+    "ssd": ["ssd.hip"],
     "rglru": ["rglru.hip"],
     "lightning": ["lightning.hip"],
     "moe": ["moe.hip"],
 }
-HEADERS = ["attn_split.h", "common.h", "gemm_tile.h", "hybrid.h", "moe.h"]
+HEADERS = ["attn_split.h", "common.h", "gemm_tile.h", "hybrid.h", "mingru.h",
+           "moe.h"]
 # Packed fp32 VALU forms are kept out of all device code: some of them
 # have returned wrong results on this hardware.  (The host pass warns that
 # it does not know the feature.)

@@ -1,6 +1,9 @@
 // gqa_attn.hip — grouped-query attention over a paged cache, without
-// rotation: RMS norm over the whole query and key projections, a query
-// factor per position, a sigmoid gate per output element.
+// rotation: RMS norm over the whole query and key projections; as options
+// a query factor per position, a sigmoid gate per output element, chunks
+// (a token sees the earlier ones of its own chunk of positions), a bias by
+// head and distance, a sink per head in the softmax.  Where values are the
+// projected keys ahead of their norm, ov is ok.
 //
 // Page p of a sequence holds positions 64p .. 64p+63, per key/value head as
 //   K [64, DP]   a key per row, zero-padded from dim to DP
@@ -13,6 +16,7 @@
 #include "attn_split.h"
 #include "gemm_tile.h"
 #include "hybrid.h"
+#include "mingru.h"
 
 #define PAGE 64
 #define TILE_PAIRS 64        // (token, head) pairs of a block over runs
@@ -20,7 +24,10 @@
 struct GqaArgs {
   const float* P;            // fp32 projections [rows, ldp], biases added
   const float *qnorm, *knorm;   // [H*d], [G*d]
-  const float* temp;         // query factor per position
+  const float* temp;         // query factor per position, nullable
+  const float* bias;         // nullable: [H, nbias] by distance, the last entry
+                             // for all beyond it; base-2 exponents
+  const float* sink;         // nullable: [H], base-2 exponents
   const int *slot, *pos;     // per row
   const int* table;          // [slots, ldt] page numbers
   void *K, *V;               // [pages, G, 64, DP], [pages, G, VP, 64]
@@ -29,11 +36,17 @@ struct GqaArgs {
   void* o;                   // [rows, ldo]
   const int *seg_row0, *seg_len, *seg_slot, *seg_pos0;
   const int *tile_seg, *tile_rr0;
-  int ldp, oq, ok, ov, og;
+  int ldp, oq, ok, ov, og;   // og < 0: no gate
   int H, G, d, vd, DP, VP, ldo, ldt;
   int rows, rbase, NS;       // rows [rbase, rbase+rows) take part
+  int chunk, nbias;          // chunk 0: every earlier position is seen
   float eps, scale;
 };
+
+// first position that position p sees
+DEVINL int first_seen(const GqaArgs& a, int p) {
+  return a.chunk ? p - p % a.chunk : 0;
+}
 
 // place of key j (0..63) in a row of V: inside each 32, score fragment i,
 // lane group g, register r hold key 16i + 4g + r
@@ -110,7 +123,7 @@ __global__ void __launch_bounds__(256) k_gqa_prep(GqaArgs a, int vblocks) {
   __syncthreads();
   sq = red[0][0] + red[0][1] + red[0][2] + red[0][3];
   sk = red[1][0] + red[1][1] + red[1][2] + red[1][3];
-  const float rq = a.temp[pos] / sqrtf(sq / (float)nq + a.eps);
+  const float rq = (a.temp ? a.temp[pos] : 1.f) / sqrtf(sq / (float)nq + a.eps);
   const float rk = 1.f / sqrtf(sk / (float)nk + a.eps);
   T* q = (T*)a.q + r * a.H * a.DP;
   if (a.d == a.DP) {                       // no padding: elements stay put
@@ -216,7 +229,9 @@ __global__ void __launch_bounds__(256) k_gqa_token(GqaArgs a) {
   const float* p = a.P + (size_t)r * a.ldp;
   const int pos = a.pos[r], kend = pos + 1;
   const int* pages = a.table + (size_t)a.slot[r] * a.ldt;
-  const int ngroup = (kend + 127) / 128, split = blockIdx.y;
+  // groups from the first key that is seen
+  const int k_lo = first_seen(a, pos), g0 = k_lo / 128;
+  const int ngroup = (kend + 127) / 128 - g0, split = blockIdx.y;
   const size_t orow = (size_t)r * a.H + h0;
   const size_t n = (size_t)a.rows * a.H;
   if (split >= ngroup) {
@@ -225,7 +240,7 @@ __global__ void __launch_bounds__(256) k_gqa_token(GqaArgs a) {
     return;
   }
   const float rq =
-      a.temp[pos] / sqrtf(sum_squares(p + a.oq, a.H * a.d, red) /
+      (a.temp ? a.temp[pos] : 1.f) / sqrtf(sum_squares(p + a.oq, a.H * a.d, red) /
                               (float)(a.H * a.d) + a.eps);
   if ((ngroup - 1) % a.NS == split) {
     // blocks of one key/value head (nqt > 1) write the same values
@@ -248,10 +263,17 @@ __global__ void __launch_bounds__(256) k_gqa_token(GqaArgs a) {
   for (int d = 0; d < ND; d++) acc[d] = {0.f, 0.f, 0.f, 0.f};
   float mrun = -INFINITY, lrun = 0.f;
   const float sc = a.scale * 1.4426950408889634f;       // base-2 exponents
+  const int hq = h0 + min(qc, nq - 1);                  // this lane's head
+  if (a.sink && split == 0 && wave == 0) {
+    mrun = a.sink[hq];
+    lrun = 1.f;
+  }
+  const float* bias = a.bias ? a.bias + (size_t)hq * a.nbias : nullptr;
 
-  for (int grp = split; grp < ngroup; grp += a.NS) {
+  for (int grp = g0 + split; grp < g0 + ngroup; grp += a.NS) {
     const int k0 = grp * 128 + wave * 32;
     if (k0 >= kend) break;
+    if (k0 + 32 <= k_lo) continue;
     const size_t pg = (size_t)pages[k0 / PAGE] * a.G + kv;
     const char* K = (const char*)((const T*)a.K +
                                   (pg * PAGE + k0 % PAGE + qc) * DP) + g * 16;
@@ -268,6 +290,12 @@ __global__ void __launch_bounds__(256) k_gqa_token(GqaArgs a) {
 #pragma unroll
       for (int u = 0; u < VV; u++)
         vf[d][u] = ld16(V + (size_t)d * 16 * PAGE * SZ + u * 16);
+    float bv[8];
+#pragma unroll
+    for (int i = 0; i < 8; i++) {
+      const int n = pos - (k0 + (i >> 2) * 16 + g * 4 + (i & 3));
+      bv[i] = bias ? bias[min(max(n, 0), a.nbias - 1)] : 0.f;
+    }
     f4v st[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
     for (int c = 0; c < NC; c++)
@@ -276,9 +304,11 @@ __global__ void __launch_bounds__(256) k_gqa_token(GqaArgs a) {
         st[i] = GemmMma<T>::mma(kf[i][c], qf[c], st[i]);
     float sv[8];
 #pragma unroll
-    for (int i = 0; i < 8; i++)
-      sv[i] = k0 + (i >> 2) * 16 + g * 4 + (i & 3) < kend
-                  ? st[i >> 2][i & 3] * sc : -INFINITY;
+    for (int i = 0; i < 8; i++) {
+      const int key = k0 + (i >> 2) * 16 + g * 4 + (i & 3);
+      sv[i] = key < kend && key >= k_lo ? fmaf(st[i >> 2][i & 3], sc, bv[i])
+                                        : -INFINITY;
+    }
     const float alpha = softmax_step<8>(sv, mrun, lrun);
     if (k0 + 32 > kend)
 #pragma unroll
@@ -302,7 +332,7 @@ __global__ void __launch_bounds__(256) k_gqa_token(GqaArgs a) {
   for (int w = 1; w < 4; w++) mt = fmaxf(mt, ms[w][qc]);
 #pragma unroll
   for (int w = 0; w < 4; w++) lt += exp2f(ms[w][qc] - mt) * ls[w][qc];
-  const float mine = exp2f(mrun - mt);
+  const float mine = exp2f(mrun - mt);          // some wave has seen a key
 #pragma unroll
   for (int half = 1; half >= 0; half--) {       // waves 2, 3, then 0, 1
     if (wave >> 1 == half)
@@ -329,7 +359,7 @@ __global__ void __launch_bounds__(256) k_gqa_token(GqaArgs a) {
 // 4 waves of 16 (token, head) pairs over key tiles of KT keys in LDS,
 // double-buffered by global_load_lds; 16-byte slots are XOR-swizzled by
 // the row, in the source address of the DMA and in the fragment reads.
-template <typename T, int DP, int VP>
+template <typename T, int DP, int VP, bool BIAS>
 __global__ void __launch_bounds__(256) k_gqa_run(GqaArgs a) {
   constexpr int SZ = sizeof(T), NC = DP * SZ / 64, ND = VP / 16, VV = SZ / 2;
   constexpr int KT = 128 / SZ, NG = KT / 32;    // 64 keys in bf16, 32 in fp32
@@ -347,9 +377,13 @@ __global__ void __launch_bounds__(256) k_gqa_run(GqaArgs a) {
   const int tok = myc / R, h = kv * R + myc - tok * R, qpos = pos0 + tok;
   const int kend = pos0 + (min(rr0 + TILE_PAIRS, nrr) - 1) / R + 1;
   const int wlast = pos0 + min(rr0 + wave * 16 + 15, nrr - 1) / R;
+  // first keys that this lane's token, the wave's first and the block's see
+  const int k_lo = first_seen(a, qpos);
+  const int w_lo = first_seen(a, pos0 + min(rr0 + wave * 16, nrr - 1) / R);
+  const int t0 = first_seen(a, pos0 + rr0 / R) / KT;
   const int ntile = (kend + KT - 1) / KT;
-  const int per = (ntile + a.NS - 1) / a.NS;
-  const int t_lo = blockIdx.z * per, t_hi = min(ntile, t_lo + per);
+  const int per = (ntile - t0 + a.NS - 1) / a.NS;
+  const int t_lo = t0 + blockIdx.z * per, t_hi = min(ntile, t_lo + per);
 
   auto stage = [&](int buf, int t) {
     const size_t pg = (size_t)pages[t * KT / PAGE] * a.G + kv;
@@ -380,6 +414,10 @@ __global__ void __launch_bounds__(256) k_gqa_run(GqaArgs a) {
     }
   };
   if (t_lo < t_hi) stage(0, t_lo);
+  float* bl = (float*)(lds + 2 * (KB + VB));     // the group's biases
+  for (int i = tid; i < (BIAS ? R * a.nbias : 0); i += 256)
+    bl[i] = a.bias[(size_t)kv * R * a.nbias + i];
+  const float* bias = bl + (h - kv * R) * a.nbias;
   f4v qf[NC], acc[ND];
   const char* qp = (const char*)((const T*)a.q +
                                  ((size_t)(row0 + tok) * a.H + h) * DP);
@@ -388,6 +426,10 @@ __global__ void __launch_bounds__(256) k_gqa_run(GqaArgs a) {
 #pragma unroll
   for (int d = 0; d < ND; d++) acc[d] = {0.f, 0.f, 0.f, 0.f};
   float mrun = -INFINITY, lrun = 0.f;
+  if (a.sink && blockIdx.z == 0) {
+    mrun = a.sink[h];
+    lrun = 1.f;
+  }
   const float sc = a.scale * 1.4426950408889634f;
   __syncthreads();
 
@@ -395,7 +437,7 @@ __global__ void __launch_bounds__(256) k_gqa_run(GqaArgs a) {
   for (int t = t_lo; t < t_hi; t++) {
     if (t + 1 < t_hi) stage(cur ^ 1, t + 1);
     const int k0 = t * KT;
-    if (k0 <= wlast) {
+    if (k0 <= wlast && k0 + KT > w_lo) {
       const char* kl = lds + cur * (KB + VB);
       const char* vl = kl + KB;
       float sv[8 * NG];
@@ -412,10 +454,12 @@ __global__ void __launch_bounds__(256) k_gqa_run(GqaArgs a) {
                 qf[c], st[i]);
           }
 #pragma unroll
-        for (int i = 0; i < 8; i++)
-          sv[j * 8 + i] =
-              k0 + j * 32 + (i >> 2) * 16 + g * 4 + (i & 3) <= qpos
-                  ? st[i >> 2][i & 3] * sc : -INFINITY;
+        for (int i = 0; i < 8; i++) {
+          const int n = qpos - (k0 + j * 32 + (i >> 2) * 16 + g * 4 + (i & 3));
+          float v = st[i >> 2][i & 3] * sc;
+          if constexpr (BIAS) v += bias[min(max(n, 0), a.nbias - 1)];
+          sv[j * 8 + i] = n >= 0 && n <= qpos - k_lo ? v : -INFINITY;
+        }
       }
       const float alpha = softmax_step<8 * NG>(sv, mrun, lrun);
       if (__any(alpha != 1.f)) {
@@ -447,14 +491,16 @@ __global__ void __launch_bounds__(256) k_gqa_run(GqaArgs a) {
   const size_t r = row0 + tok;
   if (a.NS == 1) {
     const float inv = 1.f / lrun;
-    const float* gate = a.P + r * a.ldp + a.og + h * a.vd;
+    const float* gate =
+        a.og < 0 ? nullptr : a.P + r * a.ldp + a.og + h * a.vd;
     T* o = (T*)a.o + r * a.ldo + h * a.vd;
 #pragma unroll
     for (int d = 0; d < ND; d++)
 #pragma unroll
       for (int j = 0; j < 4; j++) {
         const int i = d * 16 + g * 4 + j;
-        if (i < a.vd) o[i] = El<T>::st(acc[d][j] * inv * sigmoid_f(gate[i]));
+        if (i < a.vd)
+          o[i] = El<T>::st(acc[d][j] * inv * (gate ? sigmoid_f(gate[i]) : 1.f));
       }
   } else {
     const size_t pr = (size_t)blockIdx.z * a.rows * a.H +
@@ -471,17 +517,24 @@ __global__ void __launch_bounds__(256) k_gqa_run(GqaArgs a) {
   }
 }
 
-// merge the splits and gate, one block per (row, head)
+// merge the splits and gate, one block per (row, head); further blocks step
+// a gated recurrence that stands beside the attention
 template <typename T>
-__global__ void __launch_bounds__(256) k_gqa_merge(GqaArgs a) {
+__global__ void __launch_bounds__(256) k_gqa_merge(GqaArgs a, MingruArgs m) {
   __shared__ __attribute__((aligned(16))) float sh[MERGE_LDS];
+  const int beside = (int)blockIdx.x - a.rows * a.H;
+  if (beside >= 0) {
+    mingru_token<T>(m, beside);
+    return;
+  }
   const int rl = blockIdx.x / a.H, h = blockIdx.x - rl * a.H;
   const size_t r = a.rbase + rl;
-  const float* gate = a.P + r * a.ldp + a.og + h * a.vd;
+  const float* gate = a.og < 0 ? nullptr : a.P + r * a.ldp + a.og + h * a.vd;
   T* o = (T*)a.o + r * a.ldo + h * a.vd;
   merge_splits(a.part, a.ml, (size_t)a.rows * a.H, blockIdx.x, a.NS, a.VP, sh,
                [&](int i, float v) {
-                 if (i < a.vd) o[i] = El<T>::st(v * sigmoid_f(gate[i]));
+                 if (i < a.vd)
+                   o[i] = El<T>::st(v * (gate ? sigmoid_f(gate[i]) : 1.f));
                });
 }
 
@@ -489,7 +542,8 @@ __global__ void __launch_bounds__(256) k_gqa_merge(GqaArgs a) {
 static bool bad_shape(const GqaArgs& a) {
   return a.rows < 1 || a.rbase < 0 || a.G < 1 || a.H < 1 || a.H % a.G ||
          a.d < 1 || a.d > a.DP || a.vd < 1 || a.vd > a.VP ||
-         a.ldo < a.H * a.vd || a.NS < 1 || a.NS > MAX_SPLITS;
+         a.ldo < a.H * a.vd || a.NS < 1 || a.NS > MAX_SPLITS || a.chunk < 0 ||
+         (a.bias && a.nbias < 1);
 }
 
 extern "C" hipError_t launch_gqa_prep(int f32, const GqaArgs* a,
@@ -509,11 +563,18 @@ static hipError_t attn_go(const GqaArgs& a, int tiles, hipStream_t s) {
     hipLaunchKernelGGL((k_gqa_token<T, DP, VP>), dim3(a.rows * a.G * nqt, a.NS),
                        dim3(256), 0, s, a);
   } else {
-    constexpr size_t lds =
-        2 * ((128 / sizeof(T)) * DP * sizeof(T) + (size_t)VP * 128);
-    RAISE_LDS((k_gqa_run<T, DP, VP>));
-    hipLaunchKernelGGL((k_gqa_run<T, DP, VP>), dim3(tiles, a.G, a.NS),
-                       dim3(256), lds, s, a);
+    size_t lds = 2 * ((128 / sizeof(T)) * DP * sizeof(T) + (size_t)VP * 128);
+    if (a.bias) {
+      lds += (size_t)(a.H / a.G) * a.nbias * sizeof(float);
+      if (lds > 159 * 1024) return hipErrorInvalidValue;
+      RAISE_LDS((k_gqa_run<T, DP, VP, true>));
+      hipLaunchKernelGGL((k_gqa_run<T, DP, VP, true>), dim3(tiles, a.G, a.NS),
+                         dim3(256), lds, s, a);
+    } else {
+      RAISE_LDS((k_gqa_run<T, DP, VP, false>));
+      hipLaunchKernelGGL((k_gqa_run<T, DP, VP, false>), dim3(tiles, a.G, a.NS),
+                         dim3(256), lds, s, a);
+    }
   }
   return hipGetLastError();
 }
@@ -542,11 +603,15 @@ extern "C" hipError_t launch_gqa_run(int f32, const GqaArgs* a, int tiles,
   return f32 ? attn<float>(*a, tiles, s) : attn<u16>(*a, tiles, s);
 }
 
+// m (nullable): its single tokens take their step in the same launch
 extern "C" hipError_t launch_gqa_merge(int f32, const GqaArgs* a,
-                                       hipStream_t s) {
-  if (bad_shape(*a)) return hipErrorInvalidValue;
-  dim3 grid(a->rows * a->H);
-  if (f32) hipLaunchKernelGGL(k_gqa_merge<float>, grid, dim3(256), 0, s, *a);
-  else hipLaunchKernelGGL(k_gqa_merge<u16>, grid, dim3(256), 0, s, *a);
+                                      const MingruArgs* m, hipStream_t s) {
+  if (bad_shape(*a) || (m && (mingru_bad_shape(*m) || m->rows < 1)))
+    return hipErrorInvalidValue;
+  const MingruArgs side = m ? *m : MingruArgs{};
+  dim3 grid(a->rows * a->H + (m ? mingru_token_blocks(side) : 0));
+  if (f32)
+    hipLaunchKernelGGL(k_gqa_merge<float>, grid, dim3(256), 0, s, *a, side);
+  else hipLaunchKernelGGL(k_gqa_merge<u16>, grid, dim3(256), 0, s, *a, side);
   return hipGetLastError();
 }

@@ -20,6 +20,48 @@ k_embed_rows(const T* __restrict__ table, const int* __restrict__ ids,
   }
 }
 
+// ---- embedding of tokens and token pairs ---------------------------------
+// x = table[cur] + pairs[(before * mul_before + cur * mul_cur) mod buckets],
+// the last row of pairs at position 0, once for each of S streams.  The token
+// before a sequence's next one is kept in last[slot]; the runs' last tokens
+// are written by a launch of their own, since their first rows read the entry.
+struct PairEmbed {
+  const void *table, *pairs;   // [vocab, W], [buckets + 1, W]
+  const int *ids, *slot, *pos;
+  int* last;                   // [slots]
+  float* x;                    // [rows, S, W]
+  const int *seg_row0, *seg_len, *seg_slot;   // runs
+  long mul_before, mul_cur;
+  int W, S, M, nd, nseg, buckets;   // rows [0, nd) are single tokens
+};
+
+template <typename T>
+__global__ void __launch_bounds__(256) k_embed_pairs(PairEmbed a) {
+  const int r = blockIdx.x, W = a.W, cur = a.ids[r], slot = a.slot[r];
+  long row = a.buckets;
+  if (a.pos[r] > 0) {
+    const bool inside = r > 0 && a.slot[r - 1] == slot;   // of a run
+    const long before = inside ? a.ids[r - 1] : a.last[slot];
+    row = (before * a.mul_before + cur * a.mul_cur) % a.buckets;
+  }
+  if (r < a.nd) {
+    __syncthreads();                     // everyone has the entry
+    if (threadIdx.x == 0) a.last[slot] = cur;
+  }
+  const T* t = (const T*)a.table + (size_t)cur * W;
+  const T* p = (const T*)a.pairs + (size_t)row * W;
+  for (int i = threadIdx.x; i < W; i += 256) {
+    const float v = El<T>::ld(t[i]) + El<T>::ld(p[i]);
+    for (int q = 0; q < a.S; q++) a.x[((size_t)r * a.S + q) * W + i] = v;
+  }
+}
+
+__global__ void __launch_bounds__(256) k_last_tokens(PairEmbed a) {
+  const int g = blockIdx.x * 256 + threadIdx.x;
+  if (g < a.nseg)
+    a.last[a.seg_slot[g]] = a.ids[a.seg_row0[g] + a.seg_len[g] - 1];
+}
+
 // ---- staging a row of the residual for a projection --------------------
 // v = x [+ y / rms(y) * gb] [+ xadd]            (y: the last sublayer's output)
 // out = v / rms(v) * g [* sigmoid(gate)]
@@ -164,6 +206,173 @@ DEVINL void stage_row(const RowStage& s, size_t row, bool keep, float* red,
   for (int u = 0; u < U; u++) finish(tid + u * NT, xv[u], gv[u]);
   for (int i = tid + U * NT; i < max(W, s.Kp); i += NT)
     finish(i, i < W ? late(i) : 0.f, s.g && i < W ? s.g[i] : 0.f);
+}
+
+// ---- staging a row of several residual streams ----------------------------
+// With the output y of the sublayer before (or two halves of it,
+// y = (y / rms(y) gb + y2 / rms(y2) gb2) / 2), all streams at once:
+//   x_t <- sum_s mix[s][t] x_s + feed[t] y
+// then u = sum_s in[s] x_s and out = u / rms(u) * g, g a single number.
+#define MAX_STREAMS 8
+struct HyperStage {
+  const float* x;           // [rows, S, W]
+  const float *y, *y2;      // nullable, [rows, W]
+  const float *gb, *gb2;    // with y2
+  const float *mix, *feed;  // with y: [S, S], [S]
+  const float *in, *g;      // [S], [1]; null: only xout is wanted
+  float* xout;              // nullable: receives the streams
+  int W, Kp, S;
+  float eps;
+};
+
+// HS streams, or s.S of them where HS is 0
+template <int NT, int U, int HS, class Put>
+DEVINL void stage_hyper(const HyperStage& s, size_t row, bool keep, float* red,
+                        Put put) {
+  constexpr int MS = HS ? HS : MAX_STREAMS;
+  const int tid = threadIdx.x, W = s.W, S = HS ? HS : s.S;
+  const float* x = s.x + row * S * W;
+  const float* y = s.y ? s.y + row * W : nullptr;
+  const float* y2 = s.y2 ? s.y2 + row * W : nullptr;
+  float xv[U][MS], yv[U], zv[U], ga[U], gc[U];
+#pragma unroll
+  for (int u = 0; u < U; u++) {
+    const int i = tid + u * NT;
+#pragma unroll
+    for (int t = 0; t < MS; t++)
+      xv[u][t] = t < S && i < W ? x[(size_t)t * W + i] : 0.f;
+    yv[u] = y && i < W ? y[i] : 0.f;
+    zv[u] = y2 && i < W ? y2[i] : 0.f;
+    ga[u] = y2 && i < W ? s.gb[i] : 0.f;
+    gc[u] = y2 && i < W ? s.gb2[i] : 0.f;
+  }
+  float ra = 1.f, rc = 0.f;
+  if (y2) {
+    float sa = 0.f, sc = 0.f;
+#pragma unroll
+    for (int u = 0; u < U; u++) {
+      sa += yv[u] * yv[u];
+      sc += zv[u] * zv[u];
+    }
+    for (int i = tid + U * NT; i < W; i += NT) {
+      sa += y[i] * y[i];
+      sc += y2[i] * y2[i];
+    }
+    ra = 0.5f / sqrtf(block_sum(sa, red) / (float)W + s.eps);
+    rc = 0.5f / sqrtf(block_sum(sc, red) / (float)W + s.eps);
+  }
+  // the streams of one element, and what the next sublayer reads of them
+  auto turn = [&](float (&v)[MS], float yo) {
+    if (y) {
+      float n[MS];
+#pragma unroll
+      for (int t = 0; t < MS; t++) {
+        n[t] = 0.f;
+        if (t < S) {
+          n[t] = s.feed[t] * yo;
+#pragma unroll
+          for (int q = 0; q < MS; q++)
+            if (q < S) n[t] = fmaf(s.mix[q * S + t], v[q], n[t]);
+        }
+      }
+#pragma unroll
+      for (int t = 0; t < MS; t++) v[t] = n[t];
+    }
+    float u = 0.f;
+    if (s.in)
+#pragma unroll
+      for (int t = 0; t < MS; t++)
+        if (t < S) u = fmaf(s.in[t], v[t], u);
+    return u;
+  };
+  auto late = [&](int i, float (&v)[MS]) {   // elements beyond the registers
+#pragma unroll
+    for (int t = 0; t < MS; t++) v[t] = t < S ? x[(size_t)t * W + i] : 0.f;
+    float yo = y ? y[i] : 0.f;
+    if (y2) yo = yo * ra * s.gb[i] + y2[i] * rc * s.gb2[i];
+    return turn(v, yo);
+  };
+  float uv[U], ss = 0.f;
+#pragma unroll
+  for (int u = 0; u < U; u++) {
+    const float yo = y2 ? yv[u] * ra * ga[u] + zv[u] * rc * gc[u] : yv[u];
+    uv[u] = turn(xv[u], yo);
+    ss += uv[u] * uv[u];
+  }
+  float rn = 0.f;
+  if (s.in) {
+    for (int i = tid + U * NT; i < W; i += NT) {
+      float v[MS];
+      const float u = late(i, v);
+      ss += u * u;
+    }
+    rn = s.g[0] / sqrtf(block_sum(ss, red) / (float)W + s.eps);
+  }
+  auto finish = [&](int i, float u, const float (&v)[MS]) {
+    if (s.in && i < s.Kp) put(i, i < W ? u * rn : 0.f);
+    if (keep && s.xout && i < W)         // may be x: its reads are done
+#pragma unroll
+      for (int t = 0; t < MS; t++)
+        if (t < S) s.xout[(row * S + t) * W + i] = v[t];
+  };
+#pragma unroll
+  for (int u = 0; u < U; u++) finish(tid + u * NT, uv[u], xv[u]);
+  for (int i = tid + U * NT; i < max(W, s.Kp); i += NT) {
+    float v[MS];
+    const float u = i < W ? late(i, v) : 0.f;
+    finish(i, u, v);
+  }
+}
+
+template <typename T, int U, int HS>
+__global__ void __launch_bounds__(256)
+k_hyper_rows(HyperStage s, const int* __restrict__ rows, T* __restrict__ out) {
+  __shared__ float red[4];
+  T* o = out + (size_t)blockIdx.x * s.Kp;
+  stage_hyper<256, U, HS>(s, rows ? rows[blockIdx.x] : blockIdx.x, true, red,
+                          [&](int i, float v) { o[i] = El<T>::st(v); });
+}
+
+// ---- staging a row normed in equal parts -----------------------------------
+// out = x / rms(x over its part) * g; rn holds MAX_GROUPS floats
+#define MAX_GROUPS 1024
+template <int NT, class Put>
+DEVINL void stage_groups(const RowStage& s, int groups, size_t row, float* rn,
+                         Put put) {
+  constexpr int NW = NT / 64;
+  const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, W = s.W;
+  const int gw = W / groups, parts = max(1, NW / groups);
+  const float* x = s.x + row * W;
+  for (int k = wave; k < groups * parts; k += NW) {
+    const int grp = k / parts, p = k - grp * parts;
+    float ss = 0.f;
+#pragma unroll 4
+    for (int i = p * 64 + lane; i < gw; i += parts * 64)
+      ss += x[grp * gw + i] * x[grp * gw + i];
+    ss = wave_reduce_sum(ss);
+    if (lane == 0) rn[k] = ss;
+  }
+  __syncthreads();
+#pragma unroll 4
+  for (int i = tid; i < s.Kp; i += NT) {
+    float v = 0.f;
+    if (i < W) {
+      float ss = 0.f;
+      const int grp = i / gw;
+      for (int p = 0; p < parts; p++) ss += rn[grp * parts + p];
+      v = x[i] / sqrtf(ss / (float)gw + s.eps) * s.g[i];
+    }
+    put(i, v);
+  }
+}
+
+template <typename T>
+__global__ void __launch_bounds__(256)
+k_group_rows(RowStage s, int groups, T* __restrict__ out) {
+  __shared__ float rn[MAX_GROUPS];
+  T* o = out + (size_t)blockIdx.x * s.Kp;
+  stage_groups<256>(s, groups, blockIdx.x, rn,
+                    [&](int i, float v) { o[i] = El<T>::st(v); });
 }
 
 // one block per row; `rows` (nullable) picks the source row of each output
@@ -499,12 +708,15 @@ k_cat_rows(const float* __restrict__ x, const float* __restrict__ x0,
 
 // ---- one row: y[n] = W[n] . staged row, one wave per NR outputs ----------
 // The row is staged into LDS as T: normed or convolved (stage_row),
-// concatenated [x | x0], or through the polynomial activation; block 0 can persist it to hout, and the residual to xout.  A row
-// that is T already (hin) is read where it lies.  A wave always has its
-// next slab of weights on the way, the first one during the staging.
+// concatenated [x | x0], through the polynomial activation, from several
+// streams (stage_hyper) or normed in parts; block 0 can persist it to hout,
+// and the residual to xout.  A row that is T already (hin) is read where it
+// lies; there blockIdx.y picks one of up to two products.  A wave always has
+// its next slab of weights on the way, the first one during the staging.
 enum { EPI_F32 = 0, EPI_RESADD = 1, EPI_SOFTCAP = 2, EPI_T = 3, EPI_TGATE = 4,
-       EPI_RELU2 = 5, EPI_ROTARY = 6 };
-enum { ROW_NORM = 0, ROW_CAT = 1, ROW_PLAIN = 2, ROW_CONV = 3, ROW_POLY = 4 };
+       EPI_RELU2 = 5, EPI_ROTARY = 6, EPI_GELU = 7 };
+enum { ROW_NORM = 0, ROW_CAT = 1, ROW_PLAIN = 2, ROW_CONV = 3, ROW_POLY = 4,
+       ROW_HYPER = 5, ROW_GROUPS = 6 };
 
 struct LinRowArgs {
   const void* Wt;           // [N, Kp]
@@ -514,32 +726,42 @@ struct LinRowArgs {
   void* hout;               // nullable
   const float* bias;        // nullable
   const float* act;         // ROW_POLY: four coefficients; the row is s.x
-  void* y;                  // fp32, or T for EPI_RELU2
+  void* y;                  // fp32, or T for EPI_RELU2 and EPI_GELU
   int N, stage, epi;
   float cap;
+  int groups;               // ROW_GROUPS
+  int Z, K2;                // ROW_PLAIN: products, and K of the second,
+  long xz, wz, yz;          // which lies this many elements further on
+  HyperStage h;             // ROW_HYPER (s has W and Kp, too)
 };
 
 DEVINL float relu2_f(float v) {
   v = fmaxf(v, 0.f);
   return v * v;
 }
+DEVINL float gelu_f(float v) {
+  return 0.5f * v * (1.f + erff(v * 0.7071067811865476f));
+}
 
 #define LIN_NT 512
-template <typename T, int MODE, int U, int NR>
+template <typename T, int MODE, int U, int NR, int HS = 0>
 __global__ void __launch_bounds__(LIN_NT) k_lin_row(LinRowArgs a) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  __shared__ float red[LIN_NT / 64 * (MODE == ROW_POLY ? 3 : 1)];
+  __shared__ float red[MODE == ROW_GROUPS ? MAX_GROUPS
+                                          : LIN_NT / 64 * (MODE == ROW_POLY ? 3 : 1)];
   constexpr int V = El<T>::V, S = 64 * V, NK = 8 / NR;
   T* xs = (T*)smem;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
-  const int N = a.N, Kp = a.s.Kp;
+  const int z = MODE == ROW_PLAIN ? blockIdx.y : 0;
+  const int N = a.N, Kp = z ? a.K2 : a.s.Kp;
+  const T* Wt = (const T*)a.Wt + (MODE == ROW_PLAIN ? z * a.wz : 0);
   const int step = gridDim.x * (LIN_NT / 64) * NR;
   int n = (blockIdx.x * (LIN_NT / 64) + wave) * NR, k0 = 0;
   f4v w[NR][NK], next[NR][NK];
   auto slab = [&](f4v (&to)[NR][NK], int n0, int kb) {
 #pragma unroll
     for (int i = 0; i < NR; i++) {
-      const T* wr = (const T*)a.Wt + (size_t)min(n0 + i, N - 1) * Kp;
+      const T* wr = Wt + (size_t)min(n0 + i, N - 1) * Kp;
 #pragma unroll
       for (int u = 0; u < NK; u++) {
         const int k = kb + u * S + lane * V;
@@ -557,6 +779,15 @@ __global__ void __launch_bounds__(LIN_NT) k_lin_row(LinRowArgs a) {
       xs[i] = v;
       if (a.hout && first) ((T*)a.hout)[i] = v;
     });
+  } else if constexpr (MODE == ROW_HYPER) {
+    stage_hyper<LIN_NT, U, HS>(a.h, row, first, red, [&](int i, float f) {
+      T v = El<T>::st(f);
+      xs[i] = v;
+      if (a.hout && first) ((T*)a.hout)[i] = v;
+    });
+  } else if constexpr (MODE == ROW_GROUPS) {
+    stage_groups<LIN_NT>(a.s, a.groups, row, red,
+                         [&](int i, float f) { xs[i] = El<T>::st(f); });
   } else if constexpr (MODE == ROW_POLY) {
     const int W = a.s.W;
     const float* z = a.s.x + row * W;
@@ -581,7 +812,7 @@ __global__ void __launch_bounds__(LIN_NT) k_lin_row(LinRowArgs a) {
     for (int i = tid; i < Kp; i += LIN_NT)
       xs[i] = El<T>::st(i < W ? x[i] : i < 2 * W ? x0[i - W] : 0.f);
   }
-  const T* xr = MODE == ROW_PLAIN ? (const T*)a.hin : xs;
+  const T* xr = MODE == ROW_PLAIN ? (const T*)a.hin + z * a.xz : xs;
   if (MODE != ROW_PLAIN) __syncthreads();
   float acc[NR];
 #pragma unroll
@@ -611,6 +842,8 @@ __global__ void __launch_bounds__(LIN_NT) k_lin_row(LinRowArgs a) {
           if (a.bias) v += a.bias[n + i];
           if (a.cap > 0.f) v = a.cap * tanhf(v / a.cap);
           if (a.epi == EPI_RELU2) ((T*)a.y)[n + i] = El<T>::st(relu2_f(v));
+          else if (a.epi == EPI_GELU) ((T*)a.y)[n + i] = El<T>::st(gelu_f(v));
+          else if (MODE == ROW_PLAIN) ((float*)a.y)[z * a.yz + n + i] = v;
           else ((float*)a.y)[n + i] = v;
         }
       }
@@ -641,6 +874,7 @@ struct GemmArgs {
   int M, N, K, ldx, ldw, ldy, ldg, epi, gz, gc;
   float mult;               // EPI_RESADD multiplier / EPI_SOFTCAP cap
   long xz, wz, yz;          // per-z (head) element offsets
+  int K2;                   // K, and ldw, of z > 0
   struct Rotary r;          // EPI_ROTARY
 };
 
@@ -654,6 +888,7 @@ DEVINL void gemm_store(const GemmArgs& a, int z, int row, int col, float v) {
     ((float*)a.Y)[o] = a.mult > 0.f ? a.mult * tanhf(v / a.mult) : v;
   else if constexpr (EPI == EPI_T) ((T*)a.Y)[o] = El<T>::st(v);
   else if constexpr (EPI == EPI_RELU2) ((T*)a.Y)[o] = El<T>::st(relu2_f(v));
+  else if constexpr (EPI == EPI_GELU) ((T*)a.Y)[o] = El<T>::st(gelu_f(v));
   else
     ((T*)a.Y)[o] = El<T>::st(
         v * sigmoid_f(a.gate[(size_t)row * a.ldg + z * a.gz + col * a.gc]));
@@ -705,6 +940,7 @@ template <class Body> DEVINL void with_epilogue(int epi, Body body) {
     case EPI_TGATE: body(std::integral_constant<int, EPI_TGATE>()); break;
     case EPI_RELU2: body(std::integral_constant<int, EPI_RELU2>()); break;
     case EPI_ROTARY: body(std::integral_constant<int, EPI_ROTARY>()); break;
+    case EPI_GELU: body(std::integral_constant<int, EPI_GELU>()); break;
   }
 }
 
@@ -714,12 +950,13 @@ __global__ void __launch_bounds__(256) k_gemm(GemmArgs a) {
   const int bm = blockIdx.y * BM, bn = blockIdx.x * BN, z = blockIdx.z;
   const T* X = (const T*)a.X + (size_t)z * a.xz;
   const T* W = (const T*)a.W + (size_t)z * a.wz;
+  const int K = z ? a.K2 : a.K, ldw = z ? a.K2 : a.ldw;
   f4v acc[BM / 32][BN / 32];
   gemm_mainloop<BM, BN, T>(
       acc, lds,
       [&](int r) { return X + (size_t)min(bm + r, a.M - 1) * a.ldx; },
-      [&](int r) { return W + (size_t)min(bn + r, a.N - 1) * a.ldw; }, 0,
-      a.K / GemmMma<T>::BK);
+      [&](int r) { return W + (size_t)min(bn + r, a.N - 1) * ldw; }, 0,
+      K / GemmMma<T>::BK);
   float bias[BN / 32];
 #pragma unroll
   for (int j = 0; j < BN / 32; j++)
@@ -748,9 +985,10 @@ __global__ void __launch_bounds__(64 * NW) k_gemm_skinny(GemmArgs a) {
   constexpr int U = MF == 1 ? 8 : 4;
   const int tid = threadIdx.x, wave = wave_index(), lane = tid & 63;
   const int lr = lane & 15, gq = lane >> 4, z = blockIdx.z;
-  const int n0 = blockIdx.x * NB, nch = a.K * (int)sizeof(T) / 64;
+  const int K = z ? a.K2 : a.K, ldw = z ? a.K2 : a.ldw;
+  const int n0 = blockIdx.x * NB, nch = K * (int)sizeof(T) / 64;
   const char* wr = (const char*)((const T*)a.W + (size_t)z * a.wz +
-                                 (size_t)min(n0 + lr, a.N - 1) * a.ldw) +
+                                 (size_t)min(n0 + lr, a.N - 1) * ldw) +
                    gq * 16;
   const char* xr[MF];
 #pragma unroll
@@ -811,6 +1049,72 @@ extern "C" hipError_t launch_embed_rows(int f32, const void* table,
           hipLaunchKernelGGL(k_embed_rows<float>, dim3(M), dim3(256), 0, s,
                              (const float*)table, (const int*)ids, (float*)x,
                              (float*)x0, W, scale));
+  return hipGetLastError();
+}
+
+extern "C" hipError_t launch_embed_pairs(int f32, const PairEmbed* a,
+                                         hipStream_t s) {
+  if (a->M < 1 || a->W < 1 || a->S < 1 || a->nd < 0 || a->nd > a->M ||
+      a->nseg < 0 || a->buckets < 1 || a->mul_before < 0 || a->mul_cur < 0)
+    return hipErrorInvalidValue;
+  BY_TYPE(f32,
+          hipLaunchKernelGGL(k_embed_pairs<u16>, dim3(a->M), dim3(256), 0, s, *a),
+          hipLaunchKernelGGL(k_embed_pairs<float>, dim3(a->M), dim3(256), 0, s,
+                             *a));
+  if (a->nseg)
+    hipLaunchKernelGGL(k_last_tokens, dim3((a->nseg + 255) / 256), dim3(256), 0,
+                       s, *a);
+  return hipGetLastError();
+}
+
+static bool bad_hyper(const HyperStage& s) {
+  return s.W < 1 || s.S < 1 || s.S > MAX_STREAMS || !s.x || !s.in != !s.g ||
+         (s.in && s.Kp < s.W) || (s.y && (!s.mix || !s.feed)) ||
+         (s.y2 && (!s.y || !s.gb || !s.gb2)) || (!s.in && !s.xout);
+}
+
+template <typename T, int U>
+static void hyper_go(const HyperStage& s, const int* rows, T* out, int M,
+                     hipStream_t st) {
+  if (s.S == 2)
+    hipLaunchKernelGGL((k_hyper_rows<T, U, 2>), dim3(M), dim3(256), 0, st, s,
+                       rows, out);
+  else if (s.S == 4)
+    hipLaunchKernelGGL((k_hyper_rows<T, U, 4>), dim3(M), dim3(256), 0, st, s,
+                       rows, out);
+  else
+    hipLaunchKernelGGL((k_hyper_rows<T, 1, 0>), dim3(M), dim3(256), 0, st, s,
+                       rows, out);
+}
+
+extern "C" hipError_t launch_hyper_rows(int f32, const HyperStage* s,
+                                        const void* rows, void* out, int M,
+                                        hipStream_t st) {
+  if (bad_hyper(*s) || M < 1 || (s->in && !out) || (s->xout && rows))
+    return hipErrorInvalidValue;
+  const int* r = (const int*)rows;
+  if (s->W <= 2048)
+    BY_TYPE(f32, (hyper_go<u16, 8>(*s, r, (u16*)out, M, st)),
+            (hyper_go<float, 8>(*s, r, (float*)out, M, st)));
+  else
+    BY_TYPE(f32, (hyper_go<u16, 16>(*s, r, (u16*)out, M, st)),
+            (hyper_go<float, 16>(*s, r, (float*)out, M, st)));
+  return hipGetLastError();
+}
+
+static bool bad_groups(const RowStage& s, int groups) {
+  return s.W < 1 || !s.x || !s.g || s.Kp < s.W || groups < 1 ||
+         groups > MAX_GROUPS || s.W % groups;
+}
+
+extern "C" hipError_t launch_group_rows(int f32, const RowStage* s, int groups,
+                                        void* out, int M, hipStream_t st) {
+  if (bad_groups(*s, groups) || M < 1) return hipErrorInvalidValue;
+  BY_TYPE(f32,
+          hipLaunchKernelGGL(k_group_rows<u16>, dim3(M), dim3(256), 0, st, *s,
+                             groups, (u16*)out),
+          hipLaunchKernelGGL(k_group_rows<float>, dim3(M), dim3(256), 0, st, *s,
+                             groups, (float*)out));
   return hipGetLastError();
 }
 
@@ -929,28 +1233,33 @@ extern "C" hipError_t launch_cat_rows(int f32, const void* x, const void* x0,
   return hipGetLastError();
 }
 
-template <typename T, int MODE, int U, int NR>
+template <typename T, int MODE, int U, int NR, int HS>
 static hipError_t lin_row_nr(const LinRowArgs& a, hipStream_t s) {
   constexpr int per = LIN_NT / 64 * NR;
-  RAISE_LDS((k_lin_row<T, MODE, U, NR>));
+  RAISE_LDS((k_lin_row<T, MODE, U, NR, HS>));
   int blocks = (a.N + per - 1) / per;
   const int rounds = (blocks + 511) / 512;       // alike in every block
   blocks = (blocks + rounds - 1) / rounds;
-  hipLaunchKernelGGL((k_lin_row<T, MODE, U, NR>), dim3(blocks), dim3(LIN_NT),
+  hipLaunchKernelGGL((k_lin_row<T, MODE, U, NR, HS>),
+                     dim3(blocks, MODE == ROW_PLAIN ? a.Z : 1), dim3(LIN_NT),
                      MODE == ROW_PLAIN ? 0 : (size_t)a.s.Kp * sizeof(T), s, a);
   return hipGetLastError();
 }
 
-template <typename T, int MODE, int U>
+template <typename T, int MODE, int U, int HS = 0>
 static hipError_t lin_row_go(const LinRowArgs& a, hipStream_t s) {
-  return a.N <= 4096 ? lin_row_nr<T, MODE, U, 1>(a, s)
-                     : lin_row_nr<T, MODE, U, 2>(a, s);
+  return a.N <= 4096 ? lin_row_nr<T, MODE, U, 1, HS>(a, s)
+                     : lin_row_nr<T, MODE, U, 2, HS>(a, s);
 }
 
 template <typename T>
 static hipError_t lin_row(const LinRowArgs& a, hipStream_t s) {
   if (a.N < 1 || a.s.Kp < 64 || a.s.Kp % 64 ||
-      (a.epi != EPI_F32 && a.epi != EPI_RELU2))
+      (a.epi != EPI_F32 && a.epi != EPI_RELU2 && a.epi != EPI_GELU))
+    return hipErrorInvalidValue;
+  if (a.Z < 1 || a.Z > 2 ||
+      (a.Z == 2 && (a.stage != ROW_PLAIN || a.K2 < 64 || a.K2 % 64 ||
+                    a.epi != EPI_F32)))
     return hipErrorInvalidValue;
   if (a.stage == ROW_PLAIN)
     return a.hin ? lin_row_go<T, ROW_PLAIN, 1>(a, s) : hipErrorInvalidValue;
@@ -970,7 +1279,23 @@ static hipError_t lin_row(const LinRowArgs& a, hipStream_t s) {
     return a.s.W <= 2048 ? lin_row_go<T, ROW_CONV, 4>(a, s)
                          : lin_row_go<T, ROW_CONV, 8>(a, s);
   }
+  if (a.stage == ROW_GROUPS)
+    return bad_groups(a.s, a.groups) ? hipErrorInvalidValue
+                                     : lin_row_go<T, ROW_GROUPS, 1>(a, s);
   // other blocks read x while block 0 writes xout
+  if (a.stage == ROW_HYPER) {
+    const HyperStage& h = a.h;
+    if (bad_hyper(h) || !h.in || h.xout == h.x || h.W != a.s.W ||
+        h.Kp != a.s.Kp)
+      return hipErrorInvalidValue;
+    if (h.S == 2)
+      return h.W <= 2048 ? lin_row_go<T, ROW_HYPER, 4, 2>(a, s)
+                         : lin_row_go<T, ROW_HYPER, 8, 2>(a, s);
+    if (h.S == 4)
+      return h.W <= 2048 ? lin_row_go<T, ROW_HYPER, 4, 4>(a, s)
+                         : lin_row_go<T, ROW_HYPER, 8, 4>(a, s);
+    return lin_row_go<T, ROW_HYPER, 1, 0>(a, s);
+  }
   if (a.stage != ROW_NORM || bad_stage(a.s) || !a.s.g || a.s.xout == a.s.x) return hipErrorInvalidValue;
   return a.s.W <= 2048 ? lin_row_go<T, ROW_NORM, 4>(a, s)
                        : lin_row_go<T, ROW_NORM, 8>(a, s);
@@ -1019,12 +1344,13 @@ extern "C" hipError_t launch_gemm_rows(int f32, const void* X, const void* W,
                                        int ldy, int ldg, int epi, float mult,
                                        int Z, long xz, long wz, long yz,
                                        int gz, int gc, const Rotary* rotary,
-                                       hipStream_t s) {
+                                       int K2, hipStream_t s) {
   if (M < 1 || N < 1 || K < 64 || K % 64 || ldx < K || ldw < K || Z < 1 ||
-      epi < 0 || epi > EPI_ROTARY || (epi == EPI_TGATE && !gate))
+      K2 < 64 || K2 % 64 || ldx < K2 ||
+      epi < 0 || epi > EPI_GELU || (epi == EPI_TGATE && !gate))
     return hipErrorInvalidValue;
   GemmArgs a = {X, W, Y, (const float*)gate, (const float*)bias, M, N, K, ldx,
-                ldw, ldy, ldg, epi, gz, gc, mult, xz, wz, yz, {}};
+                ldw, ldy, ldg, epi, gz, gc, mult, xz, wz, yz, K2, {}};
   if (epi == EPI_ROTARY) {
     if (!rotary || rotary->split % 2 || rotary->RT < 2 || rotary->RT % 2 ||
         rotary->dims % 2 || rotary->dims > rotary->RT || Z != 1 ||

@@ -21,12 +21,20 @@ sublayers read the residual through a short causal convolution, latent
 attention with a query latent, a sliding window and a sink, polynomial
 dense feed-forwards or sigmoid-routed experts, layers that use another
 layer's tensors.
+
+Dogalorn: several residual streams that every sublayer reads and rewrites
+through small learned mixes, an embedding of token pairs, pairs of mixers
+side by side (chunked attention with distance biases whose values are its
+keys, a gated recurrence), state-space mixers, biased gelu feed-forwards,
+norms with a single gain, shared tensors.
 """
 
 from __future__ import annotations
 
 from dataclasses import dataclass, field
 from typing import Dict, List, Optional, Tuple
+
+import numpy as np
 
 Shapes = Dict[str, Tuple[int, ...]]
 
@@ -270,6 +278,9 @@ class AttentionSpec:
     kind = "attention"
     libs = ("gqa",)
     recurrent = False
+    inputs = ("q", "k", "v", "g")
+    chunk = bias_max = None
+    sink = False
 
     @classmethod
     def from_dict(cls, m: dict, where: str):
@@ -302,6 +313,185 @@ class AttentionSpec:
                 p + "k": (k, width), p + "k.b": (k,), p + "k.norm": (k,),
                 p + "v": (v, width), p + "v.b": (v,), p + "g": (o, width),
                 p + "o": (width, o)}
+
+
+@dataclass
+class ChunkedAttentionSpec:
+    """Grouped-query attention without rotation, bias or gate.  A token sees
+    the earlier ones of its chunk of `chunk` positions; the values are the
+    keys ahead of their norm.  Scores are multiplied by a number per head
+    and get a bias by distance, from a table whose rows are buckets: exact
+    below half of them, logarithmic up to bias_max.  The softmax has one
+    more term, of score 0."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    bias_max: float
+    chunk: int
+    kind = "attention"
+    libs = ("gqa",)
+    recurrent = False
+    inputs = ("q", "k")
+    sink = True
+    buckets = 32                 # of random weights; a checkpoint has its own
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str):
+        s = cls(heads=_get(m, "heads", where),
+                kv_heads=_get(m, "kv_heads", where),
+                dim=_get(m, "dim", where), vdim=_get(m, "vdim", where),
+                scale=float(_get(m, "scale", where)),
+                bias_max=_get(m, "bias_max", where),
+                chunk=_get(_get(m, "mask", where), "size", where + ".mask"))
+        _positive(where, heads=s.heads, kv_heads=s.kv_heads, dim=s.dim,
+                  vdim=s.vdim)
+        _positive(where + ".mask", size=s.chunk)
+        if s.heads % s.kv_heads:
+            raise ValueError(f"config.json: {where}: {s.heads} heads do not "
+                             f"divide over {s.kv_heads} kv_heads")
+        if s.dim != s.vdim:
+            raise ValueError(f"config.json: {where}: the values are the keys, "
+                             f"but dim {s.dim} is not vdim {s.vdim}")
+        if not s.bias_max > 0:
+            raise ValueError(f"config.json: {where}.bias_max must be "
+                             f"positive, got {s.bias_max!r}")
+        return s
+
+    def to_dict(self) -> dict:
+        return {"heads": self.heads, "kv_heads": self.kv_heads,
+                "dim": self.dim, "vdim": self.vdim, "scale": self.scale,
+                "bias_max": self.bias_max, "mask": {"size": self.chunk}}
+
+    def shapes(self, p: str, width: int) -> Shapes:
+        q, k = self.heads * self.dim, self.kv_heads * self.dim
+        return {p + "q": (q, width), p + "q.norm": (q,),
+                p + "k": (k, width), p + "k.norm": (k,),
+                p + "rel": (self.buckets, self.heads),
+                p + "temp": (self.heads,), p + "o": (width, q)}
+
+    def open_rows(self, p: str):
+        return [p + "rel"]
+
+
+@dataclass
+class MinGRUSpec:
+    """Gated recurrence whose gate and candidate read the current token
+    only, element by element."""
+    width: int
+    kind = "mingru"
+    libs = ("mingru",)
+    recurrent = True
+    inputs = ("z", "x", "g")
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str):
+        s = cls(width=_get(m, "width", where))
+        _positive(where, width=s.width)
+        return s
+
+    def to_dict(self) -> dict:
+        return {"width": self.width}
+
+    def shapes(self, p: str, width: int) -> Shapes:
+        C = self.width
+        return {p + "z": (C, width), p + "z.b": (C,), p + "x": (C, width),
+                p + "x.b": (C,), p + "g": (C, width), p + "o": (width, C)}
+
+
+@dataclass
+class PairSpec:
+    """Two mixers that read the same input; the result is half the sum of
+    their normed outputs."""
+    left: object
+    right: object
+    kind = "parallel"
+    left_class = ChunkedAttentionSpec
+    right_class = MinGRUSpec
+
+    @property
+    def libs(self):
+        return (*self.left.libs, *self.right.libs)
+
+    @property
+    def recurrent(self):
+        return self.left.recurrent or self.right.recurrent
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str):
+        return cls(*(c.from_dict(_get(m, k, where), f"{where}.{k}")
+                     for k, c in (("left", cls.left_class),
+                                  ("right", cls.right_class))))
+
+    def to_dict(self) -> dict:
+        return {"left": self.left.to_dict(), "right": self.right.to_dict()}
+
+    def shapes(self, p: str, width: int) -> Shapes:
+        return {**self.left.shapes(p + "left.", width),
+                **self.right.shapes(p + "right.", width),
+                p + "left.out": (width,), p + "right.out": (width,)}
+
+    def open_rows(self, p: str):
+        return [n for k in ("left", "right")
+                for n in open_rows(getattr(self, k), f"{p}{k}.")]
+
+
+def open_rows(spec, p: str):
+    """Tensors of a mixer whose number of rows the checkpoint decides."""
+    return spec.open_rows(p) if hasattr(spec, "open_rows") else []
+
+
+@dataclass
+class SSDSpec:
+    """State-space recurrence (Mamba-2): x, B and C behind a causal
+    convolution of `conv` taps, a step size per head and token, the state a
+    [state, vdim] matrix per head; the gated output is normed in
+    norm_groups equal parts."""
+    heads: int
+    vdim: int
+    state: int
+    groups: int
+    conv: int
+    norm_groups: int
+    kind = "mamba2"
+    libs = ("ssd",)
+    recurrent = True
+    inputs = ("in",)
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str):
+        names = ("heads", "vdim", "state", "groups", "conv", "norm_groups")
+        s = cls(**{k: _get(m, k, where) for k in names})
+        _positive(where, **{k: getattr(s, k) for k in names})
+        if s.heads % s.groups:
+            raise ValueError(f"config.json: {where}: {s.heads} heads do not "
+                             f"divide over {s.groups} groups")
+        if s.inner % s.norm_groups:
+            raise ValueError(f"config.json: {where}: {s.inner} values do not "
+                             f"divide into {s.norm_groups} norm_groups")
+        return s
+
+    @property
+    def inner(self) -> int:
+        return self.heads * self.vdim
+
+    @property
+    def channels(self) -> int:
+        """What passes the convolution: x, B and C."""
+        return self.inner + 2 * self.groups * self.state
+
+    def to_dict(self) -> dict:
+        return {"heads": self.heads, "vdim": self.vdim, "state": self.state,
+                "groups": self.groups, "conv": self.conv,
+                "norm_groups": self.norm_groups}
+
+    def shapes(self, p: str, width: int) -> Shapes:
+        H, C = self.heads, self.channels
+        return {p + "in": (self.inner + C + H, width),
+                p + "conv": (C, self.conv), p + "conv.b": (C,),
+                p + "dt_bias": (H,), p + "A_log": (H,), p + "D": (H,),
+                p + "norm": (self.inner,), p + "o": (width, self.inner)}
 
 
 @dataclass
@@ -404,12 +594,44 @@ class PolyDenseSpec(DenseSpec):
         return {**super().shapes(p, width), p + "act": (4,)}
 
 
+@dataclass
+class GeluDenseSpec(DenseSpec):
+    """act = the exact gelu; both matrices have biases."""
+    act = "gelu"
+
+    def shapes(self, p: str, width: int) -> Shapes:
+        return {**super().shapes(p, width), p + "up.b": (self.ff,),
+                p + "down.b": (width,)}
+
+
+@dataclass
+class BigramSpec:
+    """Embedding of token pairs: row (previous * mul_prev + current *
+    mul_cur) mod buckets; one more row for a sequence's first token."""
+    buckets: int
+    mul_prev: int
+    mul_cur: int
+
+    @classmethod
+    def from_dict(cls, m: dict, where: str):
+        names = ("buckets", "mul_prev", "mul_cur")
+        s = cls(**{k: _get(m, k, where) for k in names})
+        _positive(where, **{k: getattr(s, k) for k in names})
+        return s
+
+    def to_dict(self) -> dict:
+        return {"buckets": self.buckets, "mul_prev": self.mul_prev,
+                "mul_cur": self.mul_cur}
+
+
 @dataclass(frozen=True)
 class Design:
     """What a design fixes about its layers.  ``parallel``: one norm feeds
     mixer and feed-forward; ``sandwich``: each has a norm before and after
     it; ``post``: each has a norm after it and a short convolution over
-    time ahead of it.  ``project``: W_in [x; x0] ahead of every pass of the
+    time ahead of it; ``hyper``: each reads a mix of several residual
+    streams through a norm with one gain and rewrites them all.
+    ``project``: W_in [x; x0] ahead of every pass of the
     loop; ``add``: x + x0 ahead of every pass but the first.  ``share``: a
     layer may use another one's tensors."""
     model_type: str
@@ -435,6 +657,8 @@ DESIGNS = {
                       (DenseSpec,)),
     "Fidizen": Design("fidizen", "post", None, (WindowedLatentSpec,),
                       (PolyDenseSpec, SigmoidMoESpec), share=True),
+    "Dogalorn": Design("dogalorn", "hyper", None, (PairSpec, SSDSpec),
+                       (GeluDenseSpec,), share=True),
 }
 
 
@@ -464,6 +688,9 @@ class LayeredConfig:
     residual_mult: float = 1.0
     logit_softcap: Optional[float] = None
     conv_taps: int = 1            # of the sublayers' input convolutions
+    streams: int = 0              # copies of the residual, 0: it is plain
+    bigram: Optional[BigramSpec] = None
+    logit_scale: float = 1.0
     max_position_embeddings: int = 131072
     bos_token_id: Optional[int] = None
     eos_token_id: Optional[int] = None
@@ -537,8 +764,8 @@ class LayeredConfig:
 
     @property
     def recurrent(self) -> bool:
-        return self.conv_taps > 1 or any(l.mixer.recurrent
-                                         for l in self.layers)
+        return (self.conv_taps > 1 or self.bigram is not None or
+                any(l.mixer.recurrent for l in self.layers))
 
     @classmethod
     def matches(cls, d: dict) -> bool:
@@ -576,6 +803,14 @@ class LayeredConfig:
         if design.block == "post":
             taps = _get(_get(d, "canon", "top level"), "taps", "canon")
             _positive("canon", taps=taps)
+        streams, bigram, logit_scale = 0, None, 1.0
+        if design.block == "hyper":
+            streams = _get(d, "streams", "top level")
+            _positive("top level", streams=streams)
+            bigram = BigramSpec.from_dict(
+                _get(_get(d, "embedding", "top level"), "bigram",
+                     "embedding"), "embedding.bigram")
+            logit_scale = float(_get(d, "logit_scale", "top level"))
         width, vocab = _get(d, "width", "top level"), _get(d, "vocab",
                                                            "top level")
         _positive("top level", width=width, vocab=vocab)
@@ -589,7 +824,8 @@ class LayeredConfig:
             embed_scale=float(d.get("embedding", {}).get("scale", 1.0)),
             residual_mult=float(d.get("residual_mult", 1.0)),
             logit_softcap=float(cap) if cap else None,
-            conv_taps=taps,
+            conv_taps=taps, streams=streams, bigram=bigram,
+            logit_scale=logit_scale,
             max_position_embeddings=d.get("max_position_embeddings", 131072),
             bos_token_id=d.get("bos_token_id"),
             eos_token_id=d.get("eos_token_id"))
@@ -608,6 +844,10 @@ class LayeredConfig:
         if self.design.block == "post":
             d.update({"embedding": {"scale": self.embed_scale},
                       "canon": {"taps": self.conv_taps}})
+        if self.design.block == "hyper":
+            d.update({"embedding": {"bigram": self.bigram.to_dict()},
+                      "streams": self.streams,
+                      "logit_scale": self.logit_scale})
         if self.design.block == "parallel":
             d.update({"embedding": {"scale": self.embed_scale},
                       "residual_mult": self.residual_mult,
@@ -630,10 +870,21 @@ class LayeredConfig:
             out["loop.in"] = (W, 2 * W)
         sandwich = self.design.block == "sandwich"
         post = self.design.block == "post"
+        S, hyper = self.streams, self.design.block == "hyper"
+        if hyper:
+            out["final.norm"] = ()
+        if self.bigram:
+            out["bigram"] = (self.bigram.buckets + 1, W)
         for i, l in enumerate(self.layers):
             if l.weights_of is not None:
                 continue
-            out[f"l{i}.norm1"] = (W,)
+            out[f"l{i}.norm1"] = () if hyper else (W,)
+            if hyper:
+                if l.mlp:
+                    out[f"l{i}.norm2"] = ()
+                for q in (1, 2) if l.mlp else (1,):
+                    out.update({f"l{i}.hc{q}.in": (S,), f"l{i}.hc{q}.out": (S,),
+                                f"l{i}.hc{q}.mix": (S, S)})
             if post:
                 out[f"l{i}.canon1"] = (W, self.conv_taps)
                 if l.mlp:
@@ -647,6 +898,21 @@ class LayeredConfig:
                     out[f"l{i}.norm2"] = out[f"l{i}.norm2b"] = (W,)
                 out.update(l.mlp.shapes(f"l{i}.mlp.", W))
         return out
+
+    def open_rows(self):
+        """Names of tensors whose number of rows the checkpoint decides."""
+        return {n for i, l in enumerate(self.layers) if l.weights_of is None
+                for n in open_rows(l.mixer, f"l{i}.mix.")}
+
+    def weight_base(self, name: str, shape):
+        """What random weights scatter around: 1 for norms, streams that
+        stay as they are and are read evenly."""
+        if ".hc" in name:
+            return (np.eye(*shape) if name.endswith("mix") else
+                    np.full(shape, 1.0 / shape[0] if name.endswith("in")
+                            else 1.0))
+        return 1.0 if "norm" in name or name.endswith(
+            ("left.out", "right.out")) else 0.0
 
 
 # ----------------------------------------------------------------------
@@ -746,7 +1012,47 @@ def _windowed_stack(n, heads, ff) -> list:
             for i in range(n)]
 
 
+def _pair(heads, kv_heads, dim, width, chunk, bias_max) -> tuple:
+    return "parallel", {
+        "left": dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim,
+                     scale=dim ** -0.5, bias_max=bias_max,
+                     mask={"size": chunk}),
+        "right": {"width": width}}
+
+
+def _ssd(heads, vdim, state, groups, norm_groups=1, conv=4) -> tuple:
+    return "mamba2", dict(heads=heads, vdim=vdim, state=state, groups=groups,
+                          conv=conv, norm_groups=norm_groups)
+
+
+def _dogalorn(vocab, width, layers, ff, streams=2, share=(), buckets=65521,
+              logit_scale=1.0) -> dict:
+    """layers: (type, sizes) pairs; share: owners of further layers."""
+    entries = [{"type": t, "mixer": m, "mlp": {"kind": "dense", "ff": ff}}
+               for t, m in layers]
+    entries += [{**entries[j], "weights_of": j} for j in share]
+    return {"architecture": "Dogalorn", "vocab": vocab, "width": width,
+            "norm": {"eps": 1e-6}, "streams": streams,
+            "logit_scale": logit_scale, "layers": entries,
+            "embedding": {"bigram": {"buckets": buckets, "mul_prev": 31,
+                                     "mul_cur": 7919}}}
+
+
+def _paired_stack(n, heads, width) -> list:
+    """Pairs of attention and recurrence, and state-space layers, in turn."""
+    kinds = [_pair(heads, heads // 4, 128, width, 1024, 128),
+             _ssd(width // 32, 64, 128, 1)]
+    return [kinds[i % 2] for i in range(n)]
+
+
 LAYERED_PRESETS = {
+    "tiny-dogalorn": _dogalorn(
+        336, 72, [_pair(6, 3, 20, 108, 40, 30), _ssd(6, 20, 24, 2, 3),
+                  _pair(4, 4, 28, 60, 70, 50)], 104, streams=3, share=(0, 1),
+        buckets=500, logit_scale=0.5),
+    "dogalorn-2k": _dogalorn(32000, 2048, _paired_stack(8, 16, 2048), 8192),
+    "dogalorn-4k": _dogalorn(32000, 4096, _paired_stack(4, 32, 4096), 16384),
+
     "tiny-fidizen": _fidizen(
         352, 72,
         [_windowed(_poly(104), 5, 20, 12, 28, 44, 36, 70),

@@ -257,15 +257,23 @@ def validate_weights(cfg: ModelConfig, w) -> None:
     trusted — materializing every tensor just to check it would double
     the load cost."""
     expect = hf_weight_shapes(cfg)
+    loose = cfg.open_rows() if isinstance(cfg, LayeredConfig) else ()
+
+    def differs(k, shape):
+        """Whether a shape is wrong; some tensors may have any rows."""
+        if k in loose and len(shape) == len(expect[k]) and shape[0] >= 1:
+            return shape[1:] != expect[k][1:]
+        return shape != expect[k]
+
     own = getattr(w, "shapes", None)
     if own is not None:
         missing = [k for k in expect if k not in own]
         bad = [(k, tuple(own[k]), expect[k]) for k in expect
-               if k in own and tuple(own[k]) != expect[k]]
+               if k in own and differs(k, tuple(own[k]))]
     else:
         missing = [k for k in expect if k not in w]
         bad = [(k, tuple(np.shape(w[k])), expect[k]) for k in expect
-               if k in w and tuple(np.shape(w[k])) != expect[k]]
+               if k in w and differs(k, tuple(np.shape(w[k])))]
     msgs = []
     if missing:
         shown = ", ".join(missing[:6])
@@ -282,18 +290,22 @@ def validate_weights(cfg: ModelConfig, w) -> None:
             + "; ".join(msgs))
 
 
+def _random_base(cfg: ModelConfig, name: str, shape):
+    """What a random tensor scatters around."""
+    if isinstance(cfg, LayeredConfig):
+        return cfg.weight_base(name, shape)
+    # Llama gamma ~1; Gemma stores gamma-1 so ~0
+    return 1.0 if "norm" in name and cfg.model_type != "gemma2" else 0.0
+
+
 def random_weights(cfg: ModelConfig, seed: int = 0,
                    scale: float = 0.02) -> Dict[str, np.ndarray]:
     """Random-init fp32 weights with HF names (norm gammas ~= identity)."""
     rng = np.random.default_rng(seed)
     w = {}
     for name, shape in hf_weight_shapes(cfg).items():
-        if "norm" in name:
-            # Llama gamma ~1; Gemma stores gamma-1 so ~0
-            base = 0.0 if cfg.model_type == "gemma2" else 1.0
-            w[name] = (base + scale * rng.standard_normal(shape)).astype(np.float32)
-        else:
-            w[name] = (scale * rng.standard_normal(shape)).astype(np.float32)
+        w[name] = np.asarray(_random_base(cfg, name, shape) + scale *
+                             rng.standard_normal(shape), np.float32)
     return w
 
 
@@ -324,10 +336,10 @@ class LazyRandomWeights:
         h = (zlib.crc32(name.encode()) ^ self.seed) & 0x7FFFFFFF
         rng = np.random.default_rng(h)  # deterministic ACROSS processes
         # (python hash() is per-process salted: TP ranks must agree)
-        if "norm" in name:
-            base = 0.0 if self.cfg.model_type == "gemma2" else 1.0
-            return (base + self.scale *
-                    rng.standard_normal(shape)).astype(np.float32)
+        base = _random_base(self.cfg, name, shape)
+        if "norm" in name or np.ndim(base) or base:
+            return np.asarray(base + self.scale * rng.standard_normal(shape),
+                              np.float32)
         a = rng.random(np.prod(shape), dtype=np.float32).reshape(shape)
         return (a - 0.5) * (2.0 * self.scale)
 

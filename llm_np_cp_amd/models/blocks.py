@@ -71,7 +71,7 @@ class SandwichBlock(Block):
         self.mixer = m = MIXERS[spec.mixer.kind](eng, spec.mixer, pk,
                                                  p + "mix.")
         self.win = pk.rows([p + "mix." + n for n in m.IN], eng.W)
-        self.bias = m.biases(eng, pk, p + "mix.")
+        self.bias = m.biases(pk, p + "mix.")
         self.ldp = self.p_floats = self.win.shape[0]
         self.g1, self.g1b = pk.f32(p + "norm1"), pk.f32(p + "norm1b")
         self.ff = None
@@ -132,5 +132,49 @@ class PostNormBlock(Block):
             eng.pend = self.g2
 
 
+class HyperMix:
+    """How a sublayer reads the residual streams (read), and how they all
+    turn (mix [from, to]) and take up its output (feed)."""
+
+    def __init__(self, pk: Packer, p: str):
+        self.read, self.feed = pk.f32(p + "in"), pk.f32(p + "out")
+        self.mix = pk.f32(p + "mix")
+
+
+class HyperBlock(Block):
+    """x_t <- sum_s mix[s, t] x_s + feed[t] f(norm(sum_s read[s] x_s)) for
+    mixer and feed-forward f.  The streams turn in the staging of the
+    projection after them."""
+
+    def __init__(self, eng, spec, pk: Packer, i: int):
+        p = f"l{i}."
+        self.mixer = m = MIXERS[spec.mixer.kind](eng, spec.mixer, pk,
+                                                 p + "mix.")
+        self.win = pk.rows([p + "mix." + n for n in m.IN], eng.W)
+        self.bias = m.biases(pk, p + "mix.")
+        self.ldp = self.p_floats = self.win.shape[0]
+        self.g1, self.c1 = pk.f32(p + "norm1"), HyperMix(pk, p + "hc1.")
+        self.ff = None
+        self.act_floats = 0
+        if spec.mlp:
+            self.ff = FEED_FORWARDS[spec.mlp.kind](eng, spec.mlp, pk,
+                                                   p + "mlp.")
+            self.act_floats = self.ff.act_floats
+            self.g2, self.c2 = pk.f32(p + "norm2"), HyperMix(pk, p + "hc2.")
+
+    def run(self, eng, b, cache):
+        T, m, ff = b.T, self.mixer, self.ff
+        eng.read_streams(self.win, eng.P, T, self.c1.read, self.g1,
+                         bias=self.bias)
+        m.run(eng, b, cache, self)
+        m.out(eng, b, self)
+        eng.turn = (self.c1, m.halves(eng) if hasattr(m, "halves") else {})
+        if ff:
+            eng.read_streams(ff.up, eng.act, T, self.c2.read, self.g2,
+                             bias=ff.bias, epi=hy.EPI_GELU)
+            eng.linear(ff.down, eng.act, eng.y, T, bias=ff.down_bias)
+            eng.turn = (self.c2, {})
+
+
 BLOCKS = {"parallel": ParallelBlock, "sandwich": SandwichBlock,
-          "post": PostNormBlock}
+          "post": PostNormBlock, "hyper": HyperBlock}

@@ -135,7 +135,18 @@ class LayeredModel(DecodeLoop):
         pk = Packer(weights, self.device, self.T)
         self.embed = pk.raw("embed").to(self.T).contiguous()
         self.head = pk.rows(["head"], self.W)
-        self.g_final = pk.f32("final.norm")
+        self.g_final = pk.f32("final.norm") * cfg.logit_scale
+        self.streams, self.pairs = cfg.streams, None
+        if cfg.streams > hy.MAX_STREAMS:
+            raise ValueError(f"{cfg.model_type}: {cfg.streams} streams "
+                             f"exceed the built kernels ({hy.MAX_STREAMS})")
+        if cfg.streams:
+            self.read_all = torch.ones(cfg.streams, device=self.device)
+        if cfg.bigram:
+            self.pairs = pk.raw("bigram").to(self.T).contiguous()
+            # the token before the next one of every slot's sequence
+            self.last = torch.zeros(self.max_batch, dtype=torch.int32,
+                                    device=self.device)
         self.win_loop = (pk.rows(["loop.in"], 2 * self.W)
                          if cfg.loop and cfg.design.loop == "project"
                          else None)
@@ -169,15 +180,18 @@ class LayeredModel(DecodeLoop):
         f32 = dict(dtype=torch.float32, device=dev)
         i32 = dict(dtype=torch.int32, device=dev)
         tt = dict(dtype=self.T, device=dev)
-        self.x = torch.zeros(PC, self.W, **f32)
-        self.xb = torch.zeros(PC, self.W, **f32)
+        S = max(self.streams, 1)
+        self.x = torch.zeros(PC, S * self.W, **f32)
+        self.xb = torch.zeros(PC, S * self.W, **f32)
         self.x0 = torch.zeros(PC, self.W, **f32) if cfg.loop else None
         self.h = torch.zeros(PC, self.Wp, **tt)
         self.cat = (torch.zeros(PC, self.win_loop.shape[1], **tt)
                     if self.win_loop is not None else None)
         self.y = (torch.zeros(PC, self.W, **f32)
                   if cfg.design.block != "parallel" else None)
-        self.pend, self.add0 = None, False
+        if self.streams:             # two halves of a pair's output
+            self.y = torch.zeros(2, PC, self.W, **f32)
+        self.pend, self.add0, self.turn = None, False, None
         layers = self.layers.values()
         self.P = torch.zeros(PC * max(l.p_floats for l in layers), **f32)
         need: Dict[str, int] = {}
@@ -185,7 +199,8 @@ class LayeredModel(DecodeLoop):
             for k, n in l.mixer.sizes(self, PC).items():
                 need[k] = max(need.get(k, 0), n)
         for k in ("q", "qn", "qa", "olat", "o", "part", "ml", "raw", "gF",
-                  "gi", "gm", "cm0", "U", "un", "decay", "local", "cq", "qf"):
+                  "gi", "gm", "cm0", "U", "un", "decay", "local", "cq", "qf",
+                  "u"):
             kw = tt if k in ("q", "qn", "qa", "olat", "o", "cq") else f32
             setattr(self, k, torch.zeros(max(need.get(k, 0), 1), **kw))
         ex = [l.experts or l.ff.experts for l in layers
@@ -241,10 +256,15 @@ class LayeredModel(DecodeLoop):
         """Embedding and every layer run over the batch; leaves the
         residual stream of its rows in self.x."""
         cfg, T = self.cfg, b.T
-        self.pend, self.add0 = None, False
-        hy.embed_rows(self.embed, b.ids, self.x, self.x0, T, cfg.embed_scale)
+        self.pend, self.add0, self.turn = None, False, None
+        if self.pairs is not None:
+            hy.embed_pairs(self.embed, self.pairs, self.last, b, self.x,
+                           self.W, self.streams, cfg.bigram)
+        else:
+            hy.embed_rows(self.embed, b.ids, self.x, self.x0, T,
+                          cfg.embed_scale)
         if layer_hook is not None:
-            layer_hook(-1, self.x[:T])
+            layer_hook(-1, self._residual(T, 1.0 / max(self.streams, 1)))
         for j, (i, comes_in) in enumerate(cfg.runs):
             if comes_in:
                 if self.win_loop is None:      # x + x0, with what comes next
@@ -255,7 +275,13 @@ class LayeredModel(DecodeLoop):
             self.layers[i].run(self, b, self.caches[j])
             if layer_hook is not None:
                 self._settle(T)
-                layer_hook(j, self.x[:T])
+                layer_hook(j, self._residual(T))
+
+    def _residual(self, T: int, scale: float = 1.0):
+        """The residual of the first T rows; of several streams the sum."""
+        x = self.x[:T]
+        return (x.view(T, self.streams, self.W).sum(1) * scale
+                if self.streams else x)
 
     def _pending(self):
         """What the residual still lacks: staging arguments, then cleared."""
@@ -267,7 +293,19 @@ class LayeredModel(DecodeLoop):
         self.pend, self.add0 = None, False
         return kw
 
+    def _turning(self):
+        """What the streams still lack: staging arguments, then cleared."""
+        kw = {"S": self.streams}
+        if self.turn is not None:
+            c, halves = self.turn
+            kw.update(y=self.y[0], mix=c.mix, feed=c.feed, **halves)
+        self.turn = None
+        return kw
+
     def _settle(self, T: int):
+        if self.turn is not None:
+            hy.hyper_rows(self.x, None, T, self.W, self.W, self.cfg.norm_eps,
+                          xout=self.x, **self._turning())
         kw = self._pending()
         if kw:
             hy.norm_rows(self.x, None, None, T, self.W, self.W,
@@ -305,22 +343,48 @@ class LayeredModel(DecodeLoop):
                      epi if cap is None else hy.EPI_SOFTCAP, mult=cap or 0.0,
                      bias=bias)
 
-    def linear(self, w, src, out, T: int):
-        """out[T, N] fp32 = w . src, rows of src as wide as w's."""
+    def read_streams(self, w, out, T: int, read, g, rows=None, bias=None,
+                     epi=hy.EPI_F32):
+        """out[T, N] = w . norm(sum of the streams weighted by read), a norm
+        with the single gain g.  What is due on the streams is done on the
+        way.  One row runs as a fused GEMV."""
+        (N, K), W, eps = w.shape, self.W, self.cfg.norm_eps
+        kw = self._turning()
+        keep = "y" in kw and rows is None
+        one = self.one_row(w, T)
+        if keep:               # one row: other blocks still read x
+            kw["xout"] = self.xb if one else self.x
+        kw.update(read=read, g=g)
+        if one:
+            hy.lin_row(w, self.x, out, W, eps, rows=rows, bias=bias, epi=epi,
+                       hyper=kw)
+            if keep:
+                self.x, self.xb = self.xb, self.x
+            return
+        hy.hyper_rows(self.x, self.h, T, W, K, eps, rows=rows, **kw)
+        hy.gemm_rows(self.h, w, out, T, K, N, epi, bias=bias)
+
+    def linear(self, w, src, out, T: int, bias=None):
+        """out[T, N] fp32 = w . src + bias, rows of src as wide as w's."""
         N, K = w.shape
         if self.one_row(w, T):
-            hy.lin_row(w, None, out, 0, 0.0, hin=src)
+            hy.lin_row(w, None, out, 0, 0.0, hin=src, bias=bias)
         else:
-            hy.gemm_rows(src, w, out, T, K, N, hy.EPI_F32)
+            hy.gemm_rows(src, w, out, T, K, N, hy.EPI_F32, bias=bias)
 
-    def normed_linear(self, w, staged, out, T: int, src, W: int, g, gate,
-                      ldg: int):
-        """out[T, N] fp32 = w . (norm(src) sigmoid(gate)), src [T, W]."""
+    def normed_linear(self, w, staged, out, T: int, src, W: int, g, gate=None,
+                      ldg: int = 0, groups: int = 1):
+        """out[T, N] fp32 = w . (norm(src) sigmoid(gate)), src [T, W], or
+        with the norm over each of `groups` equal parts."""
         (N, K), eps = w.shape, self.cfg.norm_eps
         if self.one_row(w, T):
-            hy.lin_row(w, src, out, W, eps, g=g, gate=gate, ldg=ldg)
+            hy.lin_row(w, src, out, W, eps, g=g, gate=gate, ldg=ldg,
+                       groups=groups)
         else:
-            hy.norm_rows(src, g, staged, T, W, K, eps, gate=gate, ldg=ldg)
+            if groups > 1:
+                hy.group_rows(src, g, staged, T, W, K, eps, groups)
+            else:
+                hy.norm_rows(src, g, staged, T, W, K, eps, gate=gate, ldg=ldg)
             hy.gemm_rows(staged, w, out, T, K, N, hy.EPI_F32)
 
     def conv_project(self, w, kernel, ring, b: Rows, out, narrow=False):
@@ -360,6 +424,10 @@ class LayeredModel(DecodeLoop):
 
     def _head(self, out: torch.Tensor, n: int, rows=None):
         """Final norm, head and soft cap of n rows -> out [n, vocab]."""
+        if self.streams:
+            self.read_streams(self.head, out, n, self.read_all, self.g_final,
+                              rows=rows)
+            return
         self.project(self.head, self.h, out, n, self.g_final, rows=rows,
                      cap=self.cfg.logit_softcap or 0.0)
 

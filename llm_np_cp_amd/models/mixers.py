@@ -379,7 +379,7 @@ class SandwichMixer:
     IN run as one matrix, with the biases of those that have one."""
     tile_pairs = None
 
-    def biases(self, eng, pk: Packer, p: str):
+    def biases(self, pk: Packer, p: str):
         parts = [pk.f32(p + n + ".b") if p + n + ".b" in pk.w else
                  torch.zeros(pk.w[p + n].shape[0], device=pk.device)
                  for n in self.IN]
@@ -391,12 +391,26 @@ class SandwichMixer:
         eng.linear(self.wo, eng.o, eng.y, b.T)
 
 
+def distance_bias(rel: np.ndarray, far: float, longest: int) -> np.ndarray:
+    """[heads, n] bias by distance from the buckets rel [rows, heads]: below
+    rows/2 a bucket per distance, then logarithmic up to `far`.  Every
+    distance from n - 1 on has the last value."""
+    rows, half = len(rel), len(rel) // 2
+    if rows < 2 or rows % 2 or far <= half:
+        raise ValueError(f"attention: {rows} bias buckets up to distance "
+                         f"{far} are not possible")
+    n = np.arange(min(longest, int(np.ceil(far)) + 1))
+    log = half + np.floor(np.log(np.maximum(n, half) / half) /
+                          np.log(far / half) * (rows - half))
+    return rel[np.where(n < half, n, np.minimum(rows - 1, log)).astype(int)].T
+
+
 class GroupedAttention(SandwichMixer):
     kind = "attention"
-    IN = ("q", "k", "v", "g")
 
     def __init__(self, eng, spec, pk: Packer, p: str):
         self.spec = s = spec
+        self.IN = s.inputs
         fit = [c for c in hy.HEAD_SIZES if c[0] >= s.dim and c[1] >= s.vdim]
         if not fit:
             raise ValueError(
@@ -408,13 +422,40 @@ class GroupedAttention(SandwichMixer):
         self.ldo = pad_to(H * s.vdim, 64)
         self.wo = pk.rows([p + "o"], H * s.vdim)
         self.qnorm, self.knorm = pk.f32(p + "q.norm"), pk.f32(p + "k.norm")
-        self.temp = eng.query_temperature(s.temp_coef, s.temp_every)
         q, k, v = H * s.dim, G * s.dim, G * s.vdim
+        own = "v" in s.inputs                 # else the values are the keys
         self.args = hy.GqaArgs().put(
-            qnorm=self.qnorm, knorm=self.knorm, temp=self.temp, oq=0, ok=q,
-            ov=q + k, og=q + k + v, H=H, G=G, d=s.dim, vd=s.vdim,
+            qnorm=self.qnorm, knorm=self.knorm, oq=0, ok=q,
+            ov=q + k if own else q, og=q + k + v if "g" in s.inputs else -1,
+            H=H, G=G, d=s.dim, vd=s.vdim,
             DP=self.DP, VP=self.VP, ldo=self.ldo, eps=eng.cfg.norm_eps,
-            scale=s.scale)
+            scale=s.scale, chunk=min(s.chunk or 0, eng.max_seq))
+        if s.bias_max is None:
+            self.temp = eng.query_temperature(s.temp_coef, s.temp_every)
+            self.args.put(temp=self.temp)
+        else:
+            self._biases(eng, pk, p)
+        if s.sink:
+            self.sink = torch.zeros(H, device=pk.device)
+            self.args.put(sink=self.sink)
+
+    def _biases(self, eng, pk: Packer, p: str):
+        """Distance biases, base 2, and the numbers per head folded into the
+        norm of the queries."""
+        s = self.spec
+        longest = min(s.chunk or eng.max_seq, eng.max_seq)
+        rel = distance_bias(np.asarray(pk.w[p + "rel"], np.float64),
+                            s.bias_max, longest)
+        room = (30 if self.DP == 256 else 90) * 1024
+        if self.tile_pairs * rel.shape[1] * 4 > room:
+            raise ValueError(
+                f"attention: {rel.shape[1]} distances for {self.tile_pairs} "
+                f"heads exceed the built kernels")
+        self.bias = torch.from_numpy(
+            (rel * np.log2(np.e)).astype(np.float32)).to(pk.device).contiguous()
+        self.qnorm = (self.qnorm.view(s.heads, s.dim) *
+                      pk.f32(p + "temp")[:, None]).contiguous()
+        self.args.put(bias=self.bias, nbias=rel.shape[1], qnorm=self.qnorm)
 
     def new_cache(self, eng):
         n, G = eng.cache.num_pages, self.spec.kv_heads
@@ -427,6 +468,8 @@ class GroupedAttention(SandwichMixer):
         by the cache size and the number of rows, so a captured step keeps
         its grid."""
         groups = -(-eng.cache.table.shape[1] * hy.PAGE // 128)
+        if self.spec.chunk:
+            groups = min(groups, self.spec.chunk // 128 + 2)
         blocks = rows * self.spec.kv_heads * -(-self.tile_pairs // 16)
         return int(max(1, min(64, groups, 1024 // blocks)))
 
@@ -438,7 +481,9 @@ class GroupedAttention(SandwichMixer):
         return dict(q=rows * H * self.DP, o=rows * self.ldo,
                     part=splits * H * self.VP, ml=splits * H * 2)
 
-    def run(self, eng, b, cache, layer):
+    def run(self, eng, b, cache, layer, beside=None):
+        """beside: arguments of a gated recurrence whose single tokens take
+        their step along with this one's."""
         s, H, R = self.spec, self.spec.heads, self.tile_pairs
         a = self.args.put(
             P=eng.P, slot=b.slot, pos=b.pos, table=eng.table, K=cache[0],
@@ -448,10 +493,12 @@ class GroupedAttention(SandwichMixer):
         if b.nd:
             a.put(rows=b.nd, rbase=0, NS=self.token_splits(eng, b.nd))
             hy.gqa_token(eng.f32, a)
-            hy.gqa_merge(eng.f32, a)
+            hy.gqa_merge(eng.f32, a, beside)
         if b.nd < b.T:
             rows = b.T - b.nd
             seg, rr0, n, longest = b.tiles[R]
+            if s.chunk:
+                longest = min(longest, s.chunk + hy.TILE // R)
             ns = min(eng.run_splits(n * s.kv_heads, longest),
                      eng.part.numel() // (rows * H * self.VP),
                      eng.ml.numel() // (rows * H * 2))
@@ -461,6 +508,157 @@ class GroupedAttention(SandwichMixer):
             hy.gqa_run(eng.f32, a, n)
             if ns > 1:
                 hy.gqa_merge(eng.f32, a)
+
+
+class MinGRU(SandwichMixer):
+    kind = "mingru"
+
+    def __init__(self, eng, spec, pk: Packer, p: str):
+        self.spec, self.IN, C = spec, spec.inputs, spec.width
+        self.ldo = pad_to(C, 64)
+        self.wo = pk.rows([p + "o"], C)
+        self.args = hy.MingruArgs().put(oz=0, ox=C, og=2 * C, C=C,
+                                        ldo=self.ldo)
+
+    def new_cache(self, eng):
+        return (torch.zeros(eng.cache.num_slots, self.spec.width,
+                            dtype=torch.float32, device=eng.device),)
+
+    def sizes(self, eng, rows):
+        n = eng.max_chunks(rows) * self.spec.width
+        return dict(o=rows * self.ldo, decay=n, local=n)
+
+    def bind(self, eng, b, cache, layer):
+        nd = b.nd
+        return self.args.put(
+            P=eng.P, S=cache[0], A=eng.decay, h=eng.local, out=eng.o,
+            slot=b.slot, pos=b.pos, seg_row0=b.seg_row0[nd:],
+            seg_len=b.seg_len[nd:], seg_slot=b.seg_slot[nd:],
+            seg_pos0=b.seg_pos0[nd:], chunk_row0=b.chunk_row0,
+            chunk_len=b.chunk_len, chunk_seg=b.chunk_seg, ldp=layer.ldp,
+            rows=nd, nchunk=b.nchunk)
+
+    def run(self, eng, b, cache, layer):
+        a = self.bind(eng, b, cache, layer)
+        if b.nd:
+            hy.mingru_step(eng.f32, a)
+        if b.nseg:
+            hy.mingru_run(eng.f32, a)
+
+
+class MixerPair(SandwichMixer):
+    """Attention and a gated recurrence side by side: one input projection,
+    their outputs beside each other in eng.o, one launch for both output
+    projections into the halves of eng.y.  The norms of the halves and their
+    sum are left to the staging of the next projection."""
+    kind = "parallel"
+
+    def __init__(self, eng, spec, pk: Packer, p: str):
+        self.spec = spec
+        l, r = self.parts = [
+            MIXERS[s.kind](eng, s, pk, f"{p}{k}.")
+            for k, s in (("left", spec.left), ("right", spec.right))]
+        self.IN = tuple(f"{k}.{n}" for k, m in (("left", l), ("right", r))
+                        for n in m.IN)
+        self.tile_pairs = l.tile_pairs
+        at = sum(pk.w[f"{p}left.{n}"].shape[0] for n in l.IN)
+        self.ldo = l.ldo + r.ldo
+        l.args.put(ldo=self.ldo)
+        r.args.put(ldo=self.ldo, **{o: getattr(r.args, o) + at
+                                    for o in ("oz", "ox", "og")})
+        self.wo = torch.cat([m.wo.flatten() for m in (l, r)])
+        self.W = l.wo.shape[0]
+        self.wl = self.wo[:l.wo.numel()].view_as(l.wo)
+        l.wo = r.wo = None
+        self.gl, self.gr = pk.f32(p + "left.out"), pk.f32(p + "right.out")
+
+    def new_cache(self, eng):
+        return tuple(m.new_cache(eng) for m in self.parts)
+
+    def sizes(self, eng, rows):
+        a, b = (m.sizes(eng, rows) for m in self.parts)
+        return {**{k: max(a.get(k, 0), b.get(k, 0)) for k in {*a, *b}},
+                "o": rows * self.ldo}
+
+    def run(self, eng, b, cache, layer):
+        l, r = self.parts
+        a = r.bind(eng, b, cache[1], layer).put(out=eng.o[l.ldo:])
+        l.run(eng, b, cache[0], layer, beside=a)
+        if b.nseg:
+            hy.mingru_run(eng.f32, a)
+
+    def out(self, eng, b, layer):
+        l, r = self.parts
+        W, T, half = self.W, b.T, eng.PC * self.W
+        if eng.one_row(self.wl, T):
+            hy.lin_row(self.wl, None, eng.y, 0, 0.0, hin=eng.o,
+                       second=(r.ldo, l.ldo, W * l.ldo, half))
+        else:
+            hy.gemm_rows(eng.o, self.wo, eng.y, T, self.ldo, W, hy.EPI_F32,
+                         N=W, K=l.ldo, Z=2, xz=l.ldo, wz=W * l.ldo, yz=half,
+                         K2=r.ldo)
+
+    def halves(self, eng):
+        """How the staging after it puts the output together."""
+        return dict(y2=eng.y[1], gb=self.gl, gb2=self.gr)
+
+
+class SSD(SandwichMixer):
+    kind = "mamba2"
+
+    def __init__(self, eng, spec, pk: Packer, p: str):
+        self.spec, self.IN = spec, spec.inputs
+        s = spec
+        if s.state > 8192 or s.norm_groups > hy.MAX_GROUPS:
+            raise ValueError(f"mamba2: state {s.state} or norm_groups "
+                             f"{s.norm_groups} exceed the built kernels")
+        self.ldo = pad_to(s.inner, 64)
+        self.wo = pk.rows([p + "o"], s.inner)
+        self.norm = pk.f32(p + "norm")
+        self.cw = pk.f32(p + "conv").t().contiguous()
+        self.cb, self.dtb = pk.f32(p + "conv.b"), pk.f32(p + "dt_bias")
+        self.rate = torch.from_numpy(-np.exp(np.asarray(
+            pk.w[p + "A_log"], np.float64)).astype(np.float32)).to(pk.device)
+        self.D = pk.f32(p + "D")
+        self.args = hy.SsdArgs().put(
+            cw=self.cw, cb=self.cb, dtb=self.dtb, rate=self.rate, D=self.D,
+            oz=0, ox=s.inner, odt=s.inner + s.channels, H=s.heads,
+            G=s.groups, N=s.state, vd=s.vdim, C=s.channels, taps=s.conv,
+            nvt=-(-s.vdim // 64))
+
+    def new_cache(self, eng):
+        n, s = eng.cache.num_slots, self.spec
+        kw = dict(dtype=torch.float32, device=eng.device)
+        return (torch.zeros(n, s.heads, s.state, s.vdim, **kw),
+                torch.zeros(n, s.conv, s.channels, **kw))
+
+    def sizes(self, eng, rows):
+        s = self.spec
+        return dict(o=rows * self.ldo, raw=rows * s.inner,
+                    u=rows * s.channels, gi=rows * s.heads,
+                    gF=rows * s.heads,
+                    U=eng.max_chunks(rows) * s.heads * s.state * s.vdim)
+
+    def run(self, eng, b, cache, layer):
+        nd = b.nd
+        a = self.args.put(
+            P=eng.P, S=cache[0], ring=cache[1], u=eng.u, dt=eng.gi, L=eng.gF,
+            U=eng.U, o=eng.raw, slot=b.slot, pos=b.pos,
+            seg_row0=b.seg_row0[nd:], seg_len=b.seg_len[nd:],
+            seg_slot=b.seg_slot[nd:], seg_pos0=b.seg_pos0[nd:],
+            seg_chunk0=b.seg_chunk0, chunk_row0=b.chunk_row0,
+            chunk_len=b.chunk_len, chunk_seg=b.chunk_seg, ldp=layer.ldp,
+            rows=max(nd, 1), nseg=b.nseg, nchunk=b.nchunk)
+        if nd:
+            hy.ssd_step(a)
+        if b.nseg:
+            hy.ssd_run(a)
+
+    def out(self, eng, b, layer):
+        """Normed in parts, projected."""
+        eng.normed_linear(self.wo, eng.o, eng.y, b.T, eng.raw,
+                          self.spec.inner, self.norm,
+                          groups=self.spec.norm_groups)
 
 
 class RGLRU(SandwichMixer):
@@ -591,6 +789,11 @@ class DenseFF:
         self.up[:spec.ff].copy_(up)
         self.down = pk.rows([p + "down"], spec.ff)
         self.coef = pk.f32(p + "act") if spec.act == "polynorm" else None
+        self.bias = self.down_bias = None
+        if spec.act == "gelu":
+            self.bias = torch.zeros(self.ffp, device=pk.device)
+            self.bias[:spec.ff].copy_(pk.raw(p + "up.b"))
+            self.down_bias = pk.f32(p + "down.b")
         self.act_floats = self.ffp
         self.p_floats = self.ffp if self.coef is not None else 0
 
@@ -616,4 +819,4 @@ class RoutedFF:
 
 FEED_FORWARDS = {"dense": DenseFF, "moe": RoutedFF}
 MIXERS = {c.kind: c for c in (LatentAttention, MLSTM, GroupedAttention,
-                              RGLRU, Lightning)}
+                              MinGRU, MixerPair, SSD, RGLRU, Lightning)}

@@ -28,7 +28,8 @@ def _numpy():
 # pass; None: the config names them)
 MODELS = {t: (_dense, _numpy, ("llmops",))
           for t in ("llama", "gemma2", "qwen2", "mistral", "mixtral")}
-MODELS.update({t: (_layered, None, None) for t in ("turudra", "garupel", "fidizen")})
+MODELS.update({t: (_layered, None, None)
+               for t in ("turudra", "garupel", "fidizen", "dogalorn")})
 
 
 def _entry(config):

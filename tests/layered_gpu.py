@@ -14,9 +14,13 @@ def engine(cfg, w, dtype="fp32", max_seq=320, max_batch=4, **kw):
 
     m = LayeredModel(LayeredConfig.from_dict(cfg), w, dtype=dtype,
                      max_seq=max_seq, max_batch=max_batch, **kw)
-    for c in m.caches:
-        for t in (c if isinstance(c, tuple) else (c,)):
-            t.fill_(float("nan"))
+    def spoil(c):
+        if isinstance(c, tuple):
+            for t in c:
+                spoil(t)
+        else:
+            c.fill_(float("nan"))
+    spoil(tuple(m.caches))
     return m
 
 
