@@ -96,11 +96,13 @@ def attention(w, p, m, h, eps, past):
     if past is not None:
         k, v = np.concatenate([past[0], k]), np.concatenate([past[1], v])
     rel, temp = w[p + "rel"], w[p + "temp"]
+    buckets = np.array([bucket(b, len(rel), m["bias_max"])
+                        for b in range(min(n + T, size))])
     out = np.zeros((T, H, d), h.dtype)
     for t in range(T):
         i = n + t
         js = [j for j in range(i + 1) if visible(i, j, size)]
-        bias = rel[[bucket(i - j, len(rel), m["bias_max"]) for j in js]]
+        bias = rel[buckets[i - np.array(js)]]
         for a in range(H):
             g = a // (H // G)
             s = k[js, g] @ q[t, a] * m["scale"] * temp[a] + bias[:, a]
