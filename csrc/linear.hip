@@ -747,8 +747,7 @@ DEVINL float gelu_f(float v) {
 template <typename T, int MODE, int U, int NR, int HS = 0>
 __global__ void __launch_bounds__(LIN_NT) k_lin_row(LinRowArgs a) {
   extern __shared__ __attribute__((aligned(16))) char smem[];
-  __shared__ float red[MODE == ROW_GROUPS ? MAX_GROUPS
-                                          : LIN_NT / 64 * (MODE == ROW_POLY ? 3 : 1)];
+  __shared__ float red[LIN_NT / 64 * (MODE == ROW_POLY ? 3 : 1)];
   constexpr int V = El<T>::V, S = 64 * V, NK = 8 / NR;
   T* xs = (T*)smem;
   const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
@@ -786,7 +785,7 @@ __global__ void __launch_bounds__(LIN_NT) k_lin_row(LinRowArgs a) {
       if (a.hout && first) ((T*)a.hout)[i] = v;
     });
   } else if constexpr (MODE == ROW_GROUPS) {
-    stage_groups<LIN_NT>(a.s, a.groups, row, red,
+    stage_groups<LIN_NT>(a.s, a.groups, row, (float*)(xs + Kp),
                          [&](int i, float f) { xs[i] = El<T>::st(f); });
   } else if constexpr (MODE == ROW_POLY) {
     const int W = a.s.W;
@@ -1240,9 +1239,11 @@ static hipError_t lin_row_nr(const LinRowArgs& a, hipStream_t s) {
   int blocks = (a.N + per - 1) / per;
   const int rounds = (blocks + 511) / 512;       // alike in every block
   blocks = (blocks + rounds - 1) / rounds;
+  size_t lds = MODE == ROW_PLAIN ? 0 : (size_t)a.s.Kp * sizeof(T);
+  if (MODE == ROW_GROUPS) lds += MAX_GROUPS * sizeof(float);   // sums of parts
   hipLaunchKernelGGL((k_lin_row<T, MODE, U, NR, HS>),
                      dim3(blocks, MODE == ROW_PLAIN ? a.Z : 1), dim3(LIN_NT),
-                     MODE == ROW_PLAIN ? 0 : (size_t)a.s.Kp * sizeof(T), s, a);
+                     lds, s, a);
   return hipGetLastError();
 }
 
