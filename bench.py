@@ -23,7 +23,7 @@ sys.path.insert(0, os.path.dirname(os.path.abspath(__file__)))
 
 
 COMPARE = ("turudra-2k", "turudra-4k", "garupel-2k", "garupel-4k",
-           "fidizen-2k", "fidizen-4k")
+           "fidizen-2k", "fidizen-4k", "dogalorn-2k", "dogalorn-4k")
 
 
 def compare(cases, steps, warmup, prompt=2048, batches=(1, 4, 16)):
@@ -31,8 +31,10 @@ def compare(cases, steps, warmup, prompt=2048, batches=(1, 4, 16)):
     synthetic prompts.  Beside each design stands the closest other model
     of equal width, heads and layer runs.  Windowed latent attention stands
     beside unwindowed one, a dense feed-forward beside two experts, both
-    chosen, and a shared one that hold as much; other designs stand beside
-    a transformer.  An MoE one gets one more expert
+    chosen, and a shared one that hold as much; pairs of attention and
+    recurrence beside the attention alone, state-space layers beside linear
+    attention with as large a state; other designs stand beside a
+    transformer.  An MoE one gets one more expert
     and one more choice, so its experts match the design's routed + shared
     ones in stored and in active parameters; a dense one gets two thirds of
     the hidden size, so its three matrices match the design's two."""
@@ -65,9 +67,34 @@ def compare(cases, steps, warmup, prompt=2048, batches=(1, 4, 16)):
             "width": c.hidden_size, "norm": {"eps": 1e-6},
             "residual_mult": 0.5, "layers": [layer(l) for l in c.layers]})
 
+    def grouped_design(c):
+        heads = next(l.mixer.left.heads for l in c.layers
+                     if l.mixer.kind == "parallel")
+
+        def layer(l):
+            m = l.mixer
+            if m.kind == "parallel":
+                d = m.left.to_dict()
+                kind, mix = "attention", {
+                    **{k: d[k] for k in ("heads", "kv_heads", "dim", "vdim",
+                                         "scale")},
+                    "q_temp": {"coef": 0.1, "every": 2048}}
+            else:
+                kind, mix = "lightning", dict(
+                    heads=heads, dim=m.state, vdim=m.inner // heads,
+                    decay=[1 - 2.0 ** (-3 - h % 6) for h in range(heads)])
+            return {"type": kind, "mixer": mix,
+                    "mlp": {"kind": "dense", "ff": l.mlp.ff}}
+        return "garupel", L.ModelConfig.from_hf_dict({
+            "architecture": "Garupel", "vocab": c.vocab_size,
+            "width": c.hidden_size, "norm": {"eps": 1e-6},
+            "layers": [layer(l) for l in c.layers]})
+
     def closest(c):
         if c.model_type == "fidizen":
             return latent_design(c)
+        if c.model_type == "dogalorn":
+            return grouped_design(c)
         att, ff = c.layers[0].mixer, c.layers[0].mlp
         kw = dict(vocab_size=c.vocab_size, hidden_size=c.hidden_size,
                   num_hidden_layers=len(c.runs), head_dim=128,
@@ -163,9 +190,10 @@ def main():
                          "decode throughput of the layer-list designs "
                          "beside the closest other model of equal size; "
                          "cases turudra-2k (or 2k), turudra-4k, garupel-2k, "
-                         "garupel-4k, fidizen-2k, fidizen-4k (default all), "
-                         "each optionally with :turudra, :mixtral, :garupel, "
-                         ":qwen2 or :fidizen for one side only")
+                         "garupel-4k, fidizen-2k, fidizen-4k, dogalorn-2k, "
+                         "dogalorn-4k (default all), each optionally with "
+                         ":turudra, :mixtral, :garupel, :qwen2, :fidizen or "
+                         ":dogalorn for one side only")
     args = ap.parse_args()
     if args.compare is not None:
         return compare(args.compare or COMPARE, args.steps, args.warmup)
