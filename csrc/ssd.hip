@@ -51,12 +51,12 @@ DEVINL int c_channel(const SsdArgs& a, int h) {
 }
 
 // ---- one token per row ------------------------------------------------
-// 16 waves per (head, column tile): a wave's lanes own the 64 columns, the
-// rows of S are dealt to the waves.  The first rows are on their way while
-// the convolutions are worked out.
-#define SW 16
-#define SPRE 8
+// SW waves per (head, column tile): a wave's lanes own the 64 columns, the
+// rows of S are dealt to the waves.  The first 128 rows are on their way
+// while the convolutions are worked out.
+template <int SW>
 __global__ void __launch_bounds__(64 * SW) k_ssd_step(SsdArgs a) {
+  constexpr int SPRE = 128 / SW;
   extern __shared__ float sm[];           // B[N], C[N], part[SW*64]
   const int r = blockIdx.y;
   const int h = blockIdx.x / a.nvt, vtile = blockIdx.x - h * a.nvt;
@@ -420,13 +420,19 @@ static bool bad_shape(const SsdArgs& a) {
          a.C != a.H * a.vd + 2 * a.G * a.N || a.taps < 1;
 }
 
+template <int SW> static hipError_t step_go(const SsdArgs& a, hipStream_t s) {
+  const size_t lds = (size_t)(2 * a.N + SW * VT) * sizeof(float);
+  RAISE_LDS(k_ssd_step<SW>);
+  hipLaunchKernelGGL(k_ssd_step<SW>, dim3(a.H * a.nvt, a.rows), dim3(64 * SW),
+                     lds, s, a);
+  return hipGetLastError();
+}
+
 extern "C" hipError_t launch_ssd_step(const SsdArgs* a, hipStream_t s) {
   if (bad_shape(*a)) return hipErrorInvalidValue;
-  const size_t lds = (size_t)(2 * a->N + SW * VT) * sizeof(float);
-  RAISE_LDS(k_ssd_step);
-  hipLaunchKernelGGL(k_ssd_step, dim3(a->H * a->nvt, a->rows), dim3(64 * SW),
-                     lds, s, *a);
-  return hipGetLastError();
+  // two blocks of 16 waves fill a CU; beyond that more, smaller ones
+  return a->H * a->nvt * a->rows <= 512 ? step_go<16>(*a, s)
+                                        : step_go<4>(*a, s);
 }
 
 // convolutions, local sums, scan, outputs over the segments' rows

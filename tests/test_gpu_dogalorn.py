@@ -300,6 +300,25 @@ def test_state_space_alone(a):
     check_alone(config([(ssd(**a), None)]), seed=a.get("state", 0))
 
 
+@pytest.mark.parametrize("a", [
+    dict(heads=64, vdim=8, groups=4), dict(heads=24, vdim=70, state=150)])
+def test_state_space_decode_batches(a):
+    """Few and many blocks in the step of single tokens, beside a run."""
+    cfg = config([(ssd(**a), None)])
+    w, t = weights(cfg), tokens(cfg, 60)
+    want, _ = Oracle(cfg, w).run(t)
+    m = engine(cfg, w, max_batch=17)
+    seqs = [m.open_sequence() for _ in range(17)]
+    m.step([entry(s, t[:2 * k + 1], []) for k, s in enumerate(seqs)])
+    for n in range(4):
+        got = m.step([entry(s, t[2 * k + 1 + n:][:1])
+                      for k, s in enumerate(seqs)]).cpu().numpy()
+        assert worst(got, want[1 + n:34 + n:2]) < EXACT
+    got = m.step([entry(s, t[2 * k + 5:][:1 if k else 3])
+                  for k, s in enumerate(seqs)]).cpu().numpy()
+    assert worst(got, np.concatenate([want[5:8], want[7:38:2]])) < EXACT
+
+
 @pytest.mark.parametrize("ff", [1, 40, 64, 200, 5000])
 def test_dense_alone(ff):
     """A mixer that writes nothing."""
