@@ -34,7 +34,7 @@
 //   [4096, ...) data slots [2][8][slot_bytes]
 //
 // A bounded spin (s_sleep backoff) turns a dead peer into a sticky err
-// flag + clean return instead of a GPU hang (gpurun strike protection);
+// flag + clean return instead of a GPU hang;
 // the host raises on err at the next sync point.
 
 #include <hip/hip_runtime.h>
